@@ -88,8 +88,45 @@ LAB_SYMBOLS = {
     "aq_lab_set_gemv_skip_weights": (_int, [_int]),
 }
 
+# every symbol include/astrai_seq.h declares (libastrai_seq.so)
+SEQ_LIB_PATH = os.environ.get("ASTRAI_SEQ_LIB") or os.path.join(_HERE, "lib", "libastrai_seq.so")
+_f32 = ctypes.c_float
+SEQ_SYMBOLS = {
+    "aqs_embed": (_int, [_vp, _vp, _int, _vp, _i64, _i64, _i64, _vp]),
+    "aqs_add_rmsnorm": (_int, [_vp, _vp, _i64, _int, _f32, _vp, _f32, _vp, _i64, _i64, _vp]),
+    "aqs_clamped_glu": (_int, [_vp, _i64, _int, _f32, _vp, _i64, _i64, _vp]),
+    "aqs_gated_group_norm": (_int, [_vp, _vp, _i64, _int, _vp, _f32, _vp, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_head_norm_gate": (_int, [_vp, _vp, _i64, _int, _vp, _f32, _f32, _vp, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_gemv_ok": (_int, [_i64, _i64, _i64]),
+    "aqs_gemv": (_int, [_int, _int, _int, _vp, _i64, _vp, _vp, _f32, _i64, _vp, _vp, _f32, _f32, _vp, _vp, _i64,
+        _i64, _i64, _i64, _vp]),
+    "aqs_conv_silu": (_int, [_vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_conv_push": (_int, [_vp, _i64, _int, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_delta_prep": (_int, [_vp, _i64, _vp, _i64, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp,
+        _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_delta_scan": (_int, [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64,
+        _vp]),
+    "aqs_delta_step": (_int, [_vp, _i64, _i64, _i64, _i64, _i64, _int, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _i64,
+        _vp, _vp, _vp, _f32, _f32, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_ssd_scan": (_int, [_vp, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64,
+        _i64, _vp]),
+    "aqs_ssd_step": (_int, [_vp, _i64, _i64, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64,
+        _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_attn_prep": (_int, [_vp, _i64, _i64, _i64, _i64, _int, _vp, _vp, _f32, _vp, _i64, _i64, _vp, _vp, _i64,
+        _i64, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_attn_window_ok": (_int, [_int, _i64, _i64, _i64]),
+    "aqs_attn_window": (_int, [_vp, _vp, _vp, _int, _f32, _i64, _vp, _i64, _f32, _vp, _vp, _i64, _i64, _i64, _vp,
+        _i64, _i64, _i64, _i64, _i64, _i64, _i64, _int, _vp]),
+    "aqs_attn_decode_ok": (_int, [_i64, _i64, _i64]),
+    "aqs_attn_decode_slices": (_i64, [_i64, _i64]),
+    "aqs_attn_decode": (_int, [_vp, _i64, _i64, _i64, _i64, _i64, _int, _vp, _vp, _f32, _vp, _i64, _i64, _f32,
+        _i64, _f32, _vp, _vp, _i64, _i64, _i64, _vp, _vp, _vp, _i64, _vp, _i64, _i64, _i64, _i64, _i64, _i64,
+        _vp]),
+}
+
 _lib = None
 _lab = None
+_seq = None
 
 
 def load() -> ctypes.CDLL:
@@ -108,6 +145,23 @@ def load() -> ctypes.CDLL:
         fn.restype = res
         fn.argtypes = args
     _lib = lib
+    return lib
+
+
+def load_seq() -> ctypes.CDLL:
+    """The hybrid-decoder kernels; raises if they have not been built."""
+    global _seq
+    if _seq is not None:
+        return _seq
+    if not os.path.exists(SEQ_LIB_PATH):
+        raise RuntimeError(f"{SEQ_LIB_PATH} is missing: build it with `python -m khaosz_amd.build` "
+                           "(hipcc, --offload-arch=gfx950). There is no fallback path.")
+    lib = ctypes.CDLL(SEQ_LIB_PATH)
+    for name, (res, args) in SEQ_SYMBOLS.items():
+        fn = getattr(lib, name)
+        fn.restype = res
+        fn.argtypes = args
+    _seq = lib
     return lib
 
 
@@ -145,11 +199,19 @@ class lab_library:
         return False
 
 
+def error_string(code: int) -> str:
+    if _lib is None and not os.path.exists(LIB_PATH):  # only the hybrid kernels are built
+        return {-1: "a required pointer is NULL", -2: "bad shape", -3: "unknown dtype code",
+                -4: "pointer or leading dimension is not 16-byte aligned",
+                -6: "size beyond what the kernels index"}.get(code, "hip error")
+    return load().aq_error_string(code).decode()
+
+
 def check(code: int, what: str) -> None:
     """Reference convention: errors surface as Python exceptions
     (e.g. astrai/parallel/module.py:34-37), never as return codes."""
     if code != 0:
-        msg = load().aq_error_string(code).decode()
+        msg = error_string(code)
         if code in (-2, -3, -4, -6):
             raise ValueError(f"{what}: {msg} (code {code})")
         raise RuntimeError(f"{what}: {msg} (code {code})")

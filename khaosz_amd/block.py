@@ -87,15 +87,17 @@ class PagedKV:
     table tensor is first bound: a table that was changed in place (a page mapped as a sequence grew)
     must be bound again with ``refresh=True`` -- or be a new tensor, as the reference's
     ``make_table_tensor`` produces for every step.
+    ``v_head_dim``: the values' head size where it differs from the keys'.
     ``seq_lens`` (int64 ``[B]`` on the device, optional): the positions each sequence may attend to
     in a single-token step whose sequences sit at different positions; the attention kernels apply it as
     the reference's position mask (transformer.py:40-46)."""
 
     def __init__(self, n_pages: int, page_size: int, n_kv_heads: int, head_dim: int, device, dtype,
-                 n_layers: int = 1):
+                 n_layers: int = 1, v_head_dim: Optional[int] = None):
         self.page_size = page_size
         self.k_layers = torch.zeros((n_layers, n_pages, page_size, n_kv_heads, head_dim), device=device, dtype=dtype)
-        self.v_layers = torch.zeros_like(self.k_layers)
+        self.v_layers = torch.zeros((n_layers, n_pages, page_size, n_kv_heads, v_head_dim or head_dim), device=device,
+                                    dtype=dtype)
         self.page_table: Optional[Tensor] = None
         self._attn_ws: Optional[Tensor] = None
         self._mapped = None      # host bool [B, P]

@@ -1,0 +1,658 @@
+// Sliding-window grouped-query attention on a paged cache whose keys (D) and values (E) may differ in size.
+//
+//   prep      per head vector of a new token: RMS norm of q and k (plain weight), then interleaved rotation of the
+//             first `rot` dimensions; q is stored, k and v go into their page slots.
+//   prefill   the new tokens at positions pos .. pos + S over everything cached, matrix cores (bf16).
+//   simple    the same for any sizes and for fp32: one wavefront per query and head.
+//   decode    one new token per sequence: prep's work, and the attention over slices of 64 positions in separate
+//             workgroups; `combine` merges the slices.
+//
+// Position i sees j with 0 <= i - j < window.  A head's output is multiplied by sigmoid(gate) and a constant before it
+// is stored.  Positions come from device memory, so that one captured launch serves every step.
+#include "seq_common.h"
+
+namespace sq {
+
+struct AttnDims {
+  const int* pos;        // [B]
+  const int64_t* table;  // [B, P]
+  int64_t P, n_pages;
+  int S, H, G, D, E, page, window;
+};
+
+struct PrepArgs {
+  AttnDims a;
+  const float* q_norm;  // [D]
+  const float* k_norm;
+  const float* cs;      // [max_pos, rot / 2, 2] cos, sin
+  int64_t ld, o_q, o_k, o_v, max_pos;
+  int64_t M;
+  int rot;
+  float eps;
+};
+
+constexpr int HEAD_PAIRS = 4;  // element pairs per lane: head vectors of up to 512
+
+template <typename T>
+__device__ __forceinline__ int64_t page_row(const AttnDims& a, int b, int t) {
+  const int64_t lp = t / a.page;
+  const int64_t phys = lp < a.P ? a.table[(int64_t)b * a.P + lp] : -1;
+  return phys >= 0 && phys < a.n_pages ? phys * a.page + t % a.page : -1;
+}
+
+// RMS norm and rotation of one head vector by one wavefront: lane l holds the pairs l, l + 64, ...
+template <typename T>
+__device__ __forceinline__ void norm_rotate(const T* src, const float* w, const float* cs, int D, int rot, float eps, int lane,
+                                            float (&o)[HEAD_PAIRS][2]) {
+  float ss = 0.0f;
+#pragma unroll
+  for (int i = 0; i < HEAD_PAIRS; ++i) {
+    const int d = 2 * (i * 64 + lane);
+    o[i][0] = d < D ? to_f32(src[d]) : 0.0f;
+    o[i][1] = d + 1 < D ? to_f32(src[d + 1]) : 0.0f;
+    ss += o[i][0] * o[i][0] + o[i][1] * o[i][1];
+  }
+  const float r = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
+#pragma unroll
+  for (int i = 0; i < HEAD_PAIRS; ++i) {
+    const int d = 2 * (i * 64 + lane);
+    if (d >= D) continue;
+    const float u = o[i][0] * r * w[d], v = d + 1 < D ? o[i][1] * r * w[d + 1] : 0.0f;
+    if (d + 1 < rot) {
+      const float c = cs[d], s = cs[d + 1];
+      o[i][0] = u * c - v * s;
+      o[i][1] = v * c + u * s;
+    } else {
+      o[i][0] = u;
+      o[i][1] = v;
+    }
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs p, const T* proj, T* q_out, T* kc, T* vc) {
+  const AttnDims& a = p.a;
+  const int items = a.H + 2 * a.G;
+  const int64_t it = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (it >= p.M * items) return;
+  const int lane = threadIdx.x & 63, item = (int)(it % items);
+  const int64_t m = it / items;
+  const int b = (int)(m / a.S), t = a.pos[b] + (int)(m % a.S);
+  const T* row = proj + m * p.ld;
+  if (item >= a.H + a.G) {
+    const int g = item - a.H - a.G;
+    const int64_t pr = page_row<T>(a, b, t);
+    if (pr < 0) return;
+    for (int e = lane; e < a.E; e += 64) vc[(pr * a.G + g) * a.E + e] = row[p.o_v + g * a.E + e];
+    return;
+  }
+  const bool is_q = item < a.H;
+  const int h = is_q ? item : item - a.H;
+  float o[HEAD_PAIRS][2];
+  const int tc = t < p.max_pos ? t : (int)p.max_pos - 1;
+  norm_rotate<T>(row + (is_q ? p.o_q : p.o_k) + h * a.D, is_q ? p.q_norm : p.k_norm, p.cs + (int64_t)tc * p.rot, a.D, p.rot, p.eps,
+                 lane, o);
+  T* dst;
+  if (is_q) {
+    dst = q_out + (m * a.H + h) * a.D;
+  } else {
+    const int64_t pr = page_row<T>(a, b, t);
+    if (pr < 0) return;
+    dst = kc + (pr * a.G + h) * a.D;
+  }
+#pragma unroll
+  for (int i = 0; i < HEAD_PAIRS; ++i) {
+    const int d = 2 * (i * 64 + lane);
+    if (d < a.D) dst[d] = from_f32<T>(o[i][0]);
+    if (d + 1 < a.D) dst[d + 1] = from_f32<T>(o[i][1]);
+  }
+}
+
+struct AttnOut {
+  const void* gate;  // T, [M, ld_gate] one number per head, or null
+  int64_t ld_gate, ldo;
+  float scale;       // of the output
+};
+template <typename T>
+__device__ __forceinline__ float head_factor(const AttnOut& o, int64_t m, int h) {
+  return o.gate ? o.scale * sigmoid(to_f32(reinterpret_cast<const T*>(o.gate)[m * o.ld_gate + h])) : o.scale;
+}
+
+constexpr float MASKED = -1.0e30f;
+constexpr float LOG2E = 1.44269504088896341f;
+
+// ---------------------------------------------------------------------------------------------- any sizes
+constexpr int SIMPLE_MAX = 512;
+
+template <typename T>
+__global__ __launch_bounds__(256) void attn_simple_kernel(AttnDims a, AttnOut o, float scale, const T* q, const T* kc, const T* vc,
+                                                          T* out, int64_t M) {
+  __shared__ float q_s[4][SIMPLE_MAX], p_s[4][64];
+  __shared__ int row_s[4][64];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int64_t v = (int64_t)blockIdx.x * 4 + wave;
+  const bool live = v < M * a.H;
+  const int64_t m = live ? v / a.H : 0;
+  const int h = live ? (int)(v % a.H) : 0, g = h / (a.H / a.G), b = (int)(m / a.S);
+  const int i = a.pos[b] + (int)(m % a.S), lo = i - a.window + 1 > 0 ? i - a.window + 1 : 0;
+  for (int d = lane; d < a.D; d += 64) q_s[wave][d] = to_f32(q[(m * a.H + h) * a.D + d]) * scale;
+  float acc[SIMPLE_MAX / 64], mx = MASKED, l = 0.0f;
+#pragma unroll
+  for (int e = 0; e < SIMPLE_MAX / 64; ++e) acc[e] = 0.0f;
+  // the wavefronts of a workgroup may walk different numbers of tiles: everything below is per wavefront, LDS included
+  __builtin_amdgcn_wave_barrier();
+  for (int t0 = lo; live && t0 <= i; t0 += 64) {
+    const int t = t0 + lane;
+    const int64_t pr = t <= i ? page_row<T>(a, b, t) : -1;
+    float s = t <= i ? 0.0f : -INFINITY;
+    if (pr >= 0) {
+      const T* k = kc + (pr * a.G + g) * a.D;
+      for (int d = 0; d < a.D; ++d) s = fmaf(to_f32(k[d]), q_s[wave][d], s);
+    }
+    const float mn = fmaxf(mx, wave_max(s)), al = expf(mx - mn), pv = expf(s - mn);
+    l = l * al + wave_sum(pv);
+    mx = mn;
+    p_s[wave][lane] = pv;
+    row_s[wave][lane] = (int)pr;
+    __builtin_amdgcn_wave_barrier();
+#pragma unroll
+    for (int e = 0; e < SIMPLE_MAX / 64; ++e) acc[e] *= al;
+    const int n = i - t0 + 1 < 64 ? i - t0 + 1 : 64;
+    for (int k = 0; k < n; ++k) {
+      const int r = row_s[wave][k];
+      if (r < 0) continue;
+      const float w = p_s[wave][k];
+      const T* vr = vc + ((int64_t)r * a.G + g) * a.E;
+#pragma unroll
+      for (int e = 0; e < SIMPLE_MAX / 64; ++e)
+        if (e * 64 + lane < a.E) acc[e] = fmaf(w, to_f32(vr[e * 64 + lane]), acc[e]);
+    }
+    __builtin_amdgcn_wave_barrier();
+  }
+  if (!live) return;
+  const float f = head_factor<T>(o, m, h) / l;
+#pragma unroll
+  for (int e = 0; e < SIMPLE_MAX / 64; ++e)
+    if (e * 64 + lane < a.E) out[m * o.ldo + h * a.E + e * 64 + lane] = from_f32<T>(acc[e] * f);
+}
+
+// ---------------------------------------------------------------------------------------------- prefill, matrix cores
+// The arrangement of the causal kernel of attn_prefill.hip: workgroup = (128 queries, head), 4 wavefronts of 32
+// queries, key blocks of 64; S^T = K Q^T and O^T = V^T P^T with v_mfma_f32_32x32x16_bf16, so that a lane keeps one
+// query from its scores to its output.  Here the sizes are padded to DP and EP with zeros in LDS, key blocks run
+// from the window's first to the query's own, and a page holds whole key blocks (page % 64 == 0).
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef float f32x16 __attribute__((ext_vector_type(16)));
+constexpr int WQ = 128, WK = 64;
+
+template <int DP, int EP>
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DP + EP <= 256 ? 2 : 1))) void attn_window_kernel(
+    AttnDims a, AttnOut oo, float scale_log2e, const uint16_t* q, const uint16_t* kc, const uint16_t* vc, uint16_t* out, int B) {
+  constexpr int KP = DP + 8, VP = WK + 4, DS = DP / 16, DT = EP / 32, KC = DP / 32, VC = EP / 32;
+  extern __shared__ __align__(16) uint16_t lds[];
+  uint16_t* ks = lds;            // [WK][KP]
+  uint16_t* vt = lds + WK * KP;  // [EP][VP]
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int col = lane & 31, g2 = lane >> 5;
+  const int S = a.S, nqb = (S + WQ - 1) / WQ, per = a.H * B;
+  const int qblk = nqb - 1 - (int)blockIdx.x / per, h = ((int)blockIdx.x % per) % a.H, b = ((int)blockIdx.x % per) / a.H;
+  const int kvh = h / (a.H / a.G), start = a.pos[b];
+  const int q0 = qblk * WQ, qs = q0 + wave * 32 + col;         // this lane's query within the new tokens
+  const int qp = start + qs, qw = start + q0 + wave * 32;      // its position; the wavefront's first
+  const int64_t tok0 = (int64_t)b * S;
+  const int last = start + (q0 + WQ < S ? q0 + WQ : S) - 1;    // position of the workgroup's last query
+  const int first = start + q0 - a.window + 1 > 0 ? start + q0 - a.window + 1 : 0;
+  const int D = a.D, E = a.E;
+
+  uint4 qf[DS];
+  {
+    const uint16_t* src = q + ((tok0 + (qs < S ? qs : S - 1)) * a.H + h) * D + g2 * 8;
+#pragma unroll
+    for (int st = 0; st < DS; ++st)
+      qf[st] = st * 16 + g2 * 8 < D ? *reinterpret_cast<const uint4*>(src + st * 16) : make_uint4(0, 0, 0, 0);
+  }
+  uint4 kr[KC], vr[VC];
+  auto fetch = [&](int j) __attribute__((always_inline)) {
+    const int64_t lp = (int64_t)j * WK / a.page;
+    const int64_t phys = lp < a.P ? a.table[(int64_t)b * a.P + lp] : -1;
+    const bool ok = phys >= 0 && phys < a.n_pages;
+    const int64_t base = (ok ? phys : 0) * a.page + (int64_t)j * WK % a.page;
+#pragma unroll
+    for (int c = 0; c < KC; ++c) {
+      const int idx = c * 256 + tid, key = idx / (DP / 8), ch = idx % (DP / 8);
+      kr[c] = ok && ch * 8 < D ? *reinterpret_cast<const uint4*>(kc + ((base + key) * a.G + kvh) * D + ch * 8) : make_uint4(0, 0, 0, 0);
+    }
+#pragma unroll
+    for (int c = 0; c < VC; ++c) {
+      const int ch = wave + 4 * c;
+      vr[c] = ok && ch * 8 < E ? *reinterpret_cast<const uint4*>(vc + ((base + lane) * a.G + kvh) * E + ch * 8) : make_uint4(0, 0, 0, 0);
+    }
+  };
+  auto stage = [&](int j) __attribute__((always_inline)) {
+#pragma unroll
+    for (int c = 0; c < KC; ++c) {
+      const int idx = c * 256 + tid, key = idx / (DP / 8), ch = idx % (DP / 8);
+      *reinterpret_cast<uint4*>(&ks[key * KP + ch * 8]) = kr[c];
+    }
+    // V transposed, two keys per 4-byte store (neighbouring lanes swap halves).  Rows past the last position hold
+    // whatever the page held before: a probability of zero must not meet a NaN there.
+    const bool past = j * WK + lane > last;
+    const bool odd = lane & 1;
+    const uint32_t sel = odd ? 0x03020706u : 0x05040100u;
+#pragma unroll
+    for (int c = 0; c < VC; ++c) {
+      uint32_t* dst = reinterpret_cast<uint32_t*>(&vt[((wave + 4 * c) * 8 + (odd ? 1 : 0)) * VP + (lane & ~1)]);
+      const uint32_t w[4] = {past ? 0 : vr[c].x, past ? 0 : vr[c].y, past ? 0 : vr[c].z, past ? 0 : vr[c].w};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const uint32_t other = (uint32_t)__builtin_amdgcn_mov_dpp((int)w[e], 0xB1, 0xf, 0xf, true);
+        dst[e * VP] = __builtin_amdgcn_perm(other, w[e], sel);
+      }
+    }
+  };
+
+  f32x16 o[DT];
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+    for (int r = 0; r < 16; ++r) o[dt][r] = 0.0f;
+  float m = MASKED, l = 0.0f;
+  const int j0 = first / WK, j1 = last / WK;
+  fetch(j0);
+  for (int j = j0; j <= j1; ++j) {
+    __syncthreads();
+    stage(j);
+    __syncthreads();
+    if (j < j1) fetch(j + 1);
+    const int kb = j * WK;
+    // wavefront-uniform: every key ahead of every query, or behind every window
+    if (kb > qw + 31 || kb + WK - 1 < qw - a.window + 1) continue;
+    f32x16 s[2];
+#pragma unroll
+    for (int r = 0; r < 16; ++r) s[0][r] = s[1][r] = 0.0f;
+    const uint16_t* k0 = &ks[col * KP + g2 * 8];
+#pragma unroll
+    for (int st = 0; st < DS; ++st) {
+      const bf16x8 qv = __builtin_bit_cast(bf16x8, qf[st]);
+      const uint4 f0 = *reinterpret_cast<const uint4*>(k0 + st * 16), f1 = *reinterpret_cast<const uint4*>(k0 + 32 * KP + st * 16);
+      s[0] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, f0), qv, s[0], 0, 0, 0);
+      s[1] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, f1), qv, s[1], 0, 0, 0);
+    }
+    // register r of tile kt is key kb + 32 kt + 8 (r / 4) + 4 g2 + r % 4
+    const bool edge = kb + WK - 1 > qw || kb < qw + 31 - a.window + 1;
+    float bm = -INFINITY;
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) s[kt][r] *= scale_log2e;
+    if (edge) {
+#pragma unroll
+      for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) {
+          const int t = kb + kt * 32 + 8 * (r / 4) + 4 * g2 + (r % 4);
+          if (t > qp || t <= qp - a.window) s[kt][r] = -INFINITY;
+        }
+    }
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+      for (int r = 0; r < 16; ++r) bm = fmaxf(bm, s[kt][r]);
+    bm = fmaxf(bm, __shfl_xor(bm, 32, 64));
+    // the running maximum is raised only when an exponent would pass 2^8 (see attn_prefill.hip)
+    const bool raise = __builtin_amdgcn_ballot_w64(bm > m + 8.0f) != 0;
+    float alpha = 1.0f;
+    if (raise) {
+      const float mn = fmaxf(m, bm);
+      alpha = __builtin_amdgcn_exp2f(m - mn);
+      m = mn;
+      l *= alpha;
+    }
+    uint4 pf[2][2];
+#pragma unroll
+    for (int kt = 0; kt < 2; ++kt) {
+      float pv[16];
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        pv[r] = __builtin_amdgcn_exp2f(s[kt][r] - m);
+        l += pv[r];
+      }
+#pragma unroll
+      for (int s2 = 0; s2 < 2; ++s2)
+        pf[kt][s2] = make_uint4(pack2(pv[8 * s2 + 0], pv[8 * s2 + 1]), pack2(pv[8 * s2 + 2], pv[8 * s2 + 3]),
+                                pack2(pv[8 * s2 + 4], pv[8 * s2 + 5]), pack2(pv[8 * s2 + 6], pv[8 * s2 + 7]));
+    }
+    if (raise) {
+#pragma unroll
+      for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) o[dt][r] *= alpha;
+    }
+#pragma unroll
+    for (int dt = 0; dt < DT; ++dt) {
+      const uint16_t* vrow = &vt[(dt * 32 + col) * VP + 4 * g2];
+#pragma unroll
+      for (int kk = 0; kk < 4; ++kk) {
+        const uint2 lo = *reinterpret_cast<const uint2*>(vrow + kk * 16), hi = *reinterpret_cast<const uint2*>(vrow + kk * 16 + 8);
+        o[dt] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(__builtin_bit_cast(bf16x8, make_uint4(lo.x, lo.y, hi.x, hi.y)),
+                                                        __builtin_bit_cast(bf16x8, pf[kk >> 1][kk & 1]), o[dt], 0, 0, 0);
+      }
+    }
+  }
+  l += __shfl_xor(l, 32, 64);
+  if (qs >= S) return;
+  const float f = head_factor<bf16>(oo, tok0 + qs, h) / l;
+  uint16_t* dst = out + (tok0 + qs) * oo.ldo + (int64_t)h * E + 4 * g2;
+#pragma unroll
+  for (int dt = 0; dt < DT; ++dt)
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (dt * 32 + 8 * r + 4 * g2 < E)
+        *reinterpret_cast<uint2*>(dst + dt * 32 + 8 * r) = make_uint2(pack2(o[dt][4 * r] * f, o[dt][4 * r + 1] * f),
+                                                                     pack2(o[dt][4 * r + 2] * f, o[dt][4 * r + 3] * f));
+}
+
+// ---------------------------------------------------------------------------------------------- decode
+constexpr int DEC_HB = 4;   // query heads of a KV head per workgroup
+constexpr int DEC_MAX = 256;
+
+// NC: 128-dimension pieces of a key; LV: lanes that share a value row (8 dimensions each)
+template <typename T, int NC, int LV>
+__global__ __launch_bounds__(256) void attn_decode_kernel(PrepArgs p, float scale_log2e, const T* proj, T* kc, T* vc, float* part, int NS) {
+  const AttnDims& a = p.a;
+  constexpr int RPP = 64 / LV, NP = 16 / RPP;  // value rows per pass, passes over a wavefront's 16 keys
+  __shared__ __align__(16) float q_s[DEC_HB][DEC_MAX];
+  __shared__ __align__(16) T kn_s[DEC_MAX], vn_s[DEC_MAX];
+  __shared__ float p_s[DEC_HB][64], m_s[DEC_HB], l_s[DEC_HB];
+  __shared__ __align__(16) float acc_s[4][DEC_HB][LV * 8];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int per = a.H / a.G, nb = (per + DEC_HB - 1) / DEC_HB;
+  int x = blockIdx.x;
+  const int kvh = x % a.G;
+  x /= a.G;
+  const int hb = x % nb;
+  x /= nb;
+  const int split = x % NS, b = x / NS;
+  const int pos = a.pos[b], lo = pos - a.window + 1 > 0 ? pos - a.window + 1 : 0;
+  const int t0 = (lo / 64 + split) * 64;
+  if (t0 > pos) return;  // uniform
+  const int D = a.D, E = a.E, h0 = kvh * per + hb * DEC_HB;
+  const int nh = per - hb * DEC_HB < DEC_HB ? per - hb * DEC_HB : DEC_HB;
+  const int64_t pr0 = page_row<T>(a, b, t0);  // 64 positions lie in one page
+  // keys and values of this wavefront's 16 positions, requested at once
+  const int kl = lane >> 4, ch = lane & 15, vl = lane / LV, vch = lane % LV;
+  Raw8<T> kreg[4][NC], vreg[NP];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      const int key = wave * 16 + i * 4 + kl, d = (c * 16 + ch) * 8;
+      if (pr0 >= 0 && t0 + key < pos && d < D) kreg[i][c].load(kc + ((pr0 + key) * a.G + kvh) * D + d);
+      else kreg[i][c].zero();
+    }
+#pragma unroll
+  for (int i = 0; i < NP; ++i) {
+    const int key = wave * 16 + i * RPP + vl, e = vch * 8;
+    if (pr0 >= 0 && t0 + key < pos && e < E) vreg[i].load(vc + ((pr0 + key) * a.G + kvh) * E + e);
+    else vreg[i].zero();
+  }
+  const T* row = proj + b * p.ld;
+  const float* cs = p.cs + (int64_t)(pos < p.max_pos ? pos : p.max_pos - 1) * p.rot;
+  float o[HEAD_PAIRS][2];
+  if (wave < nh) {
+    norm_rotate<T>(row + p.o_q + (h0 + wave) * D, p.q_norm, cs, D, p.rot, p.eps, lane, o);
+#pragma unroll
+    for (int i = 0; i < DEC_MAX / 128; ++i) {
+      const int d = 2 * (i * 64 + lane);
+      q_s[wave][d] = o[i][0] * scale_log2e;
+      q_s[wave][d + 1] = o[i][1] * scale_log2e;
+    }
+  }
+  const bool has_new = pos < t0 + 64;
+  if (has_new) {
+    if (wave == 3) {
+      norm_rotate<T>(row + p.o_k + kvh * D, p.k_norm, cs, D, p.rot, p.eps, lane, o);
+#pragma unroll
+      for (int i = 0; i < DEC_MAX / 128; ++i) {
+        const int d = 2 * (i * 64 + lane);
+        kn_s[d] = from_f32<T>(o[i][0]);
+        kn_s[d + 1] = from_f32<T>(o[i][1]);
+      }
+    }
+    if (wave == 2)
+      for (int e = lane; e < DEC_MAX; e += 64) vn_s[e] = e < E ? row[p.o_v + kvh * E + e] : from_f32<T>(0.0f);
+  }
+  __syncthreads();
+  if (has_new) {
+    const int key = pos - t0;  // the new token's row comes from LDS, and goes into its page
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int c = 0; c < NC; ++c)
+        if (wave * 16 + i * 4 + kl == key && (c * 16 + ch) * 8 < D) kreg[i][c].load(&kn_s[(c * 16 + ch) * 8]);
+#pragma unroll
+    for (int i = 0; i < NP; ++i)
+      if (wave * 16 + i * RPP + vl == key && vch * 8 < E) vreg[i].load(&vn_s[vch * 8]);
+    if (hb == 0 && pr0 >= 0) {
+      for (int d = tid; d < D; d += 256) kc[((pr0 + key) * a.G + kvh) * D + d] = kn_s[d];
+      for (int e = tid; e < E; e += 256) vc[((pr0 + key) * a.G + kvh) * E + e] = vn_s[e];
+    }
+  }
+  // ---- scores
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int key = wave * 16 + i * 4 + kl, t = t0 + key;
+    float s[DEC_HB];
+#pragma unroll
+    for (int h = 0; h < DEC_HB; ++h) s[h] = 0.0f;
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      const int d = (c * 16 + ch) * 8;
+      float k[8];
+      kreg[i][c].get(k);
+#pragma unroll
+      for (int h = 0; h < DEC_HB; ++h) {
+        if (h >= nh) break;
+        float qv[8];
+        load_vec<8>(&q_s[h][d], qv);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) s[h] = fmaf(k[e], qv[e], s[h]);
+      }
+    }
+#pragma unroll
+    for (int h = 0; h < DEC_HB; ++h) {
+      if (h >= nh) break;
+      const float v = row16_sum(s[h]);
+      if (ch == 0) p_s[h][key] = t >= lo && t <= pos ? v : -INFINITY;
+    }
+  }
+  __syncthreads();
+  if (wave < nh) {
+    const float s = p_s[wave][lane], mx = fmaxf(wave_max(s), MASKED), e = __builtin_amdgcn_exp2f(s - mx), sum = wave_sum(e);
+    p_s[wave][lane] = e;
+    if (lane == 0) m_s[wave] = mx, l_s[wave] = sum;
+  }
+  __syncthreads();
+  // ---- values
+  float acc[DEC_HB][8];
+#pragma unroll
+  for (int h = 0; h < DEC_HB; ++h)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) acc[h][e] = 0.0f;
+#pragma unroll
+  for (int i = 0; i < NP; ++i) {
+    float v[8];
+    vreg[i].get(v);
+#pragma unroll
+    for (int h = 0; h < DEC_HB; ++h) {
+      if (h >= nh) break;
+      const float w = p_s[h][wave * 16 + i * RPP + vl];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) acc[h][e] = fmaf(w, v[e], acc[h][e]);
+    }
+  }
+#pragma unroll
+  for (int h = 0; h < DEC_HB; ++h) {
+    if (h >= nh) break;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+#pragma unroll
+      for (int st = LV; st < 64; st <<= 1) acc[h][e] += __shfl_xor(acc[h][e], st, 64);
+      if (vl == 0) acc_s[wave][h][vch * 8 + e] = acc[h][e];
+    }
+  }
+  __syncthreads();
+  const int PW = E + 4;  // numerators, maximum, denominator
+  for (int i = tid; i < nh * E; i += 256) {
+    const int h = i / E, e = i % E;
+    part[(((int64_t)b * a.H + h0 + h) * NS + split) * PW + e] = (acc_s[0][h][e] + acc_s[1][h][e]) + (acc_s[2][h][e] + acc_s[3][h][e]);
+  }
+  if (tid < nh) {
+    float* d = part + (((int64_t)b * a.H + h0 + tid) * NS + split) * PW + E;
+    d[0] = m_s[tid];
+    d[1] = l_s[tid];
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void attn_combine_kernel(AttnDims a, AttnOut o, const float* part, T* out, int NS) {
+  const int h = blockIdx.x % a.H, b = blockIdx.x / a.H;
+  const int pos = a.pos[b], lo = pos - a.window + 1 > 0 ? pos - a.window + 1 : 0;
+  int n = pos / 64 - lo / 64 + 1;
+  n = n < NS ? n : NS;
+  const int PW = a.E + 4;
+  const float* src = part + ((int64_t)b * a.H + h) * NS * PW;
+  float mx = MASKED;
+  for (int i = 0; i < n; ++i) mx = fmaxf(mx, src[(int64_t)i * PW + a.E]);
+  float den = 0.0f;
+  for (int i = 0; i < n; ++i) den += src[(int64_t)i * PW + a.E + 1] * __builtin_amdgcn_exp2f(src[(int64_t)i * PW + a.E] - mx);
+  const float f = head_factor<T>(o, b, h) / den;
+  for (int e = threadIdx.x; e < a.E; e += 256) {
+    float num = 0.0f;
+    for (int i = 0; i < n; ++i) num = fmaf(src[(int64_t)i * PW + e], __builtin_amdgcn_exp2f(src[(int64_t)i * PW + a.E] - mx), num);
+    out[b * o.ldo + h * a.E + e] = from_f32<T>(num * f);
+  }
+}
+
+int check_dims(const AttnDims& a, int64_t B) {
+  SQ_CHECK(B >= 0 && a.S >= 0 && a.H > 0 && a.G > 0 && a.H % a.G == 0 && a.D > 0 && a.E > 0 && a.page > 0 && a.window > 0 &&
+               a.P > 0 && a.n_pages > 0, AQ_E_SHAPE);
+  SQ_CHECK(a.D <= SIMPLE_MAX && a.E <= SIMPLE_MAX && a.n_pages * a.page < ((int64_t)1 << 31) && B * a.S * (a.H + 2 * a.G) < (1 << 26), AQ_E_RANGE);
+  SQ_NEED(a.pos && a.table);
+  return AQ_OK;
+}
+
+}  // namespace sq
+
+using namespace sq;
+
+#define SQ_DIMS(B, S)                                                                                                  \
+  AttnDims a{pos, table, P, n_pages, (int)(S), (int)H, (int)G, (int)D, (int)E, (int)page, (int)(window < (1 << 30) ? window : (1 << 30))}; \
+  if (const int rc = check_dims(a, B)) return rc
+
+extern "C" int aqs_attn_prep(const void* proj, int64_t ld, int64_t o_q, int64_t o_k, int64_t o_v, int dtype, const float* q_norm,
+                             const float* k_norm, float eps, const float* cs, int64_t max_pos, int64_t rot, const int32_t* pos,
+                             const int64_t* table, int64_t P, int64_t page, int64_t n_pages, void* q_out, void* kc, void* vc,
+                             int64_t B, int64_t S, int64_t H, int64_t G, int64_t D, int64_t E, void* stream) {
+  const int64_t window = 1;
+  if (B * S == 0) return AQ_OK;
+  SQ_DIMS(B, S);
+  SQ_CHECK(rot >= 0 && rot % 2 == 0 && rot <= D && max_pos > 0, AQ_E_SHAPE);
+  SQ_CHECK(o_q >= 0 && o_k >= 0 && o_v >= 0 && o_q + H * D <= ld && o_k + G * D <= ld && o_v + G * E <= ld, AQ_E_SHAPE);
+  SQ_NEED(proj && q_norm && k_norm && (cs || rot == 0) && q_out && kc && vc);
+  PrepArgs p{a, q_norm, k_norm, cs, ld, o_q, o_k, o_v, max_pos, B * S, (int)rot, eps};
+  const unsigned grid = (unsigned)((p.M * (H + 2 * G) + 3) / 4);
+  SQ_DISPATCH(dtype, (attn_prep_kernel<T><<<grid, 256, 0, (hipStream_t)stream>>>(p, (const T*)proj, (T*)q_out, (T*)kc, (T*)vc)));
+  return launched();
+}
+
+// whether the matrix-core kernel serves these sizes
+extern "C" int aqs_attn_window_ok(int dtype, int64_t D, int64_t E, int64_t page) {
+  return dtype == AQ_BF16 && D % 8 == 0 && E % 8 == 0 && D <= 256 && E <= 256 && page % WK == 0;
+}
+
+extern "C" int aqs_attn_window(const void* q, const void* kc, const void* vc, int dtype, float scale, int64_t window, const void* gate,
+                               int64_t ld_gate, float out_scale, const int32_t* pos, const int64_t* table, int64_t P, int64_t page,
+                               int64_t n_pages, void* out, int64_t ldo, int64_t B, int64_t S, int64_t H, int64_t G, int64_t D,
+                               int64_t E, int simple, void* stream) {
+  if (B * S == 0) return AQ_OK;
+  SQ_DIMS(B, S);
+  SQ_NEED(q && kc && vc && out);
+  SQ_CHECK(ldo >= H * E && (!gate || ld_gate >= H), AQ_E_SHAPE);
+  const AttnOut o{gate, ld_gate, ldo, out_scale};
+  hipStream_t st = (hipStream_t)stream;
+  if (simple || !aqs_attn_window_ok(dtype, D, E, page) || ldo % 4 || bad_ptr16(q) || bad_ptr16(kc) || bad_ptr16(vc) || bad_ptr16(out)) {
+    const unsigned grid = (unsigned)((B * S * H + 3) / 4);
+    SQ_DISPATCH(dtype, (attn_simple_kernel<T><<<grid, 256, 0, st>>>(a, o, scale, (const T*)q, (const T*)kc, (const T*)vc, (T*)out, B * S)));
+    return launched();
+  }
+  const dim3 grid((unsigned)(((S + WQ - 1) / WQ) * H * B));
+  auto go = [&](auto dtag, auto etag) -> int {
+    constexpr int DP = decltype(dtag)::value, EP = decltype(etag)::value;
+    const size_t lds = (size_t)(WK * (DP + 8) + EP * (WK + 4)) * 2;
+    auto* k = attn_window_kernel<DP, EP>;
+    if (lds > 64 * 1024) {
+      const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      if (e != hipSuccess) return (int)e;
+    }
+    k<<<grid, 256, lds, st>>>(a, o, scale * LOG2E, (const uint16_t*)q, (const uint16_t*)kc, (const uint16_t*)vc, (uint16_t*)out, (int)B);
+    return launched();
+  };
+  auto values = [&](auto dtag) -> int {
+    if (E <= 64) return go(dtag, std::integral_constant<int, 64>{});
+    if (E <= 128) return go(dtag, std::integral_constant<int, 128>{});
+    return go(dtag, std::integral_constant<int, 256>{});
+  };
+  if (D <= 64) return values(std::integral_constant<int, 64>{});
+  if (D <= 128) return values(std::integral_constant<int, 128>{});
+  return values(std::integral_constant<int, 256>{});
+}
+
+extern "C" int aqs_attn_decode_ok(int64_t D, int64_t E, int64_t page) {
+  return D % 8 == 0 && E % 8 == 0 && D <= DEC_MAX && E <= DEC_MAX && page % 64 == 0;
+}
+
+// slices a step needs for this window when the sequence may hold up to `capacity` tokens
+extern "C" int64_t aqs_attn_decode_slices(int64_t window, int64_t capacity) {
+  const int64_t by_window = (window + 62) / 64 + 1, all = (capacity + 63) / 64;
+  return by_window < all ? by_window : all;
+}
+
+// part: [B, H, slices, E + 4] floats
+extern "C" int aqs_attn_decode(const void* proj, int64_t ld, int64_t o_q, int64_t o_k, int64_t o_v, int64_t o_gate, int dtype,
+                               const float* q_norm, const float* k_norm, float eps, const float* cs, int64_t max_pos, int64_t rot,
+                               float scale, int64_t window, float out_scale, const int32_t* pos, const int64_t* table, int64_t P,
+                               int64_t page, int64_t n_pages, void* kc, void* vc, float* part, int64_t slices, void* out, int64_t ldo,
+                               int64_t B, int64_t H, int64_t G, int64_t D, int64_t E, void* stream) {
+  if (B == 0) return AQ_OK;
+  SQ_DIMS(B, 1);
+  SQ_CHECK(aqs_attn_decode_ok(D, E, page) && rot >= 0 && rot % 2 == 0 && rot <= D && max_pos > 0, AQ_E_SHAPE);
+  SQ_CHECK(o_q >= 0 && o_k >= 0 && o_v >= 0 && o_q + H * D <= ld && o_k + G * D <= ld && o_v + G * E <= ld && o_gate + H <= ld, AQ_E_SHAPE);
+  SQ_CHECK(slices == aqs_attn_decode_slices(window, P * page) && ldo >= H * E, AQ_E_SHAPE);
+  SQ_NEED(proj && q_norm && k_norm && (cs || rot == 0) && kc && vc && part && out);
+  SQ_CHECK(!bad_ptr16(kc) && !bad_ptr16(vc), AQ_E_ALIGN);
+  PrepArgs p{a, q_norm, k_norm, cs, ld, o_q, o_k, o_v, max_pos, B, (int)rot, eps};
+  const int64_t nb = (H / G + DEC_HB - 1) / DEC_HB, grid = B * slices * nb * G;
+  SQ_CHECK(grid < (1 << 24), AQ_E_RANGE);
+  hipStream_t st = (hipStream_t)stream;
+#define SQ_DEC(NC, LV) \
+  (attn_decode_kernel<T, NC, LV><<<dim3((unsigned)grid), 256, 0, st>>>(p, scale * LOG2E, (const T*)proj, (T*)kc, (T*)vc, part, (int)slices))
+  SQ_DISPATCH(dtype,
+              if (D <= 128) {
+                if (E <= 64) SQ_DEC(1, 8);
+                else if (E <= 128) SQ_DEC(1, 16);
+                else SQ_DEC(1, 32);
+              } else {
+                if (E <= 64) SQ_DEC(2, 8);
+                else if (E <= 128) SQ_DEC(2, 16);
+                else SQ_DEC(2, 32);
+              });
+#undef SQ_DEC
+  if (const int rc = launched()) return rc;
+  SQ_DISPATCH(dtype, {
+    const AttnOut o{o_gate >= 0 ? (const void*)((const T*)proj + o_gate) : nullptr, ld, ldo, out_scale};
+    (attn_combine_kernel<T><<<dim3((unsigned)(B * H)), 256, 0, st>>>(a, o, part, (T*)out, (int)slices));
+  });
+  return launched();
+}

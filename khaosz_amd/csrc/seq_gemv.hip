@@ -1,0 +1,236 @@
+// Matrix-vector products of a decode step on bf16 (or fp32) weights [N, K], for up to 8 rows of activations, with the
+// row operation in front and the elementwise operation behind folded in:
+//
+//   in front   nothing (activations of T), RMSNorm of the fp32 residual stream, or the gated group norm that closes
+//              the state-space mixer (y * silu(z), RMS per part, weight);
+//   behind     bias, store as T or fp32; the clamped GLU of a gate row and its up row; x += mult * (W h) into the
+//              fp32 residual stream.
+//
+// A workgroup of 4 wavefronts brings the rows into LDS as fp32 (every workgroup repeats the norm: the rows are a few
+// KB and come from the caches), then each wavefront takes R weight rows at a time, 16 bytes per lane and row.  The first
+// weights are requested before the norm, so that HBM works while the rows are being prepared.
+#include "seq_common.h"
+
+namespace sq {
+
+enum { IN_PLAIN = 0, IN_RMSNORM = 1, IN_GATED_NORM = 2 };
+enum { OUT_T = 0, OUT_F32 = 1, OUT_RESIDUAL = 2, OUT_GLU = 3 };
+
+struct GemvArgs {
+  const float* xf;    // IN_RMSNORM: x [M, K]; IN_GATED_NORM: y [M, K]
+  const float* gain;  // IN_RMSNORM: w around zero; IN_GATED_NORM: plain
+  const float* bias;  // [N] or null (OUT_T)
+  float* res;         // OUT_RESIDUAL [M, N]
+  int64_t ldx, ldz, ldo;
+  int M, N, K, groups;
+  float eps, mult, limit;
+};
+
+constexpr int GEMV_MAX_M = 8;
+
+template <typename T, int IN, int OUT, int R, int MR>
+__global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const T* z, const T* w, T* out) {
+  extern __shared__ __align__(16) float xs[];  // [M, K]
+  __shared__ float red[4];
+  constexpr int U = 4;                          // 512-element steps of the row requested ahead
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int K = p.K;
+  // weight row i of this wavefront (OUT_GLU: the second half of them are the up rows of the first half)
+  constexpr int OR = OUT == OUT_GLU ? R / 2 : R;  // output columns per wavefront
+  const int n0 = (blockIdx.x * 4 + wave) * OR;
+  const int F = OUT == OUT_GLU ? p.N / 2 : p.N;   // output columns
+  const T* wr[R];
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    int n = n0 + (OUT == OUT_GLU ? i % OR : i);
+    n = n < F ? n : F - 1;
+    wr[i] = w + (int64_t)(OUT == OUT_GLU && i >= OR ? n + F : n) * K;
+  }
+  Raw8<T> first[R][U];
+#pragma unroll
+  for (int u = 0; u < U; ++u)
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+      const int k = (u * 64 + lane) * 8;
+      if (k < K) first[i][u].load(wr[i] + k);
+      else first[i][u].zero();
+    }
+  __builtin_amdgcn_sched_barrier(0);
+  // ---- rows into LDS
+  for (int m = 0; m < p.M; ++m) {
+    float* row = xs + m * K;
+    if constexpr (IN == IN_PLAIN) {
+      for (int k = tid * 8; k < K; k += 2048) {
+        Raw8<T> v;
+        v.load(x + m * p.ldx + k);
+        float f[8];
+        v.get(f);
+        reinterpret_cast<float4*>(row + k)[0] = make_float4(f[0], f[1], f[2], f[3]);
+        reinterpret_cast<float4*>(row + k)[1] = make_float4(f[4], f[5], f[6], f[7]);
+      }
+    } else if constexpr (IN == IN_RMSNORM) {
+      float ss = 0.0f;
+      for (int k = tid * 4; k < K; k += 1024) {
+        const float4 v = *reinterpret_cast<const float4*>(p.xf + m * p.ldx + k);
+        *reinterpret_cast<float4*>(row + k) = v;
+        ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+      }
+      ss = block_sum<4>(ss, red);
+      const float r = 1.0f / sqrtf(ss / (float)K + p.eps);
+      for (int k = tid * 4; k < K; k += 1024) {
+        float4 v = *reinterpret_cast<const float4*>(row + k);
+        const float4 g = *reinterpret_cast<const float4*>(p.gain + k);
+        v.x *= r * (1.0f + g.x), v.y *= r * (1.0f + g.y), v.z *= r * (1.0f + g.z), v.w *= r * (1.0f + g.w);
+        *reinterpret_cast<float4*>(row + k) = v;
+      }
+    } else {
+      const int part = K / p.groups;
+      for (int g = 0; g < p.groups; ++g) {
+        float ss = 0.0f;
+        for (int k = g * part + tid; k < (g + 1) * part; k += 256) {
+          const float v = p.xf[m * p.ldx + k] * silu(to_f32(z[m * p.ldz + k]));
+          row[k] = v;
+          ss += v * v;
+        }
+        ss = block_sum<4>(ss, red);
+        const float r = 1.0f / sqrtf(ss / (float)part + p.eps);
+        for (int k = g * part + tid; k < (g + 1) * part; k += 256) row[k] *= r * p.gain[k];
+      }
+    }
+  }
+  __syncthreads();
+  // ---- products
+  float acc[R][MR];
+#pragma unroll
+  for (int i = 0; i < R; ++i)
+#pragma unroll
+    for (int m = 0; m < MR; ++m) acc[i][m] = 0.0f;
+  auto step = [&](int k, const Raw8<T>* ws) __attribute__((always_inline)) {
+    float f[R][8];
+#pragma unroll
+    for (int i = 0; i < R; ++i) ws[i].get(f[i]);
+#pragma unroll
+    for (int m = 0; m < MR; ++m) {
+      if (m >= p.M) break;
+      float a[8];
+      load_vec<8>(xs + m * K + k, a);
+#pragma unroll
+      for (int i = 0; i < R; ++i)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[i][m] = fmaf(f[i][e], a[e], acc[i][m]);
+    }
+  };
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const int k = (u * 64 + lane) * 8;
+    Raw8<T> ws[R];
+#pragma unroll
+    for (int i = 0; i < R; ++i) ws[i] = first[i][u];
+    if (k < K) step(k, ws);
+  }
+#pragma unroll 2
+  for (int k = (U * 64 + lane) * 8; k < K; k += 512) {
+    Raw8<T> ws[R];
+#pragma unroll
+    for (int i = 0; i < R; ++i) ws[i].load(wr[i] + k);
+    step(k, ws);
+  }
+  // ---- sums over the lanes and the output
+#pragma unroll
+  for (int m = 0; m < MR; ++m) {
+    if (m >= p.M) break;
+    float s[R];
+#pragma unroll
+    for (int i = 0; i < R; ++i) s[i] = wave_sum(acc[i][m]);
+    if (lane != 0) continue;
+#pragma unroll
+    for (int i = 0; i < OR; ++i) {
+      const int n = n0 + i;
+      if (n >= F) break;
+      if constexpr (OUT == OUT_T) out[m * p.ldo + n] = from_f32<T>(s[i] + (p.bias ? p.bias[n] : 0.0f));
+      else if constexpr (OUT == OUT_F32) p.res[m * p.ldo + n] = s[i];
+      else if constexpr (OUT == OUT_RESIDUAL) p.res[m * p.ldo + n] += p.mult * s[i];
+      else out[m * p.ldo + n] = from_f32<T>(clamped_glu(s[i], s[i + OR], p.limit));
+    }
+  }
+}
+
+template <typename T, int IN, int OUT>
+int launch_gemv(const GemvArgs& p, const void* x, const void* z, const void* w, void* out, hipStream_t stream) {
+  const int F = OUT == OUT_GLU ? p.N / 2 : p.N;
+  const size_t lds = (size_t)p.M * p.K * 4;
+  auto go = [&](auto r_tag, auto m_tag) -> int {
+    constexpr int R = decltype(r_tag)::value, MR = decltype(m_tag)::value;
+    constexpr int OR = OUT == OUT_GLU ? R / 2 : R;
+    auto* k = gemv_kernel<T, IN, OUT, R, MR>;
+    if (lds > 64 * 1024) {
+      const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      if (e != hipSuccess) return (int)e;
+    }
+    k<<<dim3((unsigned)((F + 4 * OR - 1) / (4 * OR))), 256, lds, stream>>>(p, (const T*)x, (const T*)z, (const T*)w, (T*)out);
+    return launched();
+  };
+  auto rows = [&](auto m_tag) -> int {
+    // enough wavefronts first (1024 SIMDs), then more rows per wavefront for fewer reads of the activations
+    if constexpr (OUT == OUT_GLU) {
+      if (F >= 8192) return go(std::integral_constant<int, 4>{}, m_tag);
+      return go(std::integral_constant<int, 2>{}, m_tag);
+    } else {
+      if (F >= 8192) return go(std::integral_constant<int, 4>{}, m_tag);
+      if (F >= 4096) return go(std::integral_constant<int, 2>{}, m_tag);
+      return go(std::integral_constant<int, 1>{}, m_tag);
+    }
+  };
+  if (p.M == 1) return rows(std::integral_constant<int, 1>{});
+  return rows(std::integral_constant<int, GEMV_MAX_M>{});
+}
+
+}  // namespace sq
+
+using namespace sq;
+
+extern "C" int aqs_gemv_ok(int64_t M, int64_t N, int64_t K) {
+  return M > 0 && M <= GEMV_MAX_M && N > 0 && N < (1 << 24) && K > 0 && K % 8 == 0 && M * K * 4 <= 144 * 1024;
+}
+
+// in_kind: 0 plain (x of dtype, stride ldx), 1 rmsnorm (xf, gain, eps), 2 gated group norm (xf = y, x = z with stride
+// ldz, gain, eps, groups).  out_kind: 0 dtype (+ bias), 1 fp32 into res, 2 res += mult * (...), 3 clamped GLU into out.
+extern "C" int aqs_gemv(int in_kind, int out_kind, int dtype, const void* x, int64_t ldx, const float* xf, const float* gain,
+                        float eps, int64_t groups, const void* w, const float* bias, float mult, float limit, float* res, void* out,
+                        int64_t ldo, int64_t M, int64_t N, int64_t K, void* stream) {
+  SQ_CHECK(M >= 0 && N > 0 && K > 0, AQ_E_SHAPE);
+  if (M == 0) return AQ_OK;
+  SQ_CHECK(aqs_gemv_ok(M, N, K), AQ_E_SHAPE);
+  SQ_NEED(w && (out_kind == OUT_F32 || out_kind == OUT_RESIDUAL ? (const void*)res : (const void*)out));
+  SQ_CHECK(!bad_ptr16(w) && !bad_ptr16(x) && !bad_ptr16(xf) && !bad_ptr16(gain), AQ_E_ALIGN);
+  SQ_CHECK(out_kind != OUT_GLU || N % 2 == 0, AQ_E_SHAPE);
+  SQ_CHECK(ldo >= (out_kind == OUT_GLU ? N / 2 : N), AQ_E_SHAPE);
+  GemvArgs p{};
+  p.xf = xf, p.gain = gain, p.bias = bias, p.res = res, p.ldo = ldo;
+  p.M = (int)M, p.N = (int)N, p.K = (int)K, p.groups = (int)groups, p.eps = eps, p.mult = mult, p.limit = limit;
+  const void* z = nullptr;
+  if (in_kind == IN_PLAIN) {
+    SQ_NEED(x);
+    SQ_CHECK(ldx >= K && ldx % 8 == 0, AQ_E_SHAPE);
+    p.ldx = ldx;
+  } else {
+    SQ_NEED(xf && gain);
+    p.ldx = K;
+    if (in_kind == IN_GATED_NORM) {
+      SQ_NEED(x);
+      SQ_CHECK(groups > 0 && K % groups == 0 && ldx >= K, AQ_E_SHAPE);
+      z = x, p.ldz = ldx;
+    }
+  }
+  hipStream_t st = (hipStream_t)stream;
+#define SQ_GEMV(I, O) \
+  if (in_kind == I && out_kind == O) SQ_DISPATCH(dtype, return (launch_gemv<T, I, O>(p, x, z, w, out, st)))
+  SQ_GEMV(IN_PLAIN, OUT_T);
+  SQ_GEMV(IN_PLAIN, OUT_RESIDUAL);
+  SQ_GEMV(IN_RMSNORM, OUT_T);
+  SQ_GEMV(IN_RMSNORM, OUT_F32);
+  SQ_GEMV(IN_RMSNORM, OUT_GLU);
+  SQ_GEMV(IN_GATED_NORM, OUT_RESIDUAL);
+#undef SQ_GEMV
+  return AQ_E_SHAPE;
+}

@@ -14,8 +14,8 @@ graph.
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
-from typing import Dict, Optional
+from dataclasses import dataclass, fields
+from typing import Any, Dict, Optional, Sequence
 
 import torch
 import torch.nn as nn
@@ -24,6 +24,7 @@ from torch import Tensor
 
 from .block import DecoderBlock, PagedKV, RMSNorm, rotary_table
 from .linear import Linear
+from .registry import register_model
 
 
 @dataclass
@@ -43,6 +44,12 @@ class LMConfig:
     use_qk_norm: bool = False
     use_gated_attention: bool = False
 
+    @classmethod
+    def from_dict(cls, d: Dict[str, Any], shapes=None) -> "LMConfig":
+        """From a config.json; fields this model does not read are left out (config/base.py:8-98)."""
+        known = {f.name for f in fields(cls)}
+        return cls(**{k: v for k, v in d.items() if k in known and v is not None})
+
 
 class Embedding(nn.Module):
     """``F.embedding`` over a learned table (astrai/model/components/embedding.py:7-17)."""
@@ -58,12 +65,17 @@ class Embedding(nn.Module):
         return F.embedding(ids, self.weight)
 
 
+@register_model("autoregressive_lm")
 class AutoRegressiveLM(nn.Module):
     """Same attribute names and state-dict keys as the reference model
     (``embed_tokens``, ``layers.N.*``, ``norm``, ``lm_head``), so ``quantize_model`` and
     ``fuse_shared_inputs`` find their targets and a reference checkpoint's keys line up."""
 
-    def __init__(self, config: LMConfig):
+    config_class = LMConfig
+    window = None            # every layer reads all positions
+    mixed_positions = False  # sequences of one step sit at one position (cache.write)
+
+    def __init__(self, config: LMConfig, dtype: Optional[torch.dtype] = None, device=None):
         super().__init__()
         self.config = config
         head_dim = config.dim // config.n_heads
@@ -82,6 +94,31 @@ class AutoRegressiveLM(nn.Module):
         for m in self.modules():
             if m is not self and hasattr(m, "reset_parameters") and isinstance(m, (Linear, Embedding)):
                 m.reset_parameters()
+        if dtype is not None or device is not None:
+            self.to(dtype=dtype, device=device)
+
+    # ---- what the loader and the engine ask of a model
+    def tensors(self) -> Dict[str, Tensor]:
+        return {n: t for n, t in self.state_dict(keep_vars=True).items()
+                if not (self.config.tie_weight and n == "lm_head.weight")}
+
+    @property
+    def vocab_size(self) -> int:
+        return self.config.vocab_size
+
+    def step_ok(self, rows: int) -> bool:
+        return False  # a step takes its position from the host: no graph is replayed for the next one
+
+    def new_sequence_state(self, n_slots: int, n_pages: int, page: int, capacity: int) -> PagedKV:
+        return self.new_cache(n_pages, page)
+
+    def advance(self, ids: Tensor, b, state: PagedKV, starts: Sequence[int], want: Optional[Sequence[int]] = None) -> Tensor:
+        """New tokens ``ids [B, S]`` of sequences that all sit at one position; fp32 logits of the rows ``want``."""
+        if len(set(starts)) != 1:
+            raise ValueError("the sequences of one step must sit at one position")
+        out = self(ids, paged_cache=state.bind(b.table, starts[0] + b.S, refresh=True), start_pos=starts[0])["logits"]
+        rows = out.view(-1, out.shape[-1])
+        return (rows if want is None else rows[list(want)]).float()
 
     def new_cache(self, n_pages: int, page_size: int, device=None, dtype=None) -> PagedKV:
         """A paged KV cache with one set of pages per layer (``KVCache``'s storage, cache.py:187-214)."""

@@ -1,0 +1,394 @@
+"""Tensor-level operators over libastrai_seq.so (include/astrai_seq.h): the row operations, matrix-vector
+products, convolutions, linear recurrences and windowed attention of the hybrid decoders.
+
+As in ``ops``: tensors already on the GPU, layouts checked as the kernels assume them, work queued on
+torch's current stream, no CPU fallback.  ``proj`` arguments are rows of a fused projection
+``[M, ld]``; ``o_*`` are first columns of its parts.
+"""
+from __future__ import annotations
+
+from typing import NamedTuple, Optional
+
+import torch
+from torch import Tensor
+
+from . import _abi
+from .ops import _DT, _need_gpu, _OnDevice, _stream
+
+
+class Batch(NamedTuple):
+    """The sequences of one step: ``S`` new tokens each, from position ``pos[b]`` on.  ``pos`` and ``slots`` int32
+    ``[B]``, ``table`` int64 ``[B, P]`` (physical pages of each sequence, -1 where none), all on the device."""
+    pos: Tensor
+    slots: Tensor
+    table: Tensor
+    B: int
+    S: int
+
+
+def _call(name: str, dev: torch.device, *args) -> None:
+    with _OnDevice(dev):
+        rc = getattr(_abi.load_seq(), name)(*args)
+    _abi.check(rc, name)
+
+
+def _p(t: Optional[Tensor], col: int = 0):
+    return None if t is None else t.data_ptr() + col * t.element_size()
+
+
+def _rows2(t: Tensor, what: str, dtype=None) -> Tensor:
+    if t.dim() != 2 or (t.shape[0] > 1 and t.stride(1) != 1) or (dtype is not None and t.dtype != dtype):
+        raise ValueError(f"{what} must be rows [M, K] with contiguous columns, got {tuple(t.shape)} {t.dtype}")
+    return t
+
+
+def _vec(t: Optional[Tensor], n: int, what: str) -> None:
+    if t is not None and (t.dtype != torch.float32 or t.numel() != n or not t.is_contiguous()):
+        raise ValueError(f"{what} must be {n} contiguous float32 elements, got {t.dtype} {tuple(t.shape)}")
+
+
+def _batch(b: Batch, rows: int, n_slots: Optional[int] = None) -> None:
+    if b.pos.dtype != torch.int32 or b.slots.dtype != torch.int32 or b.pos.numel() != b.B or b.slots.numel() != b.B:
+        raise ValueError("pos and slots must be int32 [B]")
+    if b.table.dtype != torch.int64 or b.table.dim() != 2 or b.table.shape[0] != b.B or not b.table.is_contiguous():
+        raise ValueError("table must be contiguous int64 [B, P]")
+    if rows != b.B * b.S:
+        raise ValueError(f"{rows} rows for {b.B} sequences of {b.S} tokens")
+
+
+# ------------------------------------------------------------------------------------------------ rows
+def embed(ids: Tensor, table: Tensor) -> Tensor:
+    """fp32 rows of ``table [V, K]``; an id outside the table is a zero row."""
+    _need_gpu(ids, table)
+    if ids.dtype != torch.int64 or table.dim() != 2 or not table.is_contiguous():
+        raise ValueError("ids must be int64 and the table contiguous [V, K]")
+    ids = ids.reshape(-1).contiguous()
+    x = torch.empty((ids.numel(), table.shape[1]), dtype=torch.float32, device=table.device)
+    _call("aqs_embed", x.device, _p(ids), _p(table), _DT[table.dtype], _p(x), x.shape[0], x.shape[1], table.shape[0], _stream(x))
+    return x
+
+
+def add_rmsnorm(x: Tensor, y: Optional[Tensor], mult: float, w: Optional[Tensor], eps: float, dtype: torch.dtype,
+                norm: bool = True) -> Optional[Tensor]:
+    """``x += mult * y`` in place (fp32 ``x [M, K]``, ``y`` optional), then ``rms(x) * (1 + w)`` as ``dtype``."""
+    _need_gpu(x, y, w)
+    M, K = x.shape
+    if x.dtype != torch.float32 or not x.is_contiguous() or (y is not None and (y.shape != x.shape or y.dtype != dtype)):
+        raise ValueError("x must be contiguous float32 [M, K] and y have its shape")
+    if y is not None:
+        _rows2(y, "y")
+    _vec(w, K, "w")
+    out = torch.empty((M, K), dtype=dtype, device=x.device) if norm else None
+    if M and (norm or y is not None):
+        _call("aqs_add_rmsnorm", x.device, _p(x), _p(y), y.stride(0) if y is not None else K, _DT[dtype], float(mult), _p(w),
+              float(eps), _p(out), M, K, _stream(x))
+    return out
+
+
+def clamped_glu(gu: Tensor, limit: float) -> Tensor:
+    """``gu [M, 2F] = gate | up`` -> ``g sigmoid(1.702 g) (u + 1)`` with g capped and u clamped at ``limit``."""
+    _need_gpu(gu)
+    _rows2(gu, "gu")
+    M, F = gu.shape[0], gu.shape[1] // 2
+    out = torch.empty((M, F), dtype=gu.dtype, device=gu.device)
+    _call("aqs_clamped_glu", gu.device, _p(gu), gu.stride(0), _DT[gu.dtype], float(limit), _p(out), M, F, _stream(gu))
+    return out
+
+
+def gated_group_norm(y: Tensor, proj: Tensor, o_z: int, w: Tensor, eps: float, groups: int, out: Tensor) -> None:
+    """``out = rms(y * silu(z)) * w`` with the RMS over each of ``groups`` equal parts; z the columns of ``proj`` from
+    ``o_z`` on."""
+    _need_gpu(y, proj, w, out)
+    M, K = y.shape
+    _rows2(out, "out", proj.dtype)
+    _vec(w, K, "w")
+    if y.dtype != torch.float32 or not y.is_contiguous() or proj.shape[0] != M or o_z + K > proj.shape[1] or out.shape != y.shape:
+        raise ValueError("gated_group_norm: shapes do not fit")
+    _call("aqs_gated_group_norm", y.device, _p(y), _p(proj, o_z), proj.stride(0), _DT[proj.dtype], _p(w), float(eps), _p(out),
+          out.stride(0), M, K, int(groups), _stream(y))
+
+
+def head_norm_gate(o: Tensor, gate: Tensor, w: Tensor, eps: float, scale: float, out: Tensor) -> None:
+    """Each head of ``o [M, H, E]`` over its root mean square, times ``w [E]``, ``sigmoid(gate [M, H*E])`` and ``scale``."""
+    _need_gpu(o, gate, w, out)
+    M, H, E = o.shape
+    _rows2(out, "out", gate.dtype)
+    _vec(w, E, "w")
+    if o.dtype != torch.float32 or not o.is_contiguous() or gate.shape != (M, H * E) or out.shape != (M, H * E):
+        raise ValueError("head_norm_gate: shapes do not fit")
+    _call("aqs_head_norm_gate", o.device, _p(o), _p(gate), gate.stride(0), _DT[gate.dtype], _p(w), float(eps), float(scale),
+          _p(out), out.stride(0), M, H, E, _stream(o))
+
+
+# ------------------------------------------------------------------------------------------------ matrix-vector products
+def gemv_ok(M: int, N: int, K: int) -> bool:
+    return bool(_abi.load_seq().aqs_gemv_ok(M, N, K))
+
+
+def _gemv(in_kind, out_kind, w, x=None, ldx=0, o_x=0, xf=None, gain=None, eps=0.0, groups=1, bias=None, mult=0.0, limit=0.0,
+          res=None, out=None):
+    _need_gpu(w, x, xf, gain, bias, res, out)
+    N, K = w.shape
+    if not w.is_contiguous():
+        raise ValueError("weights must be contiguous [N, K]")
+    if xf is not None and (xf.dtype != torch.float32 or xf.dim() != 2 or xf.shape[1] != K or not xf.is_contiguous()):
+        raise ValueError(f"fp32 rows must be contiguous [M, {K}], got {tuple(xf.shape)}")
+    if x is not None and (x.dtype != w.dtype or x.dim() != 2 or o_x + K > x.shape[1]):
+        raise ValueError(f"rows must be {w.dtype} [M, {K}], got {x.dtype} {tuple(x.shape)}")
+    _vec(gain, K, "gain")
+    _vec(bias, N, "bias")
+    M = (xf if xf is not None else x).shape[0]
+    dst = res if res is not None else out
+    _call("aqs_gemv", w.device, in_kind, out_kind, _DT[w.dtype], _p(x, o_x), ldx, _p(xf), _p(gain), float(eps), int(groups), _p(w),
+          _p(bias), float(mult), float(limit), _p(res), _p(out), dst.stride(0), M, N, K, _stream(w))
+
+
+def norm_gemv(x: Tensor, gain: Tensor, eps: float, w: Tensor, bias: Optional[Tensor] = None) -> Tensor:
+    """``W (rms(x) * (1 + gain)) + bias`` for a few rows of the fp32 stream ``x [M, K]``."""
+    out = torch.empty((x.shape[0], w.shape[0]), dtype=w.dtype, device=w.device)
+    _gemv(1, 0, w, xf=x, gain=gain, eps=eps, bias=bias, out=out)
+    return out
+
+
+def norm_gemv_f32(x: Tensor, gain: Tensor, eps: float, w: Tensor) -> Tensor:
+    """The same without bias, stored in fp32 (the vocabulary projection)."""
+    out = torch.empty((x.shape[0], w.shape[0]), dtype=torch.float32, device=w.device)
+    _gemv(1, 1, w, xf=x, gain=gain, eps=eps, res=out)
+    return out
+
+
+def norm_gemv_glu(x: Tensor, gain: Tensor, eps: float, w: Tensor, limit: float) -> Tensor:
+    """``clamped_glu`` of the two halves of ``W (rms(x) * (1 + gain))``; ``w [2F, K]`` = gate rows | up rows."""
+    out = torch.empty((x.shape[0], w.shape[0] // 2), dtype=w.dtype, device=w.device)
+    _gemv(1, 3, w, xf=x, gain=gain, eps=eps, limit=limit, out=out)
+    return out
+
+
+def gemv_residual(x: Tensor, w: Tensor, mult: float, res: Tensor) -> None:
+    """``res += mult * (W x)`` in the fp32 stream ``res [M, N]``."""
+    if res.dtype != torch.float32 or res.shape != (x.shape[0], w.shape[0]) or not res.is_contiguous():
+        raise ValueError("the residual stream must be contiguous float32 [M, N]")
+    _gemv(0, 2, w, x=x, ldx=x.stride(0), mult=mult, res=res)
+
+
+def gated_norm_gemv_residual(y: Tensor, proj: Tensor, o_z: int, gain: Tensor, eps: float, groups: int, w: Tensor, mult: float,
+                             res: Tensor) -> None:
+    """``gated_group_norm`` and ``gemv_residual`` in one launch."""
+    if res.dtype != torch.float32 or res.shape != (y.shape[0], w.shape[0]) or not res.is_contiguous():
+        raise ValueError("the residual stream must be contiguous float32 [M, N]")
+    _gemv(2, 2, w, x=proj, ldx=proj.stride(0), o_x=o_z, xf=y, gain=gain, eps=eps, groups=groups, mult=mult, res=res)
+
+
+# ------------------------------------------------------------------------------------------------ convolution state
+def _ring(ring: Tensor, C: int, taps: int, dtype) -> None:
+    if ring.dim() != 3 or tuple(ring.shape[1:]) != (taps, C) or ring.dtype != dtype or not ring.is_contiguous():
+        raise ValueError(f"the convolution ring must be contiguous {dtype} [slots, {taps}, {C}], got {tuple(ring.shape)}")
+
+
+def conv_silu(proj: Tensor, o_in: int, w: Tensor, bias: Optional[Tensor], ring: Tensor, b: Batch) -> Tensor:
+    """Causal convolution (``w [C, taps]``) and SiLU of ``C`` columns of ``proj``; fp32 ``[M, C]``."""
+    _need_gpu(proj, w, bias, ring, b.pos)
+    C, taps = w.shape
+    _batch(b, proj.shape[0])
+    _ring(ring, C, taps, proj.dtype)
+    _vec(w, C * taps, "w")
+    _vec(bias, C, "bias")
+    if o_in + C > proj.shape[1]:
+        raise ValueError("conv_silu: channels outside the projection")
+    out = torch.empty((proj.shape[0], C), dtype=torch.float32, device=proj.device)
+    _call("aqs_conv_silu", proj.device, _p(proj, o_in), proj.stride(0), _DT[proj.dtype], _p(w), _p(bias), _p(ring), _p(b.slots),
+          _p(b.pos), _p(out), b.B, b.S, C, taps, _stream(proj))
+    return out
+
+
+def conv_push(proj: Tensor, o_in: int, C: int, taps: int, ring: Tensor, b: Batch) -> None:
+    """Keep the last ``taps - 1`` inputs; after everything that reads the ring's old content."""
+    _batch(b, proj.shape[0])
+    _ring(ring, C, taps, proj.dtype)
+    _call("aqs_conv_push", proj.device, _p(proj, o_in), proj.stride(0), _DT[proj.dtype], _p(ring), _p(b.slots), _p(b.pos), b.B,
+          b.S, C, taps, _stream(proj))
+
+
+# ------------------------------------------------------------------------------------------------ recurrences
+def _state(s: Tensor, *dims) -> None:
+    if s.dtype != torch.float32 or tuple(s.shape[1:]) != dims or not s.is_contiguous():
+        raise ValueError(f"the recurrent state must be contiguous float32 [slots, {dims}], got {tuple(s.shape)}")
+
+
+def delta_prep(proj: Tensor, o_qkv: int, raw: Tensor, o_beta: int, conv_w: Tensor, ring: Tensor, a_log: Tensor, dt_bias: Tensor,
+               H: int, G: int, D: int, E: int, b: Batch):
+    """Inputs of the delta rule: ``(q, k [M, G, D], v [M, H, E], decay [M, H, D], beta [M, H])`` in fp32."""
+    _need_gpu(proj, raw, conv_w, ring, a_log, dt_bias)
+    M, C, taps, dev = proj.shape[0], 2 * G * D + H * E, conv_w.shape[1], proj.device
+    _batch(b, M)
+    _ring(ring, C, taps, proj.dtype)
+    _vec(conv_w, C * taps, "conv_w")
+    _vec(a_log, H, "a_log")
+    _vec(dt_bias, H * D, "dt_bias")
+    _rows2(raw, "raw", proj.dtype)
+    if raw.shape != (M, H * D) or o_qkv + C > proj.shape[1] or o_beta + H > proj.shape[1]:
+        raise ValueError("delta_prep: shapes do not fit")
+    q = torch.empty((M, G, D), dtype=torch.float32, device=dev)
+    k = torch.empty_like(q)
+    v = torch.empty((M, H, E), dtype=torch.float32, device=dev)
+    decay = torch.empty((M, H, D), dtype=torch.float32, device=dev)
+    beta = torch.empty((M, H), dtype=torch.float32, device=dev)
+    _call("aqs_delta_prep", dev, _p(proj, o_qkv), proj.stride(0), _p(raw), raw.stride(0), _p(proj, o_beta), proj.stride(0),
+          _DT[proj.dtype], _p(conv_w), _p(ring), _p(b.slots), _p(b.pos), _p(a_log), _p(dt_bias), _p(q), _p(k), _p(v), _p(decay),
+          _p(beta), b.B, b.S, H, G, D, E, taps, _stream(proj))
+    return q, k, v, decay, beta
+
+
+def delta_scan(q: Tensor, k: Tensor, v: Tensor, decay: Tensor, beta: Tensor, state: Tensor, b: Batch) -> Tensor:
+    """The gated delta rule over the new tokens; ``state [slots, H, E, D]`` is carried on.  fp32 ``[M, H, E]``."""
+    _need_gpu(q, k, v, decay, beta, state)
+    M, G, D = q.shape
+    H, E = v.shape[1:]
+    _batch(b, M)
+    _state(state, H, E, D)
+    for t, n in ((q, M * G * D), (k, M * G * D), (v, M * H * E), (decay, M * H * D), (beta, M * H)):
+        _vec(t, n, "delta_scan input")
+    out = torch.empty((M, H, E), dtype=torch.float32, device=q.device)
+    _call("aqs_delta_scan", q.device, _p(q), _p(k), _p(v), _p(decay), _p(beta), _p(state), _p(b.slots), _p(b.pos), _p(out), b.B,
+          b.S, H, G, D, E, _stream(q))
+    return out
+
+
+def delta_step(proj: Tensor, o_qkv: int, o_beta: int, o_a1: int, o_g1: int, conv_w: Tensor, ring: Tensor, a2: Tensor, g2: Tensor,
+               a_log: Tensor, dt_bias: Tensor, norm: Tensor, eps: float, scale: float, state: Tensor, out: Tensor, H: int, G: int,
+               D: int, E: int, b: Batch) -> None:
+    """One token per sequence, from the projection's row to the normed and gated heads ``out [B, H * E]``."""
+    _need_gpu(proj, conv_w, ring, a2, g2, state, out)
+    C, taps = 2 * G * D + H * E, conv_w.shape[1]
+    _batch(b, proj.shape[0])
+    _ring(ring, C, taps, proj.dtype)
+    _state(state, H, E, D)
+    _rows2(out, "out", proj.dtype)
+    _vec(conv_w, C * taps, "conv_w")
+    _vec(a_log, H, "a_log")
+    _vec(dt_bias, H * D, "dt_bias")
+    _vec(norm, E, "norm")
+    if b.S != 1 or out.shape != (b.B, H * E) or a2.shape[0] != H * D or g2.shape[0] != H * E or a2.dtype != proj.dtype \
+            or g2.dtype != proj.dtype or not a2.is_contiguous() or not g2.is_contiguous():
+        raise ValueError("delta_step: shapes do not fit")
+    _call("aqs_delta_step", proj.device, _p(proj), proj.stride(0), o_qkv, o_beta, o_a1, o_g1, _DT[proj.dtype], _p(conv_w), _p(ring),
+          _p(b.slots), _p(b.pos), _p(a2), a2.shape[1], _p(g2), g2.shape[1], _p(a_log), _p(dt_bias), _p(norm), float(eps),
+          float(scale), _p(state), _p(out), out.stride(0), b.B, H, G, D, E, taps, _stream(proj))
+
+
+def ssd_scan(xbc: Tensor, proj: Tensor, o_dt: int, dt_bias: Tensor, a_log: Tensor, skip: Tensor, state: Tensor, H: int, G: int,
+             N: int, P: int, b: Batch) -> Tensor:
+    """The state-space recurrence over the new tokens; ``xbc`` from ``conv_silu``.  fp32 ``[M, H * P]``."""
+    _need_gpu(xbc, proj, dt_bias, a_log, skip, state)
+    M = xbc.shape[0]
+    _batch(b, M)
+    _state(state, H, P, N)
+    _vec(xbc, M * (H * P + 2 * G * N), "xbc")
+    for t in (dt_bias, a_log, skip):
+        _vec(t, H, "per-head constants")
+    if proj.shape[0] != M or o_dt + H > proj.shape[1]:
+        raise ValueError("ssd_scan: shapes do not fit")
+    out = torch.empty((M, H * P), dtype=torch.float32, device=xbc.device)
+    _call("aqs_ssd_scan", xbc.device, _p(xbc), _p(proj, o_dt), proj.stride(0), _DT[proj.dtype], _p(dt_bias), _p(a_log), _p(skip),
+          _p(state), _p(b.slots), _p(b.pos), _p(out), b.B, b.S, H, G, N, P, _stream(xbc))
+    return out
+
+
+def ssd_step(proj: Tensor, o_xbc: int, o_dt: int, conv_w: Tensor, conv_b: Tensor, ring: Tensor, dt_bias: Tensor, a_log: Tensor,
+             skip: Tensor, state: Tensor, H: int, G: int, N: int, P: int, b: Batch) -> Tensor:
+    """One token per sequence: convolution, step size, recurrence.  fp32 ``[B, H * P]``, before gate and norm."""
+    _need_gpu(proj, conv_w, conv_b, ring, state)
+    C, taps = H * P + 2 * G * N, conv_w.shape[1]
+    _batch(b, proj.shape[0])
+    _ring(ring, C, taps, proj.dtype)
+    _state(state, H, P, N)
+    _vec(conv_w, C * taps, "conv_w")
+    _vec(conv_b, C, "conv_b")
+    for t in (dt_bias, a_log, skip):
+        _vec(t, H, "per-head constants")
+    if b.S != 1:
+        raise ValueError("ssd_step takes one token per sequence")
+    y = torch.empty((b.B, H * P), dtype=torch.float32, device=proj.device)
+    _call("aqs_ssd_step", proj.device, _p(proj), proj.stride(0), o_xbc, o_dt, _DT[proj.dtype], _p(conv_w), _p(conv_b), _p(ring),
+          _p(b.slots), _p(b.pos), _p(dt_bias), _p(a_log), _p(skip), _p(state), _p(y), b.B, H, G, N, P, taps, _stream(proj))
+    return y
+
+
+# ------------------------------------------------------------------------------------------------ windowed attention
+class WindowAttnSpec(NamedTuple):
+    """Sizes and constants of a windowed attention."""
+    H: int
+    G: int
+    D: int
+    E: int
+    window: int
+    scale: float
+    rot: int
+    eps: float
+
+
+def _pages(kc: Tensor, vc: Tensor, s: WindowAttnSpec, dtype) -> None:
+    if kc.dim() != 4 or vc.dim() != 4 or kc.shape[:2] != vc.shape[:2] or tuple(kc.shape[2:]) != (s.G, s.D) \
+            or tuple(vc.shape[2:]) != (s.G, s.E) or kc.dtype != dtype or vc.dtype != dtype \
+            or not (kc.is_contiguous() and vc.is_contiguous()):
+        raise ValueError(f"caches must be contiguous {dtype} [pages, page, {s.G}, {s.D} / {s.E}], got {tuple(kc.shape)}, {tuple(vc.shape)}")
+
+
+def _rotary(cs: Tensor, s: WindowAttnSpec) -> None:
+    if cs.dtype != torch.float32 or cs.dim() != 3 or tuple(cs.shape[1:]) != (s.rot // 2, 2) or not cs.is_contiguous():
+        raise ValueError(f"the rotary table must be contiguous float32 [positions, {s.rot // 2}, 2], got {tuple(cs.shape)}")
+
+
+def attn_prep(proj: Tensor, o_q: int, o_k: int, o_v: int, q_norm: Tensor, k_norm: Tensor, cs: Tensor, kc: Tensor, vc: Tensor,
+              s: WindowAttnSpec, b: Batch) -> Tensor:
+    """Head norms and rotation of q and k; k and v into their page slots.  Returns ``q [M, H, D]``."""
+    _need_gpu(proj, q_norm, k_norm, cs, kc, vc)
+    _batch(b, proj.shape[0])
+    _pages(kc, vc, s, proj.dtype)
+    _rotary(cs, s)
+    _vec(q_norm, s.D, "q_norm")
+    _vec(k_norm, s.D, "k_norm")
+    q = torch.empty((proj.shape[0], s.H, s.D), dtype=proj.dtype, device=proj.device)
+    _call("aqs_attn_prep", proj.device, _p(proj), proj.stride(0), o_q, o_k, o_v, _DT[proj.dtype], _p(q_norm), _p(k_norm), s.eps,
+          _p(cs), cs.shape[0], s.rot, _p(b.pos), _p(b.table), b.table.shape[1], kc.shape[1], kc.shape[0], _p(q), _p(kc), _p(vc),
+          b.B, b.S, s.H, s.G, s.D, s.E, _stream(proj))
+    return q
+
+
+def attn_window(q: Tensor, kc: Tensor, vc: Tensor, proj: Tensor, o_gate: int, out_scale: float, s: WindowAttnSpec, b: Batch,
+                out: Tensor, simple: bool = False) -> None:
+    """The new tokens over their windows; ``out [M, H * E]`` gated per head by ``proj``'s columns from ``o_gate`` on
+    (none for ``o_gate < 0``) and scaled."""
+    _need_gpu(q, kc, vc, proj, out)
+    _batch(b, q.shape[0])
+    _pages(kc, vc, s, q.dtype)
+    _rows2(out, "out", q.dtype)
+    if tuple(q.shape[1:]) != (s.H, s.D) or not q.is_contiguous() or out.shape != (q.shape[0], s.H * s.E) \
+            or (o_gate >= 0 and o_gate + s.H > proj.shape[1]):
+        raise ValueError("attn_window: shapes do not fit")
+    _call("aqs_attn_window", q.device, _p(q), _p(kc), _p(vc), _DT[q.dtype], s.scale, s.window,
+          _p(proj, o_gate) if o_gate >= 0 else None, proj.stride(0), float(out_scale), _p(b.pos), _p(b.table), b.table.shape[1],
+          kc.shape[1], kc.shape[0], _p(out), out.stride(0), b.B, b.S, s.H, s.G, s.D, s.E, int(simple), _stream(q))
+
+
+def attn_decode_ok(s: WindowAttnSpec, page: int) -> bool:
+    return bool(_abi.load_seq().aqs_attn_decode_ok(s.D, s.E, page))
+
+
+def attn_decode(proj: Tensor, o_q: int, o_k: int, o_v: int, o_gate: int, q_norm: Tensor, k_norm: Tensor, cs: Tensor, kc: Tensor,
+                vc: Tensor, out_scale: float, s: WindowAttnSpec, b: Batch, out: Tensor) -> None:
+    """``attn_prep`` and ``attn_window`` for one token per sequence."""
+    _need_gpu(proj, q_norm, k_norm, cs, kc, vc, out)
+    _batch(b, proj.shape[0])
+    _pages(kc, vc, s, proj.dtype)
+    _rotary(cs, s)
+    _rows2(out, "out", proj.dtype)
+    _vec(q_norm, s.D, "q_norm")
+    _vec(k_norm, s.D, "k_norm")
+    if b.S != 1 or out.shape != (b.B, s.H * s.E):
+        raise ValueError("attn_decode: shapes do not fit")
+    n = int(_abi.load_seq().aqs_attn_decode_slices(s.window, b.table.shape[1] * kc.shape[1]))
+    part = torch.empty((b.B, s.H, n, s.E + 4), dtype=torch.float32, device=proj.device)
+    _call("aqs_attn_decode", proj.device, _p(proj), proj.stride(0), o_q, o_k, o_v, o_gate, _DT[proj.dtype], _p(q_norm), _p(k_norm),
+          s.eps, _p(cs), cs.shape[0], s.rot, s.scale, s.window, float(out_scale), _p(b.pos), _p(b.table), b.table.shape[1],
+          kc.shape[1], kc.shape[0], _p(kc), _p(vc), _p(part), n, _p(out), out.stride(0), b.B, s.H, s.G, s.D, s.E, _stream(proj))

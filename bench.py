@@ -109,7 +109,8 @@ def parse():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=200)
     ap.add_argument("--warmup", type=int, default=1000)
-    ap.add_argument("--workload", default="decode", choices=["decode", "prefill", "fp8", "block", "model"])
+    ap.add_argument("--workload", default="decode", choices=["decode", "prefill", "fp8", "block", "model", "hybrid"])
+    ap.add_argument("--width", type=int, default=None, help="hybrid workload only: one model width (1024, 2048 or 4096) instead of all")
     ap.add_argument("--m", type=int, default=16, help="decode rows (1..16)")
     ap.add_argument("--mnk", default=None, help="prefill and fp8 workloads only: M,N,K of the int8 Linear instead of configuration 3's "
                     "4096,2048,2048 (e.g. 8192,8192,8192 for a profile of the GEMM's steady state)")
@@ -645,6 +646,114 @@ def bench_model(torch, ops, args, dev):
     }
 
 
+def hybrid_config(width):
+    """A hybrid decoder of a real model's layer sizes: inner width twice the model's for the state-space layers, as many
+    128-wide delta heads as fill the width, attention of 128-wide heads over a 1024-token window."""
+    h = width // 128
+    delta = {"conv": 4, "dim": 128, "heads": h, "kv_heads": h, "vdim": 128}
+    mlp = {"ff": width * 11 // 4, "kind": "dense", "limit": 7.0}
+    mamba = {"type": "mamba2", "mlp": mlp,
+             "mixer": {"conv": 4, "groups": 1, "heads": width // 32, "norm_groups": 1, "state": 128, "vdim": 64}}
+    chan = {"type": "channel_delta", "mixer": delta, "mlp": mlp}
+    left = {"dim": 128, "heads": h, "kv_heads": max(h // 4, 1), "mask": {"size": 1024}, "rot": {"base": 10000.0, "dims": 128},
+            "scale": 128 ** -0.5, "vdim": 128}
+    par = {"type": "parallel", "mlp": mlp,
+           "mixer": {"left": left, "left_scale": 0.5, "right": delta, "right_scale": 0.5}}
+    layers = [mamba, chan, mamba, par] * 2
+    shapes = {}
+    for i, l in enumerate(layers):
+        if l["type"] != "mamba2":
+            p = f"l{i}.mix." + ("right." if l["type"] == "parallel" else "")
+            shapes[p + "a1"] = shapes[p + "g1"] = (128, width)
+    return {"architecture": "Rudilix", "layers": layers, "norm": {"eps": 1e-6}, "residual_mult": 0.5, "vocab": 10000, "width": width}, shapes
+
+
+def bench_hybrid(torch, ops, args, dev):
+    """Prefill and decode throughput of the hybrid decoder (Rudilix: 4 state-space, 2 delta and 2 attention + delta
+    layers, bf16, random weights) beside AutoRegressiveLM of the same width, depth, feed-forward and vocabulary, in
+    bf16 (stock torch around float Linears) and in W8A8 with every fusion.  Prefill: one prompt, eager launches.
+    Decode: after that prompt, HIP graph replays of one step."""
+    from khaosz_amd import AutoRegressiveLM, Engine, HybridConfig, HybridLM, LMConfig, fuse_shared_inputs, quantize_model
+
+    dt, out, page, gen = torch.bfloat16, {}, 64, 32
+    widths = [args.width] if args.width else [1024, 2048, 4096]
+    for width in widths:
+        cfg, shapes = hybrid_config(width)
+        torch.manual_seed(5)
+        m = HybridLM(HybridConfig.from_dict(cfg, shapes), dt, dev).eval()
+        for name, t in m.tensors().items():
+            if name.endswith(("A_log", "dt_bias")):
+                t.normal_(-1.0, 0.5)
+            elif name.endswith("norm") and not name.startswith("final"):
+                t.fill_(1.0)
+            elif t.dim() == 2:
+                t.normal_(0.0, t.shape[1] ** -0.5)
+        weight_bytes = sum(p.numel() * p.element_size() for p in m.parameters()) - m.embed.numel() * 2
+        ar_cfg = LMConfig(vocab_size=10000, dim=width, n_layers=8, n_heads=width // 128, n_kv_heads=max(width // 512, 1),
+                          dim_ffn=width * 11 // 4, max_len=4096 + 2 * gen)
+        ar = AutoRegressiveLM(ar_cfg).to(dev).to(dt).eval()
+        arq = AutoRegressiveLM(ar_cfg).to(dev).to(dt).eval()
+        quantize_model(arq, target_modules={"q_proj", "k_proj", "v_proj", "o_proj", "up", "gate", "down", "lm_head"})
+        fuse_shared_inputs(arq, norms=True, decode_attention=True, residuals=True)
+        row = {"hybrid_weight_bytes": weight_bytes}
+        for S in (512, 4096):
+            ids = torch.randint(0, 10000, (1, S), generator=torch.Generator().manual_seed(S)).tolist()[0]
+            e = Engine(m, S + 2 * gen, 1, page)
+
+            def prefill(i=0):
+                h = e.open()
+                e.step([h], [ids], [S - 1])
+                e.close(h)
+            r = {"hybrid": {"prefill_ms": eager_time_ms(torch, prefill, 5, 2)}}
+            for B in (1, 8):
+                e = Engine(m, B * (S + gen), B, page)
+                hs = [e.open() for _ in range(B)]
+                for h in hs:
+                    e.step([h], [ids], [])
+                for _ in range(3):
+                    e.step(hs, [[7]] * B)
+                g = e._graphs[B].graph
+                r["hybrid"][f"decode_ms_b{B}"] = eager_time_ms(torch, lambda i=0: g.replay(), 50, 5)
+                t0 = time.perf_counter()
+                for _ in range(gen - 8):
+                    e.step(hs, [[7]] * B)
+                torch.cuda.synchronize()
+                r["hybrid"][f"engine_step_ms_b{B}"] = (time.perf_counter() - t0) * 1e3 / (gen - 8)
+                del e
+            P = (S + gen + page - 1) // page
+            for name, mod in (("ar_bf16", ar), ("ar_w8a8", arq)):
+                r[name] = {}
+                for B in (1, 8):
+                    c = mod.new_cache(B * P, page)
+                    table = torch.arange(B * P, device=dev).view(B, P)
+                    x = torch.tensor([ids] * B, device=dev)
+                    if B == 1:
+                        r[name]["prefill_ms"] = eager_time_ms(
+                            torch, lambda i=0: mod(x, paged_cache=c.bind(table, S), start_pos=0)["logits"][:, -1:], 5, 2)
+                    else:
+                        mod(x, paged_cache=c.bind(table, S), start_pos=0)
+                    one = x[:, :1].contiguous()
+                    r[name][f"decode_ms_b{B}"] = graph_time_ms(
+                        torch, lambda i=0: mod(one, paged_cache=c.bind(table, S + 1), start_pos=S), 20, 5)
+                    del c
+            for d in r.values():
+                d["prefill_tok_s"] = S / (d["prefill_ms"] * 1e-3)
+                d["decode_tok_s_b1"], d["decode_tok_s_b8"] = 1e3 / d["decode_ms_b1"], 8e3 / d["decode_ms_b8"]
+            row[f"prompt_{S}"] = r
+        out[f"width_{width}"] = row
+        del m, ar, arq
+    w = out[f"width_{widths[-1] if len(widths) < 3 else 2048}"]
+    ms = w["prompt_4096"]["hybrid"]["decode_ms_b1"]
+    gbs = w["hybrid_weight_bytes"] / (ms * 1e-3) / 1e9
+    return {"workload": "hybrid decoder (Rudilix, 8 layers, bf16, random weights) beside AutoRegressiveLM of equal size: "
+                        "prefill of one prompt, decode of 1 and 8 sequences",
+            "value": w["prompt_4096"]["hybrid"]["decode_tok_s_b1"], "unit": "tok/s", "ms_per_step": ms, "dtype": "bf16",
+            "widths": out,
+            "roofline": {"bound": "hbm", "kernel": "one decode step of one sequence (weights read once)", "achieved": gbs,
+                         "peak": PEAK_HBM_GBS, "unit": "GB/s", "frac": gbs / PEAK_HBM_GBS, "traffic": None},
+            "shape": (1, 0, 0)}
+
+
 def measure_ceilings(torch, ops, dev, calibrate=True):
     """What this part delivers on trivial kernels (the lab library's probes, csrc/aq_lab.h):
       * an MFMA-only loop with constant operands (no bit toggling: the clock stays at its maximum) and with random
@@ -884,13 +993,13 @@ def main():
     dev = torch.device("cuda:0")
     torch.cuda.set_device(dev)
     fns = {"decode": bench_decode, "prefill": bench_prefill, "fp8": bench_fp8, "block": bench_block,
-           "model": bench_model}
+           "model": bench_model, "hybrid": bench_hybrid}
     with torch.inference_mode():
         # the part's own ceilings first: the roofline objects of the workloads quote them
         CEIL.update(measure_ceilings(torch, ops, dev, calibrate=False))
         main_res = fns[args.workload](torch, ops, args, dev)
         extra = {}
-        if not args.no_extra:
+        if not args.no_extra and args.workload != "hybrid":
             for name in ("decode", "prefill", "fp8", "block"):  # "model" only on request: it takes a minute
                 if name != args.workload:
                     extra[name] = fns[name](torch, ops, args, dev)
@@ -902,9 +1011,9 @@ def main():
                     extra[f"decode_m{m}"] = r
                 extra["batch_32_to_256"] = bench_few_dozen_rows(torch, ops, args, dev)
         ceilings = dict(CEIL)
-        if not args.no_extra:  # launches GEMMs of other shapes: left out of single-workload (profiling) runs
+        if not args.no_extra and args.workload != "hybrid":  # launches GEMMs of other shapes: left out of single-workload (profiling) runs
             ceilings["gemm_operand_data_and_stock_library"] = gemm_calibration(torch, ops, dev)
-        if not args.no_extra and args.workload != "model":
+        if not args.no_extra and args.workload not in ("model", "hybrid"):
             # the reference's own generation benchmark: about a minute; skipped when this run is already long
             if time.time() - t_start < 150:
                 m = bench_model(torch, ops, args, dev)
@@ -916,7 +1025,7 @@ def main():
                 extra["model"] = {"skipped": "time budget of the default run spent"}
     per_step = main_res.get("bytes_per_step") or main_res.get("ops_per_step") or main_res.get("flops_per_step")
     cpu = None
-    if not args.no_cpu and args.workload not in ("block", "model"):
+    if not args.no_cpu and args.workload not in ("block", "model", "hybrid"):
         cpu = cpu_baseline(args.workload, main_res["shape"], main_res["unit"], per_step)
         if not args.no_extra and "prefill" in extra:
             # one pass of the prefill shape as well, so both halves of the metric have a CPU figure
@@ -925,7 +1034,7 @@ def main():
     for r in [main_res, *extra.values()]:
         r.pop("shape", None)
     top = ("workload", "value", "unit", "ms_per_step", "dtype", "roofline", "eager_ms_per_step")
-    detail = {k: v for k, v in main_res.items() if k not in top} if args.workload in ("block", "model") else None
+    detail = {k: v for k, v in main_res.items() if k not in top} if args.workload in ("block", "model", "hybrid") else None
     line = {
         "metric": METRIC, "value": main_res["value"], "unit": main_res["unit"], "n_gpus": 1,
         "steps": args.steps, "warmup": args.warmup, "ms_per_step": main_res["ms_per_step"],

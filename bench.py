@@ -705,7 +705,7 @@ def bench_hybrid(torch, ops, args, dev):
                 e.step([h], [ids], [S - 1])
                 e.close(h)
             r = {"hybrid": {"prefill_ms": eager_time_ms(torch, prefill, 5, 2)}}
-            for B in (1, 8):
+            for B in (1, 4):
                 e = Engine(m, B * (S + gen), B, page)
                 hs = [e.open() for _ in range(B)]
                 for h in hs:
@@ -723,7 +723,7 @@ def bench_hybrid(torch, ops, args, dev):
             P = (S + gen + page - 1) // page
             for name, mod in (("ar_bf16", ar), ("ar_w8a8", arq)):
                 r[name] = {}
-                for B in (1, 8):
+                for B in (1, 4):
                     c = mod.new_cache(B * P, page)
                     table = torch.arange(B * P, device=dev).view(B, P)
                     x = torch.tensor([ids] * B, device=dev)
@@ -738,7 +738,7 @@ def bench_hybrid(torch, ops, args, dev):
                     del c
             for d in r.values():
                 d["prefill_tok_s"] = S / (d["prefill_ms"] * 1e-3)
-                d["decode_tok_s_b1"], d["decode_tok_s_b8"] = 1e3 / d["decode_ms_b1"], 8e3 / d["decode_ms_b8"]
+                d["decode_tok_s_b1"], d["decode_tok_s_b4"] = 1e3 / d["decode_ms_b1"], 4e3 / d["decode_ms_b4"]
             row[f"prompt_{S}"] = r
         out[f"width_{width}"] = row
         del m, ar, arq
@@ -746,7 +746,7 @@ def bench_hybrid(torch, ops, args, dev):
     ms = w["prompt_4096"]["hybrid"]["decode_ms_b1"]
     gbs = w["hybrid_weight_bytes"] / (ms * 1e-3) / 1e9
     return {"workload": "hybrid decoder (Rudilix, 8 layers, bf16, random weights) beside AutoRegressiveLM of equal size: "
-                        "prefill of one prompt, decode of 1 and 8 sequences",
+                        "prefill of one prompt, decode of 1 and 4 sequences",
             "value": w["prompt_4096"]["hybrid"]["decode_tok_s_b1"], "unit": "tok/s", "ms_per_step": ms, "dtype": "bf16",
             "widths": out,
             "roofline": {"bound": "hbm", "kernel": "one decode step of one sequence (weights read once)", "achieved": gbs,

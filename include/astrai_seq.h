@@ -43,7 +43,7 @@ int aqs_head_norm_gate(const float *o, const void *gate, int64_t ldg, int dtype,
  * out_kind 0: out of dtype (+ bias) 1: fp32 into res   2: res += mult * result
  *          3: clamped GLU of w's first N/2 rows (gate) and last N/2 rows (up), out [M, N/2]
  * Pairs served: 0-0, 0-2, 1-0, 1-1, 1-3, 2-2; sizes: aqs_gemv_ok. */
-int aqs_gemv_ok(int64_t M, int64_t N, int64_t K);
+int aqs_gemv_ok(int dtype, int64_t M, int64_t N, int64_t K);
 int aqs_gemv(int in_kind, int out_kind, int dtype, const void *x, int64_t ldx, const float *xf, const float *gain, float eps,
              int64_t groups, const void *w, const float *bias, float mult, float limit, float *res, void *out, int64_t ldo,
              int64_t M, int64_t N, int64_t K, void *stream);
@@ -82,6 +82,22 @@ int aqs_ssd_step(const void *proj, int64_t ld, int64_t o_xbc, int64_t o_dt, int 
                  void *ring, const int32_t *slots, const int32_t *pos, const float *dt_bias, const float *a_log,
                  const float *skip, float *state, float *y, int64_t B, int64_t H, int64_t G, int64_t N, int64_t P, int64_t taps,
                  void *stream);
+
+/* ---- both recurrences over long prompts, in chunks of 64 tokens, convolution included (call aqs_conv_push after).
+ * Sizes: aqs_chunked_ok(D or N, taps).  ws: scratch of at least the *_ws functions' number of floats. */
+int aqs_chunked_ok(int64_t rows, int64_t taps);
+int64_t aqs_delta_chunked_ws(int64_t B, int64_t S, int64_t H, int64_t D, int64_t E);
+int64_t aqs_ssd_chunked_ws(int64_t B, int64_t S, int64_t G, int64_t N);
+/* aqs_delta_prep and aqs_delta_scan */
+int aqs_delta_chunked(const void *qkv, int64_t ld, const void *raw, int64_t ld_raw, const void *beta_raw, int64_t ld_beta,
+                      int dtype, const float *w, const void *ring, const int32_t *slots, const int32_t *pos, const float *a_log,
+                      const float *dt_bias, float *ws, int64_t ws_floats, float *state, float *out, int64_t B, int64_t S, int64_t H,
+                      int64_t G, int64_t D, int64_t E, int64_t taps, void *stream);
+/* aqs_conv_silu and aqs_ssd_scan; xbc: the raw projection columns x | B | C */
+int aqs_ssd_chunked(const void *xbc, int64_t ld, const void *dt_raw, int64_t ld_dt, int dtype, const float *conv_w,
+                    const float *conv_b, const void *ring, const int32_t *slots, const int32_t *pos, const float *dt_bias,
+                    const float *a_log, const float *skip, float *ws, int64_t ws_floats, float *state, float *out, int64_t B,
+                    int64_t S, int64_t H, int64_t G, int64_t N, int64_t P, int64_t taps, void *stream);
 
 /* ---- sliding-window attention on pages: kc [n_pages, page, G, D], vc [n_pages, page, G, E], table [B, P] */
 /* RMS norm (plain weight) and interleaved rotation of the first `rot` dimensions of q and k; q -> q_out [M, H, D],

@@ -97,7 +97,7 @@ SEQ_SYMBOLS = {
     "aqs_clamped_glu": (_int, [_vp, _i64, _int, _f32, _vp, _i64, _i64, _vp]),
     "aqs_gated_group_norm": (_int, [_vp, _vp, _i64, _int, _vp, _f32, _vp, _i64, _i64, _i64, _i64, _vp]),
     "aqs_head_norm_gate": (_int, [_vp, _vp, _i64, _int, _vp, _f32, _f32, _vp, _i64, _i64, _i64, _i64, _vp]),
-    "aqs_gemv_ok": (_int, [_i64, _i64, _i64]),
+    "aqs_gemv_ok": (_int, [_int, _i64, _i64, _i64]),
     "aqs_gemv": (_int, [_int, _int, _int, _vp, _i64, _vp, _vp, _f32, _i64, _vp, _vp, _f32, _f32, _vp, _vp, _i64,
         _i64, _i64, _i64, _vp]),
     "aqs_conv_silu": (_int, [_vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _vp]),
@@ -112,6 +112,13 @@ SEQ_SYMBOLS = {
         _i64, _vp]),
     "aqs_ssd_step": (_int, [_vp, _i64, _i64, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64,
         _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_chunked_ok": (_int, [_i64, _i64]),
+    "aqs_delta_chunked_ws": (_i64, [_i64, _i64, _i64, _i64, _i64]),
+    "aqs_ssd_chunked_ws": (_i64, [_i64, _i64, _i64, _i64]),
+    "aqs_delta_chunked": (_int, [_vp, _i64, _vp, _i64, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _vp,
+        _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_ssd_chunked": (_int, [_vp, _i64, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _vp,
+        _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
     "aqs_attn_prep": (_int, [_vp, _i64, _i64, _i64, _i64, _int, _vp, _vp, _f32, _vp, _i64, _i64, _vp, _vp, _i64,
         _i64, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
     "aqs_attn_window_ok": (_int, [_int, _i64, _i64, _i64]),

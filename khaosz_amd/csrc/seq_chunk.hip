@@ -1,0 +1,696 @@
+// The two linear recurrences over long prompts, in chunks of 64 tokens on the fp32 matrix cores
+// (v_mfma_f32_16x16x4_f32: every operand and sum stays fp32).  seq_scan.hip does one token after the other; here the
+// tokens of a chunk meet in matrix products and only the step from chunk to chunk is sequential.
+//
+// Delta rule, one head, state S before the chunk, G_i the sum of the chunk's log decays up to and including token i:
+//     u_i + beta_i sum_{j<i} <k_i e^{G_i - G_j}, k_j> u_j  =  beta_i (v_i - S^T (k_i e^{G_i}))
+//     o_i = S^T (q_i e^{G_i}) + sum_{j<=i} <q_i e^{G_i - G_j}, k_j> u_j
+//     S  <- e^{G_C} S + sum_j (k_j e^{G_C - G_j}) u_j^T
+// so with (I + A) the unit triangular matrix on the left:  u = U0 - W S  with  W = (I + A)^-1 (beta k e^G),
+// U0 = (I + A)^-1 (beta v).  Three launches: `prep` (per chunk and head: convolution, norms, decays, A and the masked
+// query-key matrix), `solve` (W and U0, one thread per column), `scan` (per head and 16 columns of S: the chunks in order).
+//
+// A decay can be anything in (0, 1], so e^{G_i - G_j} must not be split into e^{G_i} and e^{-G_j} across a chunk.  The
+// sums are kept by blocks of 16 tokens: between blocks the split point is the later block's start, and both factors are
+// at most 1; inside a block it is the block's middle while every factor stays below 2^60, and otherwise the
+// differences are exponentiated pair by pair.
+//
+// State space (SSD), same idea with one scalar decay per head and token: y = e^{L_i} S^T C_i + sum_{j<=i} M_ij x_j + D x_i,
+// M_ij = <C_i, B_j> e^{L_i - L_j} dt_j;  S <- e^{L_C} S + sum_j e^{L_C - L_j} dt_j B_j x_j^T.  C B^T belongs to the
+// group and is computed once (`ssd_group`), the rest in one launch (`ssd_chunks`).
+#include "seq_common.h"
+
+namespace sq {
+
+constexpr int CH = 64;    // tokens per chunk
+constexpr int BL = 16;    // tokens per block
+constexpr int NB = CH / BL;
+constexpr int CT = 16;    // state columns per workgroup of the scans
+constexpr int MAX_TAPS = 4;
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+
+// D[16 x 16] += A[16 x 16] B[16 x 16], contraction in four steps of 4.  Lane l: row (A) or column (B) l % 16, and the
+// elements 4 (l / 16) .. + 4 of the contraction; D: column l % 16, rows 4 (l / 16) .. + 4.
+__device__ __forceinline__ f32x4 mma16(const float4& a, const float4& b, f32x4 c) {
+  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b.x, c, 0, 0, 0);
+  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b.y, c, 0, 0, 0);
+  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b.z, c, 0, 0, 0);
+  return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b.w, c, 0, 0, 0);
+}
+__device__ __forceinline__ float ex2(float x) { return __builtin_amdgcn_exp2f(x); }
+__device__ __forceinline__ float4 ld4(const float* p) { return *reinterpret_cast<const float4*>(p); }
+
+// Convolution + SiLU of one channel over n consecutive tokens from token t0 on; put(i, value) for each
+template <typename T, typename F>
+__device__ __forceinline__ void conv_run(const T* in, int64_t ld, int64_t tok0, int t0, int n, int pos, const T* ring, int taps, int C,
+                                         int c, const float* w, float bias, F put) {
+  float wj[MAX_TAPS], win[MAX_TAPS];  // right-aligned: entry MAX_TAPS - 1 is the current token
+#pragma unroll
+  for (int j = 0; j < MAX_TAPS; ++j) {
+    const int back = MAX_TAPS - 1 - j;
+    wj[j] = back < taps ? w[c * taps + taps - 1 - back] : 0.0f;
+    win[j] = 0.0f;
+    if (back > 0 && back < taps) {
+      const int a = pos + t0 - back;  // position
+      if (a >= pos) win[j] = to_f32(in[(tok0 + (a - pos)) * ld + c]);
+      else if (a >= 0) win[j] = to_f32(ring[(int64_t)(a % taps) * C + c]);
+    }
+  }
+  // the inputs are requested 16 at a time
+  for (int i0 = 0; i0 < n; i0 += 16) {
+    float x[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) x[i] = i0 + i < n ? to_f32(in[(tok0 + t0 + i0 + i) * ld + c]) : 0.0f;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      if (i0 + i >= n) break;
+      win[MAX_TAPS - 1] = x[i];
+      float acc = bias;
+#pragma unroll
+      for (int j = 0; j < MAX_TAPS; ++j) acc = fmaf(wj[j], win[j], acc);
+#pragma unroll
+      for (int j = 0; j + 1 < MAX_TAPS; ++j) win[j] = win[j + 1];
+      put(i0 + i, silu(acc));
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------------- delta: prep
+struct DeltaChunkArgs {
+  const int* slots;
+  const int* pos;
+  const float* conv_w;   // [C, taps]
+  const float* a_log;    // [H]
+  const float* dt_bias;  // [H * D]
+  float* A;              // [BC, H, 64, 64]  (BC = B * chunks)
+  float* QK;             // [BC, H, 64, 64]
+  float* W;              // [BC, H, 64, DP]  in: beta k e^G
+  float* U;              // [BC, H, 64, EP]  in: beta v
+  float* Q;              // [BC, H, 64, DP]  q e^G
+  float* K;              // [BC, H, DP, 64]  k e^{G_C - G}, transposed
+  float* gc;             // [BC, H, DP]      e^{G_C}
+  int64_t ld, ld_raw, ld_beta;
+  int S, NC, H, G, D, E, DP, EP, taps, C;
+};
+
+template <int DP, typename T>
+__global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p, const T* qkv, const T* raw, const T* braw, const T* ring0) {
+  constexpr int PT = DP + 4, PG = DP + 2;
+  extern __shared__ __align__(16) float lds[];
+  // log2 decays summed within their block of 16, and the sums of whole blocks.  Only differences of them are used, and
+  // one token that forgets everything must not cost the digits of the others: double.
+  double* g_s = reinterpret_cast<double*>(lds);  // [64][PG]
+  double* tot = g_s + CH * PG;                   // [NB][DP]
+  float* q_s = reinterpret_cast<float*>(tot + NB * DP);  // [64][PT]
+  float* k_s = q_s + CH * PT;
+  float* b_s = k_s + CH * PT;                    // [64] beta
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int c = blockIdx.x % p.NC, b = blockIdx.x / p.NC, h = blockIdx.y, j = h / (p.H / p.G);
+  const int t0 = c * CH, n = p.S - t0 < CH ? p.S - t0 : CH;
+  const int pos = p.pos[b], D = p.D, E = p.E;
+  const int64_t tok0 = (int64_t)b * p.S, ch = (int64_t)blockIdx.x * p.H + h;
+  const T* ring = ring0 + (int64_t)p.slots[b] * p.taps * p.C;
+
+  if (tid < CH) b_s[tid] = tid < n ? sigmoid(to_f32(braw[(tok0 + t0 + tid) * p.ld_beta + h])) : 0.0f;
+  for (int x = tid; x < 2 * DP; x += 256) {
+    float* dst = (x < DP ? q_s : k_s) + x % DP;
+    const int d = x % DP, m = d < D ? n : 0;
+    if (m) conv_run(qkv, p.ld, tok0, t0, n, pos, ring, p.taps, p.C, (x < DP ? 0 : p.G * D) + j * D + d, p.conv_w, 0.0f,
+                    [&](int i, float v) { dst[i * PT] = v; });
+    for (int i = m; i < CH; ++i) dst[i * PT] = 0.0f;
+  }
+  const float a = -expf(p.a_log[h]) * 1.44269504088896341f;
+  for (int d = tid; d < DP; d += 256) {
+    double sum = 0.0;
+    const float bias = d < D ? p.dt_bias[h * D + d] : 0.0f;
+    const T* src = raw + (tok0 + t0) * p.ld_raw + h * D + d;
+#pragma unroll 16
+    for (int i = 0; i < CH; ++i) {
+      if (i % BL == 0) sum = 0.0;
+      if (i < n && d < D) sum += (double)(a * softplus(to_f32(src[i * p.ld_raw]) + bias));
+      g_s[i * PG + d] = sum;
+      if (i % BL == BL - 1) tot[(i / BL) * DP + d] = sum;
+    }
+  }
+  __syncthreads();
+  // unit vectors: a wavefront takes 16 tokens
+  for (int i = wave * BL; i < wave * BL + BL; ++i) {
+    float sq = 0.0f, sk = 0.0f;
+    for (int d = lane; d < DP; d += 64) sq += q_s[i * PT + d] * q_s[i * PT + d], sk += k_s[i * PT + d] * k_s[i * PT + d];
+    const float rq = 1.0f / (sqrtf(wave_sum(sq) + 1e-6f) * sqrtf((float)D)), rk = 1.0f / sqrtf(wave_sum(sk) + 1e-6f);
+    for (int d = lane; d < DP; d += 64) q_s[i * PT + d] *= rq, k_s[i * PT + d] *= rk;
+  }
+  // beta v, by channel (64-token pieces of 16 so that all threads have one)
+  for (int x = tid; x < p.EP * NB; x += 256) {
+    const int e = x % p.EP, i0 = (x / p.EP) * BL;
+    float* dst = p.U + (ch * CH + i0) * p.EP + e;
+    const int m = e < E ? (n - i0 < BL ? (n - i0 > 0 ? n - i0 : 0) : BL) : 0;
+    if (m) conv_run(qkv, p.ld, tok0, t0 + i0, m, pos, ring, p.taps, p.C, 2 * p.G * D + h * E + e, p.conv_w, 0.0f,
+                    [&](int i, float v) { dst[(int64_t)i * p.EP] = b_s[i0 + i] * v; });
+    for (int i = m; i < BL; ++i) dst[(int64_t)i * p.EP] = 0.0f;
+  }
+  __syncthreads();
+  // ---- the scaled copies
+  for (int x = tid; x < CH * DP; x += 256) {
+    const int i = x / DP, d = x % DP, I = i / BL;
+    double base = g_s[i * PG + d];
+    for (int k = 0; k < I; ++k) base += tot[k * DP + d];
+    const float e = ex2((float)base);
+    p.Q[ch * CH * DP + x] = q_s[i * PT + d] * e;
+    p.W[ch * CH * DP + x] = b_s[i] * k_s[i * PT + d] * e;
+  }
+  for (int x = tid; x < DP * CH; x += 256) {
+    const int d = x / CH, i = x % CH, I = i / BL;
+    double rest = tot[I * DP + d] - g_s[i * PG + d];
+    for (int k = I + 1; k < NB; ++k) rest += tot[k * DP + d];
+    p.K[ch * DP * CH + x] = k_s[i * PT + d] * ex2((float)rest);
+  }
+  for (int d = tid; d < DP; d += 256) p.gc[ch * DP + d] = ex2((float)(tot[d] + tot[DP + d] + tot[2 * DP + d] + tot[3 * DP + d]));
+  // ---- A and QK: 10 block pairs I >= J, the four diagonal ones first (one per wavefront)
+  float* A = p.A + ch * CH * CH;
+  float* QK = p.QK + ch * CH * CH;
+  const int r16 = lane & 15, q4 = (lane >> 4) * 4;
+  for (int pair = wave; pair < NB * NB; pair += 4) {
+    // pairs 0..3: diagonal; 4..9: below it; 10..15: above, zero
+    int I, J;
+    if (pair < 4) I = J = pair;
+    else {
+      constexpr int RI[12] = {1, 2, 2, 3, 3, 3, 0, 0, 1, 0, 1, 2}, RJ[12] = {0, 0, 1, 0, 1, 2, 1, 2, 2, 3, 3, 3};
+      I = RI[pair - 4], J = RJ[pair - 4];
+    }
+    f32x4 sa = {0, 0, 0, 0}, sq = {0, 0, 0, 0};
+    const int i = I * BL + r16, jj = J * BL + r16;  // this lane's row (A operand) and column (B operand)
+    bool direct = false;
+    if (I == J) {
+      // both factors around the block's middle; 2^60 leaves room for the sums
+      float worst = 0.0f;
+      for (int d = q4; d < DP; d += 16)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) worst = fmaxf(worst, fabsf((float)(g_s[i * PG + d + r] - g_s[(I * BL + BL / 2) * PG + d + r])));
+      direct = __builtin_amdgcn_ballot_w64(worst > 60.0f) != 0;
+    }
+    if (I >= J && !direct) {
+      for (int d = q4; d < DP; d += 16) {
+        // ei: from the split point to the row; ej: from the column to the split point (the middle of a diagonal block,
+        // else the start of the row's block: the rest of the column's block and the blocks between)
+        float e_i[4], e_j[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const double gi = g_s[i * PG + d + r], gj = g_s[jj * PG + d + r];
+          double to_row = gi, to_split;
+          if (I == J) {
+            const double mid = g_s[(I * BL + BL / 2) * PG + d + r];
+            to_row = gi - mid, to_split = mid - gj;
+          } else {
+            to_split = tot[J * DP + d + r] - gj;
+            for (int k = J + 1; k < I; ++k) to_split += tot[k * DP + d + r];
+          }
+          e_i[r] = ex2((float)to_row), e_j[r] = ex2((float)to_split);
+        }
+        const float4 ei = make_float4(e_i[0], e_i[1], e_i[2], e_i[3]), ej = make_float4(e_j[0], e_j[1], e_j[2], e_j[3]);
+        const float4 ki = ld4(&k_s[i * PT + d]), qi = ld4(&q_s[i * PT + d]), kj = ld4(&k_s[jj * PT + d]);
+        const float4 bj = make_float4(kj.x * ej.x, kj.y * ej.y, kj.z * ej.z, kj.w * ej.w);
+        sa = mma16(make_float4(ki.x * ei.x, ki.y * ei.y, ki.z * ei.z, ki.w * ei.w), bj, sa);
+        sq = mma16(make_float4(qi.x * ei.x, qi.y * ei.y, qi.z * ei.z, qi.w * ei.w), bj, sq);
+      }
+    } else if (direct) {
+      // entry (row q4 + r, column r16) of the block, pair by pair
+      for (int d = 0; d < DP; ++d) {
+        const double gj = g_s[jj * PG + d];
+        const float kj = k_s[jj * PT + d];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int row = I * BL + q4 + r;
+          const float e = kj * ex2(fminf((float)(g_s[row * PG + d] - gj), 0.0f));  // rows above the diagonal are not used
+          sa[r] = fmaf(k_s[row * PT + d], e, sa[r]);
+          sq[r] = fmaf(q_s[row * PT + d], e, sq[r]);
+        }
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = I * BL + q4 + r, col = J * BL + r16;
+      A[row * CH + col] = col < row ? b_s[row] * sa[r] : 0.0f;
+      QK[row * CH + col] = col <= row ? sq[r] : 0.0f;
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------------- delta: solve
+// x <- (I + A)^-1 x, column by column: one thread holds a column of 64; A is uniform and comes through scalar loads
+__global__ __launch_bounds__(256) void delta_chunk_solve_kernel(const float* __restrict__ A, float* __restrict__ W, float* __restrict__ U,
+                                                                int DP, int EP) {
+  const int64_t ch = blockIdx.x;
+  const int col = blockIdx.y * 256 + threadIdx.x;
+  if (col >= DP + EP) return;
+  const int ld = col < DP ? DP : EP;
+  float* x = col < DP ? W + ch * CH * DP + col : U + ch * CH * EP + (col - DP);
+  const float* a = A + ch * CH * CH;
+  float v[CH];
+#pragma unroll
+  for (int i = 0; i < CH; ++i) v[i] = x[(int64_t)i * ld];
+#pragma unroll
+  for (int i = 1; i < CH; ++i) {
+    float s0 = 0.0f, s1 = 0.0f;
+#pragma unroll
+    for (int k = 0; k < i; ++k) {
+      if (k & 1) s1 = fmaf(a[i * CH + k], v[k], s1);
+      else s0 = fmaf(a[i * CH + k], v[k], s0);
+    }
+    v[i] -= s0 + s1;
+  }
+#pragma unroll
+  for (int i = 0; i < CH; ++i) x[(int64_t)i * ld] = v[i];
+}
+
+// ---------------------------------------------------------------------------------------------- delta: scan
+struct DeltaScanArgs {
+  const float *W, *U, *Q, *K, *QK, *gc;
+  float* state;  // [slots, H, E, D]
+  float* out;    // [M, H, E]
+  const int* slots;
+  const int* pos;
+  int S, NC, H, D, E, EP;
+};
+
+// rows d .. d + 4 of a state column (rows past D are zero)
+__device__ __forceinline__ f32x4 load_state4(const float* col, int d, int D, bool ok) {
+  f32x4 v = {0, 0, 0, 0};
+  if (!ok) return v;
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+    if (d + r < D) v[r] = col[d + r];
+  return v;
+}
+__device__ __forceinline__ void store_state4(float* col, int d, int D, const f32x4& v) {
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+    if (d + r < D) col[d + r] = v[r];
+}
+
+template <int DP>
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) void delta_chunk_scan_kernel(DeltaScanArgs p) {
+  constexpr int KB = DP / 16;               // groups of 16 in the contraction over rows
+  constexpr int NT = (KB + 3) / 4;          // 16-row tiles of the state per wavefront
+  constexpr int SP = DP + 4, UP = CH + 4;
+  __shared__ __align__(16) float s_s[CT * SP];  // the state, column by column
+  __shared__ __align__(16) float u_s[CT * UP];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int r16 = lane & 15, q4 = (lane >> 4) * 4;
+  const int tile = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  const int e = tile * CT + r16, D = p.D;
+  float* col = p.state + (((int64_t)p.slots[b] * p.H + h) * p.E + (e < p.E ? e : 0)) * D;
+  f32x4 s[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    const int d = (wave + 4 * t) * 16 + q4;
+    s[t] = load_state4(col, d, D, e < p.E && p.pos[b] > 0 && d < DP);
+  }
+  float4 w[KB], q[KB], k[NT][NB], a[NB], gc[NT];
+  float u0[4];
+  const int row = wave * BL + r16;          // this lane's token (A operand)
+  auto base = [&](int c) -> int64_t { return ((int64_t)b * p.NC + c) * p.H + h; };
+  auto load_w = [&](int64_t ch) __attribute__((always_inline)) {
+#pragma unroll
+    for (int x = 0; x < KB; ++x) w[x] = ld4(p.W + (ch * CH + row) * DP + x * 16 + q4);
+  };
+  auto load_q = [&](int64_t ch) __attribute__((always_inline)) {
+#pragma unroll
+    for (int x = 0; x < KB; ++x) q[x] = ld4(p.Q + (ch * CH + row) * DP + x * 16 + q4);
+  };
+  auto load_u = [&](int64_t ch) __attribute__((always_inline)) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) u0[r] = e < p.EP ? p.U[(ch * CH + wave * BL + q4 + r) * p.EP + e] : 0.0f;
+  };
+  auto load_a = [&](int64_t ch) __attribute__((always_inline)) {
+#pragma unroll
+    for (int x = 0; x < NB; ++x) a[x] = ld4(p.QK + (ch * CH + row) * CH + x * 16 + q4);
+  };
+  auto load_k = [&](int64_t ch) __attribute__((always_inline)) {
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      if (wave + 4 * t >= KB) break;
+      gc[t] = ld4(p.gc + ch * DP + (wave + 4 * t) * 16 + q4);
+#pragma unroll
+      for (int x = 0; x < NB; ++x) k[t][x] = ld4(p.K + (ch * DP + (wave + 4 * t) * 16 + r16) * CH + x * 16 + q4);
+    }
+  };
+  load_w(base(0)), load_q(base(0)), load_u(base(0)), load_a(base(0)), load_k(base(0));
+  for (int c = 0; c < p.NC; ++c) {
+    const int64_t nx = base(c + 1 < p.NC ? c + 1 : c);
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+      if (wave + 4 * t < KB) *reinterpret_cast<f32x4*>(&s_s[r16 * SP + (wave + 4 * t) * 16 + q4]) = s[t];
+    __syncthreads();
+    f32x4 ws = {0, 0, 0, 0}, o = {0, 0, 0, 0};
+#pragma unroll
+    for (int x = 0; x < KB; ++x) {
+      const float4 sv = ld4(&s_s[r16 * SP + x * 16 + q4]);
+      ws = mma16(w[x], sv, ws);
+      o = mma16(q[x], sv, o);
+    }
+    f32x4 u;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) u[r] = u0[r] - ws[r];
+    *reinterpret_cast<f32x4*>(&u_s[r16 * UP + wave * BL + q4]) = u;
+    load_w(nx), load_q(nx), load_u(nx);
+    __syncthreads();
+    float4 uv[NB];
+#pragma unroll
+    for (int x = 0; x < NB; ++x) uv[x] = ld4(&u_s[r16 * UP + x * 16 + q4]);
+#pragma unroll
+    for (int x = 0; x < NB; ++x) o = mma16(a[x], uv[x], o);
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      if (wave + 4 * t >= KB) break;
+      s[t][0] *= gc[t].x, s[t][1] *= gc[t].y, s[t][2] *= gc[t].z, s[t][3] *= gc[t].w;
+#pragma unroll
+      for (int x = 0; x < NB; ++x) s[t] = mma16(k[t][x], uv[x], s[t]);
+    }
+    load_a(nx), load_k(nx);
+    const int t0 = c * CH + wave * BL + q4;
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (t0 + r < p.S && e < p.E) p.out[(((int64_t)b * p.S + t0 + r) * p.H + h) * p.E + e] = o[r];
+  }
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    const int d = (wave + 4 * t) * 16 + q4;
+    if (e < p.E && d < DP) store_state4(col, d, D, s[t]);
+  }
+}
+
+// ---------------------------------------------------------------------------------------------- state space
+struct SsdChunkArgs {
+  const int* slots;
+  const int* pos;
+  const float* conv_w;  // [C, taps], channels x | B | C
+  const float* conv_b;
+  const float* dt_bias;
+  const float* a_log;
+  const float* skip;
+  float* CB;     // [BC, G, 64, 64]
+  float* Cm;     // [BC, G, 64, NP]
+  float* Bt;     // [BC, G, NP, 64]
+  float* state;  // [slots, H, P, N]
+  float* out;    // [M, H, P]
+  int64_t ld, ld_dt;
+  int S, NC, H, G, N, P, NP, taps, C;
+};
+
+template <int NP, typename T>
+__global__ __launch_bounds__(256) void ssd_group_kernel(SsdChunkArgs p, const T* xbc, const T* ring0) {
+  constexpr int PT = NP + 4;
+  extern __shared__ __align__(16) float lds[];
+  float* b_s = lds;            // [64][PT]
+  float* c_s = lds + CH * PT;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int c = blockIdx.x % p.NC, b = blockIdx.x / p.NC, g = blockIdx.y;
+  const int t0 = c * CH, n = p.S - t0 < CH ? p.S - t0 : CH, pos = p.pos[b], N = p.N;
+  const int64_t tok0 = (int64_t)b * p.S, ch = (int64_t)blockIdx.x * p.G + g;
+  const T* ring = ring0 + (int64_t)p.slots[b] * p.taps * p.C;
+  for (int x = tid; x < 2 * NP * NB; x += 256) {  // channel and block of 16 tokens
+    const int y = x % (2 * NP), d = y % NP, i0 = (x / (2 * NP)) * BL;
+    float* dst = (y < NP ? b_s : c_s) + i0 * PT + d;
+    const int m = d < N ? (n - i0 < BL ? (n - i0 > 0 ? n - i0 : 0) : BL) : 0;
+    const int chan = p.H * p.P + (y < NP ? 0 : p.G * N) + g * N + d;
+    if (m) conv_run(xbc, p.ld, tok0, t0 + i0, m, pos, ring, p.taps, p.C, chan, p.conv_w, p.conv_b[chan],
+                    [&](int i, float v) { dst[i * PT] = v; });
+    for (int i = m; i < BL; ++i) dst[i * PT] = 0.0f;
+  }
+  __syncthreads();
+  for (int x = tid; x < CH * NP; x += 256) p.Cm[ch * CH * NP + x] = c_s[(x / NP) * PT + x % NP];
+  for (int x = tid; x < NP * CH; x += 256) p.Bt[ch * NP * CH + x] = b_s[(x % CH) * PT + x / CH];
+  const int r16 = lane & 15, q4 = (lane >> 4) * 4;
+  for (int J = 0; J < NB; ++J) {
+    f32x4 s = {0, 0, 0, 0};
+    if (J <= wave)
+      for (int d = q4; d < NP; d += 16) s = mma16(ld4(&c_s[(wave * BL + r16) * PT + d]), ld4(&b_s[(J * BL + r16) * PT + d]), s);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) p.CB[ch * CH * CH + (wave * BL + q4 + r) * CH + J * BL + r16] = s[r];
+  }
+}
+
+template <int NP, typename T>
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) void ssd_chunks_kernel(SsdChunkArgs p, const T* xbc,
+                                                                                                    const T* dt_raw, const T* ring0) {
+  constexpr int KB = NP / 16, NT = (KB + 3) / 4, SP = NP + 4, XP = CH + 4;
+  __shared__ __align__(16) float s_s[CT * SP];
+  __shared__ __align__(16) float x_s[2][CT * XP];  // the chunk's x, column by column
+  __shared__ __align__(16) float w_s[2][CH];       // dt_j e^{L_C - L_j}
+  __shared__ __align__(16) float dt_s[2][CH];
+  __shared__ __align__(16) double l_s[2][CH];      // log2 decays summed from the chunk's start
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int r16 = lane & 15, q4 = (lane >> 4) * 4;
+  const int tile = blockIdx.x, h = blockIdx.y, b = blockIdx.z, g = h / (p.H / p.G);
+  const int e = tile * CT + r16, N = p.N, P = p.P, pos = p.pos[b];
+  const int64_t tok0 = (int64_t)b * p.S;
+  const T* ring = ring0 + (int64_t)p.slots[b] * p.taps * p.C;
+  float* col = p.state + (((int64_t)p.slots[b] * p.H + h) * P + (e < P ? e : 0)) * N;
+  f32x4 s[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    const int d = (wave + 4 * t) * 16 + q4;
+    s[t] = load_state4(col, d, N, e < P && pos > 0 && d < NP);
+  }
+  const float skip = p.skip[h], neg_a = -expf(p.a_log[h]) * 1.44269504088896341f, dtb = p.dt_bias[h];
+  const int row = wave * BL + r16;
+  float4 cm[KB], cb[NB], bt[NT][NB];
+  auto base = [&](int c) -> int64_t { return ((int64_t)b * p.NC + c) * p.G + g; };
+  auto load_c = [&](int64_t ch) __attribute__((always_inline)) {
+#pragma unroll
+    for (int x = 0; x < KB; ++x) cm[x] = ld4(p.Cm + (ch * CH + row) * NP + x * 16 + q4);
+  };
+  auto load_cb = [&](int64_t ch) __attribute__((always_inline)) {
+#pragma unroll
+    for (int x = 0; x < NB; ++x) cb[x] = ld4(p.CB + (ch * CH + row) * CH + x * 16 + q4);
+  };
+  auto load_b = [&](int64_t ch) __attribute__((always_inline)) {
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      if (wave + 4 * t >= KB) break;
+#pragma unroll
+      for (int x = 0; x < NB; ++x) bt[t][x] = ld4(p.Bt + (ch * NP + (wave + 4 * t) * 16 + r16) * CH + x * 16 + q4);
+    }
+  };
+  // x: thread = (column tid % 16, tokens 4 (tid / 16) .. + 4); its raw inputs are requested a chunk ahead
+  const int xe = tid & 15, xt = (tid >> 4) * 4, xc = h * P + tile * CT + xe;
+  const bool xok = tile * CT + xe < P;
+  float wj[MAX_TAPS], xin[4 + MAX_TAPS - 1], dtin;
+#pragma unroll
+  for (int j = 0; j < MAX_TAPS; ++j) {
+    const int back = MAX_TAPS - 1 - j;
+    wj[j] = xok && back < p.taps ? p.conv_w[xc * p.taps + p.taps - 1 - back] : 0.0f;
+  }
+  const float xb = xok ? p.conv_b[xc] : 0.0f;
+  auto load_x = [&](int c) __attribute__((always_inline)) {
+#pragma unroll
+    for (int i = 0; i < 4 + MAX_TAPS - 1; ++i) {
+      const int t = c * CH + xt + i - (MAX_TAPS - 1), a = pos + t;  // token within the portion; position
+      float v = 0.0f;
+      if (xok && t < p.S && a >= 0 && (t >= 0 || t > -p.taps)) v = t >= 0 ? to_f32(xbc[(tok0 + t) * p.ld + xc]) : to_f32(ring[(int64_t)(a % p.taps) * p.C + xc]);
+      xin[i] = v;
+    }
+    const int t = c * CH + lane;
+    dtin = t < p.S ? to_f32(dt_raw[(tok0 + t) * p.ld_dt + h]) : 0.0f;
+  };
+  load_c(base(0)), load_cb(base(0)), load_b(base(0)), load_x(0);
+  for (int c = 0; c < p.NC; ++c) {
+    const int buf = c & 1, nc = c + 1 < p.NC ? c + 1 : c;
+    const int64_t nx = base(nc);
+    // ---- this chunk's x, steps and decays; the state as an operand
+    float4 xv;
+    {
+      float y[4];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        float acc = xb;
+#pragma unroll
+        for (int j = 0; j < MAX_TAPS; ++j) acc = fmaf(wj[j], xin[i + j], acc);
+        y[i] = xok && c * CH + xt + i < p.S ? silu(acc) : 0.0f;
+      }
+      xv = make_float4(y[0], y[1], y[2], y[3]);
+    }
+    *reinterpret_cast<float4*>(&x_s[buf][xe * XP + xt]) = xv;
+    const float dt = c * CH + lane < p.S ? softplus(dtin + dtb) : 0.0f;
+    double L = (double)neg_a * (double)dt;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const double v = __shfl_up(L, o, 64);
+      if (lane >= o) L += v;
+    }
+    const double LC = __shfl(L, 63, 64);
+    if (wave == 0) {
+      dt_s[buf][lane] = dt;
+      l_s[buf][lane] = L;
+      w_s[buf][lane] = dt * ex2((float)(LC - L));
+    }
+    const float decay = ex2((float)LC);
+#pragma unroll
+    for (int t = 0; t < NT; ++t)
+      if (wave + 4 * t < KB) *reinterpret_cast<f32x4*>(&s_s[r16 * SP + (wave + 4 * t) * 16 + q4]) = s[t];
+    __syncthreads();
+    load_x(nc);
+    f32x4 y = {0, 0, 0, 0};
+#pragma unroll
+    for (int x = 0; x < KB; ++x) y = mma16(cm[x], ld4(&s_s[r16 * SP + x * 16 + q4]), y);
+    load_c(nx);
+    __syncthreads();  // the state may be overwritten
+    float4 xx[NB];
+#pragma unroll
+    for (int x = 0; x < NB; ++x) xx[x] = ld4(&x_s[buf][r16 * XP + x * 16 + q4]);
+    // rows of y: tokens wave * 16 + q4 + r
+#pragma unroll
+    for (int r = 0; r < 4; ++r) y[r] *= ex2((float)l_s[buf][wave * BL + q4 + r]);
+    const double Li = l_s[buf][row];
+#pragma unroll
+    for (int x = 0; x < NB; ++x) {
+      if (x > wave) break;  // keys ahead of every token of the wavefront
+      const float4 dj = ld4(&dt_s[buf][x * 16 + q4]);
+      float m[4] = {cb[x].x * dj.x, cb[x].y * dj.y, cb[x].z * dj.z, cb[x].w * dj.w};
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int jt = x * 16 + q4 + r;
+        m[r] = jt <= row ? m[r] * ex2((float)(Li - l_s[buf][jt])) : 0.0f;
+      }
+      y = mma16(make_float4(m[0], m[1], m[2], m[3]), xx[x], y);
+    }
+    load_cb(nx);
+#pragma unroll
+    for (int x = 0; x < NB; ++x) {
+      const float4 wv = ld4(&w_s[buf][x * 16 + q4]);
+      const float4 xw = make_float4(xx[x].x * wv.x, xx[x].y * wv.y, xx[x].z * wv.z, xx[x].w * wv.w);
+#pragma unroll
+      for (int t = 0; t < NT; ++t) {
+        if (wave + 4 * t >= KB) break;
+        if (x == 0) s[t] *= decay;
+        s[t] = mma16(bt[t][x], xw, s[t]);
+      }
+    }
+    load_b(nx);
+    const int t0 = c * CH + wave * BL + q4;
+    const float4 own = ld4(&x_s[buf][r16 * XP + wave * BL + q4]);
+    const float xo[4] = {own.x, own.y, own.z, own.w};
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (t0 + r < p.S && e < P) p.out[(((int64_t)b * p.S + t0 + r) * p.H + h) * P + e] = y[r] + skip * xo[r];
+  }
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    const int d = (wave + 4 * t) * 16 + q4;
+    if (e < P && d < NP) store_state4(col, d, N, s[t]);
+  }
+}
+
+inline int64_t pad_rows(int64_t n) { return n <= 32 ? 32 : n <= 64 ? 64 : 128; }
+inline int64_t pad16(int64_t n) { return (n + 15) / 16 * 16; }
+
+}  // namespace sq
+
+using namespace sq;
+
+#define SQ_PADDED(R, ...)            \
+  do {                               \
+    if ((R) <= 32) {                 \
+      constexpr int RP = 32;         \
+      __VA_ARGS__;                   \
+    } else if ((R) <= 64) {          \
+      constexpr int RP = 64;         \
+      __VA_ARGS__;                   \
+    } else {                         \
+      constexpr int RP = 128;        \
+      __VA_ARGS__;                   \
+    }                                \
+  } while (0)
+
+template <typename K>
+static int big_lds(K* kernel, size_t bytes) {
+  if (bytes <= 64 * 1024) return 0;
+  return (int)hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes);
+}
+
+extern "C" int aqs_chunked_ok(int64_t rows, int64_t taps) { return rows > 0 && rows <= 128 && taps > 0 && taps <= MAX_TAPS; }
+
+// floats of workspace for B sequences of S tokens
+extern "C" int64_t aqs_delta_chunked_ws(int64_t B, int64_t S, int64_t H, int64_t D, int64_t E) {
+  const int64_t DP = pad_rows(D), EP = pad16(E);
+  return B * ((S + CH - 1) / CH) * H * (2 * CH * CH + 3 * CH * DP + CH * EP + DP);
+}
+extern "C" int64_t aqs_ssd_chunked_ws(int64_t B, int64_t S, int64_t G, int64_t N) {
+  const int64_t NP = pad_rows(N);
+  return B * ((S + CH - 1) / CH) * G * (CH * CH + 2 * CH * NP);
+}
+
+extern "C" int aqs_delta_chunked(const void* qkv, int64_t ld, const void* raw, int64_t ld_raw, const void* beta_raw, int64_t ld_beta,
+                                 int dtype, const float* w, const void* ring, const int32_t* slots, const int32_t* pos,
+                                 const float* a_log, const float* dt_bias, float* ws, int64_t ws_floats, float* state, float* out,
+                                 int64_t B, int64_t S, int64_t H, int64_t G, int64_t D, int64_t E, int64_t taps, void* stream) {
+  SQ_CHECK(B >= 0 && S >= 0 && H > 0 && G > 0 && H % G == 0 && D > 0 && E > 0 && aqs_chunked_ok(D, taps), AQ_E_SHAPE);
+  SQ_CHECK(ld >= 2 * G * D + H * E && ld_raw >= H * D && ld_beta >= H, AQ_E_SHAPE);
+  const int64_t NC = (S + CH - 1) / CH;
+  SQ_CHECK(B * NC < (1 << 16) && H < 65536 && B < 65536 && E <= (1 << 16), AQ_E_RANGE);
+  if (B * S == 0) return AQ_OK;
+  SQ_NEED(qkv && raw && beta_raw && w && ring && slots && pos && a_log && dt_bias && ws && state && out);
+  SQ_CHECK(!bad_ptr16(ws), AQ_E_ALIGN);
+  SQ_CHECK(ws_floats >= aqs_delta_chunked_ws(B, S, H, D, E), AQ_E_WORKSPACE);
+  const int64_t DP = pad_rows(D), EP = pad16(E), n = B * NC * H;
+  DeltaChunkArgs a{};
+  a.slots = slots, a.pos = pos, a.conv_w = w, a.a_log = a_log, a.dt_bias = dt_bias;
+  a.A = ws;
+  a.QK = a.A + n * CH * CH;
+  a.W = a.QK + n * CH * CH;
+  a.Q = a.W + n * CH * DP;
+  a.K = a.Q + n * CH * DP;
+  a.U = a.K + n * CH * DP;
+  a.gc = a.U + n * CH * EP;
+  a.ld = ld, a.ld_raw = ld_raw, a.ld_beta = ld_beta;
+  a.S = (int)S, a.NC = (int)NC, a.H = (int)H, a.G = (int)G, a.D = (int)D, a.E = (int)E, a.DP = (int)DP, a.EP = (int)EP;
+  a.taps = (int)taps, a.C = (int)(2 * G * D + H * E);
+  hipStream_t st = (hipStream_t)stream;
+  const size_t lds = (size_t)(2 * CH * (DP + 4) + CH) * 4 + (size_t)(CH * (DP + 2) + NB * DP) * 8;
+  SQ_DISPATCH(dtype, SQ_PADDED(D, {
+                if (const int rc = big_lds(&delta_chunk_prep_kernel<RP, T>, lds)) return rc;
+                (delta_chunk_prep_kernel<RP, T><<<dim3((unsigned)(B * NC), (unsigned)H), 256, lds, st>>>(
+                    a, (const T*)qkv, (const T*)raw, (const T*)beta_raw, (const T*)ring));
+              }));
+  if (const int rc = launched()) return rc;
+  delta_chunk_solve_kernel<<<dim3((unsigned)n, (unsigned)((DP + EP + 255) / 256)), 256, 0, st>>>(a.A, a.W, a.U, (int)DP, (int)EP);
+  if (const int rc = launched()) return rc;
+  const DeltaScanArgs s{a.W, a.U, a.Q, a.K, a.QK, a.gc, state, out, slots, pos, (int)S, (int)NC, (int)H, (int)D, (int)E, (int)EP};
+  const dim3 grid((unsigned)(EP / CT), (unsigned)H, (unsigned)B);
+  SQ_PADDED(D, (delta_chunk_scan_kernel<RP><<<grid, 256, 0, st>>>(s)));
+  return launched();
+}
+
+extern "C" int aqs_ssd_chunked(const void* xbc, int64_t ld, const void* dt_raw, int64_t ld_dt, int dtype, const float* conv_w,
+                               const float* conv_b, const void* ring, const int32_t* slots, const int32_t* pos, const float* dt_bias,
+                               const float* a_log, const float* skip, float* ws, int64_t ws_floats, float* state, float* out,
+                               int64_t B, int64_t S, int64_t H, int64_t G, int64_t N, int64_t P, int64_t taps, void* stream) {
+  SQ_CHECK(B >= 0 && S >= 0 && H > 0 && G > 0 && H % G == 0 && N > 0 && P > 0 && aqs_chunked_ok(N, taps), AQ_E_SHAPE);
+  SQ_CHECK(ld >= H * P + 2 * G * N && ld_dt >= H, AQ_E_SHAPE);
+  const int64_t NC = (S + CH - 1) / CH;
+  SQ_CHECK(B * NC < (1 << 16) && H < 65536 && G < 65536 && B < 65536 && P <= (1 << 16), AQ_E_RANGE);
+  if (B * S == 0) return AQ_OK;
+  SQ_NEED(xbc && dt_raw && conv_w && conv_b && ring && slots && pos && dt_bias && a_log && skip && ws && state && out);
+  SQ_CHECK(!bad_ptr16(ws), AQ_E_ALIGN);
+  SQ_CHECK(ws_floats >= aqs_ssd_chunked_ws(B, S, G, N), AQ_E_WORKSPACE);
+  const int64_t NP = pad_rows(N), n = B * NC * G;
+  SsdChunkArgs a{};
+  a.slots = slots, a.pos = pos, a.conv_w = conv_w, a.conv_b = conv_b, a.dt_bias = dt_bias, a.a_log = a_log, a.skip = skip;
+  a.CB = ws;
+  a.Cm = a.CB + n * CH * CH;
+  a.Bt = a.Cm + n * CH * NP;
+  a.state = state, a.out = out, a.ld = ld, a.ld_dt = ld_dt;
+  a.S = (int)S, a.NC = (int)NC, a.H = (int)H, a.G = (int)G, a.N = (int)N, a.P = (int)P, a.NP = (int)NP;
+  a.taps = (int)taps, a.C = (int)(H * P + 2 * G * N);
+  hipStream_t st = (hipStream_t)stream;
+  const size_t lds = (size_t)(2 * CH * (NP + 4)) * 4;
+  SQ_DISPATCH(dtype, SQ_PADDED(N, {
+                if (const int rc = big_lds(&ssd_group_kernel<RP, T>, lds)) return rc;
+                (ssd_group_kernel<RP, T><<<dim3((unsigned)(B * NC), (unsigned)G), 256, lds, st>>>(a, (const T*)xbc, (const T*)ring));
+              }));
+  if (const int rc = launched()) return rc;
+  const dim3 grid((unsigned)((P + CT - 1) / CT), (unsigned)H, (unsigned)B);
+  SQ_DISPATCH(dtype, SQ_PADDED(N, (ssd_chunks_kernel<RP, T><<<grid, 256, 0, st>>>(a, (const T*)xbc, (const T*)dt_raw, (const T*)ring))));
+  return launched();
+}

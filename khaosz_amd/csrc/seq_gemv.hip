@@ -30,7 +30,10 @@ constexpr int GEMV_MAX_M = 8;
 
 template <typename T, int IN, int OUT, int R, int MR>
 __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const T* z, const T* w, T* out) {
-  extern __shared__ __align__(16) float xs[];  // [M, K]
+  // one row is kept in fp32; several as T, so that long rows fit
+  using X = typename std::conditional<MR == 1, float, T>::type;
+  extern __shared__ __align__(16) uint8_t xs_raw[];
+  X* xs = reinterpret_cast<X*>(xs_raw);  // [M, K]
   __shared__ float red[4];
   constexpr int U = 4;                          // 512-element steps of the row requested ahead
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -58,43 +61,95 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const
   __builtin_amdgcn_sched_barrier(0);
   // ---- rows into LDS
   for (int m = 0; m < p.M; ++m) {
-    float* row = xs + m * K;
+    X* row = xs + m * K;
+    auto put8 = [&](int k, const float* f) __attribute__((always_inline)) {
+      if constexpr (std::is_same<X, float>::value) {
+        reinterpret_cast<float4*>(row + k)[0] = make_float4(f[0], f[1], f[2], f[3]);
+        reinterpret_cast<float4*>(row + k)[1] = make_float4(f[4], f[5], f[6], f[7]);
+      } else {
+        *reinterpret_cast<uint4*>(row + k) = make_uint4(pack2(f[0], f[1]), pack2(f[2], f[3]), pack2(f[4], f[5]), pack2(f[6], f[7]));
+      }
+    };
     if constexpr (IN == IN_PLAIN) {
       for (int k = tid * 8; k < K; k += 2048) {
         Raw8<T> v;
         v.load(x + m * p.ldx + k);
         float f[8];
         v.get(f);
-        reinterpret_cast<float4*>(row + k)[0] = make_float4(f[0], f[1], f[2], f[3]);
-        reinterpret_cast<float4*>(row + k)[1] = make_float4(f[4], f[5], f[6], f[7]);
+        put8(k, f);
       }
     } else if constexpr (IN == IN_RMSNORM) {
-      float ss = 0.0f;
-      for (int k = tid * 4; k < K; k += 1024) {
-        const float4 v = *reinterpret_cast<const float4*>(p.xf + m * p.ldx + k);
-        *reinterpret_cast<float4*>(row + k) = v;
-        ss += v.x * v.x + v.y * v.y + v.z * v.z + v.w * v.w;
+      // the row stays in registers between the two passes where it fits (up to 4 pieces of 2048)
+      constexpr int KEEP = 4;
+      float keep[KEEP][8], ss = 0.0f;
+#pragma unroll
+      for (int i = 0; i < KEEP; ++i) {
+        const int k = i * 2048 + tid * 8;
+        if (k < K) load_vec<8>(p.xf + m * p.ldx + k, keep[i]);
+        else
+#pragma unroll
+          for (int e = 0; e < 8; ++e) keep[i][e] = 0.0f;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss += keep[i][e] * keep[i][e];
+      }
+      for (int k = KEEP * 2048 + tid * 8; k < K; k += 2048) {
+        float f[8];
+        load_vec<8>(p.xf + m * p.ldx + k, f);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss += f[e] * f[e];
       }
       ss = block_sum<4>(ss, red);
       const float r = 1.0f / sqrtf(ss / (float)K + p.eps);
-      for (int k = tid * 4; k < K; k += 1024) {
-        float4 v = *reinterpret_cast<const float4*>(row + k);
-        const float4 g = *reinterpret_cast<const float4*>(p.gain + k);
-        v.x *= r * (1.0f + g.x), v.y *= r * (1.0f + g.y), v.z *= r * (1.0f + g.z), v.w *= r * (1.0f + g.w);
-        *reinterpret_cast<float4*>(row + k) = v;
+      auto norm8 = [&](int k, float* f) __attribute__((always_inline)) {
+        float g[8];
+        load_vec<8>(p.gain + k, g);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) f[e] *= r * (1.0f + g[e]);
+        put8(k, f);
+      };
+#pragma unroll
+      for (int i = 0; i < KEEP; ++i) {
+        const int k = i * 2048 + tid * 8;
+        if (k < K) norm8(k, keep[i]);
+      }
+      for (int k = KEEP * 2048 + tid * 8; k < K; k += 2048) {
+        float f[8];
+        load_vec<8>(p.xf + m * p.ldx + k, f);
+        norm8(k, f);
       }
     } else {
       const int part = K / p.groups;
       for (int g = 0; g < p.groups; ++g) {
-        float ss = 0.0f;
-        for (int k = g * part + tid; k < (g + 1) * part; k += 256) {
-          const float v = p.xf[m * p.ldx + k] * silu(to_f32(z[m * p.ldz + k]));
-          row[k] = v;
+        // values of the first 16 rounds stay in registers
+        constexpr int KEEP = 16;
+        const float* yr = p.xf + m * p.ldx + g * part;
+        const T* zr = z + m * p.ldz + g * part;
+        float keep[KEEP], ss = 0.0f;
+#pragma unroll
+        for (int i = 0; i < KEEP; ++i) {
+          const int k = i * 256 + tid;
+          keep[i] = k < part ? yr[k] : 0.0f;
+        }
+#pragma unroll
+        for (int i = 0; i < KEEP; ++i) {
+          const int k = i * 256 + tid;
+          if (k < part) keep[i] *= silu(to_f32(zr[k]));
+          ss += keep[i] * keep[i];
+        }
+        for (int k = KEEP * 256 + tid; k < part; k += 256) {
+          const float v = yr[k] * silu(to_f32(zr[k]));
           ss += v * v;
         }
         ss = block_sum<4>(ss, red);
         const float r = 1.0f / sqrtf(ss / (float)part + p.eps);
-        for (int k = g * part + tid; k < (g + 1) * part; k += 256) row[k] *= r * p.gain[k];
+        X* dst = row + g * part;
+        const float* gr = p.gain + g * part;
+#pragma unroll
+        for (int i = 0; i < KEEP; ++i) {
+          const int k = i * 256 + tid;
+          if (k < part) dst[k] = from_f32<X>(keep[i] * r * gr[k]);
+        }
+        for (int k = KEEP * 256 + tid; k < part; k += 256) dst[k] = from_f32<X>(yr[k] * silu(to_f32(zr[k])) * r * gr[k]);
       }
     }
   }
@@ -113,7 +168,9 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const
     for (int m = 0; m < MR; ++m) {
       if (m >= p.M) break;
       float a[8];
-      load_vec<8>(xs + m * K + k, a);
+      Raw8<X> xr;
+      xr.load(xs + m * K + k);
+      xr.get(a);
 #pragma unroll
       for (int i = 0; i < R; ++i)
 #pragma unroll
@@ -158,7 +215,7 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const
 template <typename T, int IN, int OUT>
 int launch_gemv(const GemvArgs& p, const void* x, const void* z, const void* w, void* out, hipStream_t stream) {
   const int F = OUT == OUT_GLU ? p.N / 2 : p.N;
-  const size_t lds = (size_t)p.M * p.K * 4;
+  const size_t lds = (size_t)p.M * p.K * (p.M == 1 ? 4 : sizeof(T));
   auto go = [&](auto r_tag, auto m_tag) -> int {
     constexpr int R = decltype(r_tag)::value, MR = decltype(m_tag)::value;
     constexpr int OR = OUT == OUT_GLU ? R / 2 : R;
@@ -189,8 +246,9 @@ int launch_gemv(const GemvArgs& p, const void* x, const void* z, const void* w, 
 
 using namespace sq;
 
-extern "C" int aqs_gemv_ok(int64_t M, int64_t N, int64_t K) {
-  return M > 0 && M <= GEMV_MAX_M && N > 0 && N < (1 << 24) && K > 0 && K % 8 == 0 && M * K * 4 <= 144 * 1024;
+extern "C" int aqs_gemv_ok(int dtype, int64_t M, int64_t N, int64_t K) {
+  return M > 0 && M <= GEMV_MAX_M && N > 0 && N < (1 << 24) && K > 0 && K % 8 == 0 &&
+         M * K * (M > 1 && dtype == AQ_BF16 ? 2 : 4) <= 144 * 1024;
 }
 
 // in_kind: 0 plain (x of dtype, stride ldx), 1 rmsnorm (xf, gain, eps), 2 gated group norm (xf = y, x = z with stride
@@ -200,7 +258,7 @@ extern "C" int aqs_gemv(int in_kind, int out_kind, int dtype, const void* x, int
                         int64_t ldo, int64_t M, int64_t N, int64_t K, void* stream) {
   SQ_CHECK(M >= 0 && N > 0 && K > 0, AQ_E_SHAPE);
   if (M == 0) return AQ_OK;
-  SQ_CHECK(aqs_gemv_ok(M, N, K), AQ_E_SHAPE);
+  SQ_CHECK(aqs_gemv_ok(dtype, M, N, K), AQ_E_SHAPE);
   SQ_NEED(w && (out_kind == OUT_F32 || out_kind == OUT_RESIDUAL ? (const void*)res : (const void*)out));
   SQ_CHECK(!bad_ptr16(w) && !bad_ptr16(x) && !bad_ptr16(xf) && !bad_ptr16(gain), AQ_E_ALIGN);
   SQ_CHECK(out_kind != OUT_GLU || N % 2 == 0, AQ_E_SHAPE);

@@ -149,7 +149,7 @@ class HybridLM(nn.Module):
         read positions, slots and pages from device memory and call no library)."""
         if rows not in self._step_ok:
             self._step_ok[rows] = all(l.step_ok(rows) for l in self.layers) and \
-                seq_ops.gemv_ok(rows, self.config.vocab, self.config.width)
+                seq_ops.gemv_ok(rows, self.head)
         return self._step_ok[rows]
 
     def advance(self, ids: Tensor, b: Batch, state: List[Any], starts: Sequence[int], want: Optional[Sequence[int]] = None) -> Tensor:
@@ -182,7 +182,7 @@ class HybridLM(nn.Module):
             if list(want) != list(range(x.shape[0])):
                 rows = torch.tensor(list(want), device=x.device)
                 x, y = x[rows], y[rows]
-        if seq_ops.gemv_ok(x.shape[0], c.vocab, c.width):
+        if seq_ops.gemv_ok(x.shape[0], self.head):
             seq_ops.add_rmsnorm(x, y, c.residual_mult, None, c.norm_eps, self.dtype, norm=False)
             return seq_ops.norm_gemv_f32(x, self.final_norm, c.norm_eps, self.head)
         h = seq_ops.add_rmsnorm(x, y, c.residual_mult, self.final_norm, c.norm_eps, self.dtype)

@@ -104,9 +104,13 @@ class Mamba2Mixer(nn.Module):
 
     def prompt(self, proj: Tensor, at: Dict[str, int], b: Batch, st: Dict[str, Any], out: Tensor, scale: float) -> None:
         z, xbc, dt = self._columns(at)
-        act = seq_ops.conv_silu(proj, xbc, self.conv, self.conv_b, st["ring"], b)
+        if b.S >= seq_ops.CHUNKED_MIN and seq_ops.chunked_ok(self.N, self.taps):
+            y = seq_ops.ssd_chunked(proj, xbc, dt, self.conv, self.conv_b, st["ring"], self.dt_bias, self.a_log, self.skip, st["S"],
+                                    self.H, self.G, self.N, self.P, b)
+        else:
+            act = seq_ops.conv_silu(proj, xbc, self.conv, self.conv_b, st["ring"], b)
+            y = seq_ops.ssd_scan(act, proj, dt, self.dt_bias, self.a_log, self.skip, st["S"], self.H, self.G, self.N, self.P, b)
         seq_ops.conv_push(proj, xbc, self.channels, self.taps, st["ring"], b)
-        y = seq_ops.ssd_scan(act, proj, dt, self.dt_bias, self.a_log, self.skip, st["S"], self.H, self.G, self.N, self.P, b)
         seq_ops.gated_group_norm(y, proj, z, self._gain(scale), self.eps, self.norm_groups, out)
 
     def step(self, proj: Tensor, at: Dict[str, int], b: Batch, st: Dict[str, Any], out: Tensor, scale: float) -> None:
@@ -164,10 +168,13 @@ class ChannelDeltaMixer(nn.Module):
         qkv, a1, g1 = at["qkv"], at["a1"], at["g1"]
         raw = F.linear(proj[:, a1:a1 + self.a2.shape[1]], self.a2)
         gate = F.linear(proj[:, g1:g1 + self.g2.shape[1]], self.g2)
-        q, k, v, decay, beta = seq_ops.delta_prep(proj, qkv, raw, at["b"], self.conv, st["ring"], self.a_log, self.dt_bias, self.H,
-                                                  self.G, self.D, self.E, b)
+        args = (proj, qkv, raw, at["b"], self.conv, st["ring"], self.a_log, self.dt_bias)
+        if b.S >= seq_ops.CHUNKED_MIN and seq_ops.chunked_ok(self.D, self.taps):
+            o = seq_ops.delta_chunked(*args, st["S"], self.H, self.G, self.D, self.E, b)
+        else:
+            q, k, v, decay, beta = seq_ops.delta_prep(*args, self.H, self.G, self.D, self.E, b)
+            o = seq_ops.delta_scan(q, k, v, decay, beta, st["S"], b)
         seq_ops.conv_push(proj, qkv, sum(self.split), self.taps, st["ring"], b)
-        o = seq_ops.delta_scan(q, k, v, decay, beta, st["S"], b)
         seq_ops.head_norm_gate(o, gate, self.norm, self.eps, scale, out)
 
     def step(self, proj: Tensor, at: Dict[str, int], b: Batch, st: Dict[str, Any], out: Tensor, scale: float) -> None:
@@ -272,8 +279,7 @@ class MixerBlock(nn.Module):
             seq_ops.gemv_residual(self._run(proj, b, st, "step"), self.w_out, mult, x)
 
     def step_ok(self, rows: int) -> bool:
-        n, k = self.w_in.weight.shape
-        return seq_ops.gemv_ok(rows, n, k) and seq_ops.gemv_ok(rows, k, self.inner)
+        return seq_ops.gemv_ok(rows, self.w_in.weight) and seq_ops.gemv_ok(rows, self.w_out)
 
 
 class ClampedGLU(nn.Module):
@@ -295,5 +301,4 @@ class ClampedGLU(nn.Module):
         seq_ops.gemv_residual(seq_ops.norm_gemv_glu(x, gain, eps, self.gate_up, self.limit), self.down, mult, x)
 
     def step_ok(self, rows: int) -> bool:
-        n, k = self.gate_up.shape
-        return seq_ops.gemv_ok(rows, n, k) and seq_ops.gemv_ok(rows, k, self.ff)
+        return seq_ops.gemv_ok(rows, self.gate_up) and seq_ops.gemv_ok(rows, self.down)

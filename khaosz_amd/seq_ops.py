@@ -121,8 +121,9 @@ def head_norm_gate(o: Tensor, gate: Tensor, w: Tensor, eps: float, scale: float,
 
 
 # ------------------------------------------------------------------------------------------------ matrix-vector products
-def gemv_ok(M: int, N: int, K: int) -> bool:
-    return bool(_abi.load_seq().aqs_gemv_ok(M, N, K))
+def gemv_ok(M: int, w: Tensor) -> bool:
+    """Whether the products with ``w [N, K]`` below serve M rows."""
+    return bool(_abi.load_seq().aqs_gemv_ok(_DT[w.dtype], M, w.shape[0], w.shape[1]))
 
 
 def _gemv(in_kind, out_kind, w, x=None, ldx=0, o_x=0, xf=None, gain=None, eps=0.0, groups=1, bias=None, mult=0.0, limit=0.0,
@@ -251,6 +252,60 @@ def delta_scan(q: Tensor, k: Tensor, v: Tensor, decay: Tensor, beta: Tensor, sta
     out = torch.empty((M, H, E), dtype=torch.float32, device=q.device)
     _call("aqs_delta_scan", q.device, _p(q), _p(k), _p(v), _p(decay), _p(beta), _p(state), _p(b.slots), _p(b.pos), _p(out), b.B,
           b.S, H, G, D, E, _stream(q))
+    return out
+
+
+CHUNKED_MIN = 96  # new tokens per sequence from which the chunked kernels are the faster ones
+
+
+def chunked_ok(rows: int, taps: int) -> bool:
+    """Whether the chunked recurrences serve a state of ``rows`` rows behind a convolution of ``taps`` taps."""
+    return bool(_abi.load_seq().aqs_chunked_ok(rows, taps))
+
+
+def delta_chunked(proj: Tensor, o_qkv: int, raw: Tensor, o_beta: int, conv_w: Tensor, ring: Tensor, a_log: Tensor, dt_bias: Tensor,
+                  state: Tensor, H: int, G: int, D: int, E: int, b: Batch) -> Tensor:
+    """``delta_prep`` and ``delta_scan`` in chunks of 64 tokens on the fp32 matrix cores.  fp32 ``[M, H, E]``."""
+    _need_gpu(proj, raw, conv_w, ring, a_log, dt_bias, state)
+    M, C, taps, dev = proj.shape[0], 2 * G * D + H * E, conv_w.shape[1], proj.device
+    _batch(b, M)
+    _ring(ring, C, taps, proj.dtype)
+    _state(state, H, E, D)
+    _vec(conv_w, C * taps, "conv_w")
+    _vec(a_log, H, "a_log")
+    _vec(dt_bias, H * D, "dt_bias")
+    _rows2(raw, "raw", proj.dtype)
+    if raw.shape != (M, H * D) or o_qkv + C > proj.shape[1] or o_beta + H > proj.shape[1]:
+        raise ValueError("delta_chunked: shapes do not fit")
+    n = int(_abi.load_seq().aqs_delta_chunked_ws(b.B, b.S, H, D, E))
+    ws = torch.empty(n, dtype=torch.float32, device=dev)
+    out = torch.empty((M, H, E), dtype=torch.float32, device=dev)
+    _call("aqs_delta_chunked", dev, _p(proj, o_qkv), proj.stride(0), _p(raw), raw.stride(0), _p(proj, o_beta), proj.stride(0),
+          _DT[proj.dtype], _p(conv_w), _p(ring), _p(b.slots), _p(b.pos), _p(a_log), _p(dt_bias), _p(ws), n, _p(state), _p(out),
+          b.B, b.S, H, G, D, E, taps, _stream(proj))
+    return out
+
+
+def ssd_chunked(proj: Tensor, o_xbc: int, o_dt: int, conv_w: Tensor, conv_b: Tensor, ring: Tensor, dt_bias: Tensor, a_log: Tensor,
+                skip: Tensor, state: Tensor, H: int, G: int, N: int, P: int, b: Batch) -> Tensor:
+    """``conv_silu`` and ``ssd_scan`` in chunks of 64 tokens on the fp32 matrix cores.  fp32 ``[M, H * P]``."""
+    _need_gpu(proj, conv_w, conv_b, ring, dt_bias, a_log, skip, state)
+    M, C, taps, dev = proj.shape[0], H * P + 2 * G * N, conv_w.shape[1], proj.device
+    _batch(b, M)
+    _ring(ring, C, taps, proj.dtype)
+    _state(state, H, P, N)
+    _vec(conv_w, C * taps, "conv_w")
+    _vec(conv_b, C, "conv_b")
+    for t in (dt_bias, a_log, skip):
+        _vec(t, H, "per-head constants")
+    if o_xbc + C > proj.shape[1] or o_dt + H > proj.shape[1]:
+        raise ValueError("ssd_chunked: shapes do not fit")
+    n = int(_abi.load_seq().aqs_ssd_chunked_ws(b.B, b.S, G, N))
+    ws = torch.empty(n, dtype=torch.float32, device=dev)
+    out = torch.empty((M, H * P), dtype=torch.float32, device=dev)
+    _call("aqs_ssd_chunked", dev, _p(proj, o_xbc), proj.stride(0), _p(proj, o_dt), proj.stride(0), _DT[proj.dtype], _p(conv_w),
+          _p(conv_b), _p(ring), _p(b.slots), _p(b.pos), _p(dt_bias), _p(a_log), _p(skip), _p(ws), n, _p(state), _p(out), b.B, b.S,
+          H, G, N, P, taps, _stream(proj))
     return out
 
 

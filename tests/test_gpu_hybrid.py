@@ -107,9 +107,10 @@ def test_matrix_vector_products(dtype, M, N, K):
     x, gain, w = rnd(M, K, seed=1), rnd(K, seed=2, scale=0.3), rnd(N, K, seed=3, scale=K ** -0.5)
     bias, res, z = rnd(N, seed=4), rnd(M, N, seed=5), rnd(M, K + 8, seed=6)
     xd, gd, wd = x.to(DEV), gain.to(DEV), w.to(DEV, dtype)
+    kept = torch.float32 if M == 1 else dtype  # several rows are kept in the activations' format
     h = plain.rms_norm_plus_one(f64(x), f64(gain), 1e-5)
     close(seq_ops.norm_gemv(xd, gd, 1e-5, wd, bias.to(DEV)), h @ f64(w).T + f64(bias), dtype)
-    close(seq_ops.norm_gemv_f32(xd, gd, 1e-5, wd), h @ f64(w).T, torch.float32)
+    close(seq_ops.norm_gemv_f32(xd, gd, 1e-5, wd), h @ f64(w).T, kept)
     if N % 2 == 0:
         F = N // 2
         g, u = np.minimum(h @ f64(w[:F]).T, 0.6), np.clip(h @ f64(w[F:]).T, -0.6, 0.6)
@@ -121,7 +122,7 @@ def test_matrix_vector_products(dtype, M, N, K):
         rd = res.to(DEV)
         seq_ops.gated_norm_gemv_residual(xd, z.to(DEV, dtype), 8, gd, 1e-5, groups, wd, 0.7, rd)
         v = plain.rms((f64(x) * plain.silu(f64(z[:, 8:]))).reshape(M, groups, -1), 1e-5).reshape(M, K) * f64(gain)
-        close(rd, f64(res) + 0.7 * (v @ f64(w).T), torch.float32)
+        close(rd, f64(res) + 0.7 * (v @ f64(w).T), kept)
 
 
 # ------------------------------------------------------------------------------------------------ convolution
@@ -208,6 +209,74 @@ def test_ssd_scan(dtype, H, G, N, P):
                                         H, G, N, P, batch([at], [1], n)))
             at += n
         close(torch.cat(out), want, torch.float32)
+        assert bool((state[0] == 7).all())
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,G,D,E,taps,strength", [(1, 1, 16, 16, 1, 1.0), (4, 2, 32, 24, 3, 2.0), (3, 1, 20, 37, 4, 3.0), (2, 2, 128, 64, 4, 1.0),
+                                                   (2, 1, 100, 200, 2, 4.5), (1, 1, 64, 128, 4, 6.0)])
+def test_delta_rule_in_chunks(dtype, H, G, D, E, taps, strength):
+    """Weak to very strong decays (down to e^-hundreds a token, where a factored exponent would overflow), cut anywhere."""
+    T, C = 270, 2 * G * D + H * E
+    proj, raw, w = rnd(T, C + H + 4, seed=1), rnd(T, H * D, seed=2, scale=strength), rnd(C, taps, seed=3)
+    a_log, dt = rnd(H, seed=4, scale=0.5 * strength), rnd(H * D, seed=5)
+    raw[40:43] = 90.0                                              # forgets everything, in the middle of a chunk
+    raw[100:140] = -20.0                                           # forgets nothing
+    proj[60:64, 4:4 + C] = proj[59, 4:4 + C]                       # equal keys around a chunk's edge
+    beta = plain.sigmoid(f64(proj[:, 4 + C:]))
+    act = plain.silu(plain.causal_conv(f64(proj[:, 4:4 + C]), f64(w))[0])
+    q, k = plain.unit(act[:, :G * D].reshape(T, G, D)) * D ** -0.5, plain.unit(act[:, G * D:2 * G * D].reshape(T, G, D))
+    v = act[:, 2 * G * D:].reshape(T, H, E)
+    decay = np.exp(-np.exp(f64(a_log))[:, None] * plain.softplus(f64(raw) + f64(dt)).reshape(T, H, D))
+    run = [plain.delta_rule(np.zeros((D, E)), q[:, h // (H // G)], k[:, h // (H // G)], v[:, h], decay[:, h], beta[:, h]) for h in range(H)]
+    want, last = np.stack([o for o, _ in run], 1), np.stack([S.T for _, S in run])
+    pd, rd = proj.to(DEV, dtype), raw.to(DEV, dtype)
+    for cuts in ([270], [64, 128, 78], [65, 2, 130, 63, 10]):
+        state, at, out = torch.full((2, H, E, D), 7.0, device=DEV), 0, []
+        ring = torch.full((2, taps, C), 99.0, dtype=dtype, device=DEV)
+        for n in cuts:
+            b = batch([at], [1], n)
+            out.append(seq_ops.delta_chunked(pd[at:at + n], 4, rd[at:at + n], 4 + C, w.to(DEV), ring, a_log.to(DEV), dt.to(DEV), state, H, G, D, E, b))
+            seq_ops.conv_push(pd[at:at + n], 4, C, taps, ring, b)
+            at += n
+        close(torch.cat(out), want, torch.float32)
+        close(state[1], last, torch.float32)
+        assert bool((state[0] == 7).all())
+    # two sequences in one call, one of them in the middle of its text
+    b = batch([0, 100], [1, 0], 100)
+    two = torch.cat([pd[:100], pd[100:200]])
+    state[0].copy_(torch.zeros_like(state[0]))
+    one = seq_ops.delta_chunked(pd[:100], 4, rd[:100], 4 + C, w.to(DEV), ring, a_log.to(DEV), dt.to(DEV), state, H, G, D, E, batch([0], [0], 100))
+    seq_ops.conv_push(pd[:100], 4, C, taps, ring, batch([0], [0], 100))
+    both = seq_ops.delta_chunked(two, 4, torch.cat([rd[:100], rd[100:200]]), 4 + C, w.to(DEV), ring, a_log.to(DEV), dt.to(DEV), state, H, G, D, E, b)
+    assert torch.equal(both[:100], one)
+    close(both, want[:200], torch.float32)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,G,N,P,taps", [(1, 1, 16, 16, 1), (6, 2, 24, 16, 3), (3, 3, 10, 7, 4), (4, 1, 128, 64, 4), (2, 2, 100, 80, 2), (2, 1, 64, 200, 4)])
+def test_ssd_in_chunks(dtype, H, G, N, P, taps):
+    T, C = 270, H * P + 2 * G * N
+    proj, w, bias = rnd(T, 3 + C + H, seed=1), rnd(C, taps, seed=2), rnd(C, seed=6)
+    a_log, dtb, skip = rnd(H, seed=3), rnd(H, seed=4), rnd(H, seed=5)
+    proj[40, 3 + C:], proj[100:140, 3 + C:] = 60.0, -12.0          # forgets everything; hardly moves
+    act = plain.silu(plain.causal_conv(f64(proj[:, 3:3 + C]), f64(w), f64(bias))[0])
+    dt = plain.softplus(f64(proj[:, 3 + C:]) + f64(dtb))
+    x, B, Cc = act[:, :H * P].reshape(T, H, P), act[:, H * P:H * P + G * N].reshape(T, G, N), act[:, H * P + G * N:].reshape(T, G, N)
+    run = [plain.ssd(np.zeros((N, P)), x[:, h], B[:, h // (H // G)], Cc[:, h // (H // G)], dt[:, h], f64(a_log)[h], f64(skip)[h]) for h in range(H)]
+    want, last = np.stack([y for y, _ in run], 1).reshape(T, -1), np.stack([S.T for _, S in run])
+    pd = proj.to(DEV, dtype)
+    for cuts in ([270], [64, 128, 78], [65, 2, 130, 63, 10]):
+        state, at, out = torch.full((2, H, P, N), 7.0, device=DEV), 0, []
+        ring = torch.full((2, taps, C), 99.0, dtype=dtype, device=DEV)
+        for n in cuts:
+            b = batch([at], [1], n)
+            out.append(seq_ops.ssd_chunked(pd[at:at + n], 3, 3 + C, w.to(DEV), bias.to(DEV), ring, dtb.to(DEV), a_log.to(DEV), skip.to(DEV),
+                                           state, H, G, N, P, b))
+            seq_ops.conv_push(pd[at:at + n], 3, C, taps, ring, b)
+            at += n
+        close(torch.cat(out), want, torch.float32)
+        close(state[1], last, torch.float32)
         assert bool((state[0] == 7).all())
 
 
@@ -320,7 +389,7 @@ def test_model_whole_in_portions_and_by_token(case, dtype):
     ids = hc.prompt(case, T)
     want = oracle_logits(case, ids)
     e = Engine(hc.model(case, dtype), T, 1)
-    for cuts in ([T], [64, 64, 22], [2] * 75, [7, 2, 3, 50, 1, 1, 1, 63, 22], [1] * T, [100] + [1] * 50):
+    for cuts in ([T], [64, 64, 22], [100, 50], [2] * 75, [7, 2, 3, 50, 1, 1, 1, 63, 22], [1] * T, [100] + [1] * 50):
         h = e.open()  # the same slot and pages every time
         check(feed(e, h, ids, cuts), want, dtype)
         e.close(h)

@@ -36,7 +36,7 @@ def test_seq_arguments_are_checked_before_any_launch():
     lib, P = _abi.load_seq(), 1 << 20
     assert lib.aqs_add_rmsnorm(P, None, 8, 1, 1.0, P, 1e-6, P, 1, 0, None) == -2
     assert lib.aqs_add_rmsnorm(P, None, 8, 7, 1.0, P, 1e-6, P, 1, 8, None) == -3
-    assert lib.aqs_gemv_ok(1, 64, 20) == 0 and lib.aqs_gemv_ok(9, 64, 64) == 0 and lib.aqs_gemv_ok(8, 64, 64) == 1
+    assert lib.aqs_gemv_ok(1, 1, 64, 20) == 0 and lib.aqs_gemv_ok(1, 9, 64, 64) == 0 and lib.aqs_gemv_ok(1, 8, 64, 64) == 1
     assert lib.aqs_gemv(0, 0, 1, P, 64, None, None, 0.0, 1, P + 2, None, 1.0, 0.0, None, P, 64, 1, 64, 64, None) == -4
     assert lib.aqs_gemv(2, 3, 1, P, 64, P, P, 0.0, 1, P, None, 1.0, 0.0, P, P, 64, 1, 64, 64, None) == -2  # pair not served
     assert lib.aqs_delta_scan(P, P, P, P, P, P, P, P, P, 1, 4, 3, 2, 8, 8, None) == -2                       # heads over kv heads

@@ -7,8 +7,9 @@
 //     o_i = S^T (q_i e^{G_i}) + sum_{j<=i} <q_i e^{G_i - G_j}, k_j> u_j
 //     S  <- e^{G_C} S + sum_j (k_j e^{G_C - G_j}) u_j^T
 // so with (I + A) the unit triangular matrix on the left:  u = U0 - W S  with  W = (I + A)^-1 (beta k e^G),
-// U0 = (I + A)^-1 (beta v).  Three launches: `prep` (per chunk and head: convolution, norms, decays, A and the masked
-// query-key matrix), `solve` (W and U0, one thread per column), `scan` (per head and 16 columns of S: the chunks in order).
+// U0 = (I + A)^-1 (beta v).  Two launches: `prep` (per chunk and head: convolution, norms, decays, A and the masked
+// query-key matrix, then W and U0 by forward substitution, one thread per column), `scan` (per head and 16 columns of S:
+// the chunks in order).
 //
 // A decay can be anything in (0, 1], so e^{G_i - G_j} must not be split into e^{G_i} and e^{-G_j} across a chunk.  The
 // sums are kept by blocks of 16 tokens: between blocks the split point is the later block's start, and both factors are
@@ -37,40 +38,53 @@ __device__ __forceinline__ f32x4 mma16(const float4& a, const float4& b, f32x4 c
   c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b.z, c, 0, 0, 0);
   return __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b.w, c, 0, 0, 0);
 }
+// two of them with their dependent steps interleaved
+__device__ __forceinline__ void mma16x2(const float4& a, const float4& b, f32x4& c, const float4& x, const float4& y, f32x4& z) {
+  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b.x, c, 0, 0, 0);
+  z = __builtin_amdgcn_mfma_f32_16x16x4f32(x.x, y.x, z, 0, 0, 0);
+  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b.y, c, 0, 0, 0);
+  z = __builtin_amdgcn_mfma_f32_16x16x4f32(x.y, y.y, z, 0, 0, 0);
+  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b.z, c, 0, 0, 0);
+  z = __builtin_amdgcn_mfma_f32_16x16x4f32(x.z, y.z, z, 0, 0, 0);
+  c = __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b.w, c, 0, 0, 0);
+  z = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, y.w, z, 0, 0, 0);
+}
 __device__ __forceinline__ float ex2(float x) { return __builtin_amdgcn_exp2f(x); }
 __device__ __forceinline__ float4 ld4(const float* p) { return *reinterpret_cast<const float4*>(p); }
 
-// Convolution + SiLU of one channel over n consecutive tokens from token t0 on; put(i, value) for each
+// Convolution + SiLU of one channel over `len` (a multiple of 16) consecutive tokens from token t0 on, of which the
+// portion holds n: put(i, value), zero past n.  Inputs are requested 16 at a time at clamped addresses: a load under a
+// condition would be waited for where the condition ends.
 template <typename T, typename F>
-__device__ __forceinline__ void conv_run(const T* in, int64_t ld, int64_t tok0, int t0, int n, int pos, const T* ring, int taps, int C,
-                                         int c, const float* w, float bias, F put) {
+__device__ __forceinline__ void conv_run(const T* in, int64_t ld, int64_t tok0, int t0, int n, int len, int pos, const T* ring,
+                                         int taps, int C, int c, const float* w, float bias, F put) {
   float wj[MAX_TAPS], win[MAX_TAPS];  // right-aligned: entry MAX_TAPS - 1 is the current token
+  const T* src = in + tok0 * ld + c;
 #pragma unroll
   for (int j = 0; j < MAX_TAPS; ++j) {
     const int back = MAX_TAPS - 1 - j;
     wj[j] = back < taps ? w[c * taps + taps - 1 - back] : 0.0f;
     win[j] = 0.0f;
-    if (back > 0 && back < taps) {
+    if (n > 0 && back > 0 && back < taps) {
       const int a = pos + t0 - back;  // position
-      if (a >= pos) win[j] = to_f32(in[(tok0 + (a - pos)) * ld + c]);
+      if (a >= pos) win[j] = to_f32(src[(int64_t)(a - pos) * ld]);
       else if (a >= 0) win[j] = to_f32(ring[(int64_t)(a % taps) * C + c]);
     }
   }
-  // the inputs are requested 16 at a time
-  for (int i0 = 0; i0 < n; i0 += 16) {
-    float x[16];
+  const int lastt = n > 0 ? t0 + n - 1 : 0;
+  for (int i0 = 0; i0 < len; i0 += 16) {
+    T x[16];
 #pragma unroll
-    for (int i = 0; i < 16; ++i) x[i] = i0 + i < n ? to_f32(in[(tok0 + t0 + i0 + i) * ld + c]) : 0.0f;
+    for (int i = 0; i < 16; ++i) x[i] = src[(int64_t)(i0 + i < n ? t0 + i0 + i : lastt) * ld];
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
-      if (i0 + i >= n) break;
-      win[MAX_TAPS - 1] = x[i];
+      win[MAX_TAPS - 1] = to_f32(x[i]);
       float acc = bias;
 #pragma unroll
       for (int j = 0; j < MAX_TAPS; ++j) acc = fmaf(wj[j], win[j], acc);
 #pragma unroll
       for (int j = 0; j + 1 < MAX_TAPS; ++j) win[j] = win[j + 1];
-      put(i0 + i, silu(acc));
+      put(i0 + i, i0 + i < n ? silu(acc) : 0.0f);
     }
   }
 }
@@ -82,16 +96,22 @@ struct DeltaChunkArgs {
   const float* conv_w;   // [C, taps]
   const float* a_log;    // [H]
   const float* dt_bias;  // [H * D]
-  float* A;              // [BC, H, 64, 64]  (BC = B * chunks)
-  float* QK;             // [BC, H, 64, 64]
-  float* W;              // [BC, H, 64, DP]  in: beta k e^G
-  float* U;              // [BC, H, 64, EP]  in: beta v
+  float* QK;             // [BC, H, 64, 64]  (BC = B * chunks)
+  float* W;              // [BC, H, 64, DP]
+  float* U;              // [BC, H, 64, EP]  U0
   float* Q;              // [BC, H, 64, DP]  q e^G
   float* K;              // [BC, H, DP, 64]  k e^{G_C - G}, transposed
   float* gc;             // [BC, H, DP]      e^{G_C}
   int64_t ld, ld_raw, ld_beta;
   int S, NC, H, G, D, E, DP, EP, taps, C;
 };
+
+// block pairs of the chunk's 4 x 4: 0..3 the diagonal, 4..9 below it, 10..15 above
+__device__ __forceinline__ void pair_block(int pair, int& I, int& J) {
+  constexpr uint64_t ROWS = 0x2101'0033'3221'3210ull, COLS = 0x3332'2121'0100'3210ull;
+  I = (int)(ROWS >> (4 * pair)) & 15;
+  J = (int)(COLS >> (4 * pair)) & 15;
+}
 
 template <int DP, typename T>
 __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p, const T* qkv, const T* raw, const T* braw, const T* ring0) {
@@ -102,7 +122,7 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
   double* g_s = reinterpret_cast<double*>(lds);  // [64][PG]
   double* tot = g_s + CH * PG;                   // [NB][DP]
   float* q_s = reinterpret_cast<float*>(tot + NB * DP);  // [64][PT]
-  float* k_s = q_s + CH * PT;
+  float* k_s = q_s + CH * (PT > CH + 4 ? PT : CH + 4);  // A takes q's place in the end
   float* b_s = k_s + CH * PT;                    // [64] beta
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int c = blockIdx.x % p.NC, b = blockIdx.x / p.NC, h = blockIdx.y, j = h / (p.H / p.G);
@@ -114,22 +134,27 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
   if (tid < CH) b_s[tid] = tid < n ? sigmoid(to_f32(braw[(tok0 + t0 + tid) * p.ld_beta + h])) : 0.0f;
   for (int x = tid; x < 2 * DP; x += 256) {
     float* dst = (x < DP ? q_s : k_s) + x % DP;
-    const int d = x % DP, m = d < D ? n : 0;
-    if (m) conv_run(qkv, p.ld, tok0, t0, n, pos, ring, p.taps, p.C, (x < DP ? 0 : p.G * D) + j * D + d, p.conv_w, 0.0f,
-                    [&](int i, float v) { dst[i * PT] = v; });
-    for (int i = m; i < CH; ++i) dst[i * PT] = 0.0f;
+    const int d = x % DP;
+    conv_run(qkv, p.ld, tok0, t0, d < D ? n : 0, CH, pos, ring, p.taps, p.C, (x < DP ? 0 : p.G * D) + j * D + (d < D ? d : D - 1),
+             p.conv_w, 0.0f, [&](int i, float v) { dst[i * PT] = v; });
   }
   const float a = -expf(p.a_log[h]) * 1.44269504088896341f;
-  for (int d = tid; d < DP; d += 256) {
-    double sum = 0.0;
-    const float bias = d < D ? p.dt_bias[h * D + d] : 0.0f;
-    const T* src = raw + (tok0 + t0) * p.ld_raw + h * D + d;
-#pragma unroll 16
-    for (int i = 0; i < CH; ++i) {
-      if (i % BL == 0) sum = 0.0;
-      if (i < n && d < D) sum += (double)(a * softplus(to_f32(src[i * p.ld_raw]) + bias));
-      g_s[i * PG + d] = sum;
-      if (i % BL == BL - 1) tot[(i / BL) * DP + d] = sum;
+  for (int x = tid; x < 2 * DP; x += 256) {  // channel, and half of the chunk
+    const int d = x % DP, dc = d < D ? d : D - 1, i1 = (x / DP) * (CH / 2);
+    const float bias = p.dt_bias[h * D + dc];
+    const T* src = raw + tok0 * p.ld_raw + h * D + dc;
+    for (int i0 = i1; i0 < i1 + CH / 2; i0 += BL) {
+      T v[BL];
+#pragma unroll
+      for (int i = 0; i < BL; ++i) v[i] = src[(int64_t)(t0 + (i0 + i < n ? i0 + i : n - 1)) * p.ld_raw];
+      double sum = 0.0;
+#pragma unroll
+      for (int i = 0; i < BL; ++i) {
+        const float l = a * softplus_abs(to_f32(v[i]) + bias);
+        sum += i0 + i < n && d < D ? (double)l : 0.0;
+        g_s[(i0 + i) * PG + d] = sum;
+      }
+      tot[(i0 / BL) * DP + d] = sum;
     }
   }
   __syncthreads();
@@ -140,15 +165,6 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
     const float rq = 1.0f / (sqrtf(wave_sum(sq) + 1e-6f) * sqrtf((float)D)), rk = 1.0f / sqrtf(wave_sum(sk) + 1e-6f);
     for (int d = lane; d < DP; d += 64) q_s[i * PT + d] *= rq, k_s[i * PT + d] *= rk;
   }
-  // beta v, by channel (64-token pieces of 16 so that all threads have one)
-  for (int x = tid; x < p.EP * NB; x += 256) {
-    const int e = x % p.EP, i0 = (x / p.EP) * BL;
-    float* dst = p.U + (ch * CH + i0) * p.EP + e;
-    const int m = e < E ? (n - i0 < BL ? (n - i0 > 0 ? n - i0 : 0) : BL) : 0;
-    if (m) conv_run(qkv, p.ld, tok0, t0 + i0, m, pos, ring, p.taps, p.C, 2 * p.G * D + h * E + e, p.conv_w, 0.0f,
-                    [&](int i, float v) { dst[(int64_t)i * p.EP] = b_s[i0 + i] * v; });
-    for (int i = m; i < BL; ++i) dst[(int64_t)i * p.EP] = 0.0f;
-  }
   __syncthreads();
   // ---- the scaled copies
   for (int x = tid; x < CH * DP; x += 256) {
@@ -157,7 +173,6 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
     for (int k = 0; k < I; ++k) base += tot[k * DP + d];
     const float e = ex2((float)base);
     p.Q[ch * CH * DP + x] = q_s[i * PT + d] * e;
-    p.W[ch * CH * DP + x] = b_s[i] * k_s[i * PT + d] * e;
   }
   for (int x = tid; x < DP * CH; x += 256) {
     const int d = x / CH, i = x % CH, I = i / BL;
@@ -167,17 +182,15 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
   }
   for (int d = tid; d < DP; d += 256) p.gc[ch * DP + d] = ex2((float)(tot[d] + tot[DP + d] + tot[2 * DP + d] + tot[3 * DP + d]));
   // ---- A and QK: 10 block pairs I >= J, the four diagonal ones first (one per wavefront)
-  float* A = p.A + ch * CH * CH;
+  f32x4 a_reg[NB];  // this wavefront's blocks of A: they go to LDS when q is not needed any more
   float* QK = p.QK + ch * CH * CH;
   const int r16 = lane & 15, q4 = (lane >> 4) * 4;
-  for (int pair = wave; pair < NB * NB; pair += 4) {
+#pragma unroll
+  for (int turn = 0; turn < NB; ++turn) {
+    const int pair = wave + 4 * turn;
     // pairs 0..3: diagonal; 4..9: below it; 10..15: above, zero
     int I, J;
-    if (pair < 4) I = J = pair;
-    else {
-      constexpr int RI[12] = {1, 2, 2, 3, 3, 3, 0, 0, 1, 0, 1, 2}, RJ[12] = {0, 0, 1, 0, 1, 2, 1, 2, 2, 3, 3, 3};
-      I = RI[pair - 4], J = RJ[pair - 4];
-    }
+    pair_block(pair, I, J);
     f32x4 sa = {0, 0, 0, 0}, sq = {0, 0, 0, 0};
     const int i = I * BL + r16, jj = J * BL + r16;  // this lane's row (A operand) and column (B operand)
     bool direct = false;
@@ -230,37 +243,55 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int row = I * BL + q4 + r, col = J * BL + r16;
-      A[row * CH + col] = col < row ? b_s[row] * sa[r] : 0.0f;
+      a_reg[turn][r] = col < row ? b_s[row] * sa[r] : 0.0f;
       QK[row * CH + col] = col <= row ? sq[r] : 0.0f;
     }
   }
-}
-
-// ---------------------------------------------------------------------------------------------- delta: solve
-// x <- (I + A)^-1 x, column by column: one thread holds a column of 64; A is uniform and comes through scalar loads
-__global__ __launch_bounds__(256) void delta_chunk_solve_kernel(const float* __restrict__ A, float* __restrict__ W, float* __restrict__ U,
-                                                                int DP, int EP) {
-  const int64_t ch = blockIdx.x;
-  const int col = blockIdx.y * 256 + threadIdx.x;
-  if (col >= DP + EP) return;
-  const int ld = col < DP ? DP : EP;
-  float* x = col < DP ? W + ch * CH * DP + col : U + ch * CH * EP + (col - DP);
-  const float* a = A + ch * CH * CH;
-  float v[CH];
+  __syncthreads();
+  constexpr int PA = CH + 4;
+  float* A = q_s;  // [64][PA]
 #pragma unroll
-  for (int i = 0; i < CH; ++i) v[i] = x[(int64_t)i * ld];
+  for (int turn = 0; turn < NB; ++turn) {
+    int I, J;
+    pair_block(wave + 4 * turn, I, J);
 #pragma unroll
-  for (int i = 1; i < CH; ++i) {
-    float s0 = 0.0f, s1 = 0.0f;
-#pragma unroll
-    for (int k = 0; k < i; ++k) {
-      if (k & 1) s1 = fmaf(a[i * CH + k], v[k], s1);
-      else s0 = fmaf(a[i * CH + k], v[k], s0);
-    }
-    v[i] -= s0 + s1;
+    for (int r = 0; r < 4; ++r) A[(I * BL + q4 + r) * PA + J * BL + r16] = a_reg[turn][r];
   }
+  __syncthreads();
+  // ---- x <- (I + A)^-1 x, a column per thread: beta k e^G, and beta v straight from its convolution
+  for (int colx = tid; colx < DP + p.EP; colx += 256) {
+    float v[CH];
+    if (colx < DP) {
+      double base = 0.0;
 #pragma unroll
-  for (int i = 0; i < CH; ++i) x[(int64_t)i * ld] = v[i];
+      for (int i = 0; i < CH; ++i) {
+        v[i] = b_s[i] * k_s[i * PT + colx] * ex2((float)(base + g_s[i * PG + colx]));
+        if (i % BL == BL - 1) base += tot[(i / BL) * DP + colx];
+      }
+    } else {
+      const int e = colx - DP, ec = e < E ? e : E - 1;
+#pragma unroll
+      for (int i0 = 0; i0 < CH; i0 += BL)
+        conv_run(qkv, p.ld, tok0, t0 + i0, e < E ? (n - i0 < BL ? (n - i0 > 0 ? n - i0 : 0) : BL) : 0, BL, pos, ring, p.taps, p.C,
+                 2 * p.G * D + h * E + ec, p.conv_w, 0.0f, [&](int i, float x) { v[i0 + i] = b_s[i0 + i] * x; });
+    }
+    const int ldx = colx < DP ? DP : p.EP;
+    float* x = colx < DP ? p.W + ch * CH * DP + colx : p.U + ch * CH * p.EP + (colx - DP);
+#pragma unroll
+    for (int i = 0; i < CH; ++i) {
+      float s0 = 0.0f, s1 = 0.0f;
+#pragma unroll
+      for (int k = 0; k < i; k += 4) {  // entries at and above the diagonal are zero
+        const float4 r = ld4(&A[i * PA + k]);
+        s0 = fmaf(r.x, v[k], s0);
+        if (k + 1 < i) s1 = fmaf(r.y, v[k + 1], s1);
+        if (k + 2 < i) s0 = fmaf(r.z, v[k + 2], s0);
+        if (k + 3 < i) s1 = fmaf(r.w, v[k + 3], s1);
+      }
+      v[i] -= s0 + s1;
+      x[(int64_t)i * ldx] = v[i];
+    }
+  }
 }
 
 // ---------------------------------------------------------------------------------------------- delta: scan
@@ -297,7 +328,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
   __shared__ __align__(16) float u_s[CT * UP];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int r16 = lane & 15, q4 = (lane >> 4) * 4;
-  const int tile = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  // heads first: the tiles of a head read the same chunks, and workgroups go round robin over the XCDs and their caches
+  const int tile = blockIdx.y, h = blockIdx.x, b = blockIdx.z;
   const int e = tile * CT + r16, D = p.D;
   float* col = p.state + (((int64_t)p.slots[b] * p.H + h) * p.E + (e < p.E ? e : 0)) * D;
   f32x4 s[NT];
@@ -320,7 +352,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
   };
   auto load_u = [&](int64_t ch) __attribute__((always_inline)) {
 #pragma unroll
-    for (int r = 0; r < 4; ++r) u0[r] = e < p.EP ? p.U[(ch * CH + wave * BL + q4 + r) * p.EP + e] : 0.0f;
+    for (int r = 0; r < 4; ++r) u0[r] = p.U[(ch * CH + wave * BL + q4 + r) * p.EP + e];
   };
   auto load_a = [&](int64_t ch) __attribute__((always_inline)) {
 #pragma unroll
@@ -329,10 +361,10 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
   auto load_k = [&](int64_t ch) __attribute__((always_inline)) {
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
-      if (wave + 4 * t >= KB) break;
-      gc[t] = ld4(p.gc + ch * DP + (wave + 4 * t) * 16 + q4);
+      const int d0 = (KB >= 4 || wave < KB ? wave + 4 * t : 0) * 16;  // wavefronts without a tile read another's
+      gc[t] = ld4(p.gc + ch * DP + d0 + q4);
 #pragma unroll
-      for (int x = 0; x < NB; ++x) k[t][x] = ld4(p.K + (ch * DP + (wave + 4 * t) * 16 + r16) * CH + x * 16 + q4);
+      for (int x = 0; x < NB; ++x) k[t][x] = ld4(p.K + (ch * DP + d0 + r16) * CH + x * 16 + q4);
     }
   };
   load_w(base(0)), load_q(base(0)), load_u(base(0)), load_a(base(0)), load_k(base(0));
@@ -343,12 +375,11 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
       if (wave + 4 * t < KB) *reinterpret_cast<f32x4*>(&s_s[r16 * SP + (wave + 4 * t) * 16 + q4]) = s[t];
     __syncthreads();
     f32x4 ws = {0, 0, 0, 0}, o = {0, 0, 0, 0};
+    float4 sv[KB];
 #pragma unroll
-    for (int x = 0; x < KB; ++x) {
-      const float4 sv = ld4(&s_s[r16 * SP + x * 16 + q4]);
-      ws = mma16(w[x], sv, ws);
-      o = mma16(q[x], sv, o);
-    }
+    for (int x = 0; x < KB; ++x) sv[x] = ld4(&s_s[r16 * SP + x * 16 + q4]);
+#pragma unroll
+    for (int x = 0; x < KB; ++x) mma16x2(w[x], sv[x], ws, q[x], sv[x], o);
     f32x4 u;
 #pragma unroll
     for (int r = 0; r < 4; ++r) u[r] = u0[r] - ws[r];
@@ -359,13 +390,12 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
 #pragma unroll
     for (int x = 0; x < NB; ++x) uv[x] = ld4(&u_s[r16 * UP + x * 16 + q4]);
 #pragma unroll
-    for (int x = 0; x < NB; ++x) o = mma16(a[x], uv[x], o);
+    for (int t = 0; t < NT; ++t) s[t][0] *= gc[t].x, s[t][1] *= gc[t].y, s[t][2] *= gc[t].z, s[t][3] *= gc[t].w;
 #pragma unroll
-    for (int t = 0; t < NT; ++t) {
-      if (wave + 4 * t >= KB) break;
-      s[t][0] *= gc[t].x, s[t][1] *= gc[t].y, s[t][2] *= gc[t].z, s[t][3] *= gc[t].w;
+    for (int x = 0; x < NB; ++x) {
+      mma16x2(a[x], uv[x], o, k[0][x], uv[x], s[0]);
 #pragma unroll
-      for (int x = 0; x < NB; ++x) s[t] = mma16(k[t][x], uv[x], s[t]);
+      for (int t = 1; t < NT; ++t) s[t] = mma16(k[t][x], uv[x], s[t]);
     }
     load_a(nx), load_k(nx);
     const int t0 = c * CH + wave * BL + q4;
@@ -413,10 +443,9 @@ __global__ __launch_bounds__(256) void ssd_group_kernel(SsdChunkArgs p, const T*
     const int y = x % (2 * NP), d = y % NP, i0 = (x / (2 * NP)) * BL;
     float* dst = (y < NP ? b_s : c_s) + i0 * PT + d;
     const int m = d < N ? (n - i0 < BL ? (n - i0 > 0 ? n - i0 : 0) : BL) : 0;
-    const int chan = p.H * p.P + (y < NP ? 0 : p.G * N) + g * N + d;
-    if (m) conv_run(xbc, p.ld, tok0, t0 + i0, m, pos, ring, p.taps, p.C, chan, p.conv_w, p.conv_b[chan],
-                    [&](int i, float v) { dst[i * PT] = v; });
-    for (int i = m; i < BL; ++i) dst[i * PT] = 0.0f;
+    const int chan = p.H * p.P + (y < NP ? 0 : p.G * N) + g * N + (d < N ? d : N - 1);
+    conv_run(xbc, p.ld, tok0, t0 + i0, m, BL, pos, ring, p.taps, p.C, chan, p.conv_w, p.conv_b[chan],
+             [&](int i, float v) { dst[i * PT] = v; });
   }
   __syncthreads();
   for (int x = tid; x < CH * NP; x += 256) p.Cm[ch * CH * NP + x] = c_s[(x / NP) * PT + x % NP];
@@ -442,7 +471,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
   __shared__ __align__(16) double l_s[2][CH];      // log2 decays summed from the chunk's start
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int r16 = lane & 15, q4 = (lane >> 4) * 4;
-  const int tile = blockIdx.x, h = blockIdx.y, b = blockIdx.z, g = h / (p.H / p.G);
+  const int tile = blockIdx.y, h = blockIdx.x, b = blockIdx.z, g = h / (p.H / p.G);
   const int e = tile * CT + r16, N = p.N, P = p.P, pos = p.pos[b];
   const int64_t tok0 = (int64_t)b * p.S;
   const T* ring = ring0 + (int64_t)p.slots[b] * p.taps * p.C;
@@ -468,15 +497,17 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
   auto load_b = [&](int64_t ch) __attribute__((always_inline)) {
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
-      if (wave + 4 * t >= KB) break;
+      const int d0 = (KB >= 4 || wave < KB ? wave + 4 * t : 0) * 16;
 #pragma unroll
-      for (int x = 0; x < NB; ++x) bt[t][x] = ld4(p.Bt + (ch * NP + (wave + 4 * t) * 16 + r16) * CH + x * 16 + q4);
+      for (int x = 0; x < NB; ++x) bt[t][x] = ld4(p.Bt + (ch * NP + d0 + r16) * CH + x * 16 + q4);
     }
   };
   // x: thread = (column tid % 16, tokens 4 (tid / 16) .. + 4); its raw inputs are requested a chunk ahead
-  const int xe = tid & 15, xt = (tid >> 4) * 4, xc = h * P + tile * CT + xe;
+  const int xe = tid & 15, xt = (tid >> 4) * 4;
   const bool xok = tile * CT + xe < P;
-  float wj[MAX_TAPS], xin[4 + MAX_TAPS - 1], dtin;
+  const int xc = h * P + (xok ? tile * CT + xe : P - 1);
+  float wj[MAX_TAPS];
+  T xin[4 + MAX_TAPS - 1], dtin;  // as loaded: a conversion here would wait for the load
 #pragma unroll
   for (int j = 0; j < MAX_TAPS; ++j) {
     const int back = MAX_TAPS - 1 - j;
@@ -486,15 +517,18 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
   auto load_x = [&](int c) __attribute__((always_inline)) {
 #pragma unroll
     for (int i = 0; i < 4 + MAX_TAPS - 1; ++i) {
-      const int t = c * CH + xt + i - (MAX_TAPS - 1), a = pos + t;  // token within the portion; position
-      float v = 0.0f;
-      if (xok && t < p.S && a >= 0 && (t >= 0 || t > -p.taps)) v = t >= 0 ? to_f32(xbc[(tok0 + t) * p.ld + xc]) : to_f32(ring[(int64_t)(a % p.taps) * p.C + xc]);
-      xin[i] = v;
+      const int t = c * CH + xt + i - (MAX_TAPS - 1), tc = t < 0 ? 0 : t < p.S ? t : p.S - 1;
+      xin[i] = xbc[(tok0 + tc) * p.ld + xc];
     }
     const int t = c * CH + lane;
-    dtin = t < p.S ? to_f32(dt_raw[(tok0 + t) * p.ld_dt + h]) : 0.0f;
+    dtin = dt_raw[(tok0 + (t < p.S ? t : p.S - 1)) * p.ld_dt + h];
   };
   load_c(base(0)), load_cb(base(0)), load_b(base(0)), load_x(0);
+#pragma unroll
+  for (int i = 0; i < MAX_TAPS - 1; ++i) {  // inputs from before the portion
+    const int t = xt + i - (MAX_TAPS - 1), a = pos + t;
+    if (t < 0) xin[i] = a >= 0 && t > -p.taps ? ring[(int64_t)(a % p.taps) * p.C + xc] : from_f32<T>(0.0f);
+  }
   for (int c = 0; c < p.NC; ++c) {
     const int buf = c & 1, nc = c + 1 < p.NC ? c + 1 : c;
     const int64_t nx = base(nc);
@@ -506,13 +540,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
       for (int i = 0; i < 4; ++i) {
         float acc = xb;
 #pragma unroll
-        for (int j = 0; j < MAX_TAPS; ++j) acc = fmaf(wj[j], xin[i + j], acc);
+        for (int j = 0; j < MAX_TAPS; ++j) acc = fmaf(wj[j], to_f32(xin[i + j]), acc);
         y[i] = xok && c * CH + xt + i < p.S ? silu(acc) : 0.0f;
       }
       xv = make_float4(y[0], y[1], y[2], y[3]);
     }
     *reinterpret_cast<float4*>(&x_s[buf][xe * XP + xt]) = xv;
-    const float dt = c * CH + lane < p.S ? softplus(dtin + dtb) : 0.0f;
+    const float dt = c * CH + lane < p.S ? softplus(to_f32(dtin) + dtb) : 0.0f;
     double L = (double)neg_a * (double)dt;
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
@@ -531,9 +565,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
       if (wave + 4 * t < KB) *reinterpret_cast<f32x4*>(&s_s[r16 * SP + (wave + 4 * t) * 16 + q4]) = s[t];
     __syncthreads();
     load_x(nc);
-    f32x4 y = {0, 0, 0, 0};
+    f32x4 y = {0, 0, 0, 0}, y1 = {0, 0, 0, 0};
+    float4 sv[KB];
 #pragma unroll
-    for (int x = 0; x < KB; ++x) y = mma16(cm[x], ld4(&s_s[r16 * SP + x * 16 + q4]), y);
+    for (int x = 0; x < KB; ++x) sv[x] = ld4(&s_s[r16 * SP + x * 16 + q4]);
+#pragma unroll
+    for (int x = 0; x < KB; x += 2) mma16x2(cm[x], sv[x], y, cm[x + 1], sv[x + 1], y1);
+    y += y1;
     load_c(nx);
     __syncthreads();  // the state may be overwritten
     float4 xx[NB];
@@ -614,7 +652,7 @@ extern "C" int aqs_chunked_ok(int64_t rows, int64_t taps) { return rows > 0 && r
 // floats of workspace for B sequences of S tokens
 extern "C" int64_t aqs_delta_chunked_ws(int64_t B, int64_t S, int64_t H, int64_t D, int64_t E) {
   const int64_t DP = pad_rows(D), EP = pad16(E);
-  return B * ((S + CH - 1) / CH) * H * (2 * CH * CH + 3 * CH * DP + CH * EP + DP);
+  return B * ((S + CH - 1) / CH) * H * (CH * CH + 3 * CH * DP + CH * EP + DP);
 }
 extern "C" int64_t aqs_ssd_chunked_ws(int64_t B, int64_t S, int64_t G, int64_t N) {
   const int64_t NP = pad_rows(N);
@@ -636,8 +674,7 @@ extern "C" int aqs_delta_chunked(const void* qkv, int64_t ld, const void* raw, i
   const int64_t DP = pad_rows(D), EP = pad16(E), n = B * NC * H;
   DeltaChunkArgs a{};
   a.slots = slots, a.pos = pos, a.conv_w = w, a.a_log = a_log, a.dt_bias = dt_bias;
-  a.A = ws;
-  a.QK = a.A + n * CH * CH;
+  a.QK = ws;
   a.W = a.QK + n * CH * CH;
   a.Q = a.W + n * CH * DP;
   a.K = a.Q + n * CH * DP;
@@ -647,17 +684,15 @@ extern "C" int aqs_delta_chunked(const void* qkv, int64_t ld, const void* raw, i
   a.S = (int)S, a.NC = (int)NC, a.H = (int)H, a.G = (int)G, a.D = (int)D, a.E = (int)E, a.DP = (int)DP, a.EP = (int)EP;
   a.taps = (int)taps, a.C = (int)(2 * G * D + H * E);
   hipStream_t st = (hipStream_t)stream;
-  const size_t lds = (size_t)(2 * CH * (DP + 4) + CH) * 4 + (size_t)(CH * (DP + 2) + NB * DP) * 8;
+  const size_t lds = (size_t)(CH * (DP + 4) + CH * (DP + 4 > CH + 4 ? DP + 4 : CH + 4) + CH) * 4 + (size_t)(CH * (DP + 2) + NB * DP) * 8;
   SQ_DISPATCH(dtype, SQ_PADDED(D, {
                 if (const int rc = big_lds(&delta_chunk_prep_kernel<RP, T>, lds)) return rc;
                 (delta_chunk_prep_kernel<RP, T><<<dim3((unsigned)(B * NC), (unsigned)H), 256, lds, st>>>(
                     a, (const T*)qkv, (const T*)raw, (const T*)beta_raw, (const T*)ring));
               }));
   if (const int rc = launched()) return rc;
-  delta_chunk_solve_kernel<<<dim3((unsigned)n, (unsigned)((DP + EP + 255) / 256)), 256, 0, st>>>(a.A, a.W, a.U, (int)DP, (int)EP);
-  if (const int rc = launched()) return rc;
   const DeltaScanArgs s{a.W, a.U, a.Q, a.K, a.QK, a.gc, state, out, slots, pos, (int)S, (int)NC, (int)H, (int)D, (int)E, (int)EP};
-  const dim3 grid((unsigned)(EP / CT), (unsigned)H, (unsigned)B);
+  const dim3 grid((unsigned)H, (unsigned)(EP / CT), (unsigned)B);
   SQ_PADDED(D, (delta_chunk_scan_kernel<RP><<<grid, 256, 0, st>>>(s)));
   return launched();
 }
@@ -690,7 +725,7 @@ extern "C" int aqs_ssd_chunked(const void* xbc, int64_t ld, const void* dt_raw, 
                 (ssd_group_kernel<RP, T><<<dim3((unsigned)(B * NC), (unsigned)G), 256, lds, st>>>(a, (const T*)xbc, (const T*)ring));
               }));
   if (const int rc = launched()) return rc;
-  const dim3 grid((unsigned)((P + CT - 1) / CT), (unsigned)H, (unsigned)B);
+  const dim3 grid((unsigned)H, (unsigned)((P + CT - 1) / CT), (unsigned)B);
   SQ_DISPATCH(dtype, SQ_PADDED(N, (ssd_chunks_kernel<RP, T><<<grid, 256, 0, st>>>(a, (const T*)xbc, (const T*)dt_raw, (const T*)ring))));
   return launched();
 }

@@ -121,10 +121,16 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
 }
 
 // ---- elementwise functions (fp32)
-__device__ __forceinline__ float sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
-__device__ __forceinline__ float silu(float x) { return x / (1.0f + expf(-x)); }
-// log(1 + exp(x)) without overflow
+// e^x and 1 / (1 + e^-x) from the hardware's exp2 and reciprocal (each within an ulp or two)
+__device__ __forceinline__ float exp_fast(float x) { return __builtin_amdgcn_exp2f(x * 1.44269504088896341f); }
+__device__ __forceinline__ float sigmoid(float x) { return __builtin_amdgcn_rcpf(1.0f + exp_fast(-x)); }
+__device__ __forceinline__ float silu(float x) { return x * sigmoid(x); }
+// log(1 + exp(x)) without overflow, to full relative precision
 __device__ __forceinline__ float softplus(float x) { return fmaxf(x, 0.0f) + log1pf(expf(-fabsf(x))); }
+// the same within 1e-7 absolutely: enough where only exp(-a softplus) is used
+__device__ __forceinline__ float softplus_abs(float x) {
+  return fmaxf(x, 0.0f) + 0.693147180559945309f * __builtin_amdgcn_logf(1.0f + exp_fast(-fabsf(x)));
+}
 // g * sigmoid(1.702 g) * (u + 1) of the clamped pair: the gate from above only, the linear part on both sides
 __device__ __forceinline__ float clamped_glu(float g, float u, float limit) {
   g = fminf(g, limit);

@@ -8,7 +8,7 @@
 //     S  <- e^{G_C} S + sum_j (k_j e^{G_C - G_j}) u_j^T
 // so with (I + A) the unit triangular matrix on the left:  u = U0 - W S  with  W = (I + A)^-1 (beta k e^G),
 // U0 = (I + A)^-1 (beta v).  Two launches: `prep` (per chunk and head: convolution, norms, decays, A and the masked
-// query-key matrix, then W and U0 by forward substitution, one thread per column), `scan` (per head and 16 columns of S:
+// query-key matrix, W and U0), `scan` (per head and 16 columns of S:
 // the chunks in order).
 //
 // A decay can be anything in (0, 1], so e^{G_i - G_j} must not be split into e^{G_i} and e^{-G_j} across a chunk.  The
@@ -113,6 +113,16 @@ __device__ __forceinline__ void pair_block(int pair, int& I, int& J) {
   J = (int)(COLS >> (4 * pair)) & 15;
 }
 
+constexpr int PA = CH + 4, PI = BL + 4;  // row pitches of A and of the inverted blocks
+constexpr int max_of(int a, int b) { return a > b ? a : b; }
+// floats of LDS: decays (later A and the inverses), q (later v), k, beta
+template <int DP>
+struct PrepLds {
+  static constexpr int DECAYS = max_of(2 * (CH * (DP + 2) + NB * DP), CH * PA + NB * BL * PI);
+  static constexpr int QUERIES = CH * max_of(DP + 4, PA);
+  static constexpr int TOTAL = DECAYS + QUERIES + CH * (DP + 4) + CH;
+};
+
 template <int DP, typename T>
 __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p, const T* qkv, const T* raw, const T* braw, const T* ring0) {
   constexpr int PT = DP + 4, PG = DP + 2;
@@ -121,8 +131,8 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
   // one token that forgets everything must not cost the digits of the others: double.
   double* g_s = reinterpret_cast<double*>(lds);  // [64][PG]
   double* tot = g_s + CH * PG;                   // [NB][DP]
-  float* q_s = reinterpret_cast<float*>(tot + NB * DP);  // [64][PT]
-  float* k_s = q_s + CH * (PT > CH + 4 ? PT : CH + 4);  // A takes q's place in the end
+  float* q_s = lds + PrepLds<DP>::DECAYS;        // [64][PT], later v
+  float* k_s = q_s + PrepLds<DP>::QUERIES;
   float* b_s = k_s + CH * PT;                    // [64] beta
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int c = blockIdx.x % p.NC, b = blockIdx.x / p.NC, h = blockIdx.y, j = h / (p.H / p.G);
@@ -166,19 +176,23 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
     for (int d = lane; d < DP; d += 64) q_s[i * PT + d] *= rq, k_s[i * PT + d] *= rk;
   }
   __syncthreads();
-  // ---- the scaled copies
-  for (int x = tid; x < CH * DP; x += 256) {
-    const int i = x / DP, d = x % DP, I = i / BL;
-    double base = g_s[i * PG + d];
+  // ---- the scaled copies of q and k: a thread takes a channel of a block
+  for (int x = tid; x < NB * DP; x += 256) {
+    const int d = x % DP, I = x / DP;
+    double base = 0.0, rest = tot[I * DP + d];
     for (int k = 0; k < I; ++k) base += tot[k * DP + d];
-    const float e = ex2((float)base);
-    p.Q[ch * CH * DP + x] = q_s[i * PT + d] * e;
-  }
-  for (int x = tid; x < DP * CH; x += 256) {
-    const int d = x / CH, i = x % CH, I = i / BL;
-    double rest = tot[I * DP + d] - g_s[i * PG + d];
     for (int k = I + 1; k < NB; ++k) rest += tot[k * DP + d];
-    p.K[ch * DP * CH + x] = k_s[i * PT + d] * ex2((float)rest);
+    float kt[BL];
+#pragma unroll
+    for (int i = 0; i < BL; ++i) {
+      const int t = I * BL + i;
+      const double g = g_s[t * PG + d];
+      p.Q[(ch * CH + t) * DP + d] = q_s[t * PT + d] * ex2((float)(base + g));
+      kt[i] = k_s[t * PT + d] * ex2((float)(rest - g));
+    }
+#pragma unroll
+    for (int i = 0; i < BL; i += 4)
+      *reinterpret_cast<float4*>(p.K + (ch * DP + d) * CH + I * BL + i) = make_float4(kt[i], kt[i + 1], kt[i + 2], kt[i + 3]);
   }
   for (int d = tid; d < DP; d += 256) p.gc[ch * DP + d] = ex2((float)(tot[d] + tot[DP + d] + tot[2 * DP + d] + tot[3 * DP + d]));
   // ---- A and QK: 10 block pairs I >= J, the four diagonal ones first (one per wavefront)
@@ -247,9 +261,28 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
       QK[row * CH + col] = col <= row ? sq[r] : 0.0f;
     }
   }
-  __syncthreads();
-  constexpr int PA = CH + 4;
-  float* A = q_s;  // [64][PA]
+  // ---- (I + A)^-1 by blocks of 16: X_I = T_I (R_I - sum_{J<I} A_IJ X_J), T_I the inverse of a diagonal block.  A column
+  // tile of R in the accumulator layout of mma16 is at the same time its right operand, so a wavefront solves a
+  // tile of 16 columns in registers.
+  constexpr int WT = (DP / 16 + 3) / 4;  // tiles of W per wavefront
+  f32x4 x[WT][NB];
+#pragma unroll
+  for (int t = 0; t < WT; ++t) {
+    const int d = ((wave + 4 * t) * 16 + r16) % DP;
+    double base = 0.0;
+#pragma unroll
+    for (int I = 0; I < NB; ++I) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int i = I * BL + q4 + r;
+        x[t][I][r] = b_s[i] * k_s[i * PT + d] * ex2((float)(base + g_s[i * PG + d]));
+      }
+      base += tot[I * DP + d];
+    }
+  }
+  __syncthreads();  // q, k and the decays are done with
+  float* A = reinterpret_cast<float*>(g_s);  // [64][PA]
+  float* T_s = A + CH * PA;                  // [NB][16][PI]
 #pragma unroll
   for (int turn = 0; turn < NB; ++turn) {
     int I, J;
@@ -258,39 +291,77 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
     for (int r = 0; r < 4; ++r) A[(I * BL + q4 + r) * PA + J * BL + r16] = a_reg[turn][r];
   }
   __syncthreads();
-  // ---- x <- (I + A)^-1 x, a column per thread: beta k e^G, and beta v straight from its convolution
-  for (int colx = tid; colx < DP + p.EP; colx += 256) {
-    float v[CH];
-    if (colx < DP) {
-      double base = 0.0;
+  if (wave == 0) {  // lane: column lane % 16 of block lane / 16
+    const float* blk = A + (lane >> 4) * BL * (PA + 1);
+    float v[BL];
 #pragma unroll
-      for (int i = 0; i < CH; ++i) {
-        v[i] = b_s[i] * k_s[i * PT + colx] * ex2((float)(base + g_s[i * PG + colx]));
-        if (i % BL == BL - 1) base += tot[(i / BL) * DP + colx];
+    for (int i = 0; i < BL; ++i) {
+      float sum = i == r16 ? 1.0f : 0.0f;
+#pragma unroll
+      for (int k = 0; k < i; k += 4) {
+        const float4 a4 = ld4(&blk[i * PA + k]);
+        sum = fmaf(-a4.x, v[k], sum);
+        if (k + 1 < i) sum = fmaf(-a4.y, v[k + 1], sum);
+        if (k + 2 < i) sum = fmaf(-a4.z, v[k + 2], sum);
+        if (k + 3 < i) sum = fmaf(-a4.w, v[k + 3], sum);
       }
-    } else {
-      const int e = colx - DP, ec = e < E ? e : E - 1;
-#pragma unroll
-      for (int i0 = 0; i0 < CH; i0 += BL)
-        conv_run(qkv, p.ld, tok0, t0 + i0, e < E ? (n - i0 < BL ? (n - i0 > 0 ? n - i0 : 0) : BL) : 0, BL, pos, ring, p.taps, p.C,
-                 2 * p.G * D + h * E + ec, p.conv_w, 0.0f, [&](int i, float x) { v[i0 + i] = b_s[i0 + i] * x; });
+      v[i] = sum;
+      T_s[((lane >> 4) * BL + i) * PI + r16] = sum;
     }
-    const int ldx = colx < DP ? DP : p.EP;
-    float* x = colx < DP ? p.W + ch * CH * DP + colx : p.U + ch * CH * p.EP + (colx - DP);
+  }
+  // beta v into q's space, 64 channels at a time: thread = (channel, block of 16 tokens)
+  float* v_s = q_s;  // [64][PA]
+  auto convolve_v = [&](int e0) __attribute__((always_inline)) {
+    const int e = e0 + (tid & 63), ec = e < E ? e : E - 1, i0 = wave * BL;
+    conv_run(qkv, p.ld, tok0, t0 + i0, e < E ? (n - i0 < BL ? (n - i0 > 0 ? n - i0 : 0) : BL) : 0, BL, pos, ring, p.taps, p.C,
+             2 * p.G * D + h * E + ec, p.conv_w, 0.0f, [&](int i, float v) { v_s[(i0 + i) * PA + (tid & 63)] = b_s[i0 + i] * v; });
+  };
+  convolve_v(0);
+  __syncthreads();
+  float4 am[NB][NB], tm[NB];
 #pragma unroll
-    for (int i = 0; i < CH; ++i) {
-      float s0 = 0.0f, s1 = 0.0f;
+  for (int I = 0; I < NB; ++I) {
+    tm[I] = ld4(&T_s[(I * BL + r16) * PI + q4]);
 #pragma unroll
-      for (int k = 0; k < i; k += 4) {  // entries at and above the diagonal are zero
-        const float4 r = ld4(&A[i * PA + k]);
-        s0 = fmaf(r.x, v[k], s0);
-        if (k + 1 < i) s1 = fmaf(r.y, v[k + 1], s1);
-        if (k + 2 < i) s0 = fmaf(r.z, v[k + 2], s0);
-        if (k + 3 < i) s1 = fmaf(r.w, v[k + 3], s1);
-      }
-      v[i] -= s0 + s1;
-      x[(int64_t)i * ldx] = v[i];
+    for (int J = 0; J < I; ++J) {
+      am[I][J] = ld4(&A[(I * BL + r16) * PA + J * BL + q4]);
+      am[I][J] = make_float4(-am[I][J].x, -am[I][J].y, -am[I][J].z, -am[I][J].w);
     }
+  }
+  auto solve = [&](f32x4 (&y)[NB]) __attribute__((always_inline)) {
+#pragma unroll
+    for (int I = 0; I < NB; ++I) {
+#pragma unroll
+      for (int J = 0; J < I; ++J) y[I] = mma16(am[I][J], make_float4(y[J][0], y[J][1], y[J][2], y[J][3]), y[I]);
+      y[I] = mma16(tm[I], make_float4(y[I][0], y[I][1], y[I][2], y[I][3]), f32x4{0, 0, 0, 0});
+    }
+  };
+  auto store = [&](const f32x4 (&y)[NB], float* dst, int ld) __attribute__((always_inline)) {
+#pragma unroll
+    for (int I = 0; I < NB; ++I)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) dst[(int64_t)(I * BL + q4 + r) * ld] = y[I][r];
+  };
+#pragma unroll
+  for (int t = 0; t < WT; ++t) {
+    if ((wave + 4 * t) * 16 >= DP) break;
+    solve(x[t]);
+    store(x[t], p.W + ch * CH * DP + (wave + 4 * t) * 16 + r16, DP);
+  }
+  for (int e0 = 0; e0 < p.EP; e0 += 64) {
+    if (e0) {
+      __syncthreads();
+      convolve_v(e0);
+      __syncthreads();
+    }
+    if (e0 + wave * 16 >= p.EP) continue;
+    f32x4 y[NB];
+#pragma unroll
+    for (int I = 0; I < NB; ++I)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) y[I][r] = v_s[(I * BL + q4 + r) * PA + wave * 16 + r16];
+    solve(y);
+    store(y, p.U + ch * CH * p.EP + e0 + wave * 16 + r16, p.EP);
   }
 }
 
@@ -320,7 +391,7 @@ __device__ __forceinline__ void store_state4(float* col, int d, int D, const f32
 }
 
 template <int DP>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) void delta_chunk_scan_kernel(DeltaScanArgs p) {
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) void delta_chunk_scan_kernel(DeltaScanArgs p) {
   constexpr int KB = DP / 16;               // groups of 16 in the contraction over rows
   constexpr int NT = (KB + 3) / 4;          // 16-row tiles of the state per wavefront
   constexpr int SP = DP + 4, UP = CH + 4;
@@ -338,70 +409,69 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     const int d = (wave + 4 * t) * 16 + q4;
     s[t] = load_state4(col, d, D, e < p.E && p.pos[b] > 0 && d < DP);
   }
-  float4 w[KB], q[KB], k[NT][NB], a[NB], gc[NT];
-  float u0[4];
+  // everything a chunk brings, in registers; the next chunk's is requested before this one's work begins
+  struct Chunk {
+    float4 w[KB], q[KB], k[NT][NB], a[NB], gc[NT];
+    float u0[4];
+  };
+  Chunk c0, c1;
   const int row = wave * BL + r16;          // this lane's token (A operand)
-  auto base = [&](int c) -> int64_t { return ((int64_t)b * p.NC + c) * p.H + h; };
-  auto load_w = [&](int64_t ch) __attribute__((always_inline)) {
+  auto load = [&](Chunk& r, int c) __attribute__((always_inline)) {
+    const int64_t ch = ((int64_t)b * p.NC + (c < p.NC ? c : p.NC - 1)) * p.H + h;
 #pragma unroll
-    for (int x = 0; x < KB; ++x) w[x] = ld4(p.W + (ch * CH + row) * DP + x * 16 + q4);
-  };
-  auto load_q = [&](int64_t ch) __attribute__((always_inline)) {
+    for (int x = 0; x < KB; ++x) {
+      r.w[x] = ld4(p.W + (ch * CH + row) * DP + x * 16 + q4);
+      r.q[x] = ld4(p.Q + (ch * CH + row) * DP + x * 16 + q4);
+    }
 #pragma unroll
-    for (int x = 0; x < KB; ++x) q[x] = ld4(p.Q + (ch * CH + row) * DP + x * 16 + q4);
-  };
-  auto load_u = [&](int64_t ch) __attribute__((always_inline)) {
+    for (int i = 0; i < 4; ++i) r.u0[i] = p.U[(ch * CH + wave * BL + q4 + i) * p.EP + e];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) u0[r] = p.U[(ch * CH + wave * BL + q4 + r) * p.EP + e];
-  };
-  auto load_a = [&](int64_t ch) __attribute__((always_inline)) {
-#pragma unroll
-    for (int x = 0; x < NB; ++x) a[x] = ld4(p.QK + (ch * CH + row) * CH + x * 16 + q4);
-  };
-  auto load_k = [&](int64_t ch) __attribute__((always_inline)) {
+    for (int x = 0; x < NB; ++x) r.a[x] = ld4(p.QK + (ch * CH + row) * CH + x * 16 + q4);
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
       const int d0 = (KB >= 4 || wave < KB ? wave + 4 * t : 0) * 16;  // wavefronts without a tile read another's
-      gc[t] = ld4(p.gc + ch * DP + d0 + q4);
+      r.gc[t] = ld4(p.gc + ch * DP + d0 + q4);
 #pragma unroll
-      for (int x = 0; x < NB; ++x) k[t][x] = ld4(p.K + (ch * DP + d0 + r16) * CH + x * 16 + q4);
+      for (int x = 0; x < NB; ++x) r.k[t][x] = ld4(p.K + (ch * DP + d0 + r16) * CH + x * 16 + q4);
     }
   };
-  load_w(base(0)), load_q(base(0)), load_u(base(0)), load_a(base(0)), load_k(base(0));
-  for (int c = 0; c < p.NC; ++c) {
-    const int64_t nx = base(c + 1 < p.NC ? c + 1 : c);
+  auto chunk = [&](const Chunk& r, Chunk& next, int c) __attribute__((always_inline)) {
 #pragma unroll
     for (int t = 0; t < NT; ++t)
       if (wave + 4 * t < KB) *reinterpret_cast<f32x4*>(&s_s[r16 * SP + (wave + 4 * t) * 16 + q4]) = s[t];
+    load(next, c + 1);
     __syncthreads();
     f32x4 ws = {0, 0, 0, 0}, o = {0, 0, 0, 0};
     float4 sv[KB];
 #pragma unroll
     for (int x = 0; x < KB; ++x) sv[x] = ld4(&s_s[r16 * SP + x * 16 + q4]);
 #pragma unroll
-    for (int x = 0; x < KB; ++x) mma16x2(w[x], sv[x], ws, q[x], sv[x], o);
+    for (int x = 0; x < KB; ++x) mma16x2(r.w[x], sv[x], ws, r.q[x], sv[x], o);
     f32x4 u;
 #pragma unroll
-    for (int r = 0; r < 4; ++r) u[r] = u0[r] - ws[r];
+    for (int i = 0; i < 4; ++i) u[i] = r.u0[i] - ws[i];
     *reinterpret_cast<f32x4*>(&u_s[r16 * UP + wave * BL + q4]) = u;
-    load_w(nx), load_q(nx), load_u(nx);
     __syncthreads();
     float4 uv[NB];
 #pragma unroll
     for (int x = 0; x < NB; ++x) uv[x] = ld4(&u_s[r16 * UP + x * 16 + q4]);
 #pragma unroll
-    for (int t = 0; t < NT; ++t) s[t][0] *= gc[t].x, s[t][1] *= gc[t].y, s[t][2] *= gc[t].z, s[t][3] *= gc[t].w;
+    for (int t = 0; t < NT; ++t) s[t][0] *= r.gc[t].x, s[t][1] *= r.gc[t].y, s[t][2] *= r.gc[t].z, s[t][3] *= r.gc[t].w;
 #pragma unroll
     for (int x = 0; x < NB; ++x) {
-      mma16x2(a[x], uv[x], o, k[0][x], uv[x], s[0]);
+      mma16x2(r.a[x], uv[x], o, r.k[0][x], uv[x], s[0]);
 #pragma unroll
-      for (int t = 1; t < NT; ++t) s[t] = mma16(k[t][x], uv[x], s[t]);
+      for (int t = 1; t < NT; ++t) s[t] = mma16(r.k[t][x], uv[x], s[t]);
     }
-    load_a(nx), load_k(nx);
     const int t0 = c * CH + wave * BL + q4;
 #pragma unroll
-    for (int r = 0; r < 4; ++r)
-      if (t0 + r < p.S && e < p.E) p.out[(((int64_t)b * p.S + t0 + r) * p.H + h) * p.E + e] = o[r];
+    for (int i = 0; i < 4; ++i)
+      if (t0 + i < p.S && e < p.E) p.out[(((int64_t)b * p.S + t0 + i) * p.H + h) * p.E + e] = o[i];
+  };
+  load(c0, 0);
+  for (int c = 0; c < p.NC; c += 2) {
+    chunk(c0, c1, c);
+    if (c + 1 < p.NC) chunk(c1, c0, c + 1);
   }
 #pragma unroll
   for (int t = 0; t < NT; ++t) {
@@ -461,7 +531,7 @@ __global__ __launch_bounds__(256) void ssd_group_kernel(SsdChunkArgs p, const T*
 }
 
 template <int NP, typename T>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) void ssd_chunks_kernel(SsdChunkArgs p, const T* xbc,
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) void ssd_chunks_kernel(SsdChunkArgs p, const T* xbc,
                                                                                                     const T* dt_raw, const T* ring0) {
   constexpr int KB = NP / 16, NT = (KB + 3) / 4, SP = NP + 4, XP = CH + 4;
   __shared__ __align__(16) float s_s[CT * SP];
@@ -484,54 +554,53 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
   }
   const float skip = p.skip[h], neg_a = -expf(p.a_log[h]) * 1.44269504088896341f, dtb = p.dt_bias[h];
   const int row = wave * BL + r16;
-  float4 cm[KB], cb[NB], bt[NT][NB];
-  auto base = [&](int c) -> int64_t { return ((int64_t)b * p.NC + c) * p.G + g; };
-  auto load_c = [&](int64_t ch) __attribute__((always_inline)) {
-#pragma unroll
-    for (int x = 0; x < KB; ++x) cm[x] = ld4(p.Cm + (ch * CH + row) * NP + x * 16 + q4);
-  };
-  auto load_cb = [&](int64_t ch) __attribute__((always_inline)) {
-#pragma unroll
-    for (int x = 0; x < NB; ++x) cb[x] = ld4(p.CB + (ch * CH + row) * CH + x * 16 + q4);
-  };
-  auto load_b = [&](int64_t ch) __attribute__((always_inline)) {
-#pragma unroll
-    for (int t = 0; t < NT; ++t) {
-      const int d0 = (KB >= 4 || wave < KB ? wave + 4 * t : 0) * 16;
-#pragma unroll
-      for (int x = 0; x < NB; ++x) bt[t][x] = ld4(p.Bt + (ch * NP + d0 + r16) * CH + x * 16 + q4);
-    }
-  };
   // x: thread = (column tid % 16, tokens 4 (tid / 16) .. + 4); its raw inputs are requested a chunk ahead
   const int xe = tid & 15, xt = (tid >> 4) * 4;
   const bool xok = tile * CT + xe < P;
   const int xc = h * P + (xok ? tile * CT + xe : P - 1);
   float wj[MAX_TAPS];
-  T xin[4 + MAX_TAPS - 1], dtin;  // as loaded: a conversion here would wait for the load
+  // what a chunk brings, in registers; the next chunk's is requested before this one's work begins.  x and dt as
+  // loaded: a conversion here would wait for the load.
+  struct Chunk {
+    float4 cm[KB], cb[NB], bt[NT][NB];
+    T xin[4 + MAX_TAPS - 1], dtin;
+  };
+  Chunk c0, c1;
 #pragma unroll
   for (int j = 0; j < MAX_TAPS; ++j) {
     const int back = MAX_TAPS - 1 - j;
     wj[j] = xok && back < p.taps ? p.conv_w[xc * p.taps + p.taps - 1 - back] : 0.0f;
   }
   const float xb = xok ? p.conv_b[xc] : 0.0f;
-  auto load_x = [&](int c) __attribute__((always_inline)) {
+  auto load = [&](Chunk& q, int c) __attribute__((always_inline)) {
+    if (c >= p.NC) c = p.NC - 1;
+    const int64_t ch = ((int64_t)b * p.NC + c) * p.G + g;
 #pragma unroll
     for (int i = 0; i < 4 + MAX_TAPS - 1; ++i) {
       const int t = c * CH + xt + i - (MAX_TAPS - 1), tc = t < 0 ? 0 : t < p.S ? t : p.S - 1;
-      xin[i] = xbc[(tok0 + tc) * p.ld + xc];
+      q.xin[i] = xbc[(tok0 + tc) * p.ld + xc];
     }
     const int t = c * CH + lane;
-    dtin = dt_raw[(tok0 + (t < p.S ? t : p.S - 1)) * p.ld_dt + h];
+    q.dtin = dt_raw[(tok0 + (t < p.S ? t : p.S - 1)) * p.ld_dt + h];
+#pragma unroll
+    for (int x = 0; x < KB; ++x) q.cm[x] = ld4(p.Cm + (ch * CH + row) * NP + x * 16 + q4);
+#pragma unroll
+    for (int x = 0; x < NB; ++x) q.cb[x] = ld4(p.CB + (ch * CH + row) * CH + x * 16 + q4);
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      const int d0 = (KB >= 4 || wave < KB ? wave + 4 * t : 0) * 16;
+#pragma unroll
+      for (int x = 0; x < NB; ++x) q.bt[t][x] = ld4(p.Bt + (ch * NP + d0 + r16) * CH + x * 16 + q4);
+    }
   };
-  load_c(base(0)), load_cb(base(0)), load_b(base(0)), load_x(0);
+  load(c0, 0);
 #pragma unroll
   for (int i = 0; i < MAX_TAPS - 1; ++i) {  // inputs from before the portion
     const int t = xt + i - (MAX_TAPS - 1), a = pos + t;
-    if (t < 0) xin[i] = a >= 0 && t > -p.taps ? ring[(int64_t)(a % p.taps) * p.C + xc] : from_f32<T>(0.0f);
+    if (t < 0) c0.xin[i] = a >= 0 && t > -p.taps ? ring[(int64_t)(a % p.taps) * p.C + xc] : from_f32<T>(0.0f);
   }
-  for (int c = 0; c < p.NC; ++c) {
-    const int buf = c & 1, nc = c + 1 < p.NC ? c + 1 : c;
-    const int64_t nx = base(nc);
+  auto chunk = [&](const Chunk& q, Chunk& next, int c) __attribute__((always_inline)) {
+    const int buf = c & 1;
     // ---- this chunk's x, steps and decays; the state as an operand
     float4 xv;
     {
@@ -540,13 +609,13 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
       for (int i = 0; i < 4; ++i) {
         float acc = xb;
 #pragma unroll
-        for (int j = 0; j < MAX_TAPS; ++j) acc = fmaf(wj[j], to_f32(xin[i + j]), acc);
+        for (int j = 0; j < MAX_TAPS; ++j) acc = fmaf(wj[j], to_f32(q.xin[i + j]), acc);
         y[i] = xok && c * CH + xt + i < p.S ? silu(acc) : 0.0f;
       }
       xv = make_float4(y[0], y[1], y[2], y[3]);
     }
     *reinterpret_cast<float4*>(&x_s[buf][xe * XP + xt]) = xv;
-    const float dt = c * CH + lane < p.S ? softplus(to_f32(dtin) + dtb) : 0.0f;
+    const float dt = c * CH + lane < p.S ? softplus(to_f32(q.dtin) + dtb) : 0.0f;
     double L = (double)neg_a * (double)dt;
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
@@ -563,16 +632,15 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
 #pragma unroll
     for (int t = 0; t < NT; ++t)
       if (wave + 4 * t < KB) *reinterpret_cast<f32x4*>(&s_s[r16 * SP + (wave + 4 * t) * 16 + q4]) = s[t];
+    load(next, c + 1);
     __syncthreads();
-    load_x(nc);
     f32x4 y = {0, 0, 0, 0}, y1 = {0, 0, 0, 0};
     float4 sv[KB];
 #pragma unroll
     for (int x = 0; x < KB; ++x) sv[x] = ld4(&s_s[r16 * SP + x * 16 + q4]);
 #pragma unroll
-    for (int x = 0; x < KB; x += 2) mma16x2(cm[x], sv[x], y, cm[x + 1], sv[x + 1], y1);
+    for (int x = 0; x < KB; x += 2) mma16x2(q.cm[x], sv[x], y, q.cm[x + 1], sv[x + 1], y1);
     y += y1;
-    load_c(nx);
     __syncthreads();  // the state may be overwritten
     float4 xx[NB];
 #pragma unroll
@@ -585,7 +653,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
     for (int x = 0; x < NB; ++x) {
       if (x > wave) break;  // keys ahead of every token of the wavefront
       const float4 dj = ld4(&dt_s[buf][x * 16 + q4]);
-      float m[4] = {cb[x].x * dj.x, cb[x].y * dj.y, cb[x].z * dj.z, cb[x].w * dj.w};
+      float m[4] = {q.cb[x].x * dj.x, q.cb[x].y * dj.y, q.cb[x].z * dj.z, q.cb[x].w * dj.w};
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int jt = x * 16 + q4 + r;
@@ -593,25 +661,26 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) voi
       }
       y = mma16(make_float4(m[0], m[1], m[2], m[3]), xx[x], y);
     }
-    load_cb(nx);
 #pragma unroll
     for (int x = 0; x < NB; ++x) {
       const float4 wv = ld4(&w_s[buf][x * 16 + q4]);
       const float4 xw = make_float4(xx[x].x * wv.x, xx[x].y * wv.y, xx[x].z * wv.z, xx[x].w * wv.w);
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
-        if (wave + 4 * t >= KB) break;
         if (x == 0) s[t] *= decay;
-        s[t] = mma16(bt[t][x], xw, s[t]);
+        s[t] = mma16(q.bt[t][x], xw, s[t]);
       }
     }
-    load_b(nx);
     const int t0 = c * CH + wave * BL + q4;
     const float4 own = ld4(&x_s[buf][r16 * XP + wave * BL + q4]);
     const float xo[4] = {own.x, own.y, own.z, own.w};
 #pragma unroll
     for (int r = 0; r < 4; ++r)
       if (t0 + r < p.S && e < P) p.out[(((int64_t)b * p.S + t0 + r) * p.H + h) * P + e] = y[r] + skip * xo[r];
+  };
+  for (int c = 0; c < p.NC; c += 2) {
+    chunk(c0, c1, c);
+    if (c + 1 < p.NC) chunk(c1, c0, c + 1);
   }
 #pragma unroll
   for (int t = 0; t < NT; ++t) {
@@ -684,8 +753,8 @@ extern "C" int aqs_delta_chunked(const void* qkv, int64_t ld, const void* raw, i
   a.S = (int)S, a.NC = (int)NC, a.H = (int)H, a.G = (int)G, a.D = (int)D, a.E = (int)E, a.DP = (int)DP, a.EP = (int)EP;
   a.taps = (int)taps, a.C = (int)(2 * G * D + H * E);
   hipStream_t st = (hipStream_t)stream;
-  const size_t lds = (size_t)(CH * (DP + 4) + CH * (DP + 4 > CH + 4 ? DP + 4 : CH + 4) + CH) * 4 + (size_t)(CH * (DP + 2) + NB * DP) * 8;
   SQ_DISPATCH(dtype, SQ_PADDED(D, {
+                constexpr size_t lds = PrepLds<RP>::TOTAL * sizeof(float);
                 if (const int rc = big_lds(&delta_chunk_prep_kernel<RP, T>, lds)) return rc;
                 (delta_chunk_prep_kernel<RP, T><<<dim3((unsigned)(B * NC), (unsigned)H), 256, lds, st>>>(
                     a, (const T*)qkv, (const T*)raw, (const T*)beta_raw, (const T*)ring));

@@ -50,6 +50,25 @@ __device__ __forceinline__ void mma16x2(const float4& a, const float4& b, f32x4&
   z = __builtin_amdgcn_mfma_f32_16x16x4f32(x.w, y.w, z, 0, 0, 0);
 }
 __device__ __forceinline__ float ex2(float x) { return __builtin_amdgcn_exp2f(x); }
+// The scans read their operands from memory a fragment at a time: 64 lanes x 4 floats of one 16 x 16 block, in lane
+// order, so that a load is 1 KB of consecutive memory (rows of a plain matrix would be 16 half-used cache lines).
+constexpr int FRAG = 256;
+// accumulator layout (column l % 16, rows 4 (l / 16) + r) -> left-operand layout (row l' % 16, columns 4 (l' / 16) + s)
+// of the same block: a 4 x 4 transpose inside every quad of lanes; the result belongs to fragment lane frag_lane(l).
+__device__ __forceinline__ float quad_xor1(float v) {
+  return __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0xB1, 0xf, 0xf, true));
+}
+__device__ __forceinline__ float quad_xor2(float v) {
+  return __int_as_float(__builtin_amdgcn_mov_dpp(__float_as_int(v), 0x4E, 0xf, 0xf, true));
+}
+__device__ __forceinline__ f32x4 quad_transpose(f32x4 v, int lane) {
+  const bool o1 = lane & 1, o2 = lane & 2;
+  const float a = quad_xor1(o1 ? v[0] : v[1]), b = quad_xor1(o1 ? v[2] : v[3]);
+  v = o1 ? f32x4{a, v[1], b, v[3]} : f32x4{v[0], a, v[2], b};
+  const float c = quad_xor2(o2 ? v[0] : v[2]), d = quad_xor2(o2 ? v[1] : v[3]);
+  return o2 ? f32x4{c, d, v[2], v[3]} : f32x4{v[0], v[1], c, d};
+}
+__device__ __forceinline__ int frag_lane(int lane) { return ((lane >> 2) & 3) * 16 + (lane >> 4) * 4 + (lane & 3); }
 __device__ __forceinline__ float4 ld4(const float* p) { return *reinterpret_cast<const float4*>(p); }
 
 // Convolution + SiLU of one channel over `len` (a multiple of 16) consecutive tokens from token t0 on, of which the
@@ -96,11 +115,12 @@ struct DeltaChunkArgs {
   const float* conv_w;   // [C, taps]
   const float* a_log;    // [H]
   const float* dt_bias;  // [H * D]
-  float* QK;             // [BC, H, 64, 64]  (BC = B * chunks)
-  float* W;              // [BC, H, 64, DP]
-  float* U;              // [BC, H, 64, EP]  U0
-  float* Q;              // [BC, H, 64, DP]  q e^G
-  float* K;              // [BC, H, DP, 64]  k e^{G_C - G}, transposed
+  // per chunk and head (BC = B * chunks), in fragments of 16 x 16
+  float* QK;             // [BC, H, 64 x 64]  left operands
+  float* W;              // [BC, H, 64 x DP]  left operands
+  float* Q;              // [BC, H, 64 x DP]  q e^G, left operands
+  float* K;              // [BC, H, DP x 64]  k e^{G_C - G} transposed, left operands
+  float* U;              // [BC, H, 64 x EP]  U0, accumulators
   float* gc;             // [BC, H, DP]      e^{G_C}
   int64_t ld, ld_raw, ld_beta;
   int S, NC, H, G, D, E, DP, EP, taps, C;
@@ -176,29 +196,34 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
     for (int d = lane; d < DP; d += 64) q_s[i * PT + d] *= rq, k_s[i * PT + d] *= rk;
   }
   __syncthreads();
-  // ---- the scaled copies of q and k: a thread takes a channel of a block
-  for (int x = tid; x < NB * DP; x += 256) {
-    const int d = x % DP, I = x / DP;
-    double base = 0.0, rest = tot[I * DP + d];
-    for (int k = 0; k < I; ++k) base += tot[k * DP + d];
-    for (int k = I + 1; k < NB; ++k) rest += tot[k * DP + d];
-    float kt[BL];
+  const int r16 = lane & 15, q4 = (lane >> 4) * 4;
+  // ---- the scaled copies of q and k, a fragment per wavefront and turn
+  for (int f = wave; f < NB * (DP / 16); f += 4) {
+    {
+      const int I = f / (DP / 16), d = (f % (DP / 16)) * 16 + q4, t = I * BL + r16;
+      float o[4];
 #pragma unroll
-    for (int i = 0; i < BL; ++i) {
-      const int t = I * BL + i;
-      const double g = g_s[t * PG + d];
-      p.Q[(ch * CH + t) * DP + d] = q_s[t * PT + d] * ex2((float)(base + g));
-      kt[i] = k_s[t * PT + d] * ex2((float)(rest - g));
+      for (int r = 0; r < 4; ++r) {
+        double g = g_s[t * PG + d + r];
+        for (int k = 0; k < I; ++k) g += tot[k * DP + d + r];
+        o[r] = q_s[t * PT + d + r] * ex2((float)g);
+      }
+      *reinterpret_cast<float4*>(p.Q + ch * CH * DP + f * FRAG + lane * 4) = make_float4(o[0], o[1], o[2], o[3]);
     }
+    {
+      const int d = (f / NB) * 16 + r16, J = f % NB, t = J * BL + q4;
+      double rest = tot[J * DP + d];
+      for (int k = J + 1; k < NB; ++k) rest += tot[k * DP + d];
+      float o[4];
 #pragma unroll
-    for (int i = 0; i < BL; i += 4)
-      *reinterpret_cast<float4*>(p.K + (ch * DP + d) * CH + I * BL + i) = make_float4(kt[i], kt[i + 1], kt[i + 2], kt[i + 3]);
+      for (int r = 0; r < 4; ++r) o[r] = k_s[(t + r) * PT + d] * ex2((float)(rest - g_s[(t + r) * PG + d]));
+      *reinterpret_cast<float4*>(p.K + ch * DP * CH + f * FRAG + lane * 4) = make_float4(o[0], o[1], o[2], o[3]);
+    }
   }
   for (int d = tid; d < DP; d += 256) p.gc[ch * DP + d] = ex2((float)(tot[d] + tot[DP + d] + tot[2 * DP + d] + tot[3 * DP + d]));
   // ---- A and QK: 10 block pairs I >= J, the four diagonal ones first (one per wavefront)
   f32x4 a_reg[NB];  // this wavefront's blocks of A: they go to LDS when q is not needed any more
   float* QK = p.QK + ch * CH * CH;
-  const int r16 = lane & 15, q4 = (lane >> 4) * 4;
 #pragma unroll
   for (int turn = 0; turn < NB; ++turn) {
     const int pair = wave + 4 * turn;
@@ -258,8 +283,9 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
     for (int r = 0; r < 4; ++r) {
       const int row = I * BL + q4 + r, col = J * BL + r16;
       a_reg[turn][r] = col < row ? b_s[row] * sa[r] : 0.0f;
-      QK[row * CH + col] = col <= row ? sq[r] : 0.0f;
+      sq[r] = col <= row ? sq[r] : 0.0f;
     }
+    *reinterpret_cast<f32x4*>(QK + (I * NB + J) * FRAG + frag_lane(lane) * 4) = quad_transpose(sq, lane);
   }
   // ---- (I + A)^-1 by blocks of 16: X_I = T_I (R_I - sum_{J<I} A_IJ X_J), T_I the inverse of a diagonal block.  A column
   // tile of R in the accumulator layout of mma16 is at the same time its right operand, so a wavefront solves a
@@ -336,17 +362,13 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
       y[I] = mma16(tm[I], make_float4(y[I][0], y[I][1], y[I][2], y[I][3]), f32x4{0, 0, 0, 0});
     }
   };
-  auto store = [&](const f32x4 (&y)[NB], float* dst, int ld) __attribute__((always_inline)) {
-#pragma unroll
-    for (int I = 0; I < NB; ++I)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) dst[(int64_t)(I * BL + q4 + r) * ld] = y[I][r];
-  };
 #pragma unroll
   for (int t = 0; t < WT; ++t) {
     if ((wave + 4 * t) * 16 >= DP) break;
     solve(x[t]);
-    store(x[t], p.W + ch * CH * DP + (wave + 4 * t) * 16 + r16, DP);
+#pragma unroll
+    for (int I = 0; I < NB; ++I)
+      *reinterpret_cast<f32x4*>(p.W + ch * CH * DP + (I * (DP / 16) + wave + 4 * t) * FRAG + frag_lane(lane) * 4) = quad_transpose(x[t][I], lane);
   }
   for (int e0 = 0; e0 < p.EP; e0 += 64) {
     if (e0) {
@@ -361,7 +383,9 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
 #pragma unroll
       for (int r = 0; r < 4; ++r) y[I][r] = v_s[(I * BL + q4 + r) * PA + wave * 16 + r16];
     solve(y);
-    store(y, p.U + ch * CH * p.EP + e0 + wave * 16 + r16, p.EP);
+#pragma unroll
+    for (int I = 0; I < NB; ++I)
+      *reinterpret_cast<f32x4*>(p.U + ch * CH * p.EP + (I * (p.EP / 16) + e0 / 16 + wave) * FRAG + lane * 4) = y[I];
   }
 }
 
@@ -412,27 +436,25 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
   // everything a chunk brings, in registers; the next chunk's is requested before this one's work begins
   struct Chunk {
     float4 w[KB], q[KB], k[NT][NB], a[NB], gc[NT];
-    float u0[4];
+    f32x4 u0;
   };
   Chunk c0, c1;
-  const int row = wave * BL + r16;          // this lane's token (A operand)
   auto load = [&](Chunk& r, int c) __attribute__((always_inline)) {
     const int64_t ch = ((int64_t)b * p.NC + (c < p.NC ? c : p.NC - 1)) * p.H + h;
 #pragma unroll
     for (int x = 0; x < KB; ++x) {
-      r.w[x] = ld4(p.W + (ch * CH + row) * DP + x * 16 + q4);
-      r.q[x] = ld4(p.Q + (ch * CH + row) * DP + x * 16 + q4);
+      r.w[x] = ld4(p.W + ch * CH * DP + (wave * KB + x) * FRAG + lane * 4);
+      r.q[x] = ld4(p.Q + ch * CH * DP + (wave * KB + x) * FRAG + lane * 4);
     }
+    r.u0 = *reinterpret_cast<const f32x4*>(p.U + ch * CH * p.EP + (wave * (p.EP / 16) + tile) * FRAG + lane * 4);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) r.u0[i] = p.U[(ch * CH + wave * BL + q4 + i) * p.EP + e];
-#pragma unroll
-    for (int x = 0; x < NB; ++x) r.a[x] = ld4(p.QK + (ch * CH + row) * CH + x * 16 + q4);
+    for (int x = 0; x < NB; ++x) r.a[x] = ld4(p.QK + ch * CH * CH + (wave * NB + x) * FRAG + lane * 4);
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
-      const int d0 = (KB >= 4 || wave < KB ? wave + 4 * t : 0) * 16;  // wavefronts without a tile read another's
-      r.gc[t] = ld4(p.gc + ch * DP + d0 + q4);
+      const int dt = KB >= 4 || wave < KB ? wave + 4 * t : 0;  // wavefronts without a tile read another's
+      r.gc[t] = ld4(p.gc + ch * DP + dt * 16 + q4);
 #pragma unroll
-      for (int x = 0; x < NB; ++x) r.k[t][x] = ld4(p.K + (ch * DP + d0 + r16) * CH + x * 16 + q4);
+      for (int x = 0; x < NB; ++x) r.k[t][x] = ld4(p.K + ch * DP * CH + (dt * NB + x) * FRAG + lane * 4);
     }
   };
   auto chunk = [&](const Chunk& r, Chunk& next, int c) __attribute__((always_inline)) {
@@ -447,9 +469,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     for (int x = 0; x < KB; ++x) sv[x] = ld4(&s_s[r16 * SP + x * 16 + q4]);
 #pragma unroll
     for (int x = 0; x < KB; ++x) mma16x2(r.w[x], sv[x], ws, r.q[x], sv[x], o);
-    f32x4 u;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) u[i] = r.u0[i] - ws[i];
+    const f32x4 u = r.u0 - ws;
     *reinterpret_cast<f32x4*>(&u_s[r16 * UP + wave * BL + q4]) = u;
     __syncthreads();
     float4 uv[NB];
@@ -489,9 +509,10 @@ struct SsdChunkArgs {
   const float* dt_bias;
   const float* a_log;
   const float* skip;
-  float* CB;     // [BC, G, 64, 64]
-  float* Cm;     // [BC, G, 64, NP]
-  float* Bt;     // [BC, G, NP, 64]
+  // per chunk and group, left operands in fragments of 16 x 16
+  float* CB;     // [BC, G, 64 x 64]
+  float* Cm;     // [BC, G, 64 x NP]
+  float* Bt;     // [BC, G, NP x 64]  B transposed
   float* state;  // [slots, H, P, N]
   float* out;    // [M, H, P]
   int64_t ld, ld_dt;
@@ -518,15 +539,18 @@ __global__ __launch_bounds__(256) void ssd_group_kernel(SsdChunkArgs p, const T*
              [&](int i, float v) { dst[i * PT] = v; });
   }
   __syncthreads();
-  for (int x = tid; x < CH * NP; x += 256) p.Cm[ch * CH * NP + x] = c_s[(x / NP) * PT + x % NP];
-  for (int x = tid; x < NP * CH; x += 256) p.Bt[ch * NP * CH + x] = b_s[(x % CH) * PT + x / CH];
   const int r16 = lane & 15, q4 = (lane >> 4) * 4;
+  for (int f = wave; f < NB * (NP / 16); f += 4) {
+    const int I = f / (NP / 16), d = (f % (NP / 16)) * 16 + q4;
+    *reinterpret_cast<float4*>(p.Cm + ch * CH * NP + f * FRAG + lane * 4) = ld4(&c_s[(I * BL + r16) * PT + d]);
+    const float* src = &b_s[((f % NB) * BL + q4) * PT + (f / NB) * 16 + r16];
+    *reinterpret_cast<float4*>(p.Bt + ch * NP * CH + f * FRAG + lane * 4) = make_float4(src[0], src[PT], src[2 * PT], src[3 * PT]);
+  }
   for (int J = 0; J < NB; ++J) {
     f32x4 s = {0, 0, 0, 0};
     if (J <= wave)
       for (int d = q4; d < NP; d += 16) s = mma16(ld4(&c_s[(wave * BL + r16) * PT + d]), ld4(&b_s[(J * BL + r16) * PT + d]), s);
-#pragma unroll
-    for (int r = 0; r < 4; ++r) p.CB[ch * CH * CH + (wave * BL + q4 + r) * CH + J * BL + r16] = s[r];
+    *reinterpret_cast<f32x4*>(p.CB + ch * CH * CH + (wave * NB + J) * FRAG + frag_lane(lane) * 4) = quad_transpose(s, lane);
   }
 }
 
@@ -583,14 +607,14 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     const int t = c * CH + lane;
     q.dtin = dt_raw[(tok0 + (t < p.S ? t : p.S - 1)) * p.ld_dt + h];
 #pragma unroll
-    for (int x = 0; x < KB; ++x) q.cm[x] = ld4(p.Cm + (ch * CH + row) * NP + x * 16 + q4);
+    for (int x = 0; x < KB; ++x) q.cm[x] = ld4(p.Cm + ch * CH * NP + (wave * KB + x) * FRAG + lane * 4);
 #pragma unroll
-    for (int x = 0; x < NB; ++x) q.cb[x] = ld4(p.CB + (ch * CH + row) * CH + x * 16 + q4);
+    for (int x = 0; x < NB; ++x) q.cb[x] = ld4(p.CB + ch * CH * CH + (wave * NB + x) * FRAG + lane * 4);
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
-      const int d0 = (KB >= 4 || wave < KB ? wave + 4 * t : 0) * 16;
+      const int dt = KB >= 4 || wave < KB ? wave + 4 * t : 0;
 #pragma unroll
-      for (int x = 0; x < NB; ++x) q.bt[t][x] = ld4(p.Bt + (ch * NP + d0 + r16) * CH + x * 16 + q4);
+      for (int x = 0; x < NB; ++x) q.bt[t][x] = ld4(p.Bt + ch * NP * CH + (dt * NB + x) * FRAG + lane * 4);
     }
   };
   load(c0, 0);

@@ -439,36 +439,38 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     f32x4 u0;
   };
   Chunk c0, c1;
-  auto load = [&](Chunk& r, int c) __attribute__((always_inline)) {
-    const int64_t ch = ((int64_t)b * p.NC + (c < p.NC ? c : p.NC - 1)) * p.H + h;
-#pragma unroll
-    for (int x = 0; x < KB; ++x) {
+  auto index = [&](int c) -> int64_t { return ((int64_t)b * p.NC + (c < p.NC ? c : p.NC - 1)) * p.H + h; };
+  auto load_wq = [&](Chunk& r, int64_t ch, int x) __attribute__((always_inline)) {
       r.w[x] = ld4(p.W + ch * CH * DP + (wave * KB + x) * FRAG + lane * 4);
       r.q[x] = ld4(p.Q + ch * CH * DP + (wave * KB + x) * FRAG + lane * 4);
-    }
+  };
+  const int dt[2] = {KB >= 4 || wave < KB ? wave : 0, wave + 4};  // wavefronts without a tile read another's
+  auto load_ak = [&](Chunk& r, int64_t ch, int x) __attribute__((always_inline)) {
+    r.a[x] = ld4(p.QK + ch * CH * CH + (wave * NB + x) * FRAG + lane * 4);
+#pragma unroll
+    for (int t = 0; t < NT; ++t) r.k[t][x] = ld4(p.K + ch * DP * CH + (dt[t] * NB + x) * FRAG + lane * 4);
+  };
+  auto load_rest = [&](Chunk& r, int64_t ch) __attribute__((always_inline)) {
+#pragma unroll
+    for (int t = 0; t < NT; ++t) r.gc[t] = ld4(p.gc + ch * DP + dt[t] * 16 + q4);
     r.u0 = *reinterpret_cast<const f32x4*>(p.U + ch * CH * p.EP + (wave * (p.EP / 16) + tile) * FRAG + lane * 4);
-#pragma unroll
-    for (int x = 0; x < NB; ++x) r.a[x] = ld4(p.QK + ch * CH * CH + (wave * NB + x) * FRAG + lane * 4);
-#pragma unroll
-    for (int t = 0; t < NT; ++t) {
-      const int dt = KB >= 4 || wave < KB ? wave + 4 * t : 0;  // wavefronts without a tile read another's
-      r.gc[t] = ld4(p.gc + ch * DP + dt * 16 + q4);
-#pragma unroll
-      for (int x = 0; x < NB; ++x) r.k[t][x] = ld4(p.K + ch * DP * CH + (dt * NB + x) * FRAG + lane * 4);
-    }
   };
   auto chunk = [&](const Chunk& r, Chunk& next, int c) __attribute__((always_inline)) {
 #pragma unroll
     for (int t = 0; t < NT; ++t)
       if (wave + 4 * t < KB) *reinterpret_cast<f32x4*>(&s_s[r16 * SP + (wave + 4 * t) * 16 + q4]) = s[t];
-    load(next, c + 1);
+    const int64_t nx = index(c + 1);
     __syncthreads();
     f32x4 ws = {0, 0, 0, 0}, o = {0, 0, 0, 0};
     float4 sv[KB];
 #pragma unroll
     for (int x = 0; x < KB; ++x) sv[x] = ld4(&s_s[r16 * SP + x * 16 + q4]);
 #pragma unroll
-    for (int x = 0; x < KB; ++x) mma16x2(r.w[x], sv[x], ws, r.q[x], sv[x], o);
+    for (int x = 0; x < KB; ++x) {  // loads between the products: in a row they would hold up the wavefronts
+      mma16x2(r.w[x], sv[x], ws, r.q[x], sv[x], o);
+      load_wq(next, nx, x);
+      __builtin_amdgcn_sched_barrier(0);
+    }
     const f32x4 u = r.u0 - ws;
     *reinterpret_cast<f32x4*>(&u_s[r16 * UP + wave * BL + q4]) = u;
     __syncthreads();
@@ -482,13 +484,20 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
       mma16x2(r.a[x], uv[x], o, r.k[0][x], uv[x], s[0]);
 #pragma unroll
       for (int t = 1; t < NT; ++t) s[t] = mma16(r.k[t][x], uv[x], s[t]);
+      load_ak(next, nx, x);
+      __builtin_amdgcn_sched_barrier(0);
     }
+    load_rest(next, nx);
     const int t0 = c * CH + wave * BL + q4;
 #pragma unroll
     for (int i = 0; i < 4; ++i)
       if (t0 + i < p.S && e < p.E) p.out[(((int64_t)b * p.S + t0 + i) * p.H + h) * p.E + e] = o[i];
   };
-  load(c0, 0);
+#pragma unroll
+  for (int x = 0; x < KB; ++x) load_wq(c0, index(0), x);
+#pragma unroll
+  for (int x = 0; x < NB; ++x) load_ak(c0, index(0), x);
+  load_rest(c0, index(0));
   for (int c = 0; c < p.NC; c += 2) {
     chunk(c0, c1, c);
     if (c + 1 < p.NC) chunk(c1, c0, c + 1);
@@ -596,9 +605,9 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     wj[j] = xok && back < p.taps ? p.conv_w[xc * p.taps + p.taps - 1 - back] : 0.0f;
   }
   const float xb = xok ? p.conv_b[xc] : 0.0f;
-  auto load = [&](Chunk& q, int c) __attribute__((always_inline)) {
+  auto index = [&](int c) -> int64_t { return ((int64_t)b * p.NC + (c < p.NC ? c : p.NC - 1)) * p.G + g; };
+  auto load_x = [&](Chunk& q, int c) __attribute__((always_inline)) {
     if (c >= p.NC) c = p.NC - 1;
-    const int64_t ch = ((int64_t)b * p.NC + c) * p.G + g;
 #pragma unroll
     for (int i = 0; i < 4 + MAX_TAPS - 1; ++i) {
       const int t = c * CH + xt + i - (MAX_TAPS - 1), tc = t < 0 ? 0 : t < p.S ? t : p.S - 1;
@@ -606,18 +615,21 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     }
     const int t = c * CH + lane;
     q.dtin = dt_raw[(tok0 + (t < p.S ? t : p.S - 1)) * p.ld_dt + h];
-#pragma unroll
-    for (int x = 0; x < KB; ++x) q.cm[x] = ld4(p.Cm + ch * CH * NP + (wave * KB + x) * FRAG + lane * 4);
-#pragma unroll
-    for (int x = 0; x < NB; ++x) q.cb[x] = ld4(p.CB + ch * CH * CH + (wave * NB + x) * FRAG + lane * 4);
-#pragma unroll
-    for (int t = 0; t < NT; ++t) {
-      const int dt = KB >= 4 || wave < KB ? wave + 4 * t : 0;
-#pragma unroll
-      for (int x = 0; x < NB; ++x) q.bt[t][x] = ld4(p.Bt + ch * NP * CH + (dt * NB + x) * FRAG + lane * 4);
-    }
   };
-  load(c0, 0);
+  auto load_c = [&](Chunk& q, int64_t ch, int x) __attribute__((always_inline)) {
+    q.cm[x] = ld4(p.Cm + ch * CH * NP + (wave * KB + x) * FRAG + lane * 4);
+  };
+  const int dt4[2] = {KB >= 4 || wave < KB ? wave : 0, wave + 4};  // wavefronts without a tile read another's
+  auto load_b = [&](Chunk& q, int64_t ch, int x) __attribute__((always_inline)) {
+    q.cb[x] = ld4(p.CB + ch * CH * CH + (wave * NB + x) * FRAG + lane * 4);
+#pragma unroll
+    for (int t = 0; t < NT; ++t) q.bt[t][x] = ld4(p.Bt + ch * NP * CH + (dt4[t] * NB + x) * FRAG + lane * 4);
+  };
+  load_x(c0, 0);
+#pragma unroll
+  for (int x = 0; x < KB; ++x) load_c(c0, index(0), x);
+#pragma unroll
+  for (int x = 0; x < NB; ++x) load_b(c0, index(0), x);
 #pragma unroll
   for (int i = 0; i < MAX_TAPS - 1; ++i) {  // inputs from before the portion
     const int t = xt + i - (MAX_TAPS - 1), a = pos + t;
@@ -656,14 +668,20 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
 #pragma unroll
     for (int t = 0; t < NT; ++t)
       if (wave + 4 * t < KB) *reinterpret_cast<f32x4*>(&s_s[r16 * SP + (wave + 4 * t) * 16 + q4]) = s[t];
-    load(next, c + 1);
+    const int64_t nx = index(c + 1);
     __syncthreads();
     f32x4 y = {0, 0, 0, 0}, y1 = {0, 0, 0, 0};
     float4 sv[KB];
 #pragma unroll
     for (int x = 0; x < KB; ++x) sv[x] = ld4(&s_s[r16 * SP + x * 16 + q4]);
 #pragma unroll
-    for (int x = 0; x < KB; x += 2) mma16x2(q.cm[x], sv[x], y, q.cm[x + 1], sv[x + 1], y1);
+    for (int x = 0; x < KB; x += 2) {  // loads between the products: in a row they would hold up the wavefronts
+      mma16x2(q.cm[x], sv[x], y, q.cm[x + 1], sv[x + 1], y1);
+      load_c(next, nx, x);
+      load_c(next, nx, x + 1);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    load_x(next, c + 1);
     y += y1;
     __syncthreads();  // the state may be overwritten
     float4 xx[NB];
@@ -694,6 +712,8 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
         if (x == 0) s[t] *= decay;
         s[t] = mma16(q.bt[t][x], xw, s[t]);
       }
+      load_b(next, nx, x);
+      __builtin_amdgcn_sched_barrier(0);
     }
     const int t0 = c * CH + wave * BL + q4;
     const float4 own = ld4(&x_s[buf][r16 * XP + wave * BL + q4]);

@@ -87,7 +87,7 @@ int aqs_ssd_step(const void *proj, int64_t ld, int64_t o_xbc, int64_t o_dt, int 
  * Sizes: aqs_chunked_ok(D or N, taps).  ws: scratch of at least the *_ws functions' number of floats. */
 int aqs_chunked_ok(int64_t rows, int64_t taps);
 int64_t aqs_delta_chunked_ws(int64_t B, int64_t S, int64_t H, int64_t D, int64_t E);
-int64_t aqs_ssd_chunked_ws(int64_t B, int64_t S, int64_t G, int64_t N);
+int64_t aqs_ssd_chunked_ws(int64_t B, int64_t S, int64_t H, int64_t G, int64_t N);
 /* aqs_delta_prep and aqs_delta_scan */
 int aqs_delta_chunked(const void *qkv, int64_t ld, const void *raw, int64_t ld_raw, const void *beta_raw, int64_t ld_beta,
                       int dtype, const float *w, const void *ring, const int32_t *slots, const int32_t *pos, const float *a_log,

@@ -114,7 +114,7 @@ SEQ_SYMBOLS = {
         _i64, _i64, _i64, _i64, _i64, _vp]),
     "aqs_chunked_ok": (_int, [_i64, _i64]),
     "aqs_delta_chunked_ws": (_i64, [_i64, _i64, _i64, _i64, _i64]),
-    "aqs_ssd_chunked_ws": (_i64, [_i64, _i64, _i64, _i64]),
+    "aqs_ssd_chunked_ws": (_i64, [_i64, _i64, _i64, _i64, _i64]),
     "aqs_delta_chunked": (_int, [_vp, _i64, _vp, _i64, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _vp,
         _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
     "aqs_ssd_chunked": (_int, [_vp, _i64, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _vp,

@@ -18,7 +18,8 @@
 //
 // State space (SSD), same idea with one scalar decay per head and token: y = e^{L_i} S^T C_i + sum_{j<=i} M_ij x_j + D x_i,
 // M_ij = <C_i, B_j> e^{L_i - L_j} dt_j;  S <- e^{L_C} S + sum_j e^{L_C - L_j} dt_j B_j x_j^T.  C B^T belongs to the
-// group and is computed once (`ssd_group`), the rest in one launch (`ssd_chunks`).
+// group and is computed once (`ssd_group`), M per head (`ssd_steps`), and the chunks run in order like the delta rule's
+// (`ssd_chunks`).
 #include "seq_common.h"
 
 namespace sq {
@@ -133,18 +134,19 @@ __device__ __forceinline__ void pair_block(int pair, int& I, int& J) {
   J = (int)(COLS >> (4 * pair)) & 15;
 }
 
-constexpr int PA = CH + 4, PI = BL + 4;  // row pitches of A and of the inverted blocks
+constexpr int PREP_WAVES = 8, PREP_THREADS = 64 * PREP_WAVES;
+constexpr int PA = CH + 4, PI = BL + 4, PV = 128 + 4;  // row pitches of A, of the inverted blocks and of v
 constexpr int max_of(int a, int b) { return a > b ? a : b; }
 // floats of LDS: decays (later A and the inverses), q (later v), k, beta
 template <int DP>
 struct PrepLds {
   static constexpr int DECAYS = max_of(2 * (CH * (DP + 2) + NB * DP), CH * PA + NB * BL * PI);
-  static constexpr int QUERIES = CH * max_of(DP + 4, PA);
+  static constexpr int QUERIES = CH * max_of(DP + 4, PV);
   static constexpr int TOTAL = DECAYS + QUERIES + CH * (DP + 4) + CH;
 };
 
 template <int DP, typename T>
-__global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p, const T* qkv, const T* raw, const T* braw, const T* ring0) {
+__global__ __launch_bounds__(PREP_THREADS) void delta_chunk_prep_kernel(DeltaChunkArgs p, const T* qkv, const T* raw, const T* braw, const T* ring0) {
   constexpr int PT = DP + 4, PG = DP + 2;
   extern __shared__ __align__(16) float lds[];
   // log2 decays summed within their block of 16, and the sums of whole blocks.  Only differences of them are used, and
@@ -162,43 +164,45 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
   const T* ring = ring0 + (int64_t)p.slots[b] * p.taps * p.C;
 
   if (tid < CH) b_s[tid] = tid < n ? sigmoid(to_f32(braw[(tok0 + t0 + tid) * p.ld_beta + h])) : 0.0f;
-  for (int x = tid; x < 2 * DP; x += 256) {
-    float* dst = (x < DP ? q_s : k_s) + x % DP;
-    const int d = x % DP;
-    conv_run(qkv, p.ld, tok0, t0, d < D ? n : 0, CH, pos, ring, p.taps, p.C, (x < DP ? 0 : p.G * D) + j * D + (d < D ? d : D - 1),
-             p.conv_w, 0.0f, [&](int i, float v) { dst[i * PT] = v; });
+  for (int x = tid; x < 4 * DP; x += PREP_THREADS) {  // q or k channel, and half of the chunk
+    const int y = x % (2 * DP), d = y % DP, i0 = x / (2 * DP) * (CH / 2), m = n - i0 < CH / 2 ? n - i0 : CH / 2;
+    float* dst = (y < DP ? q_s : k_s) + i0 * PT + d;
+    conv_run(qkv, p.ld, tok0, t0 + i0, d < D && m > 0 ? m : 0, CH / 2, pos, ring, p.taps, p.C,
+             (y < DP ? 0 : p.G * D) + j * D + (d < D ? d : D - 1), p.conv_w, 0.0f, [&](int i, float v) { dst[i * PT] = v; });
   }
   const float a = -expf(p.a_log[h]) * 1.44269504088896341f;
-  for (int x = tid; x < 2 * DP; x += 256) {  // channel, and half of the chunk
-    const int d = x % DP, dc = d < D ? d : D - 1, i1 = (x / DP) * (CH / 2);
+  for (int x = tid; x < NB * DP; x += PREP_THREADS) {  // channel and block
+    const int d = x % DP, dc = d < D ? d : D - 1, i0 = (x / DP) * BL;
     const float bias = p.dt_bias[h * D + dc];
     const T* src = raw + tok0 * p.ld_raw + h * D + dc;
-    for (int i0 = i1; i0 < i1 + CH / 2; i0 += BL) {
-      T v[BL];
+    T v[BL];
 #pragma unroll
-      for (int i = 0; i < BL; ++i) v[i] = src[(int64_t)(t0 + (i0 + i < n ? i0 + i : n - 1)) * p.ld_raw];
-      double sum = 0.0;
+    for (int i = 0; i < BL; ++i) v[i] = src[(int64_t)(t0 + (i0 + i < n ? i0 + i : n - 1)) * p.ld_raw];
+    double sum = 0.0;
 #pragma unroll
-      for (int i = 0; i < BL; ++i) {
-        const float l = a * softplus_abs(to_f32(v[i]) + bias);
-        sum += i0 + i < n && d < D ? (double)l : 0.0;
-        g_s[(i0 + i) * PG + d] = sum;
-      }
-      tot[(i0 / BL) * DP + d] = sum;
+    for (int i = 0; i < BL; ++i) {
+      const float l = a * softplus_abs(to_f32(v[i]) + bias);
+      sum += i0 + i < n && d < D ? (double)l : 0.0;
+      g_s[(i0 + i) * PG + d] = sum;
     }
+    tot[(i0 / BL) * DP + d] = sum;
   }
   __syncthreads();
-  // unit vectors: a wavefront takes 16 tokens
-  for (int i = wave * BL; i < wave * BL + BL; ++i) {
+  // unit vectors: 16 lanes take a token
+  for (int i = wave * 4 + (lane >> 4); i < CH; i += 4 * PREP_WAVES) {
     float sq = 0.0f, sk = 0.0f;
-    for (int d = lane; d < DP; d += 64) sq += q_s[i * PT + d] * q_s[i * PT + d], sk += k_s[i * PT + d] * k_s[i * PT + d];
-    const float rq = 1.0f / (sqrtf(wave_sum(sq) + 1e-6f) * sqrtf((float)D)), rk = 1.0f / sqrtf(wave_sum(sk) + 1e-6f);
-    for (int d = lane; d < DP; d += 64) q_s[i * PT + d] *= rq, k_s[i * PT + d] *= rk;
+    float* qr = &q_s[i * PT + (lane & 15)];
+    float* kr = &k_s[i * PT + (lane & 15)];
+#pragma unroll
+    for (int d = 0; d < DP; d += 16) sq += qr[d] * qr[d], sk += kr[d] * kr[d];
+    const float rq = 1.0f / (sqrtf(row16_sum(sq) + 1e-6f) * sqrtf((float)D)), rk = 1.0f / sqrtf(row16_sum(sk) + 1e-6f);
+#pragma unroll
+    for (int d = 0; d < DP; d += 16) qr[d] *= rq, kr[d] *= rk;
   }
   __syncthreads();
   const int r16 = lane & 15, q4 = (lane >> 4) * 4;
   // ---- the scaled copies of q and k, a fragment per wavefront and turn
-  for (int f = wave; f < NB * (DP / 16); f += 4) {
+  for (int f = wave; f < NB * (DP / 16); f += PREP_WAVES) {
     {
       const int I = f / (DP / 16), d = (f % (DP / 16)) * 16 + q4, t = I * BL + r16;
       float o[4];
@@ -220,13 +224,14 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
       *reinterpret_cast<float4*>(p.K + ch * DP * CH + f * FRAG + lane * 4) = make_float4(o[0], o[1], o[2], o[3]);
     }
   }
-  for (int d = tid; d < DP; d += 256) p.gc[ch * DP + d] = ex2((float)(tot[d] + tot[DP + d] + tot[2 * DP + d] + tot[3 * DP + d]));
+  for (int d = tid; d < DP; d += PREP_THREADS) p.gc[ch * DP + d] = ex2((float)(tot[d] + tot[DP + d] + tot[2 * DP + d] + tot[3 * DP + d]));
   // ---- A and QK: 10 block pairs I >= J, the four diagonal ones first (one per wavefront)
-  f32x4 a_reg[NB];  // this wavefront's blocks of A: they go to LDS when q is not needed any more
+  constexpr int TURNS = NB * NB / PREP_WAVES;
+  f32x4 a_reg[TURNS];  // this wavefront's blocks of A: they go to LDS when q is not needed any more
   float* QK = p.QK + ch * CH * CH;
 #pragma unroll
-  for (int turn = 0; turn < NB; ++turn) {
-    const int pair = wave + 4 * turn;
+  for (int turn = 0; turn < TURNS; ++turn) {
+    const int pair = wave + PREP_WAVES * turn;
     // pairs 0..3: diagonal; 4..9: below it; 10..15: above, zero
     int I, J;
     pair_block(pair, I, J);
@@ -290,11 +295,11 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
   // ---- (I + A)^-1 by blocks of 16: X_I = T_I (R_I - sum_{J<I} A_IJ X_J), T_I the inverse of a diagonal block.  A column
   // tile of R in the accumulator layout of mma16 is at the same time its right operand, so a wavefront solves a
   // tile of 16 columns in registers.
-  constexpr int WT = (DP / 16 + 3) / 4;  // tiles of W per wavefront
+  constexpr int WT = (DP / 16 + PREP_WAVES - 1) / PREP_WAVES;  // tiles of W per wavefront
   f32x4 x[WT][NB];
 #pragma unroll
   for (int t = 0; t < WT; ++t) {
-    const int d = ((wave + 4 * t) * 16 + r16) % DP;
+    const int d = ((wave + PREP_WAVES * t) * 16 + r16) % DP;
     double base = 0.0;
 #pragma unroll
     for (int I = 0; I < NB; ++I) {
@@ -310,9 +315,9 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
   float* A = reinterpret_cast<float*>(g_s);  // [64][PA]
   float* T_s = A + CH * PA;                  // [NB][16][PI]
 #pragma unroll
-  for (int turn = 0; turn < NB; ++turn) {
+  for (int turn = 0; turn < TURNS; ++turn) {
     int I, J;
-    pair_block(wave + 4 * turn, I, J);
+    pair_block(wave + PREP_WAVES * turn, I, J);
 #pragma unroll
     for (int r = 0; r < 4; ++r) A[(I * BL + q4 + r) * PA + J * BL + r16] = a_reg[turn][r];
   }
@@ -335,12 +340,12 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
       T_s[((lane >> 4) * BL + i) * PI + r16] = sum;
     }
   }
-  // beta v into q's space, 64 channels at a time: thread = (channel, block of 16 tokens)
-  float* v_s = q_s;  // [64][PA]
+  // beta v into q's space, 128 channels at a time: thread = (channel, block of 16 tokens)
+  float* v_s = q_s;  // [64][PV]
   auto convolve_v = [&](int e0) __attribute__((always_inline)) {
-    const int e = e0 + (tid & 63), ec = e < E ? e : E - 1, i0 = wave * BL;
+    const int e = e0 + (tid & 127), ec = e < E ? e : E - 1, i0 = (tid >> 7) * BL;
     conv_run(qkv, p.ld, tok0, t0 + i0, e < E ? (n - i0 < BL ? (n - i0 > 0 ? n - i0 : 0) : BL) : 0, BL, pos, ring, p.taps, p.C,
-             2 * p.G * D + h * E + ec, p.conv_w, 0.0f, [&](int i, float v) { v_s[(i0 + i) * PA + (tid & 63)] = b_s[i0 + i] * v; });
+             2 * p.G * D + h * E + ec, p.conv_w, 0.0f, [&](int i, float v) { v_s[(i0 + i) * PV + (tid & 127)] = b_s[i0 + i] * v; });
   };
   convolve_v(0);
   __syncthreads();
@@ -364,13 +369,13 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
   };
 #pragma unroll
   for (int t = 0; t < WT; ++t) {
-    if ((wave + 4 * t) * 16 >= DP) break;
+    if ((wave + PREP_WAVES * t) * 16 >= DP) break;
     solve(x[t]);
 #pragma unroll
     for (int I = 0; I < NB; ++I)
-      *reinterpret_cast<f32x4*>(p.W + ch * CH * DP + (I * (DP / 16) + wave + 4 * t) * FRAG + frag_lane(lane) * 4) = quad_transpose(x[t][I], lane);
+      *reinterpret_cast<f32x4*>(p.W + ch * CH * DP + (I * (DP / 16) + wave + PREP_WAVES * t) * FRAG + frag_lane(lane) * 4) = quad_transpose(x[t][I], lane);
   }
-  for (int e0 = 0; e0 < p.EP; e0 += 64) {
+  for (int e0 = 0; e0 < p.EP; e0 += 128) {
     if (e0) {
       __syncthreads();
       convolve_v(e0);
@@ -381,7 +386,7 @@ __global__ __launch_bounds__(256) void delta_chunk_prep_kernel(DeltaChunkArgs p,
 #pragma unroll
     for (int I = 0; I < NB; ++I)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) y[I][r] = v_s[(I * BL + q4 + r) * PA + wave * 16 + r16];
+      for (int r = 0; r < 4; ++r) y[I][r] = v_s[(I * BL + q4 + r) * PV + wave * 16 + r16];
     solve(y);
 #pragma unroll
     for (int I = 0; I < NB; ++I)
@@ -522,6 +527,11 @@ struct SsdChunkArgs {
   float* CB;     // [BC, G, 64 x 64]
   float* Cm;     // [BC, G, 64 x NP]
   float* Bt;     // [BC, G, NP x 64]  B transposed
+  // per chunk and head
+  float* Mx;     // [BC, H, 64 x 64]  <C_i, B_j> e^{L_i - L_j} dt_j, left operands (blocks above the diagonal are not written)
+  float* el;     // [BC, H, 64]  e^{L_i}
+  float* wj;     // [BC, H, 64]  dt_j e^{L_C - L_j}
+  float* dc;     // [BC, H]      e^{L_C}
   float* state;  // [slots, H, P, N]
   float* out;    // [M, H, P]
   int64_t ld, ld_dt;
@@ -563,15 +573,51 @@ __global__ __launch_bounds__(256) void ssd_group_kernel(SsdChunkArgs p, const T*
   }
 }
 
+template <typename T>
+__global__ __launch_bounds__(256) void ssd_steps_kernel(SsdChunkArgs p, const T* dt_raw) {
+  __shared__ double l_s[CH];  // log2 decays summed from the chunk's start; differences of them are exponentiated
+  __shared__ __align__(16) float dt_s[CH];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int c = blockIdx.x % p.NC, b = blockIdx.x / p.NC, h = blockIdx.y, g = h / (p.H / p.G);
+  const int64_t ch = (int64_t)blockIdx.x * p.H + h, cg = (int64_t)blockIdx.x * p.G + g;
+  if (wave == 0) {
+    const int t = c * CH + lane;
+    const float raw = to_f32(dt_raw[((int64_t)b * p.S + (t < p.S ? t : p.S - 1)) * p.ld_dt + h]);
+    const float dt = t < p.S ? softplus(raw + p.dt_bias[h]) : 0.0f;
+    double L = (double)(-expf(p.a_log[h]) * 1.44269504088896341f) * (double)dt;
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const double v = __shfl_up(L, o, 64);
+      if (lane >= o) L += v;
+    }
+    const double LC = __shfl(L, 63, 64);
+    l_s[lane] = L;
+    dt_s[lane] = dt;
+    p.el[ch * CH + lane] = ex2((float)L);
+    p.wj[ch * CH + lane] = dt * ex2((float)(LC - L));
+    if (lane == 0) p.dc[ch] = ex2((float)LC);
+  }
+  __syncthreads();
+  const int row = wave * BL + (lane & 15), q4 = (lane >> 4) * 4;
+  const double Li = l_s[row];
+  for (int J = 0; J <= wave; ++J) {
+    const float4 cb = ld4(p.CB + cg * CH * CH + (wave * NB + J) * FRAG + lane * 4);
+    float m[4] = {cb.x, cb.y, cb.z, cb.w};
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int j = J * BL + q4 + r;
+      m[r] = j <= row ? m[r] * dt_s[j] * ex2((float)(Li - l_s[j])) : 0.0f;
+    }
+    *reinterpret_cast<float4*>(p.Mx + ch * CH * CH + (wave * NB + J) * FRAG + lane * 4) = make_float4(m[0], m[1], m[2], m[3]);
+  }
+}
+
 template <int NP, typename T>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) void ssd_chunks_kernel(SsdChunkArgs p, const T* xbc,
-                                                                                                    const T* dt_raw, const T* ring0) {
+                                                                                                    const T* ring0) {
   constexpr int KB = NP / 16, NT = (KB + 3) / 4, SP = NP + 4, XP = CH + 4;
   __shared__ __align__(16) float s_s[CT * SP];
   __shared__ __align__(16) float x_s[2][CT * XP];  // the chunk's x, column by column
-  __shared__ __align__(16) float w_s[2][CH];       // dt_j e^{L_C - L_j}
-  __shared__ __align__(16) float dt_s[2][CH];
-  __shared__ __align__(16) double l_s[2][CH];      // log2 decays summed from the chunk's start
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int r16 = lane & 15, q4 = (lane >> 4) * 4;
   const int tile = blockIdx.y, h = blockIdx.x, b = blockIdx.z, g = h / (p.H / p.G);
@@ -585,18 +631,18 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     const int d = (wave + 4 * t) * 16 + q4;
     s[t] = load_state4(col, d, N, e < P && pos > 0 && d < NP);
   }
-  const float skip = p.skip[h], neg_a = -expf(p.a_log[h]) * 1.44269504088896341f, dtb = p.dt_bias[h];
-  const int row = wave * BL + r16;
+  const float skip = p.skip[h];
   // x: thread = (column tid % 16, tokens 4 (tid / 16) .. + 4); its raw inputs are requested a chunk ahead
   const int xe = tid & 15, xt = (tid >> 4) * 4;
   const bool xok = tile * CT + xe < P;
   const int xc = h * P + (xok ? tile * CT + xe : P - 1);
   float wj[MAX_TAPS];
-  // what a chunk brings, in registers; the next chunk's is requested before this one's work begins.  x and dt as
+  // what a chunk brings, in registers; the next chunk's is requested before this one's work begins.  x as
   // loaded: a conversion here would wait for the load.
   struct Chunk {
-    float4 cm[KB], cb[NB], bt[NT][NB];
-    T xin[4 + MAX_TAPS - 1], dtin;
+    float4 cm[KB], m[NB], bt[NT][NB], w[NB], el;
+    T xin[4 + MAX_TAPS - 1];
+    float dc;
   };
   Chunk c0, c1;
 #pragma unroll
@@ -613,15 +659,18 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
       const int t = c * CH + xt + i - (MAX_TAPS - 1), tc = t < 0 ? 0 : t < p.S ? t : p.S - 1;
       q.xin[i] = xbc[(tok0 + tc) * p.ld + xc];
     }
-    const int t = c * CH + lane;
-    q.dtin = dt_raw[(tok0 + (t < p.S ? t : p.S - 1)) * p.ld_dt + h];
+    const int64_t chh = ((int64_t)b * p.NC + c) * p.H + h;
+    q.el = ld4(p.el + chh * CH + wave * BL + q4);
+    q.dc = p.dc[chh];
   };
   auto load_c = [&](Chunk& q, int64_t ch, int x) __attribute__((always_inline)) {
     q.cm[x] = ld4(p.Cm + ch * CH * NP + (wave * KB + x) * FRAG + lane * 4);
   };
   const int dt4[2] = {KB >= 4 || wave < KB ? wave : 0, wave + 4};  // wavefronts without a tile read another's
   auto load_b = [&](Chunk& q, int64_t ch, int x) __attribute__((always_inline)) {
-    q.cb[x] = ld4(p.CB + ch * CH * CH + (wave * NB + x) * FRAG + lane * 4);
+    const int64_t chh = ch / p.G * p.H + h;
+    q.m[x] = ld4(p.Mx + chh * CH * CH + (wave * NB + x) * FRAG + lane * 4);
+    q.w[x] = ld4(p.wj + chh * CH + x * 16 + q4);
 #pragma unroll
     for (int t = 0; t < NT; ++t) q.bt[t][x] = ld4(p.Bt + ch * NP * CH + (dt4[t] * NB + x) * FRAG + lane * 4);
   };
@@ -637,7 +686,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
   }
   auto chunk = [&](const Chunk& q, Chunk& next, int c) __attribute__((always_inline)) {
     const int buf = c & 1;
-    // ---- this chunk's x, steps and decays; the state as an operand
+    // ---- this chunk's x; the state as an operand
     float4 xv;
     {
       float y[4];
@@ -651,20 +700,6 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
       xv = make_float4(y[0], y[1], y[2], y[3]);
     }
     *reinterpret_cast<float4*>(&x_s[buf][xe * XP + xt]) = xv;
-    const float dt = c * CH + lane < p.S ? softplus(to_f32(q.dtin) + dtb) : 0.0f;
-    double L = (double)neg_a * (double)dt;
-#pragma unroll
-    for (int o = 1; o < 64; o <<= 1) {
-      const double v = __shfl_up(L, o, 64);
-      if (lane >= o) L += v;
-    }
-    const double LC = __shfl(L, 63, 64);
-    if (wave == 0) {
-      dt_s[buf][lane] = dt;
-      l_s[buf][lane] = L;
-      w_s[buf][lane] = dt * ex2((float)(LC - L));
-    }
-    const float decay = ex2((float)LC);
 #pragma unroll
     for (int t = 0; t < NT; ++t)
       if (wave + 4 * t < KB) *reinterpret_cast<f32x4*>(&s_s[r16 * SP + (wave + 4 * t) * 16 + q4]) = s[t];
@@ -687,29 +722,19 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     float4 xx[NB];
 #pragma unroll
     for (int x = 0; x < NB; ++x) xx[x] = ld4(&x_s[buf][r16 * XP + x * 16 + q4]);
-    // rows of y: tokens wave * 16 + q4 + r
-#pragma unroll
-    for (int r = 0; r < 4; ++r) y[r] *= ex2((float)l_s[buf][wave * BL + q4 + r]);
-    const double Li = l_s[buf][row];
+    y[0] *= q.el.x, y[1] *= q.el.y, y[2] *= q.el.z, y[3] *= q.el.w;  // tokens wave * 16 + q4 + r
 #pragma unroll
     for (int x = 0; x < NB; ++x) {
       if (x > wave) break;  // keys ahead of every token of the wavefront
-      const float4 dj = ld4(&dt_s[buf][x * 16 + q4]);
-      float m[4] = {q.cb[x].x * dj.x, q.cb[x].y * dj.y, q.cb[x].z * dj.z, q.cb[x].w * dj.w};
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int jt = x * 16 + q4 + r;
-        m[r] = jt <= row ? m[r] * ex2((float)(Li - l_s[buf][jt])) : 0.0f;
-      }
-      y = mma16(make_float4(m[0], m[1], m[2], m[3]), xx[x], y);
+      y = mma16(q.m[x], xx[x], y);
     }
 #pragma unroll
     for (int x = 0; x < NB; ++x) {
-      const float4 wv = ld4(&w_s[buf][x * 16 + q4]);
+      const float4 wv = q.w[x];
       const float4 xw = make_float4(xx[x].x * wv.x, xx[x].y * wv.y, xx[x].z * wv.z, xx[x].w * wv.w);
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
-        if (x == 0) s[t] *= decay;
+        if (x == 0) s[t] *= q.dc;
         s[t] = mma16(q.bt[t][x], xw, s[t]);
       }
       load_b(next, nx, x);
@@ -767,9 +792,9 @@ extern "C" int64_t aqs_delta_chunked_ws(int64_t B, int64_t S, int64_t H, int64_t
   const int64_t DP = pad_rows(D), EP = pad16(E);
   return B * ((S + CH - 1) / CH) * H * (CH * CH + 3 * CH * DP + CH * EP + DP);
 }
-extern "C" int64_t aqs_ssd_chunked_ws(int64_t B, int64_t S, int64_t G, int64_t N) {
+extern "C" int64_t aqs_ssd_chunked_ws(int64_t B, int64_t S, int64_t H, int64_t G, int64_t N) {
   const int64_t NP = pad_rows(N);
-  return B * ((S + CH - 1) / CH) * G * (CH * CH + 2 * CH * NP);
+  return B * ((S + CH - 1) / CH) * (G * (CH * CH + 2 * CH * NP) + H * (CH * CH + 2 * CH + 1));
 }
 
 extern "C" int aqs_delta_chunked(const void* qkv, int64_t ld, const void* raw, int64_t ld_raw, const void* beta_raw, int64_t ld_beta,
@@ -800,7 +825,7 @@ extern "C" int aqs_delta_chunked(const void* qkv, int64_t ld, const void* raw, i
   SQ_DISPATCH(dtype, SQ_PADDED(D, {
                 constexpr size_t lds = PrepLds<RP>::TOTAL * sizeof(float);
                 if (const int rc = big_lds(&delta_chunk_prep_kernel<RP, T>, lds)) return rc;
-                (delta_chunk_prep_kernel<RP, T><<<dim3((unsigned)(B * NC), (unsigned)H), 256, lds, st>>>(
+                (delta_chunk_prep_kernel<RP, T><<<dim3((unsigned)(B * NC), (unsigned)H), PREP_THREADS, lds, st>>>(
                     a, (const T*)qkv, (const T*)raw, (const T*)beta_raw, (const T*)ring));
               }));
   if (const int rc = launched()) return rc;
@@ -821,13 +846,17 @@ extern "C" int aqs_ssd_chunked(const void* xbc, int64_t ld, const void* dt_raw, 
   if (B * S == 0) return AQ_OK;
   SQ_NEED(xbc && dt_raw && conv_w && conv_b && ring && slots && pos && dt_bias && a_log && skip && ws && state && out);
   SQ_CHECK(!bad_ptr16(ws), AQ_E_ALIGN);
-  SQ_CHECK(ws_floats >= aqs_ssd_chunked_ws(B, S, G, N), AQ_E_WORKSPACE);
+  SQ_CHECK(ws_floats >= aqs_ssd_chunked_ws(B, S, H, G, N), AQ_E_WORKSPACE);
   const int64_t NP = pad_rows(N), n = B * NC * G;
   SsdChunkArgs a{};
   a.slots = slots, a.pos = pos, a.conv_w = conv_w, a.conv_b = conv_b, a.dt_bias = dt_bias, a.a_log = a_log, a.skip = skip;
   a.CB = ws;
   a.Cm = a.CB + n * CH * CH;
   a.Bt = a.Cm + n * CH * NP;
+  a.Mx = a.Bt + n * CH * NP;
+  a.el = a.Mx + B * NC * H * CH * CH;
+  a.wj = a.el + B * NC * H * CH;
+  a.dc = a.wj + B * NC * H * CH;
   a.state = state, a.out = out, a.ld = ld, a.ld_dt = ld_dt;
   a.S = (int)S, a.NC = (int)NC, a.H = (int)H, a.G = (int)G, a.N = (int)N, a.P = (int)P, a.NP = (int)NP;
   a.taps = (int)taps, a.C = (int)(H * P + 2 * G * N);
@@ -839,6 +868,8 @@ extern "C" int aqs_ssd_chunked(const void* xbc, int64_t ld, const void* dt_raw, 
               }));
   if (const int rc = launched()) return rc;
   const dim3 grid((unsigned)H, (unsigned)((P + CT - 1) / CT), (unsigned)B);
-  SQ_DISPATCH(dtype, SQ_PADDED(N, (ssd_chunks_kernel<RP, T><<<grid, 256, 0, st>>>(a, (const T*)xbc, (const T*)dt_raw, (const T*)ring))));
+  SQ_DISPATCH(dtype, (ssd_steps_kernel<T><<<dim3((unsigned)(B * NC), (unsigned)H), 256, 0, st>>>(a, (const T*)dt_raw)));
+  if (const int rc = launched()) return rc;
+  SQ_DISPATCH(dtype, SQ_PADDED(N, (ssd_chunks_kernel<RP, T><<<grid, 256, 0, st>>>(a, (const T*)xbc, (const T*)ring))));
   return launched();
 }

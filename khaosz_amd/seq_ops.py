@@ -300,7 +300,7 @@ def ssd_chunked(proj: Tensor, o_xbc: int, o_dt: int, conv_w: Tensor, conv_b: Ten
         _vec(t, H, "per-head constants")
     if o_xbc + C > proj.shape[1] or o_dt + H > proj.shape[1]:
         raise ValueError("ssd_chunked: shapes do not fit")
-    n = int(_abi.load_seq().aqs_ssd_chunked_ws(b.B, b.S, G, N))
+    n = int(_abi.load_seq().aqs_ssd_chunked_ws(b.B, b.S, H, G, N))
     ws = torch.empty(n, dtype=torch.float32, device=dev)
     out = torch.empty((M, H * P), dtype=torch.float32, device=dev)
     _call("aqs_ssd_chunked", dev, _p(proj, o_xbc), proj.stride(0), _p(proj, o_dt), proj.stride(0), _DT[proj.dtype], _p(conv_w),

@@ -31,8 +31,6 @@ struct PrepArgs {
   float eps;
 };
 
-constexpr int HEAD_PAIRS = 4;  // element pairs per lane: head vectors of up to 512
-
 template <typename T>
 __device__ __forceinline__ int64_t page_row(const AttnDims& a, int b, int t) {
   const int64_t lp = t / a.page;
@@ -40,36 +38,37 @@ __device__ __forceinline__ int64_t page_row(const AttnDims& a, int b, int t) {
   return phys >= 0 && phys < a.n_pages ? phys * a.page + t % a.page : -1;
 }
 
-// RMS norm and rotation of one head vector by one wavefront: lane l holds the pairs l, l + 64, ...
-template <typename T>
+// RMS norm and rotation of one head vector by one wavefront: lane l holds the NP pairs l, l + 64, ... (zeros past D)
+template <int NP, typename T>
 __device__ __forceinline__ void norm_rotate(const T* src, const float* w, const float* cs, int D, int rot, float eps, int lane,
-                                            float (&o)[HEAD_PAIRS][2]) {
+                                            float (&o)[NP][2]) {
+  T raw[NP][2];
+#pragma unroll
+  for (int i = 0; i < NP; ++i) {
+    const int d = 2 * (i * 64 + lane);
+    raw[i][0] = src[d < D ? d : 0];
+    raw[i][1] = src[d + 1 < D ? d + 1 : 0];
+  }
   float ss = 0.0f;
 #pragma unroll
-  for (int i = 0; i < HEAD_PAIRS; ++i) {
+  for (int i = 0; i < NP; ++i) {
     const int d = 2 * (i * 64 + lane);
-    o[i][0] = d < D ? to_f32(src[d]) : 0.0f;
-    o[i][1] = d + 1 < D ? to_f32(src[d + 1]) : 0.0f;
+    o[i][0] = d < D ? to_f32(raw[i][0]) : 0.0f;
+    o[i][1] = d + 1 < D ? to_f32(raw[i][1]) : 0.0f;
     ss += o[i][0] * o[i][0] + o[i][1] * o[i][1];
   }
   const float r = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
 #pragma unroll
-  for (int i = 0; i < HEAD_PAIRS; ++i) {
-    const int d = 2 * (i * 64 + lane);
-    if (d >= D) continue;
-    const float u = o[i][0] * r * w[d], v = d + 1 < D ? o[i][1] * r * w[d + 1] : 0.0f;
-    if (d + 1 < rot) {
-      const float c = cs[d], s = cs[d + 1];
-      o[i][0] = u * c - v * s;
-      o[i][1] = v * c + u * s;
-    } else {
-      o[i][0] = u;
-      o[i][1] = v;
-    }
+  for (int i = 0; i < NP; ++i) {
+    const int d = 2 * (i * 64 + lane), dr = d + 1 < rot ? d : 0;
+    const float u = o[i][0] * r * w[d < D ? d : 0], v = o[i][1] * r * w[d + 1 < D ? d + 1 : 0];
+    const float c = rot ? cs[dr] : 1.0f, s = rot ? cs[dr + 1] : 0.0f;
+    o[i][0] = d + 1 < rot ? u * c - v * s : u;
+    o[i][1] = d + 1 < rot ? v * c + u * s : v;
   }
 }
 
-template <typename T>
+template <int NP, typename T>
 __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs p, const T* proj, T* q_out, T* kc, T* vc) {
   const AttnDims& a = p.a;
   const int items = a.H + 2 * a.G;
@@ -83,14 +82,21 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs p, const T* pro
     const int g = item - a.H - a.G;
     const int64_t pr = page_row<T>(a, b, t);
     if (pr < 0) return;
-    for (int e = lane; e < a.E; e += 64) vc[(pr * a.G + g) * a.E + e] = row[p.o_v + g * a.E + e];
+    const T* src = row + p.o_v + g * a.E;
+    T* dst = vc + (pr * a.G + g) * a.E;
+    if (((uintptr_t)src | (uintptr_t)dst | (a.E * sizeof(T))) % 8 == 0) {  // uniform
+      const uint2* s8 = reinterpret_cast<const uint2*>(src);
+      for (int e = lane; e < (int)(a.E * sizeof(T) / 8); e += 64) reinterpret_cast<uint2*>(dst)[e] = s8[e];
+    } else {
+      for (int e = lane; e < a.E; e += 64) dst[e] = src[e];
+    }
     return;
   }
   const bool is_q = item < a.H;
   const int h = is_q ? item : item - a.H;
-  float o[HEAD_PAIRS][2];
+  float o[NP][2];
   const int tc = t < p.max_pos ? t : (int)p.max_pos - 1;
-  norm_rotate<T>(row + (is_q ? p.o_q : p.o_k) + h * a.D, is_q ? p.q_norm : p.k_norm, p.cs + (int64_t)tc * p.rot, a.D, p.rot, p.eps,
+  norm_rotate<NP, T>(row + (is_q ? p.o_q : p.o_k) + h * a.D, is_q ? p.q_norm : p.k_norm, p.cs + (int64_t)tc * p.rot, a.D, p.rot, p.eps,
                  lane, o);
   T* dst;
   if (is_q) {
@@ -101,7 +107,7 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs p, const T* pro
     dst = kc + (pr * a.G + h) * a.D;
   }
 #pragma unroll
-  for (int i = 0; i < HEAD_PAIRS; ++i) {
+  for (int i = 0; i < NP; ++i) {
     const int d = 2 * (i * 64 + lane);
     if (d < a.D) dst[d] = from_f32<T>(o[i][0]);
     if (d + 1 < a.D) dst[d + 1] = from_f32<T>(o[i][1]);
@@ -399,11 +405,11 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(PrepArgs p, float scal
   }
   const T* row = proj + b * p.ld;
   const float* cs = p.cs + (int64_t)(pos < p.max_pos ? pos : p.max_pos - 1) * p.rot;
-  float o[HEAD_PAIRS][2];
+  float o[NC][2];
   if (wave < nh) {
-    norm_rotate<T>(row + p.o_q + (h0 + wave) * D, p.q_norm, cs, D, p.rot, p.eps, lane, o);
+    norm_rotate<NC, T>(row + p.o_q + (h0 + wave) * D, p.q_norm, cs, D, p.rot, p.eps, lane, o);
 #pragma unroll
-    for (int i = 0; i < DEC_MAX / 128; ++i) {
+    for (int i = 0; i < NC; ++i) {
       const int d = 2 * (i * 64 + lane);
       q_s[wave][d] = o[i][0] * scale_log2e;
       q_s[wave][d + 1] = o[i][1] * scale_log2e;
@@ -412,9 +418,9 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(PrepArgs p, float scal
   const bool has_new = pos < t0 + 64;
   if (has_new) {
     if (wave == 3) {
-      norm_rotate<T>(row + p.o_k + kvh * D, p.k_norm, cs, D, p.rot, p.eps, lane, o);
+      norm_rotate<NC, T>(row + p.o_k + kvh * D, p.k_norm, cs, D, p.rot, p.eps, lane, o);
 #pragma unroll
-      for (int i = 0; i < DEC_MAX / 128; ++i) {
+      for (int i = 0; i < NC; ++i) {
         const int d = 2 * (i * 64 + lane);
         kn_s[d] = from_f32<T>(o[i][0]);
         kn_s[d + 1] = from_f32<T>(o[i][1]);
@@ -517,21 +523,47 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(PrepArgs p, float scal
 
 template <typename T>
 __global__ __launch_bounds__(256) void attn_combine_kernel(AttnDims a, AttnOut o, const float* part, T* out, int NS) {
-  const int h = blockIdx.x % a.H, b = blockIdx.x / a.H;
+  __shared__ float w_s[256];
+  __shared__ float red[4];
+  const int tid = threadIdx.x, h = blockIdx.x % a.H, b = blockIdx.x / a.H;
   const int pos = a.pos[b], lo = pos - a.window + 1 > 0 ? pos - a.window + 1 : 0;
   int n = pos / 64 - lo / 64 + 1;
   n = n < NS ? n : NS;
   const int PW = a.E + 4;
   const float* src = part + ((int64_t)b * a.H + h) * NS * PW;
+  // all slices' maxima, then weights 256 slices at a time
   float mx = MASKED;
-  for (int i = 0; i < n; ++i) mx = fmaxf(mx, src[(int64_t)i * PW + a.E]);
-  float den = 0.0f;
-  for (int i = 0; i < n; ++i) den += src[(int64_t)i * PW + a.E + 1] * __builtin_amdgcn_exp2f(src[(int64_t)i * PW + a.E] - mx);
+  for (int i = tid; i < n; i += 256) mx = fmaxf(mx, src[(int64_t)i * PW + a.E]);
+  mx = wave_max(mx);
+  if ((tid & 63) == 0) red[tid >> 6] = mx;
+  __syncthreads();
+  mx = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+  float den = 0.0f, num[SIMPLE_MAX / 256] = {};
+  for (int i0 = 0; i0 < n; i0 += 256) {
+    const int m = n - i0 < 256 ? n - i0 : 256;
+    __syncthreads();
+    if (tid < m) {
+      const float* ml = src + (int64_t)(i0 + tid) * PW + a.E;
+      const float w = __builtin_amdgcn_exp2f(ml[0] - mx);
+      w_s[tid] = w;
+      den += w * ml[1];
+    }
+    __syncthreads();
+#pragma unroll
+    for (int k = 0; k < SIMPLE_MAX / 256; ++k) {
+      const int e = k * 256 + tid;
+      if (e >= a.E) break;
+      const float* col = src + (int64_t)i0 * PW + e;
+#pragma unroll 8
+      for (int i = 0; i < m; ++i) num[k] = fmaf(col[(int64_t)i * PW], w_s[i], num[k]);
+    }
+  }
+  den = block_sum<4>(den, red);
   const float f = head_factor<T>(o, b, h) / den;
-  for (int e = threadIdx.x; e < a.E; e += 256) {
-    float num = 0.0f;
-    for (int i = 0; i < n; ++i) num = fmaf(src[(int64_t)i * PW + e], __builtin_amdgcn_exp2f(src[(int64_t)i * PW + a.E] - mx), num);
-    out[b * o.ldo + h * a.E + e] = from_f32<T>(num * f);
+#pragma unroll
+  for (int k = 0; k < SIMPLE_MAX / 256; ++k) {
+    const int e = k * 256 + tid;
+    if (e < a.E) out[b * o.ldo + h * a.E + e] = from_f32<T>(num[k] * f);
   }
 }
 
@@ -563,7 +595,10 @@ extern "C" int aqs_attn_prep(const void* proj, int64_t ld, int64_t o_q, int64_t 
   SQ_NEED(proj && q_norm && k_norm && (cs || rot == 0) && q_out && kc && vc);
   PrepArgs p{a, q_norm, k_norm, cs, ld, o_q, o_k, o_v, max_pos, B * S, (int)rot, eps};
   const unsigned grid = (unsigned)((p.M * (H + 2 * G) + 3) / 4);
-  SQ_DISPATCH(dtype, (attn_prep_kernel<T><<<grid, 256, 0, (hipStream_t)stream>>>(p, (const T*)proj, (T*)q_out, (T*)kc, (T*)vc)));
+  hipStream_t st = (hipStream_t)stream;
+#define SQ_PREP(NP) (attn_prep_kernel<NP, T><<<grid, 256, 0, st>>>(p, (const T*)proj, (T*)q_out, (T*)kc, (T*)vc))
+  SQ_DISPATCH(dtype, if (D <= 128) SQ_PREP(1); else if (D <= 256) SQ_PREP(2); else SQ_PREP(4));
+#undef SQ_PREP
   return launched();
 }
 

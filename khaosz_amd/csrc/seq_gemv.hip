@@ -35,7 +35,7 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const
   extern __shared__ __align__(16) uint8_t xs_raw[];
   X* xs = reinterpret_cast<X*>(xs_raw);  // [M, K]
   __shared__ float red[4];
-  constexpr int U = 4;                          // 512-element steps of the row requested ahead
+  constexpr int U = R >= 4 ? 2 : 8 / R;         // 512-element steps of the rows in one block; the next block is in flight
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int K = p.K;
   // weight row i of this wavefront (OUT_GLU: the second half of them are the up rows of the first half)
@@ -49,15 +49,16 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const
     n = n < F ? n : F - 1;
     wr[i] = w + (int64_t)(OUT == OUT_GLU && i >= OR ? n + F : n) * K;
   }
-  Raw8<T> first[R][U];
+  Raw8<T> w0[R][U], w1[R][U];
+  auto load = [&](Raw8<T> (&dst)[R][U], int k0) __attribute__((always_inline)) {
 #pragma unroll
-  for (int u = 0; u < U; ++u)
+    for (int u = 0; u < U; ++u) {
+      const int k = k0 + (u * 64 + lane) * 8, kc = k < K ? k : 0;
 #pragma unroll
-    for (int i = 0; i < R; ++i) {
-      const int k = (u * 64 + lane) * 8;
-      if (k < K) first[i][u].load(wr[i] + k);
-      else first[i][u].zero();
+      for (int i = 0; i < R; ++i) dst[i][u].load(wr[i] + kc);
     }
+  };
+  load(w0, 0);
   __builtin_amdgcn_sched_barrier(0);
   // ---- rows into LDS
   for (int m = 0; m < p.M; ++m) {
@@ -125,15 +126,16 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const
         const float* yr = p.xf + m * p.ldx + g * part;
         const T* zr = z + m * p.ldz + g * part;
         float keep[KEEP], ss = 0.0f;
+        T zk[KEEP];
 #pragma unroll
         for (int i = 0; i < KEEP; ++i) {
-          const int k = i * 256 + tid;
-          keep[i] = k < part ? yr[k] : 0.0f;
+          const int k = i * 256 + tid, kc = k < part ? k : part - 1;
+          keep[i] = yr[kc];
+          zk[i] = zr[kc];
         }
 #pragma unroll
         for (int i = 0; i < KEEP; ++i) {
-          const int k = i * 256 + tid;
-          if (k < part) keep[i] *= silu(to_f32(zr[k]));
+          keep[i] = i * 256 + tid < part ? keep[i] * silu(to_f32(zk[i])) : 0.0f;
           ss += keep[i] * keep[i];
         }
         for (int k = KEEP * 256 + tid; k < part; k += 256) {
@@ -160,37 +162,35 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const
   for (int i = 0; i < R; ++i)
 #pragma unroll
     for (int m = 0; m < MR; ++m) acc[i][m] = 0.0f;
-  auto step = [&](int k, const Raw8<T>* ws) __attribute__((always_inline)) {
-    float f[R][8];
+  auto block = [&](const Raw8<T> (&ws)[R][U], int k0) __attribute__((always_inline)) {
 #pragma unroll
-    for (int i = 0; i < R; ++i) ws[i].get(f[i]);
+    for (int u = 0; u < U; ++u) {
+      const int k = k0 + (u * 64 + lane) * 8;
+      if (k >= K) continue;
+      float f[R][8];
 #pragma unroll
-    for (int m = 0; m < MR; ++m) {
-      if (m >= p.M) break;
-      float a[8];
-      Raw8<X> xr;
-      xr.load(xs + m * K + k);
-      xr.get(a);
+      for (int i = 0; i < R; ++i) ws[i][u].get(f[i]);
 #pragma unroll
-      for (int i = 0; i < R; ++i)
+      for (int m = 0; m < MR; ++m) {
+        if (m >= p.M) break;
+        float a[8];
+        Raw8<X> xr;
+        xr.load(xs + m * K + k);
+        xr.get(a);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) acc[i][m] = fmaf(f[i][e], a[e], acc[i][m]);
+        for (int i = 0; i < R; ++i)
+#pragma unroll
+          for (int e = 0; e < 8; ++e) acc[i][m] = fmaf(f[i][e], a[e], acc[i][m]);
+      }
     }
   };
-#pragma unroll
-  for (int u = 0; u < U; ++u) {
-    const int k = (u * 64 + lane) * 8;
-    Raw8<T> ws[R];
-#pragma unroll
-    for (int i = 0; i < R; ++i) ws[i] = first[i][u];
-    if (k < K) step(k, ws);
-  }
-#pragma unroll 2
-  for (int k = (U * 64 + lane) * 8; k < K; k += 512) {
-    Raw8<T> ws[R];
-#pragma unroll
-    for (int i = 0; i < R; ++i) ws[i].load(wr[i] + k);
-    step(k, ws);
+  constexpr int STEP = U * 512;
+  for (int k0 = 0; k0 < K; k0 += 2 * STEP) {
+    if (k0 + STEP < K) load(w1, k0 + STEP);
+    block(w0, k0);
+    if (k0 + STEP >= K) break;
+    if (k0 + 2 * STEP < K) load(w0, k0 + 2 * STEP);
+    block(w1, k0 + STEP);
   }
   // ---- sums over the lanes and the output
 #pragma unroll

@@ -41,6 +41,28 @@ __device__ __forceinline__ float conv_at(const ConvSrc& s, const T* in, int64_t 
   return acc;
 }
 
+// The same for the single token of a step at position pos (row: its inputs, channel c).  Up to four taps are requested at
+// once at addresses that are always valid: a load under a condition would be waited for where the condition ends.
+template <typename T>
+__device__ __forceinline__ float conv_step(const ConvSrc& s, const T* row, int pos, const T* ring, int c) {
+  if (s.taps > 4) return conv_at(s, row, 0, 0, pos, ring, c, pos);
+  T x[4];
+  float w[4];
+#pragma unroll
+  for (int back = 0; back < 4; ++back) {
+    const bool on = back < s.taps && back <= pos;
+    const int slot = on && back ? (pos - back) % s.taps : 0;
+    const T* src = back ? ring + (int64_t)slot * s.C + c : row + c;
+    x[back] = *src;
+    const float v = s.w[c * s.taps + (back < s.taps ? s.taps - 1 - back : 0)];
+    w[back] = on ? v : 0.0f;
+  }
+  float acc = s.bias ? s.bias[c] : 0.0f;
+#pragma unroll
+  for (int back = 3; back >= 0; --back) acc = w[back] != 0.0f ? fmaf(w[back], to_f32(x[back]), acc) : acc;
+  return acc;
+}
+
 // out[m, c] = silu(conv) in fp32
 template <typename T>
 __global__ __launch_bounds__(256) void conv_silu_kernel(const T* in, int64_t ld, ConvSrc s, const T* ring, const int* slots,
@@ -333,20 +355,28 @@ struct DeltaStepArgs {
 constexpr int STEP_WAVES = 8;
 constexpr int STEP_MAX = 256;  // rows and columns of a head's state
 
-// sum_k w[row, k] x[k], four lanes per row; every lane of the quad gets it
+// sum_k w[row, k] x[k] by four lanes (sub 0..3); every lane of the quad gets it.  n a multiple of 8.  Four pieces per
+// lane are requested at once.
 template <typename T>
-__device__ __forceinline__ float quad_dot(const T* w, const T* x, int n, int sub, bool ok) {
+__device__ __forceinline__ float quad_dot(const T* w, const T* x, int n, int sub) {
   float acc = 0.0f;
-  for (int c = sub * 8; c < n; c += 32) {
-    Raw8<T> a, b;
-    if (ok) a.load(w + c);
-    else a.zero();
-    b.load(x + c);
-    float fa[8], fb[8];
-    a.get(fa);
-    b.get(fb);
+  for (int c0 = 0; c0 < n; c0 += 128) {
+    Raw8<T> a[4], b[4];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) acc = fmaf(fa[i], fb[i], acc);
+    for (int i = 0; i < 4; ++i) {
+      const int c = c0 + i * 32 + sub * 8;
+      a[i].load(w + (c < n ? c : 0));
+      b[i].load(x + (c < n ? c : 0));
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      float fa[8], fb[8], part = 0.0f;
+      a[i].get(fa);
+      b[i].get(fb);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) part = fmaf(fa[e], fb[e], part);
+      acc += c0 + i * 32 + sub * 8 < n ? part : 0.0f;
+    }
   }
   SQ_DPP_ADD(acc, 0xB1);
   SQ_DPP_ADD(acc, 0x4E);
@@ -380,19 +410,19 @@ __global__ __launch_bounds__(STEP_WAVES * 64) void delta_step_kernel(DeltaStepAr
     const int which = i < D ? 0 : i < 2 * D ? 1 : 2;
     const int d = i - which * D;
     const int c = which == 2 ? 2 * p.G * D + h * E + d : (which * p.G + j) * D + d;
-    const float x = silu(conv_at(p.s, cin, p.ld, 0, pos, rg, c, pos));
+    const float x = silu(conv_step(p.s, cin, pos, rg, c));
     (which == 0 ? q_s : which == 1 ? k_s : v_s)[d] = x;
     if (which == 2 || h % per == 0) rg[(int64_t)(pos % p.s.taps) * p.s.C + c] = cin[c];
   }
   const float a = expf(p.a_log[h]);
   for (int d0 = 0; d0 < D; d0 += TH / 4) {
     const int d = d0 + tid / 4;
-    const float raw = quad_dot<T>(a2 + (int64_t)(h * D + (d < D ? d : 0)) * p.rank_a, row + p.o_a1, p.rank_a, tid & 3, d < D);
+    const float raw = quad_dot<T>(a2 + (int64_t)(h * D + (d < D ? d : 0)) * p.rank_a, row + p.o_a1, p.rank_a, tid & 3);
     if (d < D && (tid & 3) == 0) g_s[d] = expf(-a * softplus(raw + p.dt_bias[h * D + d]));
   }
   for (int e0 = 0; e0 < E; e0 += TH / 4) {
     const int e = e0 + tid / 4;
-    const float raw = quad_dot<T>(g2 + (int64_t)(h * E + (e < E ? e : 0)) * p.rank_g, row + p.o_g1, p.rank_g, tid & 3, e < E);
+    const float raw = quad_dot<T>(g2 + (int64_t)(h * E + (e < E ? e : 0)) * p.rank_g, row + p.o_g1, p.rank_g, tid & 3);
     if (e < E && (tid & 3) == 0) gate_s[e] = sigmoid(raw);
   }
   const float beta = sigmoid(to_f32(row[p.o_beta + h]));
@@ -475,7 +505,7 @@ __global__ __launch_bounds__(256) void ssd_step_kernel(SsdStepArgs p, const T* p
     const int which = i < N ? 0 : i < 2 * N ? 1 : 2;
     const int d = i - which * N;
     const int c = which == 2 ? h * P + d : inner + (which * p.G + j) * N + d;
-    const float x = silu(conv_at(p.s, cin, p.ld, 0, pos, rg, c, pos));
+    const float x = silu(conv_step(p.s, cin, pos, rg, c));
     (which == 0 ? b_s : which == 1 ? c_s : x_s)[d] = x;
     if (which == 2 || h % per == 0) rg[(int64_t)(pos % p.s.taps) * p.s.C + c] = cin[c];
   }

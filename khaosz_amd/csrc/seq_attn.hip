@@ -40,77 +40,95 @@ __device__ __forceinline__ int64_t page_row(const AttnDims& a, int b, int t) {
 
 // RMS norm and rotation of one head vector by one wavefront: lane l holds the NP pairs l, l + 64, ... (zeros past D)
 template <int NP, typename T>
+struct HeadVec {
+  T raw[NP][2];
+  __device__ __forceinline__ void load(const T* src, int D, int lane) {
+#pragma unroll
+    for (int i = 0; i < NP; ++i) {
+      const int d = 2 * (i * 64 + lane);
+      raw[i][0] = src[d < D ? d : 0];
+      raw[i][1] = src[d + 1 < D ? d + 1 : 0];
+    }
+  }
+  __device__ __forceinline__ void norm_rotate(const float* w, const float* cs, int D, int rot, float eps, int lane, float (&o)[NP][2]) const {
+    float ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < NP; ++i) {
+      const int d = 2 * (i * 64 + lane);
+      o[i][0] = d < D ? to_f32(raw[i][0]) : 0.0f;
+      o[i][1] = d + 1 < D ? to_f32(raw[i][1]) : 0.0f;
+      ss += o[i][0] * o[i][0] + o[i][1] * o[i][1];
+    }
+    const float r = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
+#pragma unroll
+    for (int i = 0; i < NP; ++i) {
+      const int d = 2 * (i * 64 + lane), dr = d + 1 < rot ? d : 0;
+      const float u = o[i][0] * r * w[d < D ? d : 0], v = o[i][1] * r * w[d + 1 < D ? d + 1 : 0];
+      const float c = rot ? cs[dr] : 1.0f, s = rot ? cs[dr + 1] : 0.0f;
+      o[i][0] = d + 1 < rot ? u * c - v * s : u;
+      o[i][1] = d + 1 < rot ? v * c + u * s : v;
+    }
+  }
+};
+template <int NP, typename T>
 __device__ __forceinline__ void norm_rotate(const T* src, const float* w, const float* cs, int D, int rot, float eps, int lane,
                                             float (&o)[NP][2]) {
-  T raw[NP][2];
-#pragma unroll
-  for (int i = 0; i < NP; ++i) {
-    const int d = 2 * (i * 64 + lane);
-    raw[i][0] = src[d < D ? d : 0];
-    raw[i][1] = src[d + 1 < D ? d + 1 : 0];
-  }
-  float ss = 0.0f;
-#pragma unroll
-  for (int i = 0; i < NP; ++i) {
-    const int d = 2 * (i * 64 + lane);
-    o[i][0] = d < D ? to_f32(raw[i][0]) : 0.0f;
-    o[i][1] = d + 1 < D ? to_f32(raw[i][1]) : 0.0f;
-    ss += o[i][0] * o[i][0] + o[i][1] * o[i][1];
-  }
-  const float r = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
-#pragma unroll
-  for (int i = 0; i < NP; ++i) {
-    const int d = 2 * (i * 64 + lane), dr = d + 1 < rot ? d : 0;
-    const float u = o[i][0] * r * w[d < D ? d : 0], v = o[i][1] * r * w[d + 1 < D ? d + 1 : 0];
-    const float c = rot ? cs[dr] : 1.0f, s = rot ? cs[dr + 1] : 0.0f;
-    o[i][0] = d + 1 < rot ? u * c - v * s : u;
-    o[i][1] = d + 1 < rot ? v * c + u * s : v;
-  }
+  HeadVec<NP, T> v;
+  v.load(src, D, lane);
+  v.norm_rotate(w, cs, D, rot, eps, lane, o);
 }
 
-template <int NP, typename T>
+constexpr int PREP_VECS = 4;  // head vectors of a token per wavefront, their loads together
+
+// VP: value elements per lane
+template <int NP, int VP, typename T>
 __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs p, const T* proj, T* q_out, T* kc, T* vc) {
   const AttnDims& a = p.a;
-  const int items = a.H + 2 * a.G;
+  const int items = a.H + 2 * a.G, groups = (items + PREP_VECS - 1) / PREP_VECS;
   const int64_t it = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (it >= p.M * items) return;
-  const int lane = threadIdx.x & 63, item = (int)(it % items);
-  const int64_t m = it / items;
+  if (it >= p.M * groups) return;
+  const int lane = threadIdx.x & 63, item0 = (int)(it % groups) * PREP_VECS;
+  const int64_t m = it / groups;
   const int b = (int)(m / a.S), t = a.pos[b] + (int)(m % a.S);
   const T* row = proj + m * p.ld;
-  if (item >= a.H + a.G) {
-    const int g = item - a.H - a.G;
-    const int64_t pr = page_row<T>(a, b, t);
-    if (pr < 0) return;
-    const T* src = row + p.o_v + g * a.E;
-    T* dst = vc + (pr * a.G + g) * a.E;
-    if (((uintptr_t)src | (uintptr_t)dst | (a.E * sizeof(T))) % 8 == 0) {  // uniform
-      const uint2* s8 = reinterpret_cast<const uint2*>(src);
-      for (int e = lane; e < (int)(a.E * sizeof(T) / 8); e += 64) reinterpret_cast<uint2*>(dst)[e] = s8[e];
-    } else {
-      for (int e = lane; e < a.E; e += 64) dst[e] = src[e];
-    }
-    return;
-  }
-  const bool is_q = item < a.H;
-  const int h = is_q ? item : item - a.H;
-  float o[NP][2];
-  const int tc = t < p.max_pos ? t : (int)p.max_pos - 1;
-  norm_rotate<NP, T>(row + (is_q ? p.o_q : p.o_k) + h * a.D, is_q ? p.q_norm : p.k_norm, p.cs + (int64_t)tc * p.rot, a.D, p.rot, p.eps,
-                 lane, o);
-  T* dst;
-  if (is_q) {
-    dst = q_out + (m * a.H + h) * a.D;
-  } else {
-    const int64_t pr = page_row<T>(a, b, t);
-    if (pr < 0) return;
-    dst = kc + (pr * a.G + h) * a.D;
-  }
+  HeadVec<NP, T> x[PREP_VECS];
+  T val[PREP_VECS][VP];
 #pragma unroll
-  for (int i = 0; i < NP; ++i) {
-    const int d = 2 * (i * 64 + lane);
-    if (d < a.D) dst[d] = from_f32<T>(o[i][0]);
-    if (d + 1 < a.D) dst[d + 1] = from_f32<T>(o[i][1]);
+  for (int k = 0; k < PREP_VECS; ++k) {
+    const int item = item0 + k < items ? item0 + k : items - 1;
+    if (item < a.H + a.G) {  // uniform
+      x[k].load(row + (item < a.H ? p.o_q + item * a.D : p.o_k + (item - a.H) * a.D), a.D, lane);
+    } else {
+      const T* src = row + p.o_v + (item - a.H - a.G) * a.E;
+#pragma unroll
+      for (int i = 0; i < VP; ++i) val[k][i] = src[i * 64 + lane < a.E ? i * 64 + lane : 0];
+    }
+  }
+  const int64_t pr = page_row<T>(a, b, t);
+  const float* cs = p.cs + (int64_t)(t < p.max_pos ? t : p.max_pos - 1) * p.rot;
+#pragma unroll
+  for (int k = 0; k < PREP_VECS; ++k) {
+    const int item = item0 + k;
+    if (item >= items) return;
+    if (item >= a.H + a.G) {
+      if (pr < 0) continue;
+      T* dst = vc + (pr * a.G + item - a.H - a.G) * a.E;
+#pragma unroll
+      for (int i = 0; i < VP; ++i)
+        if (i * 64 + lane < a.E) dst[i * 64 + lane] = val[k][i];
+      continue;
+    }
+    const bool is_q = item < a.H;
+    float o[NP][2];
+    x[k].norm_rotate(is_q ? p.q_norm : p.k_norm, cs, a.D, p.rot, p.eps, lane, o);
+    if (!is_q && pr < 0) continue;
+    T* dst = is_q ? q_out + (m * a.H + item) * a.D : kc + (pr * a.G + item - a.H) * a.D;
+#pragma unroll
+    for (int i = 0; i < NP; ++i) {
+      const int d = 2 * (i * 64 + lane);
+      if (d < a.D) dst[d] = from_f32<T>(o[i][0]);
+      if (d + 1 < a.D) dst[d + 1] = from_f32<T>(o[i][1]);
+    }
   }
 }
 
@@ -594,10 +612,11 @@ extern "C" int aqs_attn_prep(const void* proj, int64_t ld, int64_t o_q, int64_t 
   SQ_CHECK(o_q >= 0 && o_k >= 0 && o_v >= 0 && o_q + H * D <= ld && o_k + G * D <= ld && o_v + G * E <= ld, AQ_E_SHAPE);
   SQ_NEED(proj && q_norm && k_norm && (cs || rot == 0) && q_out && kc && vc);
   PrepArgs p{a, q_norm, k_norm, cs, ld, o_q, o_k, o_v, max_pos, B * S, (int)rot, eps};
-  const unsigned grid = (unsigned)((p.M * (H + 2 * G) + 3) / 4);
+  const int64_t groups = (H + 2 * G + PREP_VECS - 1) / PREP_VECS;
+  const unsigned grid = (unsigned)((p.M * groups + 3) / 4);
   hipStream_t st = (hipStream_t)stream;
-#define SQ_PREP(NP) (attn_prep_kernel<NP, T><<<grid, 256, 0, st>>>(p, (const T*)proj, (T*)q_out, (T*)kc, (T*)vc))
-  SQ_DISPATCH(dtype, if (D <= 128) SQ_PREP(1); else if (D <= 256) SQ_PREP(2); else SQ_PREP(4));
+#define SQ_PREP(NP, VP) (attn_prep_kernel<NP, VP, T><<<grid, 256, 0, st>>>(p, (const T*)proj, (T*)q_out, (T*)kc, (T*)vc))
+  SQ_DISPATCH(dtype, if (D <= 128 && E <= 128) SQ_PREP(1, 2); else if (D <= 256 && E <= 256) SQ_PREP(2, 4); else SQ_PREP(4, 8));
 #undef SQ_PREP
   return launched();
 }

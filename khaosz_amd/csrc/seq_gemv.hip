@@ -35,7 +35,7 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const
   extern __shared__ __align__(16) uint8_t xs_raw[];
   X* xs = reinterpret_cast<X*>(xs_raw);  // [M, K]
   __shared__ float red[4];
-  constexpr int U = R >= 4 ? 2 : 8 / R;         // 512-element steps of the rows in one block; the next block is in flight
+  constexpr int U = 8 / R;                      // 512-element steps of the rows in one block; the next block is in flight
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int K = p.K;
   // weight row i of this wavefront (OUT_GLU: the second half of them are the up rows of the first half)
@@ -121,37 +121,41 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const
     } else {
       const int part = K / p.groups;
       for (int g = 0; g < p.groups; ++g) {
-        // values of the first 16 rounds stay in registers
-        constexpr int KEEP = 16;
+        // 16 or 32 values per thread stay in registers between the two passes; a longer part is read again
         const float* yr = p.xf + m * p.ldx + g * part;
         const T* zr = z + m * p.ldz + g * part;
-        float keep[KEEP], ss = 0.0f;
-        T zk[KEEP];
-#pragma unroll
-        for (int i = 0; i < KEEP; ++i) {
-          const int k = i * 256 + tid, kc = k < part ? k : part - 1;
-          keep[i] = yr[kc];
-          zk[i] = zr[kc];
-        }
-#pragma unroll
-        for (int i = 0; i < KEEP; ++i) {
-          keep[i] = i * 256 + tid < part ? keep[i] * silu(to_f32(zk[i])) : 0.0f;
-          ss += keep[i] * keep[i];
-        }
-        for (int k = KEEP * 256 + tid; k < part; k += 256) {
-          const float v = yr[k] * silu(to_f32(zr[k]));
-          ss += v * v;
-        }
-        ss = block_sum<4>(ss, red);
-        const float r = 1.0f / sqrtf(ss / (float)part + p.eps);
         X* dst = row + g * part;
         const float* gr = p.gain + g * part;
+        auto run = [&](auto keep_tag) __attribute__((always_inline)) {
+          constexpr int KEEP = decltype(keep_tag)::value;
+          float keep[KEEP], ss = 0.0f;
+          T zk[KEEP];
 #pragma unroll
-        for (int i = 0; i < KEEP; ++i) {
-          const int k = i * 256 + tid;
-          if (k < part) dst[k] = from_f32<X>(keep[i] * r * gr[k]);
-        }
-        for (int k = KEEP * 256 + tid; k < part; k += 256) dst[k] = from_f32<X>(yr[k] * silu(to_f32(zr[k])) * r * gr[k]);
+          for (int i = 0; i < KEEP; ++i) {
+            const int k = i * 256 + tid, kc = k < part ? k : part - 1;
+            keep[i] = yr[kc];
+            zk[i] = zr[kc];
+          }
+#pragma unroll
+          for (int i = 0; i < KEEP; ++i) {
+            keep[i] = i * 256 + tid < part ? keep[i] * silu(to_f32(zk[i])) : 0.0f;
+            ss += keep[i] * keep[i];
+          }
+          for (int k = KEEP * 256 + tid; k < part; k += 256) {
+            const float v = yr[k] * silu(to_f32(zr[k]));
+            ss += v * v;
+          }
+          ss = block_sum<4>(ss, red);
+          const float r = 1.0f / sqrtf(ss / (float)part + p.eps);
+#pragma unroll
+          for (int i = 0; i < KEEP; ++i) {
+            const int k = i * 256 + tid;
+            if (k < part) dst[k] = from_f32<X>(keep[i] * r * gr[k]);
+          }
+          for (int k = KEEP * 256 + tid; k < part; k += 256) dst[k] = from_f32<X>(yr[k] * silu(to_f32(zr[k])) * r * gr[k]);
+        };
+        if (part <= 4096) run(std::integral_constant<int, 16>{});
+        else run(std::integral_constant<int, 32>{});
       }
     }
   }
@@ -228,15 +232,10 @@ int launch_gemv(const GemvArgs& p, const void* x, const void* z, const void* w, 
     return launched();
   };
   auto rows = [&](auto m_tag) -> int {
-    // enough wavefronts first (1024 SIMDs), then more rows per wavefront for fewer reads of the activations
-    if constexpr (OUT == OUT_GLU) {
-      if (F >= 8192) return go(std::integral_constant<int, 4>{}, m_tag);
-      return go(std::integral_constant<int, 2>{}, m_tag);
-    } else {
-      if (F >= 8192) return go(std::integral_constant<int, 4>{}, m_tag);
-      if (F >= 4096) return go(std::integral_constant<int, 2>{}, m_tag);
-      return go(std::integral_constant<int, 1>{}, m_tag);
-    }
+    // two rows per wavefront once that still leaves four wavefronts per SIMD (four rows were slower: 13.6 against 10.1 us
+    // for 8704 x 2048, 29.7 against 26.9 us for 16896 x 4096)
+    if (OUT == OUT_GLU || F >= 4096) return go(std::integral_constant<int, 2>{}, m_tag);
+    return go(std::integral_constant<int, OUT == OUT_GLU ? 2 : 1>{}, m_tag);
   };
   if (p.M == 1) return rows(std::integral_constant<int, 1>{});
   return rows(std::integral_constant<int, GEMV_MAX_M>{});

@@ -116,23 +116,42 @@ __global__ __launch_bounds__(ROW_THREADS) void gated_group_norm_kernel(const flo
 }
 
 // Every head of o [M, H, E] fp32 over its root mean square, times w [E], times sigmoid(gate), times scale -> out.
-// One wavefront per head vector.
-template <typename T>
+// A wavefront takes four head vectors, their loads together; NE elements of each per lane.
+template <int NE, typename T>
 __global__ __launch_bounds__(ROW_THREADS) void head_norm_gate_kernel(const float* o, const T* gate, int64_t ldg, const float* w,
                                                                      float eps, float scale, T* out, int64_t ldo, int64_t M,
                                                                      int H, int E) {
+  constexpr int VPW = 4;
   const int lane = threadIdx.x & 63;
-  const int64_t v = (int64_t)blockIdx.x * (ROW_THREADS / 64) + (threadIdx.x >> 6);
-  if (v >= M * H) return;
-  const int64_t m = v / H;
-  const int h = (int)(v - m * H);
-  const float* src = o + v * E;
-  float ss = 0.0f;
-  for (int e = lane; e < E; e += 64) ss += src[e] * src[e];
-  ss = wave_sum(ss);
-  const float r = 1.0f / sqrtf(ss / (float)E + eps);
-  for (int e = lane; e < E; e += 64)
-    out[m * ldo + h * E + e] = from_f32<T>(src[e] * r * w[e] * sigmoid(to_f32(gate[m * ldg + h * E + e])) * scale);
+  const int64_t v0 = ((int64_t)blockIdx.x * (ROW_THREADS / 64) + (threadIdx.x >> 6)) * VPW, nv = M * H;
+  float x[VPW][NE];
+  T gt[VPW][NE];
+#pragma unroll
+  for (int k = 0; k < VPW; ++k) {
+    const int64_t v = v0 + k < nv ? v0 + k : nv - 1, m = v / H;
+    const int h = (int)(v - m * H);
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int e = i * 64 + lane, ec = e < E ? e : E - 1;
+      x[k][i] = o[v * E + ec];
+      gt[k][i] = gate[m * ldg + h * E + ec];
+    }
+  }
+#pragma unroll
+  for (int k = 0; k < VPW; ++k) {
+    const int64_t v = v0 + k, m = v / H;
+    if (v >= nv) return;
+    const int h = (int)(v - m * H);
+    float ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < NE; ++i) ss += i * 64 + lane < E ? x[k][i] * x[k][i] : 0.0f;
+    const float r = scale / sqrtf(wave_sum(ss) / (float)E + eps);
+#pragma unroll
+    for (int i = 0; i < NE; ++i) {
+      const int e = i * 64 + lane;
+      if (e < E) out[m * ldo + h * E + e] = from_f32<T>(x[k][i] * r * w[e] * sigmoid(to_f32(gt[k][i])));
+    }
+  }
 }
 
 }  // namespace sq
@@ -201,8 +220,12 @@ extern "C" int aqs_head_norm_gate(const float* o, const void* gate, int64_t ldg,
   if (M == 0) return AQ_OK;
   SQ_NEED(o && gate && w && out);
   SQ_CHECK(M * H < (int64_t)1 << 26, AQ_E_RANGE);
-  const unsigned grid = (unsigned)((M * H + 3) / 4);
-  SQ_DISPATCH(dtype, (head_norm_gate_kernel<T><<<grid, ROW_THREADS, 0, (hipStream_t)stream>>>(
-                         o, (const T*)gate, ldg, w, eps, scale, (T*)out, ldo, M, (int)H, (int)E)));
+  SQ_CHECK(E <= 512, AQ_E_RANGE);
+  const unsigned grid = (unsigned)((M * H + 15) / 16);
+#define SQ_HEADS(NE)                                                                                                       \
+  (head_norm_gate_kernel<NE, T><<<grid, ROW_THREADS, 0, (hipStream_t)stream>>>(o, (const T*)gate, ldg, w, eps, scale,      \
+                                                                               (T*)out, ldo, M, (int)H, (int)E))
+  SQ_DISPATCH(dtype, if (E <= 64) SQ_HEADS(1); else if (E <= 128) SQ_HEADS(2); else if (E <= 256) SQ_HEADS(4); else SQ_HEADS(8));
+#undef SQ_HEADS
   return launched();
 }

@@ -23,6 +23,7 @@ struct GemvArgs {
   float* res;         // OUT_RESIDUAL [M, N]
   int64_t ldx, ldz, ldo;
   int M, N, K, groups;
+  int vec;            // IN_GATED_NORM: parts and z in whole 16-byte pieces
   float eps, mult, limit;
 };
 
@@ -121,41 +122,71 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemvArgs p, const T* x, const
     } else {
       const int part = K / p.groups;
       for (int g = 0; g < p.groups; ++g) {
-        // 16 or 32 values per thread stay in registers between the two passes; a longer part is read again
         const float* yr = p.xf + m * p.ldx + g * part;
         const T* zr = z + m * p.ldz + g * part;
-        X* dst = row + g * part;
         const float* gr = p.gain + g * part;
-        auto run = [&](auto keep_tag) __attribute__((always_inline)) {
-          constexpr int KEEP = decltype(keep_tag)::value;
-          float keep[KEEP], ss = 0.0f;
-          T zk[KEEP];
+        float ss = 0.0f;
+        if (p.vec) {
+          // 8 values at a time; the first 4 pieces of 2048 stay in registers between the two passes
+          constexpr int KEEP = 4;
+          float keep[KEEP][8];
+          Raw8<T> zk[KEEP];
 #pragma unroll
           for (int i = 0; i < KEEP; ++i) {
-            const int k = i * 256 + tid, kc = k < part ? k : part - 1;
-            keep[i] = yr[kc];
-            zk[i] = zr[kc];
+            const int k = i * 2048 + tid * 8, kc = k < part ? k : 0;
+            if (i * 2048 < part) {  // uniform
+              load_vec<8>(yr + kc, keep[i]);
+              zk[i].load(zr + kc);
+            }
           }
+          auto gate8 = [&](float* v, const Raw8<T>& zv) __attribute__((always_inline)) {
+            float f[8];
+            zv.get(f);
 #pragma unroll
-          for (int i = 0; i < KEEP; ++i) {
-            keep[i] = i * 256 + tid < part ? keep[i] * silu(to_f32(zk[i])) : 0.0f;
-            ss += keep[i] * keep[i];
+            for (int e = 0; e < 8; ++e) {
+              v[e] *= silu(f[e]);
+              ss += v[e] * v[e];
+            }
+          };
+#pragma unroll
+          for (int i = 0; i < KEEP; ++i)
+            if (i * 2048 + tid * 8 < part) gate8(keep[i], zk[i]);
+          for (int k = KEEP * 2048 + tid * 8; k < part; k += 2048) {
+            float v[8];
+            Raw8<T> zv;
+            load_vec<8>(yr + k, v);
+            zv.load(zr + k);
+            gate8(v, zv);
           }
-          for (int k = KEEP * 256 + tid; k < part; k += 256) {
+          ss = block_sum<4>(ss, red);
+          const float r = 1.0f / sqrtf(ss / (float)part + p.eps);
+          auto put = [&](int k, float* v) __attribute__((always_inline)) {
+            float gv[8];
+            load_vec<8>(gr + k, gv);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) v[e] *= r * gv[e];
+            put8(g * part + k, v);
+          };
+#pragma unroll
+          for (int i = 0; i < KEEP; ++i)
+            if (i * 2048 + tid * 8 < part) put(i * 2048 + tid * 8, keep[i]);
+          for (int k = KEEP * 2048 + tid * 8; k < part; k += 2048) {
+            float v[8];
+            Raw8<T> zv;
+            load_vec<8>(yr + k, v);
+            zv.load(zr + k);
+            gate8(v, zv);
+            put(k, v);
+          }
+        } else {
+          for (int k = tid; k < part; k += 256) {
             const float v = yr[k] * silu(to_f32(zr[k]));
             ss += v * v;
           }
           ss = block_sum<4>(ss, red);
           const float r = 1.0f / sqrtf(ss / (float)part + p.eps);
-#pragma unroll
-          for (int i = 0; i < KEEP; ++i) {
-            const int k = i * 256 + tid;
-            if (k < part) dst[k] = from_f32<X>(keep[i] * r * gr[k]);
-          }
-          for (int k = KEEP * 256 + tid; k < part; k += 256) dst[k] = from_f32<X>(yr[k] * silu(to_f32(zr[k])) * r * gr[k]);
-        };
-        if (part <= 4096) run(std::integral_constant<int, 16>{});
-        else run(std::integral_constant<int, 32>{});
+          for (int k = tid; k < part; k += 256) row[g * part + k] = from_f32<X>(yr[k] * silu(to_f32(zr[k])) * r * gr[k]);
+        }
       }
     }
   }
@@ -259,7 +290,7 @@ extern "C" int aqs_gemv(int in_kind, int out_kind, int dtype, const void* x, int
   if (M == 0) return AQ_OK;
   SQ_CHECK(aqs_gemv_ok(dtype, M, N, K), AQ_E_SHAPE);
   SQ_NEED(w && (out_kind == OUT_F32 || out_kind == OUT_RESIDUAL ? (const void*)res : (const void*)out));
-  SQ_CHECK(!bad_ptr16(w) && !bad_ptr16(x) && !bad_ptr16(xf) && !bad_ptr16(gain), AQ_E_ALIGN);
+  SQ_CHECK(!bad_ptr16(w) && (in_kind == IN_GATED_NORM || !bad_ptr16(x)) && !bad_ptr16(xf) && !bad_ptr16(gain), AQ_E_ALIGN);
   SQ_CHECK(out_kind != OUT_GLU || N % 2 == 0, AQ_E_SHAPE);
   SQ_CHECK(ldo >= (out_kind == OUT_GLU ? N / 2 : N), AQ_E_SHAPE);
   GemvArgs p{};
@@ -277,6 +308,7 @@ extern "C" int aqs_gemv(int in_kind, int out_kind, int dtype, const void* x, int
       SQ_NEED(x);
       SQ_CHECK(groups > 0 && K % groups == 0 && ldx >= K, AQ_E_SHAPE);
       z = x, p.ldz = ldx;
+      p.vec = K / groups % 8 == 0 && ldx % 8 == 0 && !bad_ptr16(x);
     }
   }
   hipStream_t st = (hipStream_t)stream;

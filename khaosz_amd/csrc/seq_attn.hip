@@ -33,9 +33,9 @@ struct PrepArgs {
 
 template <typename T>
 __device__ __forceinline__ int64_t page_row(const AttnDims& a, int b, int t) {
-  const int64_t lp = t / a.page;
+  const int lp = (int)((uint32_t)t / (uint32_t)a.page);
   const int64_t phys = lp < a.P ? a.table[(int64_t)b * a.P + lp] : -1;
-  return phys >= 0 && phys < a.n_pages ? phys * a.page + t % a.page : -1;
+  return phys >= 0 && phys < a.n_pages ? phys * a.page + (t - lp * a.page) : -1;
 }
 
 // RMS norm and rotation of one head vector by one wavefront: lane l holds the NP pairs l, l + 64, ... (zeros past D)
@@ -85,11 +85,11 @@ template <int NP, int VP, typename T>
 __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs p, const T* proj, T* q_out, T* kc, T* vc) {
   const AttnDims& a = p.a;
   const int items = a.H + 2 * a.G, groups = (items + PREP_VECS - 1) / PREP_VECS;
-  const int64_t it = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (it >= p.M * groups) return;
-  const int lane = threadIdx.x & 63, item0 = (int)(it % groups) * PREP_VECS;
-  const int64_t m = it / groups;
-  const int b = (int)(m / a.S), t = a.pos[b] + (int)(m % a.S);
+  const uint32_t it = blockIdx.x * 4 + (threadIdx.x >> 6), mu = it / (uint32_t)groups;  // fewer than 2^26 of them
+  if (mu >= p.M) return;
+  const int lane = threadIdx.x & 63, item0 = (int)(it - mu * groups) * PREP_VECS;
+  const int64_t m = mu;
+  const int b = (int)(mu / (uint32_t)a.S), t = a.pos[b] + (int)(mu - (uint32_t)b * a.S);
   const T* row = proj + m * p.ld;
   HeadVec<NP, T> x[PREP_VECS];
   T val[PREP_VECS][VP];
@@ -129,6 +129,79 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(PrepArgs p, const T* pro
       if (d < a.D) dst[d] = from_f32<T>(o[i][0]);
       if (d + 1 < a.D) dst[d + 1] = from_f32<T>(o[i][1]);
     }
+  }
+}
+
+// The same where every head vector is whole 16-byte pieces: 16 lanes take a vector, 8 elements each and piece (NC pieces of
+// 128), a wavefront four vectors at once.
+template <typename T>
+__device__ __forceinline__ void store8(T* dst, const float* v);
+template <>
+__device__ __forceinline__ void store8<bf16>(bf16* dst, const float* v) {
+  *reinterpret_cast<uint4*>(dst) = make_uint4(pack2(v[0], v[1]), pack2(v[2], v[3]), pack2(v[4], v[5]), pack2(v[6], v[7]));
+}
+template <>
+__device__ __forceinline__ void store8<float>(float* dst, const float* v) {
+  reinterpret_cast<float4*>(dst)[0] = make_float4(v[0], v[1], v[2], v[3]);
+  reinterpret_cast<float4*>(dst)[1] = make_float4(v[4], v[5], v[6], v[7]);
+}
+template <int NC, typename T>
+__global__ __launch_bounds__(256) void attn_prep_vec_kernel(PrepArgs p, const T* proj, T* q_out, T* kc, T* vc) {
+  const AttnDims& a = p.a;
+  const int items = a.H + 2 * a.G, groups = (items + 3) / 4;
+  const uint32_t it = blockIdx.x * 4 + (threadIdx.x >> 6), mu = it / (uint32_t)groups;  // fewer than 2^26 of them
+  if (mu >= p.M) return;
+  const int lane = threadIdx.x & 63, l16 = lane & 15, my = (int)(it - mu * groups) * 4 + (lane >> 4);
+  const bool live = my < items;
+  const int item = live ? my : items - 1;
+  const int64_t m = mu;
+  const int b = (int)(mu / (uint32_t)a.S), t = a.pos[b] + (int)(mu - (uint32_t)b * a.S);
+  const bool is_q = item < a.H, is_v = item >= a.H + a.G;
+  const int n = is_v ? a.E : a.D, g = is_q ? item : is_v ? item - a.H - a.G : item - a.H;
+  const T* src = proj + m * p.ld + (is_q ? p.o_q : is_v ? p.o_v : p.o_k) + g * n;
+  const float* w = is_q ? p.q_norm : p.k_norm;
+  const float* cs = p.cs + (int64_t)(t < p.max_pos ? t : p.max_pos - 1) * p.rot;
+  Raw8<T> raw[NC];
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int d = (c * 16 + l16) * 8;
+    raw[c].load(src + (d < n ? d : 0));
+  }
+  // cosines and sines of the lane's pairs, and the weights: requested at valid addresses whether they are used or not
+  float2 turn[NC][4];
+  float wv[NC][8];
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int d = (c * 16 + l16) * 8;
+    load_vec<8>(w + (d < a.D ? d : 0), wv[c]);
+#pragma unroll
+    for (int e = 0; e < 4; ++e)
+      turn[c][e] = p.rot ? *reinterpret_cast<const float2*>(cs + (d + 2 * e < p.rot ? d + 2 * e : 0)) : make_float2(1.0f, 0.0f);
+  }
+  const int64_t pr = page_row<T>(a, b, t);
+  float x[NC][8], ss = 0.0f;
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    raw[c].get(x[c]);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ss += (c * 16 + l16) * 8 < n ? x[c][e] * x[c][e] : 0.0f;
+  }
+  const float r = 1.0f / sqrtf(row16_sum(ss) / (float)a.D + p.eps);
+#pragma unroll
+  for (int c = 0; c < NC; ++c) {
+    const int d = (c * 16 + l16) * 8;
+    if (d >= n || !live) continue;
+    if (!is_v) {
+#pragma unroll
+      for (int e = 0; e < 8; e += 2) {
+        const float u = x[c][e] * r * wv[c][e], v = x[c][e + 1] * r * wv[c][e + 1];
+        const float2 cs2 = d + e < p.rot ? turn[c][e / 2] : make_float2(1.0f, 0.0f);
+        x[c][e] = u * cs2.x - v * cs2.y;
+        x[c][e + 1] = v * cs2.x + u * cs2.y;
+      }
+    }
+    if (!is_q && pr < 0) continue;
+    store8<T>((is_q ? q_out + (m * a.H + g) * a.D : is_v ? vc + (pr * a.G + g) * a.E : kc + (pr * a.G + g) * a.D) + d, x[c]);
   }
 }
 
@@ -403,8 +476,14 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(PrepArgs p, float scal
   if (t0 > pos) return;  // uniform
   const int D = a.D, E = a.E, h0 = kvh * per + hb * DEC_HB;
   const int nh = per - hb * DEC_HB < DEC_HB ? per - hb * DEC_HB : DEC_HB;
-  const int64_t pr0 = page_row<T>(a, b, t0);  // 64 positions lie in one page
-  // keys and values of this wavefront's 16 positions, requested at once
+  // the new token's projections first: they do not wait for the page table
+  const T* row = proj + b * p.ld;
+  HeadVec<NC, T> qraw, kraw;
+  qraw.load(row + p.o_q + (h0 + (wave < nh ? wave : 0)) * D, D, lane);
+  kraw.load(row + p.o_k + kvh * D, D, lane);
+  // keys and values of this wavefront's 16 positions, requested at once.  64 positions lie in one page, all of whose rows
+  // may be read; what lies past the sequence is masked or zeroed below.
+  const int64_t pr0 = page_row<T>(a, b, t0), prc = pr0 >= 0 ? pr0 : 0;
   const int kl = lane >> 4, ch = lane & 15, vl = lane / LV, vch = lane % LV;
   Raw8<T> kreg[4][NC], vreg[NP];
 #pragma unroll
@@ -412,31 +491,28 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(PrepArgs p, float scal
 #pragma unroll
     for (int c = 0; c < NC; ++c) {
       const int key = wave * 16 + i * 4 + kl, d = (c * 16 + ch) * 8;
-      if (pr0 >= 0 && t0 + key < pos && d < D) kreg[i][c].load(kc + ((pr0 + key) * a.G + kvh) * D + d);
-      else kreg[i][c].zero();
+      kreg[i][c].load(kc + ((prc + key) * a.G + kvh) * D + (d < D ? d : 0));
     }
 #pragma unroll
   for (int i = 0; i < NP; ++i) {
     const int key = wave * 16 + i * RPP + vl, e = vch * 8;
-    if (pr0 >= 0 && t0 + key < pos && e < E) vreg[i].load(vc + ((pr0 + key) * a.G + kvh) * E + e);
-    else vreg[i].zero();
+    vreg[i].load(vc + ((prc + key) * a.G + kvh) * E + (e < E ? e : 0));
   }
-  const T* row = proj + b * p.ld;
   const float* cs = p.cs + (int64_t)(pos < p.max_pos ? pos : p.max_pos - 1) * p.rot;
   float o[NC][2];
   if (wave < nh) {
-    norm_rotate<NC, T>(row + p.o_q + (h0 + wave) * D, p.q_norm, cs, D, p.rot, p.eps, lane, o);
+    qraw.norm_rotate(p.q_norm, cs, D, p.rot, p.eps, lane, o);
 #pragma unroll
     for (int i = 0; i < NC; ++i) {
       const int d = 2 * (i * 64 + lane);
-      q_s[wave][d] = o[i][0] * scale_log2e;
+      q_s[wave][d] = o[i][0] * scale_log2e;  // zero past D, where the key pieces repeat the row's start
       q_s[wave][d + 1] = o[i][1] * scale_log2e;
     }
   }
   const bool has_new = pos < t0 + 64;
   if (has_new) {
     if (wave == 3) {
-      norm_rotate<NC, T>(row + p.o_k + kvh * D, p.k_norm, cs, D, p.rot, p.eps, lane, o);
+      kraw.norm_rotate(p.k_norm, cs, D, p.rot, p.eps, lane, o);
 #pragma unroll
       for (int i = 0; i < NC; ++i) {
         const int d = 2 * (i * 64 + lane);
@@ -447,6 +523,9 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(PrepArgs p, float scal
     if (wave == 2)
       for (int e = lane; e < DEC_MAX; e += 64) vn_s[e] = e < E ? row[p.o_v + kvh * E + e] : from_f32<T>(0.0f);
   }
+#pragma unroll
+  for (int i = 0; i < NP; ++i)
+    if (pr0 < 0 || t0 + wave * 16 + i * RPP + vl >= pos) vreg[i].zero();
   __syncthreads();
   if (has_new) {
     const int key = pos - t0;  // the new token's row comes from LDS, and goes into its page
@@ -615,6 +694,13 @@ extern "C" int aqs_attn_prep(const void* proj, int64_t ld, int64_t o_q, int64_t 
   const int64_t groups = (H + 2 * G + PREP_VECS - 1) / PREP_VECS;
   const unsigned grid = (unsigned)((p.M * groups + 3) / 4);
   hipStream_t st = (hipStream_t)stream;
+  if (D % 8 == 0 && E % 8 == 0 && D <= 256 && E <= 256 && ld % 8 == 0 && o_q % 8 == 0 && o_k % 8 == 0 && o_v % 8 == 0 && !bad_ptr16(proj) &&
+      !bad_ptr16(q_out) && !bad_ptr16(kc) && !bad_ptr16(vc) && !bad_ptr16(q_norm) && !bad_ptr16(k_norm)) {
+    const unsigned vgrid = (unsigned)((p.M * ((H + 2 * G + 3) / 4) + 3) / 4);
+    SQ_DISPATCH(dtype, if (D <= 128 && E <= 128)(attn_prep_vec_kernel<1, T><<<vgrid, 256, 0, st>>>(p, (const T*)proj, (T*)q_out, (T*)kc, (T*)vc));
+                else (attn_prep_vec_kernel<2, T><<<vgrid, 256, 0, st>>>(p, (const T*)proj, (T*)q_out, (T*)kc, (T*)vc)));
+    return launched();
+  }
 #define SQ_PREP(NP, VP) (attn_prep_kernel<NP, VP, T><<<grid, 256, 0, st>>>(p, (const T*)proj, (T*)q_out, (T*)kc, (T*)vc))
   SQ_DISPATCH(dtype, if (D <= 128 && E <= 128) SQ_PREP(1, 2); else if (D <= 256 && E <= 256) SQ_PREP(2, 4); else SQ_PREP(4, 8));
 #undef SQ_PREP

@@ -83,9 +83,10 @@ __global__ __launch_bounds__(ROW_THREADS) void add_rmsnorm_kernel(float* x, cons
 // gu [M, 2F] = gate | up  ->  out [M, F]
 template <typename T, int V>
 __global__ __launch_bounds__(ROW_THREADS) void glu_kernel(const T* gu, int64_t ld, float limit, T* out, int64_t M, int64_t F) {
-  const int64_t per = F / V, n = M * per;
-  for (int64_t i = (int64_t)blockIdx.x * ROW_THREADS + threadIdx.x; i < n; i += (int64_t)gridDim.x * ROW_THREADS) {
-    const int64_t m = i / per, f = (i - m * per) * V;
+  // one row of blocks per F, rows of the matrix in the grid's second dimension: no division
+  const int64_t f = ((int64_t)blockIdx.x * ROW_THREADS + threadIdx.x) * V;
+  if (f >= F) return;
+  for (int64_t m = blockIdx.y; m < M; m += gridDim.y) {
     float g[V], u[V];
     Pack<T, V>::load(gu + m * ld + f, g);
     Pack<T, V>::load(gu + m * ld + F + f, u);
@@ -123,25 +124,28 @@ __global__ __launch_bounds__(ROW_THREADS) void head_norm_gate_kernel(const float
                                                                      int H, int E) {
   constexpr int VPW = 4;
   const int lane = threadIdx.x & 63;
-  const int64_t v0 = ((int64_t)blockIdx.x * (ROW_THREADS / 64) + (threadIdx.x >> 6)) * VPW, nv = M * H;
+  // fewer than 2^26 vectors: 32-bit divisions
+  const uint32_t v0 = (blockIdx.x * (ROW_THREADS / 64) + (threadIdx.x >> 6)) * VPW, nv = (uint32_t)(M * H);
   float x[VPW][NE];
   T gt[VPW][NE];
 #pragma unroll
   for (int k = 0; k < VPW; ++k) {
-    const int64_t v = v0 + k < nv ? v0 + k : nv - 1, m = v / H;
-    const int h = (int)(v - m * H);
+    const uint32_t v = v0 + k < nv ? v0 + k : nv - 1, mu = v / (uint32_t)H;
+    const int h = (int)(v - mu * H);
+    const int64_t m = mu;
 #pragma unroll
     for (int i = 0; i < NE; ++i) {
       const int e = i * 64 + lane, ec = e < E ? e : E - 1;
-      x[k][i] = o[v * E + ec];
+      x[k][i] = o[(int64_t)v * E + ec];
       gt[k][i] = gate[m * ldg + h * E + ec];
     }
   }
 #pragma unroll
   for (int k = 0; k < VPW; ++k) {
-    const int64_t v = v0 + k, m = v / H;
+    const uint32_t v = v0 + k, mu = v / (uint32_t)H;
     if (v >= nv) return;
-    const int h = (int)(v - m * H);
+    const int h = (int)(v - mu * H);
+    const int64_t m = mu;
     float ss = 0.0f;
 #pragma unroll
     for (int i = 0; i < NE; ++i) ss += i * 64 + lane < E ? x[k][i] * x[k][i] : 0.0f;
@@ -193,8 +197,9 @@ extern "C" int aqs_clamped_glu(const void* gu, int64_t ld, int dtype, float limi
   if (M == 0) return AQ_OK;
   SQ_NEED(gu && out);
   const bool v4 = F % 4 == 0 && ld % 4 == 0 && !bad_ptr16(gu) && !bad_ptr16(out);
-  const int64_t n = M * (v4 ? F / 4 : F);
-  const unsigned grid = (unsigned)((n + ROW_THREADS - 1) / ROW_THREADS < 16384 ? (n + ROW_THREADS - 1) / ROW_THREADS : 16384);
+  const int64_t nf = ((v4 ? F / 4 : F) + ROW_THREADS - 1) / ROW_THREADS;
+  SQ_CHECK(nf < (1 << 20), AQ_E_RANGE);
+  const dim3 grid((unsigned)nf, (unsigned)(M < 65535 ? M : 65535));
   SQ_DISPATCH(dtype, if (v4)(glu_kernel<T, 4><<<grid, ROW_THREADS, 0, (hipStream_t)stream>>>((const T*)gu, ld, limit, (T*)out, M, F));
               else (glu_kernel<T, 1><<<grid, ROW_THREADS, 0, (hipStream_t)stream>>>((const T*)gu, ld, limit, (T*)out, M, F)));
   return launched();

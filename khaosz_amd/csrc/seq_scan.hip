@@ -103,7 +103,7 @@ struct DeltaPrepArgs {
   int64_t M, ld, ld_raw, ld_beta;
   int S, H, G, D, E;
 };
-constexpr int PREP_MAX = 4;  // values per lane: head vectors of up to 256
+constexpr int PREP_MAX = 8;  // values per lane: head vectors of up to 512
 
 // one wavefront per head vector of a token: G queries, G keys, H values, H decays (with beta)
 template <typename T>

@@ -98,6 +98,9 @@ class Mamba2Mixer(nn.Module):
         return {"ring": torch.zeros((n_slots, self.taps, self.channels), dtype=dtype, device=device),
                 "S": torch.zeros((n_slots, self.H, self.P, self.N), dtype=torch.float32, device=device)}
 
+    def step_sizes_ok(self) -> bool:
+        return max(self.N, self.P) <= seq_ops.STEP_MAX
+
     def _columns(self, at: Dict[str, int]) -> Tuple[int, int, int]:
         z = at["in"]
         return z, z + self.out_dim, z + self.out_dim + self.channels
@@ -150,6 +153,9 @@ class ChannelDeltaMixer(nn.Module):
         # q | k | v are convolved together and have to touch; the low ranks read as whole pieces
         return [("qkv", q + k + v, False), ("b", self.H, False), ("a1", self.rank_a, False), ("g1", self.rank_g, False)]
 
+    def step_sizes_ok(self) -> bool:
+        return max(self.D, self.E) <= seq_ops.STEP_MAX
+
     def sub_parts(self) -> Dict[str, Tuple[str, int, int]]:
         """Checkpoint tensors that are slices of one part: name -> (part, first row, rows)."""
         q, k, v = self.split
@@ -196,6 +202,9 @@ class WindowAttention(nn.Module):
         self.base = float(c["rot"]["base"])
         self.out_dim = s.H * s.E
         self.q_norm, self.k_norm = _param(s.D, device=device), _param(s.D, device=device)
+
+    def step_sizes_ok(self) -> bool:
+        return True
 
     def in_parts(self) -> List[Tuple[str, int, bool]]:
         s = self.spec
@@ -279,7 +288,8 @@ class MixerBlock(nn.Module):
             seq_ops.gemv_residual(self._run(proj, b, st, "step"), self.w_out, mult, x)
 
     def step_ok(self, rows: int) -> bool:
-        return seq_ops.gemv_ok(rows, self.w_in.weight) and seq_ops.gemv_ok(rows, self.w_out)
+        return seq_ops.gemv_ok(rows, self.w_in.weight) and seq_ops.gemv_ok(rows, self.w_out) \
+            and all(m.step_sizes_ok() for m in self.mixers)
 
 
 class ClampedGLU(nn.Module):

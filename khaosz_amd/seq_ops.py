@@ -255,6 +255,7 @@ def delta_scan(q: Tensor, k: Tensor, v: Tensor, decay: Tensor, beta: Tensor, sta
     return out
 
 
+STEP_MAX = 256    # rows and columns of a head's state in the one-token kernels
 CHUNKED_MIN = 96  # new tokens per sequence from which the chunked kernels are the faster ones
 
 

@@ -47,6 +47,9 @@ CASES = {
     # heads wider than one tile, a convolution of one tap, a window longer than the tests' prompts, one repeated size
     "wide": config([layer("channel_delta", delta(2, 1, 136, 200, 4)), layer("parallel", parallel(attention(6, 1, 136, 144, 4096, 136, 1e4, 0.09), delta(2, 2, 72, 40, 1), 1.0, 1.0)),
                     layer("mamba2", mamba(2, 2, 144, 80, 1, 2), limit=7.0)], width=72, vocab=64, mult=1.0, eps=1e-6, rank=(24, 8)),
+    # state columns past what the one-token kernels hold
+    "tall": config([layer("channel_delta", delta(1, 1, 24, 264, 2)), layer("mamba2", mamba(1, 1, 16, 272, 4, 2), ff=24),
+                    layer("parallel", parallel(attention(2, 2, 264, 296, 33, 264, 1e3, 0.06), delta(2, 1, 16, 40, 3)))], width=40, vocab=48),
     # several windows inside one page and one chunk
     "short": config([layer("parallel", parallel(attention(8, 4, 64, 64, 1, 64), delta(1, 1, 64, 64, 8))),
                      layer("parallel", parallel(attention(5, 1, 32, 128, 64, 2, 90.0, 0.3), delta(4, 4, 8, 16, 2)), ff=None)], width=48, vocab=80),

@@ -93,42 +93,60 @@ SEQ_LIB_PATH = os.environ.get("ASTRAI_SEQ_LIB") or os.path.join(_HERE, "lib", "l
 _f32 = ctypes.c_float
 SEQ_SYMBOLS = {
     "aqs_embed": (_int, [_vp, _vp, _int, _vp, _i64, _i64, _i64, _vp]),
-    "aqs_add_rmsnorm": (_int, [_vp, _vp, _i64, _int, _f32, _vp, _f32, _vp, _i64, _i64, _vp]),
+    "aqs_add_rmsnorm": (_int, [_vp, _vp, _i64, _int, _vp, _vp, _i64, _vp, _f32, _vp, _f32, _f32, _vp, _i64, _i64,
+        _vp]),
     "aqs_clamped_glu": (_int, [_vp, _i64, _int, _f32, _vp, _i64, _i64, _vp]),
+    "aqs_silu_glu": (_int, [_vp, _i64, _int, _vp, _i64, _i64, _vp]),
+    "aqs_norm_gate": (_int, [_vp, _vp, _i64, _int, _vp, _f32, _vp, _i64, _i64, _i64, _vp]),
     "aqs_gated_group_norm": (_int, [_vp, _vp, _i64, _int, _vp, _f32, _vp, _i64, _i64, _i64, _i64, _vp]),
     "aqs_head_norm_gate": (_int, [_vp, _vp, _i64, _int, _vp, _f32, _f32, _vp, _i64, _i64, _i64, _i64, _vp]),
     "aqs_gemv_ok": (_int, [_int, _i64, _i64, _i64]),
-    "aqs_gemv": (_int, [_int, _int, _int, _vp, _i64, _vp, _vp, _f32, _i64, _vp, _vp, _f32, _f32, _vp, _vp, _i64,
-        _i64, _i64, _i64, _vp]),
+    "aqs_gemv": (_int, [_int, _int, _int, _vp, _i64, _vp, _vp, _vp, _vp, _vp, _f32, _f32, _i64, _vp, _vp, _f32, _f32,
+        _i64, _vp, _vp, _i64, _vp, _i64, _i64, _i64, _vp]),
     "aqs_conv_silu": (_int, [_vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _vp]),
     "aqs_conv_push": (_int, [_vp, _i64, _int, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _vp]),
-    "aqs_delta_prep": (_int, [_vp, _i64, _vp, _i64, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp,
-        _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
-    "aqs_delta_scan": (_int, [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64,
-        _vp]),
-    "aqs_delta_step": (_int, [_vp, _i64, _i64, _i64, _i64, _i64, _int, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _i64,
-        _vp, _vp, _vp, _f32, _f32, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
-    "aqs_ssd_scan": (_int, [_vp, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64,
-        _i64, _vp]),
-    "aqs_ssd_step": (_int, [_vp, _i64, _i64, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64,
+    "aqs_delta_prep": (_int, [_vp, _i64, _vp, _i64, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp,
+        _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_delta_scan": (_int, [_vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_delta_step": (_int, [_vp, _i64, _i64, _i64, _i64, _i64, _int, _vp, _vp, _vp, _vp, _vp, _i64, _vp, _i64, _vp,
+        _vp, _vp, _f32, _f32, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_ssd_scan": (_int, [_vp, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64,
+        _i64, _i64, _vp]),
+    "aqs_ssd_step": (_int, [_vp, _i64, _i64, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64,
         _i64, _i64, _i64, _i64, _i64, _vp]),
     "aqs_chunked_ok": (_int, [_i64, _i64]),
     "aqs_delta_chunked_ws": (_i64, [_i64, _i64, _i64, _i64, _i64]),
     "aqs_ssd_chunked_ws": (_i64, [_i64, _i64, _i64, _i64, _i64]),
     "aqs_delta_chunked": (_int, [_vp, _i64, _vp, _i64, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _vp,
         _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
-    "aqs_ssd_chunked": (_int, [_vp, _i64, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64, _vp,
-        _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
-    "aqs_attn_prep": (_int, [_vp, _i64, _i64, _i64, _i64, _int, _vp, _vp, _f32, _vp, _i64, _i64, _vp, _vp, _i64,
-        _i64, _i64, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_ssd_chunked": (_int, [_vp, _i64, _vp, _i64, _int, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _vp, _i64,
+        _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_attn_prep": (_int, [_vp, _i64, _i64, _i64, _i64, _int, _vp, _vp, _f32, _vp, _i64, _i64, _vp, _vp, _i64, _i64,
+        _i64, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
     "aqs_attn_window_ok": (_int, [_int, _i64, _i64, _i64]),
     "aqs_attn_window": (_int, [_vp, _vp, _vp, _int, _f32, _i64, _vp, _i64, _f32, _vp, _vp, _i64, _i64, _i64, _vp,
         _i64, _i64, _i64, _i64, _i64, _i64, _i64, _int, _vp]),
     "aqs_attn_decode_ok": (_int, [_i64, _i64, _i64]),
     "aqs_attn_decode_slices": (_i64, [_i64, _i64]),
-    "aqs_attn_decode": (_int, [_vp, _i64, _i64, _i64, _i64, _i64, _int, _vp, _vp, _f32, _vp, _i64, _i64, _f32,
-        _i64, _f32, _vp, _vp, _i64, _i64, _i64, _vp, _vp, _vp, _i64, _vp, _i64, _i64, _i64, _i64, _i64, _i64,
-        _vp]),
+    "aqs_attn_decode": (_int, [_vp, _i64, _i64, _i64, _i64, _i64, _int, _vp, _vp, _f32, _vp, _i64, _i64, _f32, _i64,
+        _f32, _vp, _vp, _i64, _i64, _i64, _vp, _vp, _vp, _i64, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_latent_prep": (_int, [_vp, _i64, _i64, _i64, _int, _vp, _vp, _f32, _vp, _i64, _vp, _vp, _i64, _i64, _i64,
+        _i64, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_latent_rotate": (_int, [_vp, _int, _vp, _i64, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_latent_window": (_int, [_vp, _vp, _i64, _vp, _i64, _i64, _int, _f32, _i64, _vp, _i64, _vp, _i64, _vp, _i64,
+        _i64, _i64, _i64, _i64, _i64, _i64, _int, _vp]),
+    "aqs_latent_decode_ok": (_int, [_i64, _i64, _i64, _i64, _i64, _i64]),
+    "aqs_latent_decode_slices": (_i64, [_i64, _i64]),
+    "aqs_latent_decode": (_int, [_vp, _i64, _i64, _i64, _vp, _vp, _vp, _int, _vp, _f32, _vp, _i64, _f32, _i64, _vp,
+        _vp, _i64, _i64, _i64, _vp, _vp, _vp, _i64, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_moe_route": (_int, [_vp, _i64, _int, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_moe_tile": (_i64, [_int, _i64, _i64, _i64, _i64]),
+    "aqs_moe_tiles": (_i64, [_i64, _i64, _i64]),
+    "aqs_moe_sort": (_int, [_vp, _i64, _i64, _i64, _vp, _vp, _vp, _i64, _vp]),
+    "aqs_moe_product": (_int, [_int, _vp, _i64, _int, _vp, _vp, _i64, _i64, _vp, _vp, _i64, _vp, _i64, _i64, _vp]),
+    "aqs_moe_step_ok": (_int, [_i64, _i64, _i64, _i64, _i64, _i64]),
+    "aqs_moe_step_up": (_int, [_vp, _vp, _int, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _vp]),
+    "aqs_moe_step_down": (_int, [_vp, _vp, _int, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),
 }
 
 _lib = None

@@ -87,7 +87,7 @@ class PagedKV:
     table tensor is first bound: a table that was changed in place (a page mapped as a sequence grew)
     must be bound again with ``refresh=True`` -- or be a new tensor, as the reference's
     ``make_table_tensor`` produces for every step.
-    ``v_head_dim``: the values' head size where it differs from the keys'.
+    ``v_head_dim``: the values' head size where it differs from the keys' (0: values are read from the keys' rows).
     ``seq_lens`` (int64 ``[B]`` on the device, optional): the positions each sequence may attend to
     in a single-token step whose sequences sit at different positions; the attention kernels apply it as
     the reference's position mask (transformer.py:40-46)."""
@@ -96,8 +96,8 @@ class PagedKV:
                  n_layers: int = 1, v_head_dim: Optional[int] = None):
         self.page_size = page_size
         self.k_layers = torch.zeros((n_layers, n_pages, page_size, n_kv_heads, head_dim), device=device, dtype=dtype)
-        self.v_layers = torch.zeros((n_layers, n_pages, page_size, n_kv_heads, v_head_dim or head_dim), device=device,
-                                    dtype=dtype)
+        v_dim = head_dim if v_head_dim is None else v_head_dim
+        self.v_layers = torch.zeros((n_layers, n_pages, page_size, n_kv_heads, v_dim), device=device, dtype=dtype)
         self.page_table: Optional[Tensor] = None
         self._attn_ws: Optional[Tensor] = None
         self._mapped = None      # host bool [B, P]

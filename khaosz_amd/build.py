@@ -34,7 +34,7 @@ SOURCES = ["abi.hip", "quant.hip", "gemm_mfma.hip", "gemv.hip", "attn_decode.hip
 LAB_SOURCES = [("gemm_mfma.hip", "gemm_mfma_lab.o", ["-DAQ_LAB"]), ("gemv.hip", "gemv_lab.o", ["-DAQ_LAB"]),
                ("lab.hip", "lab.o", [])]
 
-SEQ_SOURCES = ["seq_rows.hip", "seq_gemv.hip", "seq_scan.hip", "seq_chunk.hip", "seq_attn.hip"]
+SEQ_SOURCES = ["seq_rows.hip", "seq_gemv.hip", "seq_scan.hip", "seq_chunk.hip", "seq_attn.hip", "seq_latent.hip", "seq_moe.hip"]
 
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 FLAGS = [

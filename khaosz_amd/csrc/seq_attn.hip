@@ -7,15 +7,16 @@
 //   decode    one new token per sequence: prep's work, and the attention over slices of 64 positions in separate
 //             workgroups; `combine` merges the slices.
 //
-// Position i sees j with 0 <= i - j < window.  A head's output is multiplied by sigmoid(gate) and a constant before it
-// is stored.  Positions come from device memory, so that one captured launch serves every step.
+// Position i sees j with 0 <= i - j < window.  A head's output is multiplied by sigmoid(gate) -- one number for the head, or
+// one for each element -- and a constant before it is stored.  Prompts may also attend to packed rows in which keys and
+// values were formed from a shared latent (seq_latent.hip).  Positions come from device memory, so that one captured launch serves every step.
 #include "seq_common.h"
 
 namespace sq {
 
 struct AttnDims {
   const int* pos;        // [B]
-  const int64_t* table;  // [B, P]
+  const int64_t* table;  // [B, P]; null: packed rows, P * page of them per sequence (see page_row)
   int64_t P, n_pages;
   int S, H, G, D, E, page, window;
 };
@@ -31,8 +32,32 @@ struct PrepArgs {
   float eps;
 };
 
+// Where the elements of keys and values lie.  Row r, KV head g: the key's first D0 elements at k + r * ld_k + g * k_head, the
+// others (shared by all heads) at ks + r * ld_s; the value at v + r * ld_v + g * v_head.
+template <typename T>
+struct AttnKV {
+  const T* k;
+  const T* ks;
+  const T* v;
+  int64_t ld_k, ld_s, ld_v;
+  int k_head, v_head, D0;
+};
+template <typename T>
+AttnKV<T> paged_kv(const AttnDims& a, const void* kc, const void* vc) {
+  return {(const T*)kc, nullptr, (const T*)vc, (int64_t)a.G * a.D, 0, (int64_t)a.G * a.E, a.D, a.E, a.D};
+}
+
+// Packed rows hold the positions from the block of 64 on in which the first new token's window begins.
+__device__ __forceinline__ int packed_base(const AttnDims& a, int b) {
+  const int lo = a.pos[b] - a.window + 1;
+  return lo > 0 ? lo / 64 * 64 : 0;
+}
 template <typename T>
 __device__ __forceinline__ int64_t page_row(const AttnDims& a, int b, int t) {
+  if (!a.table) {
+    const int64_t r = t - packed_base(a, b), n = a.P * a.page;
+    return r >= 0 && r < n ? b * n + r : -1;
+  }
   const int lp = (int)((uint32_t)t / (uint32_t)a.page);
   const int64_t phys = lp < a.P ? a.table[(int64_t)b * a.P + lp] : -1;
   return phys >= 0 && phys < a.n_pages ? phys * a.page + (t - lp * a.page) : -1;
@@ -206,13 +231,14 @@ __global__ __launch_bounds__(256) void attn_prep_vec_kernel(PrepArgs p, const T*
 }
 
 struct AttnOut {
-  const void* gate;  // T, [M, ld_gate] one number per head, or null
+  const void* gate;  // T, [M, ld_gate] one number per head or (each) per element of the output, or null
   int64_t ld_gate, ldo;
   float scale;       // of the output
+  bool each;
 };
 template <typename T>
 __device__ __forceinline__ float head_factor(const AttnOut& o, int64_t m, int h) {
-  return o.gate ? o.scale * sigmoid(to_f32(reinterpret_cast<const T*>(o.gate)[m * o.ld_gate + h])) : o.scale;
+  return o.gate && !o.each ? o.scale * sigmoid(to_f32(reinterpret_cast<const T*>(o.gate)[m * o.ld_gate + h])) : o.scale;
 }
 
 constexpr float MASKED = -1.0e30f;
@@ -222,8 +248,8 @@ constexpr float LOG2E = 1.44269504088896341f;
 constexpr int SIMPLE_MAX = 512;
 
 template <typename T>
-__global__ __launch_bounds__(256) void attn_simple_kernel(AttnDims a, AttnOut o, float scale, const T* q, const T* kc, const T* vc,
-                                                          T* out, int64_t M) {
+__global__ __launch_bounds__(256) void attn_simple_kernel(AttnDims a, AttnKV<T> kv, AttnOut o, float scale, const T* q, T* out,
+                                                          int64_t M) {
   __shared__ float q_s[4][SIMPLE_MAX], p_s[4][64];
   __shared__ int row_s[4][64];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -243,8 +269,10 @@ __global__ __launch_bounds__(256) void attn_simple_kernel(AttnDims a, AttnOut o,
     const int64_t pr = t <= i ? page_row<T>(a, b, t) : -1;
     float s = t <= i ? 0.0f : -INFINITY;
     if (pr >= 0) {
-      const T* k = kc + (pr * a.G + g) * a.D;
-      for (int d = 0; d < a.D; ++d) s = fmaf(to_f32(k[d]), q_s[wave][d], s);
+      const T* k = kv.k + pr * kv.ld_k + (int64_t)g * kv.k_head;
+      for (int d = 0; d < kv.D0; ++d) s = fmaf(to_f32(k[d]), q_s[wave][d], s);
+      const T* ks = kv.ks + pr * kv.ld_s - kv.D0;
+      for (int d = kv.D0; d < a.D; ++d) s = fmaf(to_f32(ks[d]), q_s[wave][d], s);
     }
     const float mn = fmaxf(mx, wave_max(s)), al = expf(mx - mn), pv = expf(s - mn);
     l = l * al + wave_sum(pv);
@@ -259,7 +287,7 @@ __global__ __launch_bounds__(256) void attn_simple_kernel(AttnDims a, AttnOut o,
       const int r = row_s[wave][k];
       if (r < 0) continue;
       const float w = p_s[wave][k];
-      const T* vr = vc + ((int64_t)r * a.G + g) * a.E;
+      const T* vr = kv.v + (int64_t)r * kv.ld_v + (int64_t)g * kv.v_head;
 #pragma unroll
       for (int e = 0; e < SIMPLE_MAX / 64; ++e)
         if (e * 64 + lane < a.E) acc[e] = fmaf(w, to_f32(vr[e * 64 + lane]), acc[e]);
@@ -270,7 +298,10 @@ __global__ __launch_bounds__(256) void attn_simple_kernel(AttnDims a, AttnOut o,
   const float f = head_factor<T>(o, m, h) / l;
 #pragma unroll
   for (int e = 0; e < SIMPLE_MAX / 64; ++e)
-    if (e * 64 + lane < a.E) out[m * o.ldo + h * a.E + e * 64 + lane] = from_f32<T>(acc[e] * f);
+    if (e * 64 + lane < a.E) {
+      const float ge = o.each ? sigmoid(to_f32(((const T*)o.gate)[m * o.ld_gate + h * a.E + e * 64 + lane])) : 1.0f;
+      out[m * o.ldo + h * a.E + e * 64 + lane] = from_f32<T>(acc[e] * f * ge);
+    }
 }
 
 // ---------------------------------------------------------------------------------------------- prefill, matrix cores
@@ -284,7 +315,7 @@ constexpr int WQ = 128, WK = 64;
 
 template <int DP, int EP>
 __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DP + EP <= 256 ? 2 : 1))) void attn_window_kernel(
-    AttnDims a, AttnOut oo, float scale_log2e, const uint16_t* q, const uint16_t* kc, const uint16_t* vc, uint16_t* out, int B) {
+    AttnDims a, AttnKV<uint16_t> kv, AttnOut oo, float scale_log2e, const uint16_t* q, uint16_t* out, int B) {
   constexpr int KP = DP + 8, VP = WK + 4, DS = DP / 16, DT = EP / 32, KC = DP / 32, VC = EP / 32;
   extern __shared__ __align__(16) uint16_t lds[];
   uint16_t* ks = lds;            // [WK][KP]
@@ -311,19 +342,18 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DP + EP <= 
   }
   uint4 kr[KC], vr[VC];
   auto fetch = [&](int j) __attribute__((always_inline)) {
-    const int64_t lp = (int64_t)j * WK / a.page;
-    const int64_t phys = lp < a.P ? a.table[(int64_t)b * a.P + lp] : -1;
-    const bool ok = phys >= 0 && phys < a.n_pages;
-    const int64_t base = (ok ? phys : 0) * a.page + (int64_t)j * WK % a.page;
+    const int64_t row0 = page_row<uint16_t>(a, b, j * WK), base = row0 >= 0 ? row0 : 0;
+    const bool ok = row0 >= 0;
 #pragma unroll
     for (int c = 0; c < KC; ++c) {
       const int idx = c * 256 + tid, key = idx / (DP / 8), ch = idx % (DP / 8);
-      kr[c] = ok && ch * 8 < D ? *reinterpret_cast<const uint4*>(kc + ((base + key) * a.G + kvh) * D + ch * 8) : make_uint4(0, 0, 0, 0);
+      const uint16_t* src = ch * 8 < kv.D0 ? kv.k + (base + key) * kv.ld_k + kvh * kv.k_head : kv.ks + (base + key) * kv.ld_s - kv.D0;
+      kr[c] = ok && ch * 8 < D ? *reinterpret_cast<const uint4*>(src + ch * 8) : make_uint4(0, 0, 0, 0);
     }
 #pragma unroll
     for (int c = 0; c < VC; ++c) {
       const int ch = wave + 4 * c;
-      vr[c] = ok && ch * 8 < E ? *reinterpret_cast<const uint4*>(vc + ((base + lane) * a.G + kvh) * E + ch * 8) : make_uint4(0, 0, 0, 0);
+      vr[c] = ok && ch * 8 < E ? *reinterpret_cast<const uint4*>(kv.v + (base + lane) * kv.ld_v + kvh * kv.v_head + ch * 8) : make_uint4(0, 0, 0, 0);
     }
   };
   auto stage = [&](int j) __attribute__((always_inline)) {
@@ -445,9 +475,17 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DP + EP <= 
   for (int dt = 0; dt < DT; ++dt)
 #pragma unroll
     for (int r = 0; r < 4; ++r)
-      if (dt * 32 + 8 * r + 4 * g2 < E)
-        *reinterpret_cast<uint2*>(dst + dt * 32 + 8 * r) = make_uint2(pack2(o[dt][4 * r] * f, o[dt][4 * r + 1] * f),
-                                                                     pack2(o[dt][4 * r + 2] * f, o[dt][4 * r + 3] * f));
+      if (dt * 32 + 8 * r + 4 * g2 < E) {
+        float v[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = o[dt][4 * r + i] * f;
+        if (oo.each) {
+          const uint2 z = *reinterpret_cast<const uint2*>((const uint16_t*)oo.gate + (tok0 + qs) * oo.ld_gate + (int64_t)h * E + 4 * g2 + dt * 32 + 8 * r);
+          v[0] *= sigmoid(__uint_as_float(z.x << 16)), v[1] *= sigmoid(__uint_as_float(z.x & 0xffff0000u));
+          v[2] *= sigmoid(__uint_as_float(z.y << 16)), v[3] *= sigmoid(__uint_as_float(z.y & 0xffff0000u));
+        }
+        *reinterpret_cast<uint2*>(dst + dt * 32 + 8 * r) = make_uint2(pack2(v[0], v[1]), pack2(v[2], v[3]));
+      }
 }
 
 // ---------------------------------------------------------------------------------------------- decode
@@ -712,22 +750,17 @@ extern "C" int aqs_attn_window_ok(int dtype, int64_t D, int64_t E, int64_t page)
   return dtype == AQ_BF16 && D % 8 == 0 && E % 8 == 0 && D <= 256 && E <= 256 && page % WK == 0;
 }
 
-extern "C" int aqs_attn_window(const void* q, const void* kc, const void* vc, int dtype, float scale, int64_t window, const void* gate,
-                               int64_t ld_gate, float out_scale, const int32_t* pos, const int64_t* table, int64_t P, int64_t page,
-                               int64_t n_pages, void* out, int64_t ldo, int64_t B, int64_t S, int64_t H, int64_t G, int64_t D,
-                               int64_t E, int simple, void* stream) {
-  if (B * S == 0) return AQ_OK;
-  SQ_DIMS(B, S);
-  SQ_NEED(q && kc && vc && out);
-  SQ_CHECK(ldo >= H * E && (!gate || ld_gate >= H), AQ_E_SHAPE);
-  const AttnOut o{gate, ld_gate, ldo, out_scale};
-  hipStream_t st = (hipStream_t)stream;
-  if (simple || !aqs_attn_window_ok(dtype, D, E, page) || ldo % 4 || bad_ptr16(q) || bad_ptr16(kc) || bad_ptr16(vc) || bad_ptr16(out)) {
-    const unsigned grid = (unsigned)((B * S * H + 3) / 4);
-    SQ_DISPATCH(dtype, (attn_simple_kernel<T><<<grid, 256, 0, st>>>(a, o, scale, (const T*)q, (const T*)kc, (const T*)vc, (T*)out, B * S)));
-    return launched();
-  }
-  const dim3 grid((unsigned)(((S + WQ - 1) / WQ) * H * B));
+template <typename T>
+static int launch_simple(const AttnDims& a, const AttnKV<T>& kv, const AttnOut& o, float scale, const void* q, void* out, int64_t B,
+                         hipStream_t st) {
+  const unsigned grid = (unsigned)((B * a.S * a.H + 3) / 4);
+  attn_simple_kernel<T><<<grid, 256, 0, st>>>(a, kv, o, scale, (const T*)q, (T*)out, B * a.S);
+  return launched();
+}
+
+static int launch_window(const AttnDims& a, const AttnKV<uint16_t>& kv, const AttnOut& o, float scale, const void* q, void* out,
+                         int64_t B, hipStream_t st) {
+  const dim3 grid((unsigned)(((a.S + WQ - 1) / WQ) * a.H * B));
   auto go = [&](auto dtag, auto etag) -> int {
     constexpr int DP = decltype(dtag)::value, EP = decltype(etag)::value;
     const size_t lds = (size_t)(WK * (DP + 8) + EP * (WK + 4)) * 2;
@@ -736,17 +769,59 @@ extern "C" int aqs_attn_window(const void* q, const void* kc, const void* vc, in
       const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
       if (e != hipSuccess) return (int)e;
     }
-    k<<<grid, 256, lds, st>>>(a, o, scale * LOG2E, (const uint16_t*)q, (const uint16_t*)kc, (const uint16_t*)vc, (uint16_t*)out, (int)B);
+    k<<<grid, 256, lds, st>>>(a, kv, o, scale * LOG2E, (const uint16_t*)q, (uint16_t*)out, (int)B);
     return launched();
   };
   auto values = [&](auto dtag) -> int {
-    if (E <= 64) return go(dtag, std::integral_constant<int, 64>{});
-    if (E <= 128) return go(dtag, std::integral_constant<int, 128>{});
+    if (a.E <= 64) return go(dtag, std::integral_constant<int, 64>{});
+    if (a.E <= 128) return go(dtag, std::integral_constant<int, 128>{});
     return go(dtag, std::integral_constant<int, 256>{});
   };
-  if (D <= 64) return values(std::integral_constant<int, 64>{});
-  if (D <= 128) return values(std::integral_constant<int, 128>{});
+  if (a.D <= 64) return values(std::integral_constant<int, 64>{});
+  if (a.D <= 128) return values(std::integral_constant<int, 128>{});
+  if (a.D <= 192) return values(std::integral_constant<int, 192>{});
   return values(std::integral_constant<int, 256>{});
+}
+
+extern "C" int aqs_attn_window(const void* q, const void* kc, const void* vc, int dtype, float scale, int64_t window, const void* gate,
+                               int64_t ld_gate, float out_scale, const int32_t* pos, const int64_t* table, int64_t P, int64_t page,
+                               int64_t n_pages, void* out, int64_t ldo, int64_t B, int64_t S, int64_t H, int64_t G, int64_t D,
+                               int64_t E, int simple, void* stream) {
+  if (B * S == 0) return AQ_OK;
+  SQ_DIMS(B, S);
+  SQ_NEED(q && kc && vc && out);
+  SQ_CHECK(ldo >= H * E && (!gate || ld_gate >= H), AQ_E_SHAPE);
+  const AttnOut o{gate, ld_gate, ldo, out_scale, false};
+  hipStream_t st = (hipStream_t)stream;
+  if (simple || !aqs_attn_window_ok(dtype, D, E, page) || ldo % 4 || bad_ptr16(q) || bad_ptr16(kc) || bad_ptr16(vc) || bad_ptr16(out))
+    SQ_DISPATCH(dtype, return launch_simple<T>(a, paged_kv<T>(a, kc, vc), o, scale, q, out, B, st));
+  return launch_window(a, paged_kv<uint16_t>(a, kc, vc), o, scale, q, out, B, st);
+}
+
+// Keys and values of every head, formed from a shared latent: kv [B * rows, ld_kv] holds the keys' first `dim` elements
+// head by head, then the values; the keys' last `rot` elements are columns o_rot .. of packed [B * rows, ld_packed].
+extern "C" int aqs_latent_window(const void* q, const void* kv, int64_t ld_kv, const void* packed, int64_t ld_packed, int64_t o_rot,
+                                 int dtype, float scale, int64_t window, const void* gate, int64_t ld_gate, const int32_t* pos,
+                                 int64_t rows, void* out, int64_t ldo, int64_t B, int64_t S, int64_t H, int64_t dim, int64_t rot,
+                                 int64_t E, int simple, void* stream) {
+  if (B * S == 0) return AQ_OK;
+  SQ_CHECK(rows > 0 && rows % 64 == 0 && dim > 0 && rot >= 0, AQ_E_SHAPE);
+  const int64_t D = dim + rot, G = H, P = rows / 64, page = 64, n_pages = P * B;
+  const int64_t some_table[1] = {0}, *table = some_table;  // for the checks only
+  SQ_DIMS(B, S);
+  a.table = nullptr;
+  SQ_NEED(q && kv && packed && out && gate);
+  SQ_CHECK(ldo >= H * E && ld_gate >= H * E && ld_kv >= H * (dim + E) && o_rot >= 0 && ld_packed >= o_rot + rot, AQ_E_SHAPE);
+  const AttnOut o{gate, ld_gate, ldo, 1.0f, true};
+  hipStream_t st = (hipStream_t)stream;
+  auto source = [&](auto* t) {
+    using T = typename std::remove_pointer<decltype(t)>::type;
+    return AttnKV<T>{(const T*)kv, (const T*)packed + o_rot, (const T*)kv + H * dim, ld_kv, ld_packed, ld_kv, (int)dim, (int)E, (int)dim};
+  };
+  if (simple || !aqs_attn_window_ok(dtype, D, E, page) || dim % 8 || o_rot % 8 || ld_kv % 8 || ld_packed % 8 || ldo % 4 || ld_gate % 4 ||
+      bad_ptr16(q) || bad_ptr16(kv) || bad_ptr16(packed) || bad_ptr16(out) || bad_ptr16(gate))
+    SQ_DISPATCH(dtype, return launch_simple<T>(a, source((T*)nullptr), o, scale, q, out, B, st));
+  return launch_window(a, source((uint16_t*)nullptr), o, scale, q, out, B, st);
 }
 
 extern "C" int aqs_attn_decode_ok(int64_t D, int64_t E, int64_t page) {
@@ -791,7 +866,7 @@ extern "C" int aqs_attn_decode(const void* proj, int64_t ld, int64_t o_q, int64_
 #undef SQ_DEC
   if (const int rc = launched()) return rc;
   SQ_DISPATCH(dtype, {
-    const AttnOut o{o_gate >= 0 ? (const void*)((const T*)proj + o_gate) : nullptr, ld, ldo, out_scale};
+    const AttnOut o{o_gate >= 0 ? (const void*)((const T*)proj + o_gate) : nullptr, ld, ldo, out_scale, false};
     (attn_combine_kernel<T><<<dim3((unsigned)(B * H)), 256, 0, st>>>(a, o, part, (T*)out, (int)slices));
   });
   return launched();

@@ -19,7 +19,7 @@
 // State space (SSD), same idea with one scalar decay per head and token: y = e^{L_i} S^T C_i + sum_{j<=i} M_ij x_j + D x_i,
 // M_ij = <C_i, B_j> e^{L_i - L_j} dt_j;  S <- e^{L_C} S + sum_j e^{L_C - L_j} dt_j B_j x_j^T.  C B^T belongs to the
 // group and is computed once (`ssd_group`), M per head (`ssd_steps`), and the chunks run in order like the delta rule's
-// (`ssd_chunks`).
+// (`ssd_chunks`).  Linear attention with a constant decay per head is the same with dt = 1.
 #include "seq_common.h"
 
 namespace sq {
@@ -522,7 +522,8 @@ struct SsdChunkArgs {
   const float* conv_b;
   const float* dt_bias;
   const float* a_log;
-  const float* skip;
+  const float* skip;    // or null
+  const float* decay;   // [H] constant decays (step size 1), or null
   // per chunk and group, left operands in fragments of 16 x 16
   float* CB;     // [BC, G, 64 x 64]
   float* Cm;     // [BC, G, 64 x NP]
@@ -582,9 +583,16 @@ __global__ __launch_bounds__(256) void ssd_steps_kernel(SsdChunkArgs p, const T*
   const int64_t ch = (int64_t)blockIdx.x * p.H + h, cg = (int64_t)blockIdx.x * p.G + g;
   if (wave == 0) {
     const int t = c * CH + lane;
-    const float raw = to_f32(dt_raw[((int64_t)b * p.S + (t < p.S ? t : p.S - 1)) * p.ld_dt + h]);
-    const float dt = t < p.S ? softplus(raw + p.dt_bias[h]) : 0.0f;
-    double L = (double)(-expf(p.a_log[h]) * 1.44269504088896341f) * (double)dt;
+    float dt;
+    double L;
+    if (p.decay) {
+      dt = t < p.S ? 1.0f : 0.0f;
+      L = log2(fmax((double)p.decay[h], 1e-300)) * (double)dt;
+    } else {
+      const float raw = to_f32(dt_raw[((int64_t)b * p.S + (t < p.S ? t : p.S - 1)) * p.ld_dt + h]);
+      dt = t < p.S ? softplus(raw + p.dt_bias[h]) : 0.0f;
+      L = (double)(-expf(p.a_log[h]) * 1.44269504088896341f) * (double)dt;
+    }
 #pragma unroll
     for (int o = 1; o < 64; o <<= 1) {
       const double v = __shfl_up(L, o, 64);
@@ -631,7 +639,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 1))) voi
     const int d = (wave + 4 * t) * 16 + q4;
     s[t] = load_state4(col, d, N, e < P && pos > 0 && d < NP);
   }
-  const float skip = p.skip[h];
+  const float skip = p.skip ? p.skip[h] : 0.0f;
   // x: thread = (column tid % 16, tokens 4 (tid / 16) .. + 4); its raw inputs are requested a chunk ahead
   const int xe = tid & 15, xt = (tid >> 4) * 4;
   const bool xok = tile * CT + xe < P;
@@ -837,19 +845,20 @@ extern "C" int aqs_delta_chunked(const void* qkv, int64_t ld, const void* raw, i
 
 extern "C" int aqs_ssd_chunked(const void* xbc, int64_t ld, const void* dt_raw, int64_t ld_dt, int dtype, const float* conv_w,
                                const float* conv_b, const void* ring, const int32_t* slots, const int32_t* pos, const float* dt_bias,
-                               const float* a_log, const float* skip, float* ws, int64_t ws_floats, float* state, float* out,
-                               int64_t B, int64_t S, int64_t H, int64_t G, int64_t N, int64_t P, int64_t taps, void* stream) {
+                               const float* a_log, const float* skip, const float* decay, float* ws, int64_t ws_floats, float* state,
+                               float* out, int64_t B, int64_t S, int64_t H, int64_t G, int64_t N, int64_t P, int64_t taps, void* stream) {
   SQ_CHECK(B >= 0 && S >= 0 && H > 0 && G > 0 && H % G == 0 && N > 0 && P > 0 && aqs_chunked_ok(N, taps), AQ_E_SHAPE);
-  SQ_CHECK(ld >= H * P + 2 * G * N && ld_dt >= H, AQ_E_SHAPE);
+  SQ_CHECK(ld >= H * P + 2 * G * N && (decay || ld_dt >= H), AQ_E_SHAPE);
   const int64_t NC = (S + CH - 1) / CH;
   SQ_CHECK(B * NC < (1 << 16) && H < 65536 && G < 65536 && B < 65536 && P <= (1 << 16), AQ_E_RANGE);
   if (B * S == 0) return AQ_OK;
-  SQ_NEED(xbc && dt_raw && conv_w && conv_b && ring && slots && pos && dt_bias && a_log && skip && ws && state && out);
+  SQ_NEED(xbc && conv_w && conv_b && ring && slots && pos && (decay || (dt_raw && dt_bias && a_log)) && ws && state && out);
   SQ_CHECK(!bad_ptr16(ws), AQ_E_ALIGN);
   SQ_CHECK(ws_floats >= aqs_ssd_chunked_ws(B, S, H, G, N), AQ_E_WORKSPACE);
   const int64_t NP = pad_rows(N), n = B * NC * G;
   SsdChunkArgs a{};
-  a.slots = slots, a.pos = pos, a.conv_w = conv_w, a.conv_b = conv_b, a.dt_bias = dt_bias, a.a_log = a_log, a.skip = skip;
+  a.slots = slots, a.pos = pos, a.conv_w = conv_w, a.conv_b = conv_b, a.dt_bias = dt_bias, a.a_log = a_log;
+  a.skip = skip, a.decay = decay;
   a.CB = ws;
   a.Cm = a.CB + n * CH * CH;
   a.Bt = a.Cm + n * CH * NP;

@@ -1,6 +1,6 @@
 // Row operations of the hybrid decoder outside its matrix products and mixers: embedding lookup into
-// the fp32 residual stream, residual add + RMSNorm, the clamped GLU, and the gated norms that close
-// the two linear recurrences.
+// the fp32 residual stream, residual add + RMSNorm (with a norm of the branch in front of the sum, and routed experts'
+// rows collected, where a design has them), the GLUs, and the gated norms that close the linear recurrences.
 #include "seq_common.h"
 
 namespace sq {
@@ -44,22 +44,71 @@ __global__ __launch_bounds__(ROW_THREADS) void embed_kernel(const int64_t* ids, 
   for (int64_t k = threadIdx.x; k < K; k += ROW_THREADS) x[m * K + k] = ok ? to_f32(table[id * K + k]) : 0.0f;
 }
 
-// x += mult * y (y optional), then out = x / sqrt(mean(x^2) + eps) * (1 + w) (out optional)
-template <typename T, int V>
-__global__ __launch_bounds__(ROW_THREADS) void add_rmsnorm_kernel(float* x, const T* y, int64_t ldy, float mult, const float* w,
-                                                                  float eps, T* out, int K) {
+struct AddNormArgs {
+  float* x;            // [M, K]
+  const int* slots;    // [M, top] rows of `routed` that belong to a token (negative: none)
+  const float* post;   // weight of the branch's own norm
+  const float* w;      // weight of the norm behind the sum
+  int64_t ldy;
+  int top, K;
+  float mult, eps, w0;
+};
+
+// The branch's output t = y + sum_j routed[slots[m, j]] (either may be missing); POST: t <- t / rms(t) * post.
+// x += mult * t, then out = x / sqrt(mean(x^2) + eps) * (w0 + w) (out optional).
+template <typename T, int V, bool POST>
+__global__ __launch_bounds__(ROW_THREADS) void add_rmsnorm_kernel(AddNormArgs p, const T* y, const T* routed, T* out) {
   extern __shared__ __align__(16) float row[];
   __shared__ float red[ROW_THREADS / 64];
   const int64_t m = blockIdx.x;
-  float* xr = x + m * K;
-  float ss = 0.0f;
+  const int K = p.K;
+  float* xr = p.x + m * K;
+  auto branch = [&](int k, float (&b)[V]) __attribute__((always_inline)) {
+    if (y) {
+      Pack<T, V>::load(y + m * p.ldy + k, b);
+    } else {
+#pragma unroll
+      for (int i = 0; i < V; ++i) b[i] = 0.0f;
+    }
+    for (int j = 0; j < p.top; ++j) {
+      const int s = p.slots[m * p.top + j];
+      if (s < 0) continue;
+      float e[V];
+      Pack<T, V>::load(routed + (int64_t)s * K + k, e);
+#pragma unroll
+      for (int i = 0; i < V; ++i) b[i] += e[i];
+    }
+  };
+  float ry = 1.0f, ss = 0.0f;
+  if constexpr (POST) {
+    for (int k = threadIdx.x * V; k < K; k += ROW_THREADS * V) {
+      float b[V];
+      branch(k, b);
+#pragma unroll
+      for (int i = 0; i < V; ++i) {
+        ss += b[i] * b[i];
+        row[k + i] = b[i];
+      }
+    }
+    ss = block_sum<ROW_THREADS / 64>(ss, red);
+    ry = 1.0f / sqrtf(ss / (float)K + p.eps);
+    ss = 0.0f;
+  }
+  const bool add = POST || y || p.top;
   for (int k = threadIdx.x * V; k < K; k += ROW_THREADS * V) {
     float a[V], b[V];
     Pack<float, V>::load(xr + k, a);
-    if (y) {
-      Pack<T, V>::load(y + m * ldy + k, b);
+    if (add) {
+      if constexpr (POST) {
+        float g[V];
+        Pack<float, V>::load(p.post + k, g);
 #pragma unroll
-      for (int i = 0; i < V; ++i) a[i] += mult * b[i];
+        for (int i = 0; i < V; ++i) b[i] = row[k + i] * ry * g[i];
+      } else {
+        branch(k, b);
+      }
+#pragma unroll
+      for (int i = 0; i < V; ++i) a[i] += p.mult * b[i];
       Pack<float, V>::store(xr + k, a);
     }
 #pragma unroll
@@ -70,18 +119,18 @@ __global__ __launch_bounds__(ROW_THREADS) void add_rmsnorm_kernel(float* x, cons
   }
   if (!out) return;
   ss = block_sum<ROW_THREADS / 64>(ss, red);
-  const float r = 1.0f / sqrtf(ss / (float)K + eps);
+  const float r = 1.0f / sqrtf(ss / (float)K + p.eps);
   for (int k = threadIdx.x * V; k < K; k += ROW_THREADS * V) {
     float a[V], g[V];
-    Pack<float, V>::load(w + k, g);
+    Pack<float, V>::load(p.w + k, g);
 #pragma unroll
-    for (int i = 0; i < V; ++i) a[i] = row[k + i] * r * (1.0f + g[i]);
+    for (int i = 0; i < V; ++i) a[i] = row[k + i] * r * (p.w0 + g[i]);
     Pack<T, V>::store(out + m * K + k, a);
   }
 }
 
 // gu [M, 2F] = gate | up  ->  out [M, F]
-template <typename T, int V>
+template <typename T, int V, bool CLAMPED>
 __global__ __launch_bounds__(ROW_THREADS) void glu_kernel(const T* gu, int64_t ld, float limit, T* out, int64_t M, int64_t F) {
   // one row of blocks per F, rows of the matrix in the grid's second dimension: no division
   const int64_t f = ((int64_t)blockIdx.x * ROW_THREADS + threadIdx.x) * V;
@@ -91,7 +140,7 @@ __global__ __launch_bounds__(ROW_THREADS) void glu_kernel(const T* gu, int64_t l
     Pack<T, V>::load(gu + m * ld + f, g);
     Pack<T, V>::load(gu + m * ld + F + f, u);
 #pragma unroll
-    for (int e = 0; e < V; ++e) g[e] = clamped_glu(g[e], u[e], limit);
+    for (int e = 0; e < V; ++e) g[e] = CLAMPED ? clamped_glu(g[e], u[e], limit) : silu(g[e]) * u[e];
     Pack<T, V>::store(out + m * F + f, g);
   }
 }
@@ -114,6 +163,35 @@ __global__ __launch_bounds__(ROW_THREADS) void gated_group_norm_kernel(const flo
   const float r = 1.0f / sqrtf(ss / (float)group + eps);
   for (int k = threadIdx.x; k < group; k += ROW_THREADS)
     out[m * ldo + base + k] = from_f32<T>(row[k] * r * w[base + k]);
+}
+
+// y [M, K] fp32 over its root mean square, times w, times sigmoid(z)  ->  out
+template <typename T, int V>
+__global__ __launch_bounds__(ROW_THREADS) void norm_gate_kernel(const float* y, const T* z, int64_t ldz, const float* w, float eps,
+                                                                T* out, int64_t ldo, int K) {
+  extern __shared__ __align__(16) float row[];
+  __shared__ float red[ROW_THREADS / 64];
+  const int64_t m = blockIdx.x;
+  float ss = 0.0f;
+  for (int k = threadIdx.x * V; k < K; k += ROW_THREADS * V) {
+    float a[V];
+    Pack<float, V>::load(y + m * K + k, a);
+#pragma unroll
+    for (int i = 0; i < V; ++i) {
+      ss += a[i] * a[i];
+      row[k + i] = a[i];
+    }
+  }
+  ss = block_sum<ROW_THREADS / 64>(ss, red);
+  const float r = 1.0f / sqrtf(ss / (float)K + eps);
+  for (int k = threadIdx.x * V; k < K; k += ROW_THREADS * V) {
+    float a[V], g[V], f[V];
+    Pack<float, V>::load(w + k, g);
+    Pack<T, V>::load(z + m * ldz + k, f);
+#pragma unroll
+    for (int i = 0; i < V; ++i) a[i] = row[k + i] * r * g[i] * sigmoid(f[i]);
+    Pack<T, V>::store(out + m * ldo + k, a);
+  }
 }
 
 // Every head of o [M, H, E] fp32 over its root mean square, times w [E], times sigmoid(gate), times scale -> out.
@@ -172,26 +250,30 @@ extern "C" int aqs_embed(const int64_t* ids, const void* table, int dtype, float
   return launched();
 }
 
-extern "C" int aqs_add_rmsnorm(float* x, const void* y, int64_t ldy, int dtype, float mult, const float* w, float eps,
-                               void* out, int64_t M, int64_t K, void* stream) {
-  SQ_CHECK(M >= 0 && K > 0, AQ_E_SHAPE);
-  SQ_CHECK(K <= 16384, AQ_E_RANGE);
+extern "C" int aqs_add_rmsnorm(float* x, const void* y, int64_t ldy, int dtype, const void* routed, const int32_t* slots,
+                               int64_t top, const float* post, float mult, const float* w, float w0, float eps, void* out, int64_t M,
+                               int64_t K, void* stream) {
+  SQ_CHECK(M >= 0 && K > 0 && top >= 0, AQ_E_SHAPE);
+  SQ_CHECK(K <= 16384 && top <= 1024, AQ_E_RANGE);
   SQ_CHECK(!y || ldy >= K, AQ_E_SHAPE);
   SQ_CHECK(M < (1 << 24), AQ_E_RANGE);  // one workgroup a row, fewer than 2^32 threads a launch
   if (M == 0) return AQ_OK;
-  SQ_NEED(x && (out || y) && (w || !out));
-  const bool v4 = K % 4 == 0 && ldy % 4 == 0 && !bad_ptr16(x) && !bad_ptr16(y) && !bad_ptr16(w) && !bad_ptr16(out);
+  const bool branch = y || top;
+  SQ_NEED(x && (out || branch) && (w || !out) && (branch || !post) && (top == 0 || (routed && slots)));
+  const AddNormArgs a{x, slots, post, w, ldy, (int)top, (int)K, mult, eps, w0};
+  const bool v4 = K % 4 == 0 && (!y || ldy % 4 == 0) && !bad_ptr16(x) && !bad_ptr16(y) && !bad_ptr16(routed) && !bad_ptr16(post) &&
+                  !bad_ptr16(w) && !bad_ptr16(out);
   const size_t lds = (size_t)K * 4;
   const dim3 grid((unsigned)M);
-  SQ_DISPATCH(dtype, if (v4)(add_rmsnorm_kernel<T, 4><<<grid, ROW_THREADS, lds, (hipStream_t)stream>>>(
-                         x, (const T*)y, ldy, mult, w, eps, (T*)out, (int)K));
-              else (add_rmsnorm_kernel<T, 1><<<grid, ROW_THREADS, lds, (hipStream_t)stream>>>(x, (const T*)y, ldy, mult, w, eps,
-                                                                                               (T*)out, (int)K)));
+#define SQ_ADD(V, POST) \
+  (add_rmsnorm_kernel<T, V, POST><<<grid, ROW_THREADS, lds, (hipStream_t)stream>>>(a, (const T*)y, (const T*)routed, (T*)out))
+  SQ_DISPATCH(dtype, if (v4) { if (post) SQ_ADD(4, true); else SQ_ADD(4, false); }
+                     else { if (post) SQ_ADD(1, true); else SQ_ADD(1, false); });
+#undef SQ_ADD
   return launched();
 }
 
-extern "C" int aqs_clamped_glu(const void* gu, int64_t ld, int dtype, float limit, void* out, int64_t M, int64_t F,
-                               void* stream) {
+static int launch_glu(const void* gu, int64_t ld, int dtype, bool clamped, float limit, void* out, int64_t M, int64_t F, void* stream) {
   SQ_CHECK(M >= 0 && F > 0 && ld >= 2 * F, AQ_E_SHAPE);
   SQ_CHECK(M < (1 << 24), AQ_E_RANGE);  // one workgroup a row, fewer than 2^32 threads a launch
   if (M == 0) return AQ_OK;
@@ -200,8 +282,33 @@ extern "C" int aqs_clamped_glu(const void* gu, int64_t ld, int dtype, float limi
   const int64_t nf = ((v4 ? F / 4 : F) + ROW_THREADS - 1) / ROW_THREADS;
   SQ_CHECK(nf < (1 << 20), AQ_E_RANGE);
   const dim3 grid((unsigned)nf, (unsigned)(M < 65535 ? M : 65535));
-  SQ_DISPATCH(dtype, if (v4)(glu_kernel<T, 4><<<grid, ROW_THREADS, 0, (hipStream_t)stream>>>((const T*)gu, ld, limit, (T*)out, M, F));
-              else (glu_kernel<T, 1><<<grid, ROW_THREADS, 0, (hipStream_t)stream>>>((const T*)gu, ld, limit, (T*)out, M, F)));
+#define SQ_GLU(V, C) (glu_kernel<T, V, C><<<grid, ROW_THREADS, 0, (hipStream_t)stream>>>((const T*)gu, ld, limit, (T*)out, M, F))
+  SQ_DISPATCH(dtype, if (clamped) { if (v4) SQ_GLU(4, true); else SQ_GLU(1, true); }
+                     else { if (v4) SQ_GLU(4, false); else SQ_GLU(1, false); });
+#undef SQ_GLU
+  return launched();
+}
+
+extern "C" int aqs_clamped_glu(const void* gu, int64_t ld, int dtype, float limit, void* out, int64_t M, int64_t F, void* stream) {
+  return launch_glu(gu, ld, dtype, true, limit, out, M, F, stream);
+}
+
+extern "C" int aqs_silu_glu(const void* gu, int64_t ld, int dtype, void* out, int64_t M, int64_t F, void* stream) {
+  return launch_glu(gu, ld, dtype, false, 0.0f, out, M, F, stream);
+}
+
+extern "C" int aqs_norm_gate(const float* y, const void* z, int64_t ldz, int dtype, const float* w, float eps, void* out, int64_t ldo,
+                             int64_t M, int64_t K, void* stream) {
+  SQ_CHECK(M >= 0 && K > 0 && ldz >= K && ldo >= K, AQ_E_SHAPE);
+  SQ_CHECK(K <= 16384 && M < (1 << 24), AQ_E_RANGE);
+  if (M == 0) return AQ_OK;
+  SQ_NEED(y && z && w && out);
+  const bool v4 = K % 4 == 0 && ldz % 4 == 0 && ldo % 4 == 0 && !bad_ptr16(y) && !bad_ptr16(z) && !bad_ptr16(w) && !bad_ptr16(out);
+  const size_t lds = (size_t)K * 4;
+  const dim3 grid((unsigned)M);
+#define SQ_NG(V) (norm_gate_kernel<T, V><<<grid, ROW_THREADS, lds, (hipStream_t)stream>>>(y, (const T*)z, ldz, w, eps, (T*)out, ldo, (int)K))
+  SQ_DISPATCH(dtype, if (v4) SQ_NG(4); else SQ_NG(1));
+#undef SQ_NG
   return launched();
 }
 

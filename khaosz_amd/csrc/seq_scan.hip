@@ -2,6 +2,7 @@
 //
 //   gated delta rule   S <- g S (one decay per key channel), u = beta (v - S^T k), S <- S + k u^T, o = S^T q
 //   state space (SSD)  S <- a S (one decay per head),        u = dt x,             S <- S + B u^T, y = S^T C + D x
+//                      (with constant decays, dt = 1 and D = 0 it is linear attention: x = v, B = k, C = q)
 //
 // Both are "decay the rows, add an outer product, read out", so they share the scan kernel: rows of the state
 // belong to k (or B), columns to v (or x).  The state is fp32 and is stored column by column, [slot, head, column,
@@ -154,7 +155,7 @@ struct ScanArgs {
   const float* k;  // element (m, group, row) at k + m * ld_k + group * R + row; likewise q
   const float* q;
   const float* v;  // element (m, head, column) at v + m * ld_v + head * E + column
-  const float* decay;    // delta: [M, H, R]
+  const float* decay;    // delta: [M, H, R]; ssd: [H] if the decays are constants (step size 1), else null
   const float* beta;     // delta: [M, H]
   const float* dt_bias;  // ssd: [H]
   const float* a_log;    // ssd: [H]
@@ -226,7 +227,11 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs p, const T* dt_raw) 
   float s[RP];
   load_rows<RP>(col, r0, R, e < p.E && p.pos[b] > 0, s);
   float skip = 0.0f, neg_a = 0.0f, dtb = 0.0f;
-  if constexpr (!DELTA) skip = p.skip[h], neg_a = -expf(p.a_log[h]), dtb = p.dt_bias[h];
+  const bool constant = !DELTA && p.decay;
+  if constexpr (!DELTA) {
+    skip = p.skip ? p.skip[h] : 0.0f;
+    if (!constant) neg_a = -expf(p.a_log[h]), dtb = p.dt_bias[h];
+  }
   const float* src[3] = {p.k + m0 * p.ld_k + (int64_t)j * R, p.q + m0 * p.ld_q + (int64_t)j * R,
                          DELTA ? p.decay + (m0 * p.H + h) * R : nullptr};
   const int64_t ld[3] = {p.ld_k, p.ld_q, (int64_t)p.H * R};
@@ -261,6 +266,8 @@ __global__ __launch_bounds__(256) void scan_kernel(ScanArgs p, const T* dt_raw) 
     if (tid < TC && t0 + tid < p.S) {
       if constexpr (DELTA) {
         creg.x = p.beta[(m0 + t0 + tid) * p.H + h];
+      } else if (constant) {
+        creg = make_float2(p.decay[h], 1.0f);
       } else {
         const float dt = softplus(to_f32(dt_raw[(m0 + t0 + tid) * p.ld_dt + h]) + dtb);
         creg = make_float2(expf(neg_a * dt), dt);
@@ -473,7 +480,8 @@ struct SsdStepArgs {
   const int* pos;
   const float* dt_bias;
   const float* a_log;
-  const float* skip;
+  const float* skip;     // or null
+  const float* decay;    // [H] constant decays (step size 1), or null
   float* state;  // [slots, H, P, N]
   float* y;
   int64_t ld, o_xbc, o_dt;
@@ -509,8 +517,8 @@ __global__ __launch_bounds__(256) void ssd_step_kernel(SsdStepArgs p, const T* p
     (which == 0 ? b_s : which == 1 ? c_s : x_s)[d] = x;
     if (which == 2 || h % per == 0) rg[(int64_t)(pos % p.s.taps) * p.s.C + c] = cin[c];
   }
-  const float dt = softplus(to_f32(row[p.o_dt + h]) + p.dt_bias[h]);
-  const float a = expf(-expf(p.a_log[h]) * dt), skip = p.skip[h];
+  const float dt = p.decay ? 1.0f : softplus(to_f32(row[p.o_dt + h]) + p.dt_bias[h]);
+  const float a = p.decay ? p.decay[h] : expf(-expf(p.a_log[h]) * dt), skip = p.skip ? p.skip[h] : 0.0f;
   __syncthreads();
   float k[RP], q[RP];
   load_vec<RP>(&b_s[r0], k);
@@ -640,16 +648,16 @@ extern "C" int aqs_delta_scan(const float* q, const float* k, const float* v, co
 }
 
 extern "C" int aqs_ssd_scan(const float* xbc, const void* dt_raw, int64_t ld_dt, int dtype, const float* dt_bias, const float* a_log,
-                            const float* skip, float* state, const int32_t* slots, const int32_t* pos, float* out, int64_t B,
-                            int64_t S, int64_t H, int64_t G, int64_t N, int64_t P, void* stream) {
-  SQ_CHECK(B >= 0 && S >= 0 && H > 0 && G > 0 && H % G == 0 && N > 0 && P > 0 && ld_dt >= H, AQ_E_SHAPE);
+                            const float* skip, const float* decay, float* state, const int32_t* slots, const int32_t* pos, float* out,
+                            int64_t B, int64_t S, int64_t H, int64_t G, int64_t N, int64_t P, void* stream) {
+  SQ_CHECK(B >= 0 && S >= 0 && H > 0 && G > 0 && H % G == 0 && N > 0 && P > 0 && (decay || ld_dt >= H), AQ_E_SHAPE);
   SQ_CHECK(N <= STEP_MAX && S < ((int64_t)1 << 31), AQ_E_RANGE);
   if (B * S == 0) return AQ_OK;
-  SQ_NEED(xbc && dt_raw && dt_bias && a_log && skip && state && slots && pos && out);
+  SQ_NEED(xbc && (decay || (dt_raw && dt_bias && a_log)) && state && slots && pos && out);
   ScanArgs a{};
   const int64_t C = H * P + 2 * G * N;
   a.v = xbc, a.k = xbc + H * P, a.q = xbc + H * P + G * N;
-  a.dt_bias = dt_bias, a.a_log = a_log, a.skip = skip, a.state = state, a.out = out, a.slots = slots, a.pos = pos;
+  a.dt_bias = dt_bias, a.a_log = a_log, a.skip = skip, a.decay = decay, a.state = state, a.out = out, a.slots = slots, a.pos = pos;
   a.ld_k = a.ld_q = a.ld_v = C, a.ld_dt = ld_dt;
   a.S = (int)S, a.H = (int)H, a.G = (int)G, a.R = (int)N, a.E = (int)P;
   const int64_t grid = B * H * ((P + SCAN_COLS - 1) / SCAN_COLS);
@@ -686,17 +694,17 @@ extern "C" int aqs_delta_step(const void* proj, int64_t ld, int64_t o_qkv, int64
 
 extern "C" int aqs_ssd_step(const void* proj, int64_t ld, int64_t o_xbc, int64_t o_dt, int dtype, const float* conv_w,
                             const float* conv_b, void* ring, const int32_t* slots, const int32_t* pos, const float* dt_bias,
-                            const float* a_log, const float* skip, float* state, float* y, int64_t B, int64_t H, int64_t G,
-                            int64_t N, int64_t P, int64_t taps, void* stream) {
+                            const float* a_log, const float* skip, const float* decay, float* state, float* y, int64_t B,
+                            int64_t H, int64_t G, int64_t N, int64_t P, int64_t taps, void* stream) {
   SQ_CHECK(B >= 0 && H > 0 && G > 0 && H % G == 0 && N > 0 && P > 0 && taps > 0, AQ_E_SHAPE);
   SQ_CHECK(N <= STEP_MAX && P <= STEP_MAX && taps <= 64 && B <= 65535, AQ_E_RANGE);
-  SQ_CHECK(o_xbc >= 0 && o_dt >= 0 && o_xbc + H * P + 2 * G * N <= ld && o_dt + H <= ld, AQ_E_SHAPE);
+  SQ_CHECK(o_xbc >= 0 && o_xbc + H * P + 2 * G * N <= ld && (decay || (o_dt >= 0 && o_dt + H <= ld)), AQ_E_SHAPE);
   if (B == 0) return AQ_OK;
-  SQ_NEED(proj && conv_w && ring && slots && pos && dt_bias && a_log && skip && state && y);
+  SQ_NEED(proj && conv_w && ring && slots && pos && (decay || (dt_bias && a_log)) && state && y);
   SQ_CHECK(!bad_ptr16(state), AQ_E_ALIGN);
   SsdStepArgs a{};
   a.s = ConvSrc{conv_w, conv_b, (int)(H * P + 2 * G * N), (int)taps};
-  a.slots = slots, a.pos = pos, a.dt_bias = dt_bias, a.a_log = a_log, a.skip = skip, a.state = state, a.y = y;
+  a.slots = slots, a.pos = pos, a.dt_bias = dt_bias, a.a_log = a_log, a.skip = skip, a.decay = decay, a.state = state, a.y = y;
   a.ld = ld, a.o_xbc = o_xbc, a.o_dt = o_dt;
   a.H = (int)H, a.G = (int)G, a.N = (int)N, a.P = (int)P;
   const dim3 grid((unsigned)H, (unsigned)B);

@@ -1,16 +1,20 @@
-"""Decoders whose layers mix linear recurrences and windowed attention, configured layer by layer.
+"""Decoders whose layers mix linear recurrences, windowed and latent attention, configured layer by layer.
 
-``Rudilix``: embedding, pre-norm layers ``x += m mixer(norm(x)); x += m ff(norm(x))`` with mixers of three kinds
-(``mamba2``, ``channel_delta``, and ``parallel``: windowed attention beside a channel delta rule), norms with their
-weight around zero, clamped GLU feed-forwards, an untied vocabulary projection.  Which mixer a layer has, every size
-and every constant come from the configuration.
+Two designs share the layers, the model class and everything behind it:
 
-The residual stream is fp32 throughout; weights and activations are bf16 or fp32.
+* ``Rudilix``: pre-norm layers ``x += m mixer(norm(x)); x += m ff(norm(x))`` with mixers of three kinds (``mamba2``,
+  ``channel_delta``, and ``parallel``: windowed attention beside a channel delta rule), norms with their weight around zero,
+  clamped GLU feed-forwards.
+* ``Lomozen``: norms before and after each sublayer, ``x += norm'(mixer(norm(x))); x += norm'(ff(norm(x)))``, with mixers of two
+  kinds (``latent_attention``, ``lightning``), plain norm weights, routed experts with a shared one.
+
+Both have an untied vocabulary projection.  Which mixer a layer has, every size and every constant that is not the design's
+come from the configuration.  The residual stream is fp32 throughout; weights and activations are bf16 or fp32.
 """
 from __future__ import annotations
 
 from dataclasses import dataclass, field
-from typing import Any, Dict, List, Optional, Sequence
+from typing import Any, Callable, Dict, List, NamedTuple, Optional, Sequence
 
 import torch
 import torch.nn as nn
@@ -18,9 +22,19 @@ import torch.nn.functional as F
 from torch import Tensor
 
 from . import seq_ops
-from .mixers import ChannelDeltaMixer, ClampedGLU, Mamba2Mixer, MixerBlock, WindowAttention, _param
+from .mixers import (Branch, ChannelDeltaMixer, ClampedGLU, LatentAttention, LightningMixer, Mamba2Mixer, MixerBlock, RoutedExperts,
+                     WindowAttention, _param)
 from .registry import register_model
-from .seq_ops import Batch
+from .seq_ops import Batch, Stream
+
+
+class Design(NamedTuple):
+    """What a design fixes: the mixers a layer's ``type`` may name, the feed-forwards its ``kind`` may name, what is added to
+    a norm's stored weight, and whether a sublayer's output passes a norm of its own."""
+    mixers: Dict[str, Callable]
+    feed_forwards: Dict[str, Callable]
+    norm_offset: float
+    post_norms: bool
 
 
 @dataclass
@@ -34,21 +48,26 @@ class HybridConfig:
     residual_mult: float = 1.0
     # ranks of the low-rank factors, by tensor name: no other field gives them, so they come from the tensors' shapes
     ranks: Dict[str, int] = field(default_factory=dict)
+    architecture: str = "Rudilix"
+
+    @property
+    def design(self) -> Design:
+        return DESIGNS[self.architecture]
 
     @classmethod
     def from_dict(cls, d: Dict[str, Any], shapes: Optional[Dict[str, Sequence[int]]] = None) -> "HybridConfig":
+        name = d.get("architecture", "Rudilix")
+        if name not in DESIGNS:
+            raise ValueError(f"unknown design {name!r}, know {sorted(DESIGNS)}")
+        design = DESIGNS[name]
         for i, layer in enumerate(d["layers"]):
-            if layer["type"] not in LAYER_MIXERS:
-                raise ValueError(f"layer {i}: unknown mixer {layer['type']!r}, know {sorted(LAYER_MIXERS)}")
+            if layer["type"] not in design.mixers:
+                raise ValueError(f"layer {i}: unknown mixer {layer['type']!r}, know {sorted(design.mixers)}")
             mlp = layer.get("mlp")
-            if mlp is not None and mlp["kind"] != "dense":
+            if mlp is not None and mlp["kind"] not in design.feed_forwards:
                 raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
         ranks = {n: s[0] for n, s in (shapes or {}).items() if n.endswith((".a1", ".g1"))}
-        return cls(int(d["vocab"]), int(d["width"]), d["layers"], float(d["norm"]["eps"]), float(d["residual_mult"]), ranks)
-
-
-def _mamba2(cfg: HybridConfig, c, prefix: str, dtype, device):
-    return [("", Mamba2Mixer(c, cfg.norm_eps, dtype, device), 1.0)]
+        return cls(int(d["vocab"]), int(d["width"]), d["layers"], float(d["norm"]["eps"]), float(d.get("residual_mult", 1.0)), ranks, name)
 
 
 def _delta(cfg: HybridConfig, c, prefix: str, dtype, device):
@@ -66,48 +85,65 @@ def _parallel(cfg: HybridConfig, c, prefix: str, dtype, device):
     return [("left.", left, c["left_scale"]), ("right.", right, c["right_scale"])]
 
 
-LAYER_MIXERS = {"mamba2": _mamba2, "channel_delta": _delta, "parallel": _parallel}
+def _alone(mixer) -> Callable:
+    return lambda cfg, c, prefix, dtype, device: [("", mixer(c, cfg.norm_eps, dtype, device), 1.0)]
+
+
+DESIGNS = {
+    "Rudilix": Design({"mamba2": _alone(Mamba2Mixer), "channel_delta": _delta, "parallel": _parallel}, {"dense": ClampedGLU}, 1.0, False),
+    "Lomozen": Design({"latent_attention": _alone(LatentAttention), "lightning": _alone(LightningMixer)}, {"moe": RoutedExperts}, 0.0, True),
+}
 
 
 class HybridLayer(nn.Module):
     def __init__(self, cfg: HybridConfig, index: int, dtype, device=None):
         super().__init__()
-        layer = cfg.layers[index]
-        self.prefix, self.eps, self.mult = f"l{index}.", cfg.norm_eps, cfg.residual_mult
-        mixers = LAYER_MIXERS[layer["type"]](cfg, layer["mixer"], self.prefix + "mix.", dtype, device)
-        self.norm1 = _param(cfg.width, device=device)
+        layer, design = cfg.layers[index], cfg.design
+        self.prefix, self.eps, self.mult, self.w0 = f"l{index}.", cfg.norm_eps, cfg.residual_mult, design.norm_offset
+        mixers = design.mixers[layer["type"]](cfg, layer["mixer"], self.prefix + "mix.", dtype, device)
+        norm = lambda on: _param(cfg.width, device=device) if on else None
+        self.norm1, self.norm1b = norm(True), norm(design.post_norms)
         self.mixer = MixerBlock(cfg.width, mixers, dtype, device)
-        self.mlp = None
-        if layer.get("mlp") is not None:
-            self.norm2 = _param(cfg.width, device=device)
-            self.mlp = ClampedGLU(cfg.width, layer["mlp"], dtype, device)
+        mlp = layer.get("mlp")
+        self.norm2, self.norm2b = norm(mlp is not None), norm(mlp is not None and design.post_norms)
+        self.mlp = design.feed_forwards[mlp["kind"]](cfg.width, mlp, dtype, device) if mlp is not None else None
 
     def tensors(self) -> Dict[str, Tensor]:
-        out = {self.prefix + "norm1": self.norm1}
+        norms = lambda *names: {self.prefix + n: t for n in names if (t := getattr(self, n)) is not None}
+        out = norms("norm1", "norm1b")
         out.update({self.prefix + "mix." + n: t for n, t in self.mixer.tensors().items()})
+        out.update(norms("norm2", "norm2b"))
         if self.mlp is not None:
-            out[self.prefix + "norm2"] = self.norm2
             out.update({self.prefix + "mlp." + n: t for n, t in self.mlp.tensors().items()})
         return out
 
-    def prompt(self, x: Tensor, y: Optional[Tensor], b: Batch, st, dtype) -> Tensor:
-        """Adds the pending branch output ``y`` to the stream, runs the layer and returns its own pending output."""
-        h = seq_ops.add_rmsnorm(x, y, self.mult, self.norm1, self.eps, dtype)
-        y = self.mixer.prompt(h, b, st)
+    def _norm(self, x: Tensor, pending: Optional[Branch], w: Tensor, dtype) -> Tensor:
+        return add_branch(x, pending, self.mult, w, self.eps, dtype, self.w0)
+
+    def prompt(self, x: Tensor, pending: Optional[Branch], b: Batch, st, dtype) -> Branch:
+        """Adds the pending branch output to the stream, runs the layer and returns its own pending output."""
+        y = self.mixer.prompt(self._norm(x, pending, self.norm1, dtype), b, st)._replace(post=self.norm1b)
         if self.mlp is None:
             return y
-        return self.mlp.prompt(seq_ops.add_rmsnorm(x, y, self.mult, self.norm2, self.eps, dtype))
+        return self.mlp.prompt(self._norm(x, y, self.norm2, dtype))._replace(post=self.norm2b)
 
-    def step(self, x: Tensor, b: Batch, st) -> None:
-        self.mixer.step(x, self.norm1, self.eps, b, st, self.mult)
+    def step(self, s: Stream, b: Batch, st) -> None:
+        self.mixer.step(s, self.norm1, b, st, self.norm1b)
         if self.mlp is not None:
-            self.mlp.step(x, self.norm2, self.eps, self.mult)
+            self.mlp.step(s, self.norm2, self.norm2b)
 
     def step_ok(self, rows: int) -> bool:
         return self.mixer.step_ok(rows) and (self.mlp is None or self.mlp.step_ok(rows))
 
 
+def add_branch(x: Tensor, pending: Optional[Branch], mult: float, w: Optional[Tensor], eps: float, dtype, w0: float) -> Optional[Tensor]:
+    """Adds a pending branch output to the stream ``x`` in place; returns the sum normed with ``w0 + w`` if there is a ``w``."""
+    p = pending or Branch(None)
+    return seq_ops.add_rmsnorm(x, p.y, mult, w, eps, dtype, w is not None, w0, p.post, p.routed)
+
+
 @register_model("Rudilix")
+@register_model("Lomozen")
 class HybridLM(nn.Module):
     """``forward`` runs new tokens of a batch of sequences on the state that earlier calls left."""
 
@@ -138,8 +174,7 @@ class HybridLM(nn.Module):
     @property
     def window(self) -> int:
         """How many positions back any layer still reads keys (1: none does)."""
-        from .mixers import WindowAttention as W
-        return max([m.spec.window for l in self.layers for m in l.mixer.mixers if isinstance(m, W)] or [1])
+        return max([m.spec.window for l in self.layers for m in l.mixer.mixers if isinstance(m, (WindowAttention, LatentAttention))] or [1])
 
     def new_sequence_state(self, n_slots: int, n_pages: int, page: int, capacity: int) -> List[Any]:
         return [l.mixer.new_state(n_slots, n_pages, page, capacity, self.dtype, self.embed.device) for l in self.layers]
@@ -153,37 +188,38 @@ class HybridLM(nn.Module):
         return self._step_ok[rows]
 
     def advance(self, ids: Tensor, b: Batch, state: List[Any], starts: Sequence[int], want: Optional[Sequence[int]] = None) -> Tensor:
-        return self(ids, b, state, want)
+        return self(ids, b._replace(starts=tuple(starts)) if b.S > 1 or not self.step_ok(b.B) else b, state, want)
 
     def forward(self, ids: Tensor, b: Batch, state: List[Any], want: Optional[Sequence[int]] = None,
                 layer_outputs: Optional[List[Tensor]] = None) -> Tensor:
         """``ids [B, S]``; returns fp32 logits of the rows ``want`` (row = sequence * S + token; all of them if None).
         ``layer_outputs``: a list that receives the residual stream after every layer."""
-        c = self.config
+        c, w0 = self.config, self.config.design.norm_offset
         x = seq_ops.embed(ids, self.embed)
         if b.S == 1 and self.step_ok(b.B):
+            s = Stream(x, c.norm_eps, w0, c.residual_mult)
             for layer, st in zip(self.layers, state):
-                layer.step(x, b, st)
+                layer.step(s, b, st)
                 if layer_outputs is not None:
-                    layer_outputs.append(x.clone())
+                    layer_outputs.append(s.settled())
             if want is not None and list(want) != list(range(b.B)):
-                x = x[list(want)].contiguous()
-            if not x.shape[0]:
+                s.rows(list(want))
+            if not s.x.shape[0]:
                 return torch.empty((0, c.vocab), dtype=torch.float32, device=x.device)
-            return seq_ops.norm_gemv_f32(x, self.final_norm, c.norm_eps, self.head)
-        y = None
+            return s.norm_gemv_f32(self.final_norm, self.head)
+        pending = None
         for layer, st in zip(self.layers, state):
-            y = layer.prompt(x, y, b, st, self.dtype)
+            pending = layer.prompt(x, pending, b, st, self.dtype)
             if layer_outputs is not None:
-                layer_outputs.append(x + c.residual_mult * y.float())
+                layer_outputs.append(x.clone())
+                add_branch(layer_outputs[-1], pending, c.residual_mult, None, c.norm_eps, self.dtype, w0)
         if want is not None:
             if not len(want):
                 return torch.empty((0, c.vocab), dtype=torch.float32, device=x.device)
             if list(want) != list(range(x.shape[0])):
                 rows = torch.tensor(list(want), device=x.device)
-                x, y = x[rows], y[rows]
+                x, pending = x[rows], pending.rows(rows)
         if seq_ops.gemv_ok(x.shape[0], self.head):
-            seq_ops.add_rmsnorm(x, y, c.residual_mult, None, c.norm_eps, self.dtype, norm=False)
-            return seq_ops.norm_gemv_f32(x, self.final_norm, c.norm_eps, self.head)
-        h = seq_ops.add_rmsnorm(x, y, c.residual_mult, self.final_norm, c.norm_eps, self.dtype)
-        return F.linear(h, self.head).float()
+            add_branch(x, pending, c.residual_mult, None, c.norm_eps, self.dtype, w0)
+            return Stream(x, c.norm_eps, w0, c.residual_mult).norm_gemv_f32(self.final_norm, self.head)
+        return F.linear(add_branch(x, pending, c.residual_mult, self.final_norm, c.norm_eps, self.dtype, w0), self.head).float()

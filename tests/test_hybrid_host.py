@@ -34,14 +34,22 @@ def test_seq_library_exports_every_declared_symbol():
 
 def test_seq_arguments_are_checked_before_any_launch():
     lib, P = _abi.load_seq(), 1 << 20
-    assert lib.aqs_add_rmsnorm(P, None, 8, 1, 1.0, P, 1e-6, P, 1, 0, None) == -2
-    assert lib.aqs_add_rmsnorm(P, None, 8, 7, 1.0, P, 1e-6, P, 1, 8, None) == -3
+    add = lambda dtype, K, top=0, post=None: lib.aqs_add_rmsnorm(P, None, 8, dtype, None, None, top, post, 1.0, P, 1.0, 1e-6, P, 1, K, None)
+    assert add(1, 0) == -2 and add(7, 8) == -3
+    assert add(1, 8, top=2) == -1 and add(1, 8, post=P) == -1                                                # routed rows missing; nothing to norm
     assert lib.aqs_gemv_ok(1, 1, 64, 20) == 0 and lib.aqs_gemv_ok(1, 9, 64, 64) == 0 and lib.aqs_gemv_ok(1, 8, 64, 64) == 1
-    assert lib.aqs_gemv(0, 0, 1, P, 64, None, None, 0.0, 1, P + 2, None, 1.0, 0.0, None, P, 64, 1, 64, 64, None) == -4
-    assert lib.aqs_gemv(2, 3, 1, P, 64, P, P, 0.0, 1, P, None, 1.0, 0.0, P, P, 64, 1, 64, 64, None) == -2  # pair not served
+    def gemv(i, o, x=P, xf=None, yf=None, post=None, x_out=None, gain=None, w=P, routers=0, res=None, ldo=64):
+        return lib.aqs_gemv(i, o, 1, x, 64, xf, yf, post, x_out, gain, 0.0, 1e-6, 1, w, None, 1.0, 0.0, routers, res, P, ldo, None, 1, 64, 64, None)
+    assert gemv(0, 0, w=P + 2) == -4
+    assert gemv(2, 3, xf=P, gain=P, res=P) == -2                                                             # pair not served
+    assert gemv(3, 0, xf=P, gain=P) == -1                                                                    # no branch output
+    assert gemv(3, 0, xf=P, yf=P, post=P, x_out=P, gain=P) == -2                                             # the old stream is still read
+    assert gemv(0, 0, routers=8) == -2 and gemv(3, 4, xf=P, yf=P, post=P, x_out=2 * P, gain=P, res=P) == -2  # routers only with kind 4
     assert lib.aqs_delta_scan(P, P, P, P, P, P, P, P, P, 1, 4, 3, 2, 8, 8, None) == -2                       # heads over kv heads
     assert lib.aqs_delta_scan(P, P, P, P, P, P, P, P, P, 1, 4, 2, 2, 257, 8, None) == -6
-    assert lib.aqs_ssd_scan(P, P, 2, 1, P, P, P, P, P, P, P, 0, 4, 2, 2, 8, 8, None) == 0                    # nothing to do
+    assert lib.aqs_ssd_scan(P, P, 2, 1, P, P, P, None, P, P, P, P, 0, 4, 2, 2, 8, 8, None) == 0              # nothing to do
+    assert lib.aqs_ssd_scan(P, P, 0, 1, None, None, None, P, P, P, P, P, 0, 4, 2, 2, 8, 8, None) == 0        # constant decays need no steps
+    assert lib.aqs_ssd_scan(P, P, 0, 1, None, None, None, None, P, P, P, P, 1, 4, 2, 2, 8, 8, None) == -2
     assert lib.aqs_attn_window_ok(1, 24, 40, 64) == 1 and lib.aqs_attn_window_ok(0, 24, 40, 64) == 0
     assert lib.aqs_attn_window_ok(1, 20, 40, 64) == 0 and lib.aqs_attn_window_ok(1, 24, 40, 16) == 0
     for window in (1, 2, 63, 64, 65, 127, 128, 129, 300):

@@ -109,8 +109,8 @@ def parse():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=200)
     ap.add_argument("--warmup", type=int, default=1000)
-    ap.add_argument("--workload", default="decode", choices=["decode", "prefill", "fp8", "block", "model", "hybrid"])
-    ap.add_argument("--width", type=int, default=None, help="hybrid workload only: one model width (1024, 2048 or 4096) instead of all")
+    ap.add_argument("--workload", default="decode", choices=["decode", "prefill", "fp8", "block", "model", "hybrid", "lomozen"])
+    ap.add_argument("--width", type=int, default=None, help="hybrid and lomozen workloads only: one model width (1024, 2048 or 4096) instead of all")
     ap.add_argument("--m", type=int, default=16, help="decode rows (1..16)")
     ap.add_argument("--mnk", default=None, help="prefill and fp8 workloads only: M,N,K of the int8 Linear instead of configuration 3's "
                     "4096,2048,2048 (e.g. 8192,8192,8192 for a profile of the GEMM's steady state)")
@@ -668,26 +668,69 @@ def hybrid_config(width):
     return {"architecture": "Rudilix", "layers": layers, "norm": {"eps": 1e-6}, "residual_mult": 0.5, "vocab": 10000, "width": width}, shapes
 
 
+def random_hybrid(m):
+    plain = m.config.design.norm_offset == 0.0
+    for name, t in m.tensors().items():
+        if name.endswith(("A_log", "dt_bias")):
+            t.normal_(-1.0, 0.5)
+        elif name.endswith("norm") and not name.startswith("final"):
+            t.fill_(1.0)
+        elif t.dim() == 2:
+            t.normal_(0.0, t.shape[1] ** -0.5)
+        elif plain:
+            t.fill_(1.0)
+    return m
+
+
+def engine_rates(torch, m, ids, gen, page):
+    """Milliseconds of one prompt (eager launches) and, behind it, of a decode step of 1 and of 4 sequences (replays of the
+    captured step; and whole calls of Engine.step with their host work)."""
+    from khaosz_amd import Engine
+
+    S, r = len(ids), {}
+    e = Engine(m, S + 2 * gen, 1, page)
+
+    def prefill(i=0):
+        h = e.open()
+        e.step([h], [ids], [S - 1])
+        e.close(h)
+    r["prefill_ms"] = eager_time_ms(torch, prefill, 5, 2)
+    for B in (1, 4):
+        e = Engine(m, B * (S + gen), B, page)
+        hs = [e.open() for _ in range(B)]
+        for h in hs:
+            e.step([h], [ids], [])
+        for _ in range(3):
+            e.step(hs, [[7 + 3 * i] for i in range(B)])
+        g = e._graphs[B].graph
+        r[f"decode_ms_b{B}"] = eager_time_ms(torch, lambda i=0: g.replay(), 50, 5)
+        t0 = time.perf_counter()
+        for _ in range(gen - 8):
+            e.step(hs, [[7 + 3 * i] for i in range(B)])
+        torch.cuda.synchronize()
+        r[f"engine_step_ms_b{B}"] = (time.perf_counter() - t0) * 1e3 / (gen - 8)
+        del e, g
+    return r
+
+
+def add_rates(d, S):
+    d["prefill_tok_s"] = S / (d["prefill_ms"] * 1e-3)
+    d["decode_tok_s_b1"], d["decode_tok_s_b4"] = 1e3 / d["decode_ms_b1"], 4e3 / d["decode_ms_b4"]
+
+
 def bench_hybrid(torch, ops, args, dev):
     """Prefill and decode throughput of the hybrid decoder (Rudilix: 4 state-space, 2 delta and 2 attention + delta
     layers, bf16, random weights) beside AutoRegressiveLM of the same width, depth, feed-forward and vocabulary, in
     bf16 (stock torch around float Linears) and in W8A8 with every fusion.  Prefill: one prompt, eager launches.
     Decode: after that prompt, HIP graph replays of one step."""
-    from khaosz_amd import AutoRegressiveLM, Engine, HybridConfig, HybridLM, LMConfig, fuse_shared_inputs, quantize_model
+    from khaosz_amd import AutoRegressiveLM, HybridConfig, HybridLM, LMConfig, fuse_shared_inputs, quantize_model
 
     dt, out, page, gen = torch.bfloat16, {}, 64, 32
     widths = [args.width] if args.width else [1024, 2048, 4096]
     for width in widths:
         cfg, shapes = hybrid_config(width)
         torch.manual_seed(5)
-        m = HybridLM(HybridConfig.from_dict(cfg, shapes), dt, dev).eval()
-        for name, t in m.tensors().items():
-            if name.endswith(("A_log", "dt_bias")):
-                t.normal_(-1.0, 0.5)
-            elif name.endswith("norm") and not name.startswith("final"):
-                t.fill_(1.0)
-            elif t.dim() == 2:
-                t.normal_(0.0, t.shape[1] ** -0.5)
+        m = random_hybrid(HybridLM(HybridConfig.from_dict(cfg, shapes), dt, dev).eval())
         weight_bytes = sum(p.numel() * p.element_size() for p in m.parameters()) - m.embed.numel() * 2
         ar_cfg = LMConfig(vocab_size=10000, dim=width, n_layers=8, n_heads=width // 128, n_kv_heads=max(width // 512, 1),
                           dim_ffn=width * 11 // 4, max_len=4096 + 2 * gen)
@@ -698,28 +741,7 @@ def bench_hybrid(torch, ops, args, dev):
         row = {"hybrid_weight_bytes": weight_bytes}
         for S in (512, 4096):
             ids = torch.randint(0, 10000, (1, S), generator=torch.Generator().manual_seed(S)).tolist()[0]
-            e = Engine(m, S + 2 * gen, 1, page)
-
-            def prefill(i=0):
-                h = e.open()
-                e.step([h], [ids], [S - 1])
-                e.close(h)
-            r = {"hybrid": {"prefill_ms": eager_time_ms(torch, prefill, 5, 2)}}
-            for B in (1, 4):
-                e = Engine(m, B * (S + gen), B, page)
-                hs = [e.open() for _ in range(B)]
-                for h in hs:
-                    e.step([h], [ids], [])
-                for _ in range(3):
-                    e.step(hs, [[7]] * B)
-                g = e._graphs[B].graph
-                r["hybrid"][f"decode_ms_b{B}"] = eager_time_ms(torch, lambda i=0: g.replay(), 50, 5)
-                t0 = time.perf_counter()
-                for _ in range(gen - 8):
-                    e.step(hs, [[7]] * B)
-                torch.cuda.synchronize()
-                r["hybrid"][f"engine_step_ms_b{B}"] = (time.perf_counter() - t0) * 1e3 / (gen - 8)
-                del e
+            r = {"hybrid": engine_rates(torch, m, ids, gen, page)}
             P = (S + gen + page - 1) // page
             for name, mod in (("ar_bf16", ar), ("ar_w8a8", arq)):
                 r[name] = {}
@@ -737,8 +759,7 @@ def bench_hybrid(torch, ops, args, dev):
                         torch, lambda i=0: mod(one, paged_cache=c.bind(table, S + 1), start_pos=S), 20, 5)
                     del c
             for d in r.values():
-                d["prefill_tok_s"] = S / (d["prefill_ms"] * 1e-3)
-                d["decode_tok_s_b1"], d["decode_tok_s_b4"] = 1e3 / d["decode_ms_b1"], 4e3 / d["decode_ms_b4"]
+                add_rates(d, S)
             row[f"prompt_{S}"] = r
         out[f"width_{width}"] = row
         del m, ar, arq
@@ -749,6 +770,53 @@ def bench_hybrid(torch, ops, args, dev):
                         "prefill of one prompt, decode of 1 and 4 sequences",
             "value": w["prompt_4096"]["hybrid"]["decode_tok_s_b1"], "unit": "tok/s", "ms_per_step": ms, "dtype": "bf16",
             "widths": out,
+            "roofline": {"bound": "hbm", "kernel": "one decode step of one sequence (weights read once)", "achieved": gbs,
+                         "peak": PEAK_HBM_GBS, "unit": "GB/s", "frac": gbs / PEAK_HBM_GBS, "traffic": None},
+            "shape": (1, 0, 0)}
+
+
+def lomozen_config(width):
+    """A Lomozen decoder of a real model's layer sizes: 128-wide heads that fill the width, latents of 3/4 of the width and of
+    512, a 1024-token window, 64 experts of which a token uses 4, as much active feed-forward as hybrid_config."""
+    h, ff = width // 128, width * 11 // 32
+    mlp = {"kind": "moe", "router": {"experts": 64, "top": 4}, "expert": {"ff": ff}, "shared": {"ff": 4 * ff}}
+    light = {"type": "lightning", "mlp": mlp, "mixer": {"heads": h, "dim": 128, "vdim": 128, "decay": [1 - 2.0 ** -(1 + 8 * (i + 1) / h) for i in range(h)]}}
+    latent = {"type": "latent_attention", "mlp": mlp, "mixer": {
+        "heads": h, "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": width * 3 // 4, "kv_rank": 512, "mask": {"size": 1024}, "scale": 192 ** -0.5,
+        "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    return {"architecture": "Lomozen", "layers": [light, latent] * 4, "norm": {"eps": 1e-6}, "vocab": 10000, "width": width}
+
+
+def bench_lomozen(torch, ops, args, dev):
+    """Prefill and decode throughput of the Lomozen decoder (4 lightning and 4 latent attention layers, 64 experts, bf16,
+    random weights) beside the Rudilix hybrid of the same width, depth, active feed-forward and vocabulary."""
+    from khaosz_amd import HybridConfig, HybridLM
+
+    dt, out, page, gen = torch.bfloat16, {}, 64, 32
+    widths = [args.width] if args.width else [1024, 2048, 4096]
+    for width in widths:
+        row = {}
+        for name, (cfg, shapes) in (("lomozen", (lomozen_config(width), None)), ("rudilix", hybrid_config(width))):
+            torch.manual_seed(5)
+            m = random_hybrid(HybridLM(HybridConfig.from_dict(cfg, shapes), dt, dev).eval())
+            read = sum(p.numel() * p.element_size() for n, p in m.named_parameters() if n != "embed")
+            for l in m.layers:  # a step of one sequence reads the chosen experts only
+                if hasattr(l.mlp, "Ex"):
+                    read -= 2 * (l.mlp.gate_up.numel() + l.mlp.down.numel()) * (l.mlp.Ex - l.mlp.top) // l.mlp.Ex
+            row[name] = {"weight_bytes_read_by_a_step": read}
+            for S in (512, 4096):
+                ids = torch.randint(0, 10000, (1, S), generator=torch.Generator().manual_seed(S)).tolist()[0]
+                r = engine_rates(torch, m, ids, gen, page)
+                add_rates(r, S)
+                row[name][f"prompt_{S}"] = r
+            del m
+        out[f"width_{width}"] = row
+    w = out[f"width_{widths[-1] if len(widths) < 3 else 2048}"]["lomozen"]
+    ms = w["prompt_4096"]["decode_ms_b1"]
+    gbs = w["weight_bytes_read_by_a_step"] / (ms * 1e-3) / 1e9
+    return {"workload": "Lomozen decoder (8 layers, 64 experts, bf16, random weights) beside the Rudilix hybrid of equal size: prefill of one "
+                        "prompt, decode of 1 and 4 sequences",
+            "value": w["prompt_4096"]["decode_tok_s_b1"], "unit": "tok/s", "ms_per_step": ms, "dtype": "bf16", "widths": out,
             "roofline": {"bound": "hbm", "kernel": "one decode step of one sequence (weights read once)", "achieved": gbs,
                          "peak": PEAK_HBM_GBS, "unit": "GB/s", "frac": gbs / PEAK_HBM_GBS, "traffic": None},
             "shape": (1, 0, 0)}
@@ -993,13 +1061,13 @@ def main():
     dev = torch.device("cuda:0")
     torch.cuda.set_device(dev)
     fns = {"decode": bench_decode, "prefill": bench_prefill, "fp8": bench_fp8, "block": bench_block,
-           "model": bench_model, "hybrid": bench_hybrid}
+           "model": bench_model, "hybrid": bench_hybrid, "lomozen": bench_lomozen}
     with torch.inference_mode():
         # the part's own ceilings first: the roofline objects of the workloads quote them
         CEIL.update(measure_ceilings(torch, ops, dev, calibrate=False))
         main_res = fns[args.workload](torch, ops, args, dev)
         extra = {}
-        if not args.no_extra and args.workload != "hybrid":
+        if not args.no_extra and args.workload not in ("hybrid", "lomozen"):
             for name in ("decode", "prefill", "fp8", "block"):  # "model" only on request: it takes a minute
                 if name != args.workload:
                     extra[name] = fns[name](torch, ops, args, dev)
@@ -1011,9 +1079,9 @@ def main():
                     extra[f"decode_m{m}"] = r
                 extra["batch_32_to_256"] = bench_few_dozen_rows(torch, ops, args, dev)
         ceilings = dict(CEIL)
-        if not args.no_extra and args.workload != "hybrid":  # launches GEMMs of other shapes: left out of single-workload (profiling) runs
+        if not args.no_extra and args.workload not in ("hybrid", "lomozen"):  # launches GEMMs of other shapes: left out of single-workload (profiling) runs
             ceilings["gemm_operand_data_and_stock_library"] = gemm_calibration(torch, ops, dev)
-        if not args.no_extra and args.workload not in ("model", "hybrid"):
+        if not args.no_extra and args.workload not in ("model", "hybrid", "lomozen"):
             # the reference's own generation benchmark: about a minute; skipped when this run is already long
             if time.time() - t_start < 150:
                 m = bench_model(torch, ops, args, dev)
@@ -1025,7 +1093,7 @@ def main():
                 extra["model"] = {"skipped": "time budget of the default run spent"}
     per_step = main_res.get("bytes_per_step") or main_res.get("ops_per_step") or main_res.get("flops_per_step")
     cpu = None
-    if not args.no_cpu and args.workload not in ("block", "model", "hybrid"):
+    if not args.no_cpu and args.workload not in ("block", "model", "hybrid", "lomozen"):
         cpu = cpu_baseline(args.workload, main_res["shape"], main_res["unit"], per_step)
         if not args.no_extra and "prefill" in extra:
             # one pass of the prefill shape as well, so both halves of the metric have a CPU figure
@@ -1034,7 +1102,7 @@ def main():
     for r in [main_res, *extra.values()]:
         r.pop("shape", None)
     top = ("workload", "value", "unit", "ms_per_step", "dtype", "roofline", "eager_ms_per_step")
-    detail = {k: v for k, v in main_res.items() if k not in top} if args.workload in ("block", "model", "hybrid") else None
+    detail = {k: v for k, v in main_res.items() if k not in top} if args.workload in ("block", "model", "hybrid", "lomozen") else None
     line = {
         "metric": METRIC, "value": main_res["value"], "unit": main_res["unit"], "n_gpus": 1,
         "steps": args.steps, "warmup": args.warmup, "ms_per_step": main_res["ms_per_step"],

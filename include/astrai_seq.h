@@ -168,16 +168,17 @@ int aqs_latent_decode(const void *proj, int64_t ld, int64_t o_kv, int64_t o_gate
 /* The `top` best of Ex experts of every row of h: ids and scores [M, top]. */
 int aqs_moe_route(const void *h, int64_t ldh, int dtype, const void *w, int32_t *ids, float *scores, int64_t M, int64_t K, int64_t Ex,
                   int64_t top, void *stream);
-/* Slots per tile for A choices among Ex experts of width K and inner size F; the number of tiles to make room for. */
+/* Slots per tile for A choices among Ex experts of width K and inner size F; rows of `tiles` to make room for. */
 int64_t aqs_moe_tile(int dtype, int64_t A, int64_t Ex, int64_t K, int64_t F);
 int64_t aqs_moe_tiles(int64_t A, int64_t Ex, int64_t tile);
-/* A choices (ids) by expert: rows[slot] = choice, slots[choice] = slot, tiles [n_tiles, 4] = expert (-1: none), first slot, slots. */
+/* A choices (ids) by expert: rows[slot] = choice, slots[choice] = slot; tiles [n_tiles, 4]: how many there are, then expert, first
+ * slot and number of slots of each. */
 int aqs_moe_sort(const int32_t *ids, int64_t A, int64_t Ex, int64_t tile, int32_t *rows, int32_t *slots, int32_t *tiles,
                  int64_t n_tiles, void *stream);
 /* glu != 0: x by token [., ldx], w [Ex, N = 2F, K] = gate | up, out [A, F] = silu(s gate) * (s up); 0: x by slot [A, ldx],
  * w [Ex, N, K], out [A, N]. */
 int aqs_moe_product(int glu, const void *x, int64_t ldx, int dtype, const void *w, const int32_t *tiles, int64_t n_tiles, int64_t tile,
-                    const int32_t *rows, const float *scores, int64_t top, void *out, int64_t N, int64_t K, void *stream);
+                    const int32_t *rows, const float *scores, int64_t A, int64_t top, void *out, int64_t N, int64_t K, void *stream);
 /* A step of up to 8 tokens from the router's logits z [M, Ex]: act [M * top, F] of the chosen experts (w [Ex, 2F, K]), then
  * y [M, N] fp32 = sum of their down projections (w [Ex, N, F]) and of the shared expert's (sact [M, Fs], sw [N, Fs]; Fs 0: none). */
 int aqs_moe_step_ok(int64_t M, int64_t N, int64_t F, int64_t Fs, int64_t Ex, int64_t top);

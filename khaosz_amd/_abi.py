@@ -143,7 +143,8 @@ SEQ_SYMBOLS = {
     "aqs_moe_tile": (_i64, [_int, _i64, _i64, _i64, _i64]),
     "aqs_moe_tiles": (_i64, [_i64, _i64, _i64]),
     "aqs_moe_sort": (_int, [_vp, _i64, _i64, _i64, _vp, _vp, _vp, _i64, _vp]),
-    "aqs_moe_product": (_int, [_int, _vp, _i64, _int, _vp, _vp, _i64, _i64, _vp, _vp, _i64, _vp, _i64, _i64, _vp]),
+    "aqs_moe_product": (_int, [_int, _vp, _i64, _int, _vp, _vp, _i64, _i64, _vp, _vp, _i64, _i64, _vp, _i64, _i64,
+        _vp]),
     "aqs_moe_step_ok": (_int, [_i64, _i64, _i64, _i64, _i64, _i64]),
     "aqs_moe_step_up": (_int, [_vp, _vp, _int, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _vp]),
     "aqs_moe_step_down": (_int, [_vp, _vp, _int, _vp, _vp, _vp, _vp, _i64, _i64, _i64, _i64, _i64, _i64, _vp]),

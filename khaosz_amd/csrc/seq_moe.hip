@@ -106,8 +106,8 @@ __global__ __launch_bounds__(256) void route_any_kernel(RouteArgs p, const T* h,
 }
 
 // bf16 on the matrix cores: 16 tokens per workgroup, every wavefront all experts over a quarter of the contraction (steps
-// of 32 in turn).  NT: tiles of 16 experts.
-template <int NT>
+// of 32 in turn).  NT: tiles of 16 experts; KU: steps whose operands are requested together.
+template <int NT, int KU>
 __global__ __launch_bounds__(256) void route_mfma_kernel(RouteArgs p, const uint16_t* h, const uint16_t* w) {
   constexpr int ZP = NT * 16 + 4;
   __shared__ __align__(16) float z_s[4][16][ZP];
@@ -120,14 +120,21 @@ __global__ __launch_bounds__(256) void route_mfma_kernel(RouteArgs p, const uint
   f32x4 acc[NT];
 #pragma unroll
   for (int t = 0; t < NT; ++t) acc[t] = f32x4{0, 0, 0, 0};
-  for (int k0 = wave * 32; k0 < p.K; k0 += 128) {
-    const int k = k0 + q * 8, kc = k < p.K ? k : 0;
-    uint4 x = *reinterpret_cast<const uint4*>(hr + kc);
-    if (k >= p.K) x = make_uint4(0, 0, 0, 0);
+  for (int k0 = wave * 32; k0 < p.K; k0 += 128 * KU) {
+    uint4 x[KU], v[KU][NT];
 #pragma unroll
-    for (int t = 0; t < NT; ++t) {
-      const uint4 v = *reinterpret_cast<const uint4*>(wr[t] + kc);
-      acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v), __builtin_bit_cast(bf16x8, x), acc[t], 0, 0, 0);
+    for (int u = 0; u < KU; ++u) {
+      const int k = k0 + u * 128 + q * 8, kc = k < p.K ? k : 0;
+      x[u] = *reinterpret_cast<const uint4*>(hr + kc);
+#pragma unroll
+      for (int t = 0; t < NT; ++t) v[u][t] = *reinterpret_cast<const uint4*>(wr[t] + kc);
+    }
+#pragma unroll
+    for (int u = 0; u < KU; ++u) {
+      if (k0 + u * 128 + q * 8 >= p.K) x[u] = make_uint4(0, 0, 0, 0);
+#pragma unroll
+      for (int t = 0; t < NT; ++t)
+        acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v[u][t]), __builtin_bit_cast(bf16x8, x[u]), acc[t], 0, 0, 0);
     }
   }
   // column r16: token; rows 4 q + r: experts
@@ -150,34 +157,41 @@ __global__ __launch_bounds__(256) void route_mfma_kernel(RouteArgs p, const uint
 }
 
 // ---------------------------------------------------------------------------------------------- prompts: sorting
-// One workgroup per expert scans all A choices: how many belong to lower experts gives its first slot, a second pass
-// writes its own.  rows[slot] = choice (token * top + j), slots[choice] = slot.  Expert e's tiles of TM slots are numbered
-// from off / TM + e on, which leaves every expert room for its own; unused numbers are marked with expert -1.
+// One workgroup per expert counts all A choices by expert, which gives its first slot and its first tile; a second pass
+// writes its own: rows[slot] = choice (token * top + j), slots[choice] = slot.  tiles[0].x = number of tiles, tiles[1 ..] =
+// (expert, first slot, slots of the tile, -).
 constexpr int SORT_WAVES = 16;
 
 __global__ __launch_bounds__(SORT_WAVES * 64) void moe_sort_kernel(const int* ids, int A, int Ex, int TM, int* rows, int* slots,
                                                                   int4* tiles, int n_tiles) {
-  __shared__ int own_s[SORT_WAVES], low_s[SORT_WAVES];
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, e = blockIdx.x;
+  __shared__ int own_s[SORT_WAVES], count_s[MAX_EXPERTS];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, e = blockIdx.x;
+  for (int i = tid; i < Ex; i += SORT_WAVES * 64) count_s[i] = 0;
+  __syncthreads();
   const int per = ((A + SORT_WAVES - 1) / SORT_WAVES + 63) / 64 * 64, i0 = wave * per, i1 = i0 + per < A ? i0 + per : A;
-  int own = 0, low = 0;
+  int own = 0;
 #pragma unroll 4
   for (int i = i0 + lane; i < i1; i += 64) {
     const int id = ids[i];
     own += id == e;
-    low += id < e;
+    atomicAdd(&count_s[id], 1);
   }
 #pragma unroll
-  for (int o = 32; o; o >>= 1) own += __shfl_xor(own, o, 64), low += __shfl_xor(low, o, 64);
-  if (lane == 0) own_s[wave] = own, low_s[wave] = low;
+  for (int o = 32; o; o >>= 1) own += __shfl_xor(own, o, 64);
+  if (lane == 0) own_s[wave] = own;
   __syncthreads();
-  int off = 0, cnt = 0, at = 0;
-  for (int w = 0; w < SORT_WAVES; ++w) {
-    off += low_s[w];
-    at += w < wave ? own_s[w] : 0;
-    cnt += own_s[w];
+  int off = 0, t0 = 0, total = 0;  // every wavefront sums for itself
+  for (int i = lane; i < Ex; i += 64) {
+    const int c = count_s[i], t = (c + TM - 1) / TM;
+    off += i < e ? c : 0;
+    t0 += i < e ? t : 0;
+    total += t;
   }
-  at += off;
+#pragma unroll
+  for (int o = 32; o; o >>= 1) off += __shfl_xor(off, o, 64), t0 += __shfl_xor(t0, o, 64), total += __shfl_xor(total, o, 64);
+  const int cnt = count_s[e];
+  int at = off;
+  for (int w = 0; w < wave; ++w) at += own_s[w];
   for (int ib = i0; ib < i1; ib += 64) {
     const int i = ib + lane;
     const bool mine = i < i1 && ids[i] == e;
@@ -189,19 +203,17 @@ __global__ __launch_bounds__(SORT_WAVES * 64) void moe_sort_kernel(const int* id
     }
     at += __popcll(b);
   }
-  const int t0 = off / TM + e, mine = (cnt + TM - 1) / TM, t1 = e + 1 < Ex ? (off + cnt) / TM + e + 1 : n_tiles;
-  for (int t = t0 + (int)threadIdx.x; t < t1 && t < n_tiles; t += SORT_WAVES * 64) {
-    const int first = off + (t - t0) * TM, n = off + cnt - first;
-    tiles[t] = t - t0 < mine ? make_int4(e, first, n < TM ? n : TM, 0) : make_int4(-1, 0, 0, 0);
-  }
+  if (e == 0 && tid == 0) tiles[0] = make_int4(total, 0, 0, 0);
+  for (int t = tid; t * TM < cnt && 1 + t0 + t < n_tiles; t += SORT_WAVES * 64)
+    tiles[1 + t0 + t] = make_int4(e, off + t * TM, cnt - t * TM < TM ? cnt - t * TM : TM, 0);
 }
 
 // ---------------------------------------------------------------------------------------------- prompts: grouped products
 struct GroupArgs {
-  const int4* tiles;    // (expert or -1, first slot, slots, -)
+  const int4* tiles;    // [0].x: how many; [1 ..]: (expert, first slot, slots, -)
   const int* rows;      // slot -> choice
   const float* scores;  // by choice (GLU)
-  int64_t ldx;
+  int64_t ldx, x_bytes; // x_bytes: extent of x's rows (matrix cores)
   int top, N, K;        // GLU: N = 2 F weight rows per expert, gate | up
 };
 
@@ -212,8 +224,8 @@ __global__ __launch_bounds__(256) void grouped_any_kernel(GroupArgs p, const T* 
   __shared__ float x_s[BK][TM + 4], w_s[BK][64 + 4];
   __shared__ int64_t src_s[TM];
   __shared__ float sc_s[TM];
-  const int4 tile = p.tiles[blockIdx.y];
-  if (tile.x < 0) return;  // uniform
+  if ((int)blockIdx.y >= p.tiles[0].x) return;  // uniform
+  const int4 tile = p.tiles[1 + blockIdx.y];
   const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4, F = GLU ? p.N / 2 : p.N;
   const int f0 = blockIdx.x * (GLU ? 32 : 64);
   if (tid < TM) {
@@ -261,97 +273,131 @@ __global__ __launch_bounds__(256) void grouped_any_kernel(GroupArgs p, const T* 
 }
 
 // bf16 on the matrix cores.  Weights are the left operand (32 of them per accumulator's rows), slots the right one, so that a
-// lane ends with four consecutive outputs of one slot.  A workgroup of 4 wavefronts, WM of them along the slots; a
-// wavefront has 2 tiles of 32 weight rows (GLU: gate and up rows of the same outputs) and MT of 32 slots.
-constexpr int GK = 64, GP = GK + 8;  // contraction per stage, row stride in LDS
+// lane ends with four consecutive outputs of one slot.  WW x WT wavefronts, each with 2 tiles of 32 weight rows (GLU: the
+// gate and the up rows of the same 32 outputs) and JT of 32 slots.  The contraction is walked in steps of 64 through NS
+// stages in LDS, filled by direct global->LDS loads: a load brings 8 rows of 128 bytes, whose 16-byte pieces are permuted
+// (piece c of row r in place c ^ (r / 2) % 8) so that 16 rows' reads of one piece meet no bank twice.
+template <int WW_, int WT_, int JT_, int NS_>
+struct GroupShape {
+  static constexpr int WW = WW_, WT = WT_, JT = JT_, NS = NS_, NW = WW * WT, THREADS = NW * 64;
+  static constexpr int WROWS = WW * 64, TROWS = WT * JT * 32, STAGE = (WROWS + TROWS) * 128;
+  static constexpr int W_LOADS = WROWS / 8 / NW, T_LOADS = TROWS / 8 / NW, LOADS = W_LOADS + T_LOADS;
+  static_assert(NW % 2 == 0, "a wavefront's rows of all its loads are permuted alike");
+  static_assert(TROWS % (8 * NW) == 0 && NS * STAGE <= 160 * 1024 && (NS - 1) * LOADS < 64, "whole loads, LDS, counter");
+};
+using GroupWide = GroupShape<4, 2, 2, 3>;    // 256 weight rows x 128 slots
+using GroupNarrow = GroupShape<2, 1, 1, 4>;  // 128 weight rows x 32 slots: weights stream by
 
-template <int WM, int MT, bool GLU>
-__global__ __launch_bounds__(256) void grouped_mfma_kernel(GroupArgs p, const uint16_t* x, const uint16_t* w, uint16_t* out) {
-  constexpr int WN = 4 / WM, TM = WM * MT * 32, TN = WN * 64, XC = TM / 32, WC = TN / 32;
-  extern __shared__ __align__(16) uint16_t lds[];  // 2 stages of TM + TN rows
-  const int4 tile = p.tiles[blockIdx.y];
-  if (tile.x < 0) return;  // uniform
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, wm = wave % WM, wn = wave / WM;
+typedef __attribute__((address_space(3))) void lds_void;
+// until at most n vector loads are on their way, and no LDS read
+#define SQ_WAIT_VM_LDS(n) __builtin_amdgcn_s_waitcnt(0x0070 | ((n) & 15) | (((n) >> 4) << 14))
+// a workgroup barrier without the fence of __syncthreads(), which would wait for the loads of later stages
+#define SQ_RAW_BARRIER()           \
+  do {                             \
+    asm volatile("" ::: "memory"); \
+    __builtin_amdgcn_s_barrier();  \
+    asm volatile("" ::: "memory"); \
+  } while (0)
+constexpr uint32_t GROUP_OOB = 0x7ffffff0u;  // beyond every descriptor: reads zero
+
+template <class G, bool GLU>
+__device__ __forceinline__ void grouped_tile(const GroupArgs& p, const uint16_t* x, const uint16_t* w, uint16_t* out, uint8_t* smem) {
+  // consecutive workgroups go to different XCDs: number them so that each XCD takes a run of tiles, outputs first
+  const int cols = (int)gridDim.x, total = cols * p.tiles[0].x, pid = blockIdx.y * cols + blockIdx.x;
+  if (pid >= total) return;  // uniform
+  const int per = total / 8, rem = total % 8, xcd = pid % 8, id = xcd * per + (xcd < rem ? xcd : rem) + pid / 8;
+  const int4 tile = p.tiles[1 + id / cols];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), ww = wave % G::WW, wt = wave / G::WW;
   const int col = lane & 31, g2 = lane >> 5, F = GLU ? p.N / 2 : p.N, K = p.K;
-  const int f0 = blockIdx.x * (GLU ? TN / 2 : TN);
-  const int lr = tid >> 3, lc = (tid & 7) * 8;  // this thread's row (of every 32) and column in a stage
-  const uint16_t* xp[XC];
-  const uint16_t* wp[WC];
+  const int f0 = id % cols * (GLU ? G::WROWS / 2 : G::WROWS);
+  const __amdgpu_buffer_rsrc_t Wr =
+      __builtin_amdgcn_make_buffer_rsrc(const_cast<uint16_t*>(w + (int64_t)tile.x * p.N * K), 0, (int)((int64_t)p.N * K * 2), 0x00020000);
+  const __amdgpu_buffer_rsrc_t Xr = __builtin_amdgcn_make_buffer_rsrc(const_cast<uint16_t*>(x), 0, (int)p.x_bytes, 0x00020000);
+  // this lane's row of every load, and its piece of it
+  const int lr = wave * 8 + lane / 8, piece = ((lane % 8) ^ (lr / 2 % 8)) * 16;
+  uint32_t wo[G::W_LOADS], xo[G::T_LOADS];
 #pragma unroll
-  for (int i = 0; i < XC; ++i) {
-    const int r = i * 32 + lr, s = tile.y + (r < tile.z ? r : 0);
-    xp[i] = x + (int64_t)(GLU ? p.rows[s] / p.top : s) * p.ldx + lc;
+  for (int i = 0; i < G::W_LOADS; ++i) {
+    const int r = i * 8 * G::NW + lr, n = f0 + (GLU ? r / 64 * 32 + r % 32 : r);
+    wo[i] = n < F ? (uint32_t)(GLU && (r & 32) ? n + F : n) * (uint32_t)K * 2 + piece : GROUP_OOB;
   }
-  const uint16_t* we = w + (int64_t)tile.x * p.N * K + lc;
 #pragma unroll
-  for (int i = 0; i < WC; ++i) {
-    // GLU: rows of 64 alternate 32 gate and 32 up rows, a wavefront's two tiles
-    int n = f0 + (GLU ? i / 2 * 32 : i * 32) + lr;
-    n = n < F ? n : F - 1;
-    wp[i] = we + (int64_t)(GLU && (i & 1) ? n + F : n) * K;
+  for (int i = 0; i < G::T_LOADS; ++i) {
+    const int r = i * 8 * G::NW + lr, s = tile.y + (r < tile.z ? r : 0);
+    xo[i] = r < tile.z ? (uint32_t)(GLU ? p.rows[s] / p.top : s) * (uint32_t)(p.ldx * 2) + piece : GROUP_OOB;
   }
-  uint4 xr[XC], wr[WC];
-  auto fetch = [&](int k0) __attribute__((always_inline)) {
-    const bool ok = k0 + lc < K;
-    const int k = ok ? k0 : 0;
+  const int nk = (K + 63) / 64;
+  auto fetch = [&](int kt) __attribute__((always_inline)) {
+    uint8_t* st = smem + kt % G::NS * G::STAGE + wave * 1024;
+    const uint32_t k0 = (uint32_t)kt * 128;
+    const bool ok = (int)k0 + piece < K * 2;  // past the end, zeros: the number of loads in flight stays the same
 #pragma unroll
-    for (int i = 0; i < XC; ++i) {
-      xr[i] = *reinterpret_cast<const uint4*>(xp[i] + (ok ? k : -lc));
-      if (!ok) xr[i] = make_uint4(0, 0, 0, 0);
-    }
+    for (int i = 0; i < G::W_LOADS; ++i)
+      __builtin_amdgcn_raw_ptr_buffer_load_lds(Wr, (lds_void*)(st + i * 1024 * G::NW), 16, ok ? wo[i] + k0 : GROUP_OOB, 0, 0, 0);
 #pragma unroll
-    for (int i = 0; i < WC; ++i) wr[i] = *reinterpret_cast<const uint4*>(wp[i] + (ok ? k : -lc));
+    for (int i = 0; i < G::T_LOADS; ++i)
+      __builtin_amdgcn_raw_ptr_buffer_load_lds(Xr, (lds_void*)(st + G::WROWS * 128 + i * 1024 * G::NW), 16, ok ? xo[i] + k0 : GROUP_OOB, 0, 0, 0);
   };
-  auto stage = [&](int buf) __attribute__((always_inline)) {
-    uint16_t* xs = lds + buf * (TM + TN) * GP;
-    uint16_t* ws = xs + TM * GP;
-#pragma unroll
-    for (int i = 0; i < XC; ++i) *reinterpret_cast<uint4*>(&xs[(i * 32 + lr) * GP + lc]) = xr[i];
-#pragma unroll
-    for (int i = 0; i < WC; ++i) *reinterpret_cast<uint4*>(&ws[(i * 32 + lr) * GP + lc]) = wr[i];
-  };
-  f32x16 acc[2][MT];
+  f32x16 acc[2][G::JT];
 #pragma unroll
   for (int i = 0; i < 2; ++i)
 #pragma unroll
-    for (int j = 0; j < MT; ++j)
+    for (int j = 0; j < G::JT; ++j)
 #pragma unroll
       for (int r = 0; r < 16; ++r) acc[i][j][r] = 0.0f;
-  fetch(0);
-  stage(0);
-  __syncthreads();
-  int buf = 0;
-  for (int k0 = 0; k0 < K; k0 += GK, buf ^= 1) {
-    const bool more = k0 + GK < K;
-    if (more) fetch(k0 + GK);
-    const uint16_t* xs = lds + buf * (TM + TN) * GP + (wm * MT * 32 + col) * GP + g2 * 8;
-    const uint16_t* ws = lds + buf * (TM + TN) * GP + (TM + wn * 64 + col) * GP + g2 * 8;
+  // Fragments are read a quarter of a stage ahead of their products.  When the last quarter's are in registers (and the
+  // next stage has landed), a barrier frees the stage for the loads of the one NS later.
+  const int fw = (ww * 64 + col) * 128, fx = (G::WROWS + wt * G::JT * 32 + col) * 128, turn = col / 2 % 8;
+  bf16x8 a[2][2], b[2][G::JT];
+  auto read = [&](int s, int kk, int f, int to) __attribute__((always_inline)) {  // fragment f: 0, 1 of the weights, then slots
+    const uint8_t* st = smem + s % G::NS * G::STAGE + ((kk * 2 + g2) ^ turn) * 16;
+    if (f < 2) a[to][f] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(st + fw + f * 32 * 128));
+    else b[to][f - 2] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(st + fx + (f - 2) * 32 * 128));
+  };
 #pragma unroll
-    for (int kk = 0; kk < GK / 16; ++kk) {
-      bf16x8 a[2], b[MT];
+  for (int s = 0; s < G::NS; ++s) fetch(s);
+  SQ_WAIT_VM_LDS((G::NS - 1) * G::LOADS);
+  SQ_RAW_BARRIER();
+  // JN: the wavefront's tiles that hold slots at all
+  auto run = [&](auto tag) __attribute__((always_inline)) {
+    constexpr int JN = decltype(tag)::value, NF = JN ? 2 + JN : 0, NM = JN ? 2 * JN : 1;
+    auto quarter = [&](int from, int s, int kk) __attribute__((always_inline)) {  // products; the fragments of (s, kk) read beside
 #pragma unroll
-      for (int i = 0; i < 2; ++i) a[i] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(ws + i * 32 * GP + kk * 16));
+      for (int m = 0; m < 2 * JN; ++m) {
+        acc[m % 2][m / 2] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a[from][m % 2], b[from][m / 2], acc[m % 2][m / 2], 0, 0, 0);
 #pragma unroll
-      for (int j = 0; j < MT; ++j) b[j] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(xs + j * 32 * GP + kk * 16));
+        for (int f = m * NF / NM; f < (m + 1) * NF / NM; ++f) read(s, kk, f, from ^ 1);
+        __builtin_amdgcn_sched_barrier(0);
+      }
+    };
 #pragma unroll
-      for (int i = 0; i < 2; ++i)
-#pragma unroll
-        for (int j = 0; j < MT; ++j) acc[i][j] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(a[i], b[j], acc[i][j], 0, 0, 0);
+    for (int f = 0; f < NF; ++f) read(0, 0, f, 0);
+    for (int s = 0; s < nk; ++s) {
+      quarter(0, s, 1);
+      quarter(1, s, 2);
+      quarter(0, s, 3);
+      SQ_WAIT_VM_LDS((G::NS - 2) * G::LOADS);
+      SQ_RAW_BARRIER();
+      fetch(s + G::NS);
+      quarter(1, s + 1, 0);
     }
-    if (more) stage(buf ^ 1);
-    __syncthreads();
-  }
+  };
+  const int held = tile.z - wt * G::JT * 32;
+  if (held <= 0) run(std::integral_constant<int, 0>{});
+  else if (G::JT > 1 && held <= 32) run(std::integral_constant<int, 1>{});
+  else run(std::integral_constant<int, G::JT>{});
+  SQ_WAIT_VM_LDS(0);  // the padding loads, before the workgroup's LDS goes to another
   // register r of a tile: weight row 8 (r / 4) + 4 g2 + r % 4, slot col
 #pragma unroll
-  for (int j = 0; j < MT; ++j) {
-    const int r = wm * MT * 32 + j * 32 + col;
+  for (int j = 0; j < G::JT; ++j) {
+    const int r = (wt * G::JT + j) * 32 + col;
     if (r >= tile.z) continue;
     uint16_t* dst = out + (int64_t)(tile.y + r) * F;
     if constexpr (GLU) {
       const float sc = p.scores[p.rows[tile.y + r]];
 #pragma unroll
       for (int q = 0; q < 4; ++q) {
-        const int f = f0 + wn * 32 + 8 * q + 4 * g2;
+        const int f = f0 + ww * 32 + 8 * q + 4 * g2;
         if (f >= F) continue;
         float v[4];
 #pragma unroll
@@ -363,12 +409,18 @@ __global__ __launch_bounds__(256) void grouped_mfma_kernel(GroupArgs p, const ui
       for (int i = 0; i < 2; ++i)
 #pragma unroll
         for (int q = 0; q < 4; ++q) {
-          const int f = f0 + wn * 64 + i * 32 + 8 * q + 4 * g2;
+          const int f = f0 + ww * 64 + i * 32 + 8 * q + 4 * g2;
           if (f >= F) continue;
           *reinterpret_cast<uint2*>(dst + f) = make_uint2(pack2(acc[i][j][4 * q], acc[i][j][4 * q + 1]), pack2(acc[i][j][4 * q + 2], acc[i][j][4 * q + 3]));
         }
     }
   }
+}
+
+template <class G, bool GLU>
+__global__ __launch_bounds__(G::THREADS) void grouped_mfma_kernel(GroupArgs p, const uint16_t* x, const uint16_t* w, uint16_t* out) {
+  __shared__ __attribute__((aligned(1024))) uint8_t smem[G::NS * G::STAGE];
+  grouped_tile<G, GLU>(p, x, w, out, smem);
 }
 
 // ---------------------------------------------------------------------------------------------- steps of a few tokens
@@ -476,10 +528,10 @@ extern "C" int aqs_moe_route(const void* h, int64_t ldh, int dtype, const void* 
   if (dtype == AQ_BF16 && K % 8 == 0 && ldh % 8 == 0 && !bad_ptr16(h) && !bad_ptr16(w) && Ex <= 224) {
     const unsigned grid = (unsigned)((M + 15) / 16);
     const uint16_t *hp = (const uint16_t*)h, *wp = (const uint16_t*)w;
-    if (Ex <= 32) route_mfma_kernel<2><<<grid, 256, 0, st>>>(p, hp, wp);
-    else if (Ex <= 64) route_mfma_kernel<4><<<grid, 256, 0, st>>>(p, hp, wp);
-    else if (Ex <= 128) route_mfma_kernel<8><<<grid, 256, 0, st>>>(p, hp, wp);
-    else route_mfma_kernel<14><<<grid, 256, 0, st>>>(p, hp, wp);
+    if (Ex <= 32) route_mfma_kernel<2, 8><<<grid, 256, 0, st>>>(p, hp, wp);
+    else if (Ex <= 64) route_mfma_kernel<4, 6><<<grid, 256, 0, st>>>(p, hp, wp);
+    else if (Ex <= 128) route_mfma_kernel<8, 3><<<grid, 256, 0, st>>>(p, hp, wp);
+    else route_mfma_kernel<14, 2><<<grid, 256, 0, st>>>(p, hp, wp);
     return launched();
   }
   SQ_DISPATCH(dtype, (route_any_kernel<T><<<dim3((unsigned)((M + 3) / 4)), 256, 0, st>>>(p, (const T*)h, (const T*)w)));
@@ -489,7 +541,7 @@ extern "C" int aqs_moe_route(const void* h, int64_t ldh, int dtype, const void* 
 // slots per tile for A choices of Ex experts of width K and inner size F
 extern "C" int64_t aqs_moe_tile(int dtype, int64_t A, int64_t Ex, int64_t K, int64_t F) {
   if (dtype != AQ_BF16 || K % 8 || F % 8) return 64;
-  return A >= 64 * Ex ? 128 : 32;
+  return A >= 64 * Ex ? GroupWide::TROWS : GroupNarrow::TROWS;
 }
 extern "C" int64_t aqs_moe_tiles(int64_t A, int64_t Ex, int64_t tile) { return A / tile + Ex + 1; }
 
@@ -507,42 +559,35 @@ extern "C" int aqs_moe_sort(const int32_t* ids, int64_t A, int64_t Ex, int64_t t
 
 // glu != 0: x [tokens, ldx], w [Ex, N = 2 F, K] gate | up, out [A, F] = silu(s g) (s u); otherwise x [A, ldx] by slot, out [A, N].
 extern "C" int aqs_moe_product(int glu, const void* x, int64_t ldx, int dtype, const void* w, const int32_t* tiles, int64_t n_tiles,
-                               int64_t tile, const int32_t* rows, const float* scores, int64_t top, void* out, int64_t N, int64_t K,
-                               void* stream) {
-  SQ_CHECK(N > 0 && K > 0 && top > 0 && n_tiles > 0 && ldx >= K && (!glu || N % 2 == 0), AQ_E_SHAPE);
+                               int64_t tile, const int32_t* rows, const float* scores, int64_t A, int64_t top, void* out, int64_t N,
+                               int64_t K, void* stream) {
+  SQ_CHECK(N > 0 && K > 0 && A > 0 && top > 0 && A % top == 0 && n_tiles > 1 && ldx >= K && (!glu || N % 2 == 0), AQ_E_SHAPE);
   SQ_CHECK(n_tiles < 65536 && N < (1 << 24) && K < (1 << 24), AQ_E_RANGE);
   SQ_NEED(x && w && tiles && rows && out && (scores || !glu));
-  const GroupArgs p{(const int4*)tiles, rows, scores, ldx, (int)top, (int)N, (int)K};
+  // extent of x's rows: whole rows but for the last one's padding
+  const int64_t x_rows = glu ? A / top : A, x_bytes = ((x_rows - 1) * ldx + K) * 2;
+  const GroupArgs p{(const int4*)tiles, rows, scores, ldx, x_bytes, (int)top, (int)N, (int)K};
   const int64_t F = glu ? N / 2 : N;
   hipStream_t st = (hipStream_t)stream;
   if (tile == 64) {
-    const dim3 grid((unsigned)((F + (glu ? 31 : 63)) / (glu ? 32 : 64)), (unsigned)n_tiles);
+    const dim3 grid((unsigned)((F + (glu ? 31 : 63)) / (glu ? 32 : 64)), (unsigned)(n_tiles - 1));
     SQ_DISPATCH(dtype, if (glu)(grouped_any_kernel<T, true><<<grid, 256, 0, st>>>(p, (const T*)x, (const T*)w, (T*)out));
                 else (grouped_any_kernel<T, false><<<grid, 256, 0, st>>>(p, (const T*)x, (const T*)w, (T*)out)));
     return launched();
   }
   SQ_CHECK(mfma_ok(dtype, ldx, N, K, glu, x, w, out), AQ_E_ALIGN);
-  auto go = [&](auto wm_tag, auto mt_tag, auto glu_tag) -> int {
-    constexpr int WM = decltype(wm_tag)::value, MT = decltype(mt_tag)::value, TM = WM * MT * 32, TN = 4 / WM * 64;
-    constexpr bool G = decltype(glu_tag)::value;
-    auto* k = grouped_mfma_kernel<WM, MT, G>;
-    constexpr size_t lds = (size_t)2 * (TM + TN) * GP * 2;
-    if (lds > 64 * 1024) {
-      const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-      if (e != hipSuccess) return (int)e;
-    }
-    constexpr int cols = G ? TN / 2 : TN;
-    k<<<dim3((unsigned)((F + cols - 1) / cols), (unsigned)n_tiles), 256, lds, st>>>(p, (const uint16_t*)x, (const uint16_t*)w, (uint16_t*)out);
+  SQ_CHECK(x_bytes < (int64_t)GROUP_OOB - 65536 * 2 && N * K * 2 < (int64_t)GROUP_OOB - 65536 * 2, AQ_E_RANGE);
+  auto go = [&](auto shape, auto glu_tag) -> int {
+    using G = decltype(shape);
+    constexpr bool GLU = decltype(glu_tag)::value;
+    constexpr int cols = GLU ? G::WROWS / 2 : G::WROWS;
+    const dim3 grid((unsigned)((F + cols - 1) / cols), (unsigned)(n_tiles - 1));
+    grouped_mfma_kernel<G, GLU><<<grid, G::THREADS, 0, st>>>(p, (const uint16_t*)x, (const uint16_t*)w, (uint16_t*)out);
     return launched();
   };
-  using std::integral_constant;
-  if (tile == 128) {
-    if (glu) return go(integral_constant<int, 2>{}, integral_constant<int, 2>{}, std::true_type{});
-    return go(integral_constant<int, 2>{}, integral_constant<int, 2>{}, std::false_type{});
-  }
-  SQ_CHECK(tile == 32, AQ_E_SHAPE);
-  if (glu) return go(integral_constant<int, 1>{}, integral_constant<int, 1>{}, std::true_type{});
-  return go(integral_constant<int, 1>{}, integral_constant<int, 1>{}, std::false_type{});
+  SQ_CHECK(tile == GroupWide::TROWS || tile == GroupNarrow::TROWS, AQ_E_SHAPE);
+  if (tile == GroupWide::TROWS) return glu ? go(GroupWide{}, std::true_type{}) : go(GroupWide{}, std::false_type{});
+  return glu ? go(GroupNarrow{}, std::true_type{}) : go(GroupNarrow{}, std::false_type{});
 }
 
 // whether the two launches below serve these sizes

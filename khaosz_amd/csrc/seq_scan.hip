@@ -488,34 +488,37 @@ struct SsdStepArgs {
   int H, G, N, P;
 };
 
+constexpr int SSD_STEP_COLS = 32;  // state columns per workgroup: a head's columns never meet
+
 template <typename T, int RP, int NI>
 __global__ __launch_bounds__(256) void ssd_step_kernel(SsdStepArgs p, const T* proj, T* ring) {
   constexpr int TH = 256, CPI = 16;
   __shared__ __align__(16) float b_s[STEP_MAX], c_s[STEP_MAX];
-  __shared__ float x_s[STEP_MAX];
+  __shared__ float x_s[NI * CPI];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int h = blockIdx.x, b = blockIdx.y, per = p.H / p.G, j = h / per;
+  const int tiles = (p.P + NI * CPI - 1) / (NI * CPI), h = blockIdx.x / tiles, e0 = (blockIdx.x % tiles) * NI * CPI;
+  const int b = blockIdx.y, per = p.H / p.G, j = h / per, cols = p.P - e0 < NI * CPI ? p.P - e0 : NI * CPI;
   const int slot = p.slots[b], pos = p.pos[b], N = p.N, P = p.P, inner = p.H * P;
   const int r0 = (lane & 15) * RP, cl = wave * 4 + (lane >> 4);
   const T* row = proj + b * p.ld;
-  float* st = p.state + ((int64_t)slot * p.H + h) * P * N;
+  float* st = p.state + (((int64_t)slot * p.H + h) * P + e0) * N;
   float s[NI][RP];
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int e = i * CPI + cl;
-    load_rows<RP>(st + (int64_t)e * N, r0, N, e < P && pos > 0, s[i]);
+    load_rows<RP>(st + (int64_t)e * N, r0, N, e < cols && pos > 0, s[i]);
   }
   for (int d = tid; d < STEP_MAX; d += TH)
     if (d >= N) b_s[d] = c_s[d] = 0.0f;
   T* rg = ring + (int64_t)slot * p.s.taps * p.s.C;
   const T* cin = row + p.o_xbc;
-  for (int i = tid; i < 2 * N + P; i += TH) {
+  for (int i = tid; i < 2 * N + cols; i += TH) {
     const int which = i < N ? 0 : i < 2 * N ? 1 : 2;
     const int d = i - which * N;
-    const int c = which == 2 ? h * P + d : inner + (which * p.G + j) * N + d;
+    const int c = which == 2 ? h * P + e0 + d : inner + (which * p.G + j) * N + d;
     const float x = silu(conv_step(p.s, cin, pos, rg, c));
     (which == 0 ? b_s : which == 1 ? c_s : x_s)[d] = x;
-    if (which == 2 || h % per == 0) rg[(int64_t)(pos % p.s.taps) * p.s.C + c] = cin[c];
+    if (which == 2 || (h % per == 0 && e0 == 0)) rg[(int64_t)(pos % p.s.taps) * p.s.C + c] = cin[c];
   }
   const float dt = p.decay ? 1.0f : softplus(to_f32(row[p.o_dt + h]) + p.dt_bias[h]);
   const float a = p.decay ? p.decay[h] : expf(-expf(p.a_log[h]) * dt), skip = p.skip ? p.skip[h] : 0.0f;
@@ -526,14 +529,14 @@ __global__ __launch_bounds__(256) void ssd_step_kernel(SsdStepArgs p, const T* p
 #pragma unroll
   for (int i = 0; i < NI; ++i) {
     const int e = i * CPI + cl;
-    if (i * CPI >= P) break;
-    const float x = e < P ? x_s[e] : 0.0f, u = dt * x;
+    if (i * CPI >= cols) break;
+    const float x = e < cols ? x_s[e] : 0.0f, u = dt * x;
 #pragma unroll
     for (int w = 0; w < RP; ++w) s[i][w] = fmaf(k[w], u, a * s[i][w]);
     const float o = row16_sum(dot_rows<RP>(s[i], q)) + skip * x;
-    if (e < P) {
+    if (e < cols) {
       store_rows<RP>(st + (int64_t)e * N, r0, N, s[i]);
-      if ((lane & 15) == 0) p.y[(int64_t)b * inner + h * P + e] = o;
+      if ((lane & 15) == 0) p.y[(int64_t)b * inner + h * P + e0 + e] = o;
     }
   }
 }
@@ -707,8 +710,9 @@ extern "C" int aqs_ssd_step(const void* proj, int64_t ld, int64_t o_xbc, int64_t
   a.slots = slots, a.pos = pos, a.dt_bias = dt_bias, a.a_log = a_log, a.skip = skip, a.decay = decay, a.state = state, a.y = y;
   a.ld = ld, a.o_xbc = o_xbc, a.o_dt = o_dt;
   a.H = (int)H, a.G = (int)G, a.N = (int)N, a.P = (int)P;
-  const dim3 grid((unsigned)H, (unsigned)B);
-  SQ_DISPATCH(dtype, SQ_ROWS(N, SQ_ITERS((P + 15) / 16, (ssd_step_kernel<T, RP, NI><<<grid, 256, 0, (hipStream_t)stream>>>(
-                         a, (const T*)proj, (T*)ring)))));
+  constexpr int NI = SSD_STEP_COLS / 16;
+  SQ_CHECK(H * P < (1 << 24), AQ_E_RANGE);
+  const dim3 grid((unsigned)(H * ((P + SSD_STEP_COLS - 1) / SSD_STEP_COLS)), (unsigned)B);
+  SQ_DISPATCH(dtype, SQ_ROWS(N, (ssd_step_kernel<T, RP, NI><<<grid, 256, 0, (hipStream_t)stream>>>(a, (const T*)proj, (T*)ring))));
   return launched();
 }

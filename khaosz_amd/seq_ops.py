@@ -724,9 +724,10 @@ def moe_experts(h: Tensor, ids: Tensor, scores: Tensor, gate_up: Tensor, down: T
     act = torch.empty((A, F), dtype=h.dtype, device=dev)
     out = torch.empty((A, K), dtype=h.dtype, device=dev)
     _call("aqs_moe_sort", dev, _p(ids), A, Ex, tile, _p(rows), _p(slots), _p(tiles), n, _stream(h))
-    _call("aqs_moe_product", dev, 1, _p(h), h.stride(0), _DT[h.dtype], _p(gate_up), _p(tiles), n, tile, _p(rows), _p(scores), top, _p(act),
-          2 * F, K, _stream(h))
-    _call("aqs_moe_product", dev, 0, _p(act), F, _DT[h.dtype], _p(down), _p(tiles), n, tile, _p(rows), None, top, _p(out), K, F, _stream(h))
+    _call("aqs_moe_product", dev, 1, _p(h), h.stride(0), _DT[h.dtype], _p(gate_up), _p(tiles), n, tile, _p(rows), _p(scores), A, top,
+          _p(act), 2 * F, K, _stream(h))
+    _call("aqs_moe_product", dev, 0, _p(act), F, _DT[h.dtype], _p(down), _p(tiles), n, tile, _p(rows), None, A, top, _p(out), K, F,
+          _stream(h))
     return Routed(out, slots)
 
 

@@ -134,8 +134,8 @@ def test_arguments_are_checked_before_any_launch():
     assert lib.aqs_latent_decode_ok(1, 20, 8, 48, 40, 64) == 0 and lib.aqs_latent_decode_ok(1, 24, 8, 48, 40, 16) == 0
     assert lib.aqs_moe_route(P, 8, 1, P, P, P, 4, 8, 4, 5, None) == -2 and lib.aqs_moe_route(P, 8, 1, P, P, P, 4, 8, 513, 1, None) == -6
     assert lib.aqs_moe_sort(P, 8, 4, 64, P, P, P, 3, None) == -2
-    assert lib.aqs_moe_product(1, P, 8, 1, P, P, 5, 64, P, None, 1, P, 16, 8, None) == -1  # no scores
-    assert lib.aqs_moe_product(0, P, 12, 1, P, P, 5, 128, P, None, 1, P, 16, 12, None) == -4
+    assert lib.aqs_moe_product(1, P, 8, 1, P, P, 5, 64, P, None, 8, 1, P, 16, 8, None) == -1  # no scores
+    assert lib.aqs_moe_product(0, P, 12, 1, P, P, 5, 128, P, None, 8, 1, P, 16, 12, None) == -4
     assert lib.aqs_moe_step_ok(8, 64, 8, 8, 4, 4) == 1 and lib.aqs_moe_step_ok(9, 64, 8, 8, 4, 4) == 0 and lib.aqs_moe_step_ok(1, 64, 12, 8, 4, 4) == 0
     assert lib.aqs_moe_tile(1, 10, 4, 64, 64) != 64 and lib.aqs_moe_tile(0, 10, 4, 64, 64) == 64 and lib.aqs_moe_tile(1, 10, 4, 64, 12) == 64
 

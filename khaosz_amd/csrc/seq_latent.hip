@@ -340,6 +340,119 @@ __global__ __launch_bounds__(256) void latent_decode_any_kernel(LatentArgs a, fl
   }
 }
 
+// bf16 on the matrix cores: 16 heads per workgroup, so that a cache row is read once for all of them.  Scores: every wavefront 16
+// of a block's 64 positions, operands straight from memory; values: the same rows' first R elements transposed in LDS,
+// every wavefront a quarter of the columns.  KS: steps of 32 along a key; RP: R padded.
+typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+constexpr int LAT_VP = 72, LAT_SP = 68;
+
+template <int RP, int KS>
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(1, 2))) void latent_decode_mfma_kernel(
+    LatentArgs a, float scale_log2e, const uint16_t* qa, const uint16_t* kc, float* part, int NS, int span) {
+  constexpr int VC = RP / 32, NT = RP / 64;
+  extern __shared__ __align__(16) uint16_t vt[];  // [RP][LAT_VP]
+  __shared__ __align__(16) float s_s[16][LAT_SP];
+  __shared__ __align__(16) uint16_t p_s[16][LAT_VP];
+  __shared__ float m_s[16], l_s[16], al_s[16];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, q4 = lane >> 4;
+  const int groups = (a.H + 15) / 16, h0 = (blockIdx.x % groups) * 16, split = (blockIdx.x / groups) % NS, b = blockIdx.x / (groups * NS);
+  const int pos = a.pos[b], lo = pos - a.window + 1 > 0 ? pos - a.window + 1 : 0, DK = a.R + a.rot;
+  const int t0 = lo / 64 * 64 + split * span;
+  if (t0 > pos) return;  // uniform
+  const int t1 = t0 + span < pos + 1 ? t0 + span : pos + 1;
+  const int nh = a.H - h0 < 16 ? a.H - h0 : 16;
+  uint4 q[KS];
+  {
+    const uint16_t* src = qa + ((int64_t)b * a.H + h0 + (r16 < nh ? r16 : 0)) * DK;
+#pragma unroll
+    for (int k = 0; k < KS; ++k) {
+      const int d = k * 32 + q4 * 8;
+      q[k] = *reinterpret_cast<const uint4*>(src + (d < DK ? d : 0));
+    }
+  }
+  f32x4 o[NT];
+#pragma unroll
+  for (int n = 0; n < NT; ++n) o[n] = f32x4{0, 0, 0, 0};
+  if (tid < 16) m_s[tid] = MASKED, l_s[tid] = 0.0f;
+  for (int tb = t0; tb < t1; tb += 64) {
+    const int64_t pr0 = page_row(a, b, tb), row0 = pr0 >= 0 ? pr0 : 0;
+    uint4 k[KS], v[VC];
+    const uint16_t* kr = kc + (row0 + wave * 16 + r16) * DK;
+#pragma unroll
+    for (int i = 0; i < KS; ++i) {
+      const int d = i * 32 + q4 * 8;
+      k[i] = *reinterpret_cast<const uint4*>(kr + (d < DK ? d : 0));
+    }
+    const uint16_t* vr = kc + (row0 + lane) * DK;
+#pragma unroll
+    for (int c = 0; c < VC; ++c) {
+      const int d = (wave + 4 * c) * 8;
+      v[c] = *reinterpret_cast<const uint4*>(vr + (d < a.R ? d : 0));
+    }
+    f32x4 s = {0, 0, 0, 0};
+#pragma unroll
+    for (int i = 0; i < KS; ++i) {
+      if (i * 32 + q4 * 8 >= DK) k[i] = make_uint4(0, 0, 0, 0);  // past the row the loads repeat its start
+      s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, q[i]), __builtin_bit_cast(bf16x8, k[i]), s, 0, 0, 0);
+    }
+    // column r16: position tb + wave * 16 + r16; rows 4 q4 + r: heads
+    const int t = tb + wave * 16 + r16;
+    const bool on = pr0 >= 0 && t >= lo && t <= pos;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) s_s[q4 * 4 + r][wave * 16 + r16] = on ? s[r] * scale_log2e : -INFINITY;
+    // values: two positions per 4-byte store (neighbouring lanes swap halves); masked rows may hold anything
+    const bool off = !(pr0 >= 0 && tb + lane >= lo && tb + lane <= pos), odd = lane & 1;
+    const uint32_t sel = odd ? 0x03020706u : 0x05040100u;
+#pragma unroll
+    for (int c = 0; c < VC; ++c) {
+      uint32_t* dst = reinterpret_cast<uint32_t*>(&vt[((wave + 4 * c) * 8 + (odd ? 1 : 0)) * LAT_VP + (lane & ~1)]);
+      const uint32_t w[4] = {off ? 0 : v[c].x, off ? 0 : v[c].y, off ? 0 : v[c].z, off ? 0 : v[c].w};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const uint32_t other = (uint32_t)__builtin_amdgcn_mov_dpp((int)w[e], 0xB1, 0xf, 0xf, true);
+        dst[e * LAT_VP] = __builtin_amdgcn_perm(other, w[e], sel);
+      }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {  // heads 4 wave + i; lane: position
+      const int h = wave * 4 + i;
+      const float x = s_s[h][lane], old = m_s[h], mn = fmaxf(old, wave_max(x)), e = __builtin_amdgcn_exp2f(x - mn), sum = wave_sum(e);
+      const float al = __builtin_amdgcn_exp2f(old - mn), l = l_s[h] * al + sum;
+      p_s[h][lane] = (uint16_t)(pack2(e, e) & 0xffffu);
+      if (lane == 0) m_s[h] = mn, l_s[h] = l, al_s[h] = al;
+    }
+    __syncthreads();
+    bf16x8 pf[2];
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) pf[kk] = __builtin_bit_cast(bf16x8, *reinterpret_cast<const uint4*>(&p_s[r16][kk * 32 + q4 * 8]));
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[n][r] *= al_s[q4 * 4 + r];
+#pragma unroll
+      for (int kk = 0; kk < 2; ++kk) {
+        const uint4 vf = *reinterpret_cast<const uint4*>(&vt[((wave * NT + n) * 16 + r16) * LAT_VP + kk * 32 + q4 * 8]);
+        o[n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[kk], __builtin_bit_cast(bf16x8, vf), o[n], 0, 0, 0);
+      }
+    }
+    if (tb + 64 < t1) __syncthreads();  // the stages may be overwritten
+  }
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int h = q4 * 4 + r;
+    if (h >= nh) continue;
+    float* dst = part + (((int64_t)b * a.H + h0 + h) * NS + split) * (a.R + 4);
+#pragma unroll
+    for (int n = 0; n < NT; ++n) {
+      const int d = (wave * NT + n) * 16 + r16;
+      if (d < a.R) dst[d] = o[n][r];
+    }
+    if (wave == 0 && r16 == 0) dst[a.R] = m_s[h], dst[a.R + 1] = l_s[h];
+  }
+}
+
 // Slices of head h merged, W_uv [H * E, R] applied, times sigmoid(gate [B, H * E]).  Workgroup: OUT_ROWS values of a head.
 constexpr int OUT_ROWS = 32, LAT_MAX_SLICES = 64, LAT_MAX_R = 1024;
 
@@ -519,8 +632,28 @@ extern "C" int aqs_latent_decode(const void* proj, int64_t ld, int64_t o_kv, int
     if (DK <= 576) return any(std::integral_constant<int, 9>{}, t);
     return any(std::integral_constant<int, 18>{}, t);
   };
+  auto cores = [&](auto r_tag, auto k_tag) -> int {
+    constexpr int RP = decltype(r_tag)::value, KS = decltype(k_tag)::value;
+    auto* k = latent_decode_mfma_kernel<RP, KS>;
+    constexpr size_t lds = (size_t)RP * LAT_VP * 2;
+    if (lds > 48 * 1024) {  // besides what the kernel declares
+      const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(k), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+      if (e != hipSuccess) return (int)e;
+    }
+    k<<<dim3((unsigned)(B * ((H + 15) / 16) * slices)), 256, lds, st>>>(a, scale * LOG2E, (const uint16_t*)qa, (const uint16_t*)kc, part, NS, span);
+    return launched();
+  };
+  using std::integral_constant;
   int rc = AQ_OK;
-  SQ_DISPATCH(dtype, rc = pieces((T*)nullptr));
+  if (dtype == AQ_BF16 && R <= 512 && rot <= 128) {
+    if (R <= 64) rc = cores(integral_constant<int, 64>{}, integral_constant<int, 6>{});
+    else if (R <= 128) rc = cores(integral_constant<int, 128>{}, integral_constant<int, 8>{});
+    else if (R <= 256) rc = cores(integral_constant<int, 256>{}, integral_constant<int, 12>{});
+    else if (DK <= 576) rc = cores(integral_constant<int, 512>{}, integral_constant<int, 18>{});
+    else rc = cores(integral_constant<int, 512>{}, integral_constant<int, 20>{});
+  } else {
+    SQ_DISPATCH(dtype, rc = pieces((T*)nullptr));
+  }
   if (rc) return rc;
   const dim3 ogrid((unsigned)(H * outs), (unsigned)B);
   SQ_DISPATCH(dtype, (latent_out_kernel<T><<<ogrid, 256, 0, st>>>(a, (int)E, part, NS, span, (const T*)uv, (const T*)proj + o_gate, ld, (T*)out, ldo)));

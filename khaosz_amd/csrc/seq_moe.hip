@@ -105,12 +105,12 @@ __global__ __launch_bounds__(256) void route_any_kernel(RouteArgs p, const T* h,
   });
 }
 
-// bf16 on the matrix cores: 16 tokens per workgroup, every wavefront all experts over a quarter of the contraction (steps
-// of 32 in turn).  NT: tiles of 16 experts; KU: steps whose operands are requested together.
-template <int NT, int KU>
-__global__ __launch_bounds__(256) void route_mfma_kernel(RouteArgs p, const uint16_t* h, const uint16_t* w) {
+// bf16 on the matrix cores: 16 tokens per workgroup, every wavefront all experts over its share of the contraction (steps
+// of 32 in turn).  NT: tiles of 16 experts; KU: steps whose operands are requested together; NW: wavefronts.
+template <int NT, int KU, int NW>
+__global__ __launch_bounds__(NW * 64) void route_mfma_kernel(RouteArgs p, const uint16_t* h, const uint16_t* w) {
   constexpr int ZP = NT * 16 + 4;
-  __shared__ __align__(16) float z_s[4][16][ZP];
+  __shared__ __align__(16) float z_s[NW][16][ZP];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, q = lane >> 4;
   const int64_t m0 = (int64_t)blockIdx.x * 16;
   const uint16_t* hr = h + (m0 + r16 < p.M ? m0 + r16 : p.M - 1) * p.ldh;
@@ -120,18 +120,18 @@ __global__ __launch_bounds__(256) void route_mfma_kernel(RouteArgs p, const uint
   f32x4 acc[NT];
 #pragma unroll
   for (int t = 0; t < NT; ++t) acc[t] = f32x4{0, 0, 0, 0};
-  for (int k0 = wave * 32; k0 < p.K; k0 += 128 * KU) {
+  for (int k0 = wave * 32; k0 < p.K; k0 += NW * 32 * KU) {
     uint4 x[KU], v[KU][NT];
 #pragma unroll
     for (int u = 0; u < KU; ++u) {
-      const int k = k0 + u * 128 + q * 8, kc = k < p.K ? k : 0;
+      const int k = k0 + u * NW * 32 + q * 8, kc = k < p.K ? k : 0;
       x[u] = *reinterpret_cast<const uint4*>(hr + kc);
 #pragma unroll
       for (int t = 0; t < NT; ++t) v[u][t] = *reinterpret_cast<const uint4*>(wr[t] + kc);
     }
 #pragma unroll
     for (int u = 0; u < KU; ++u) {
-      if (k0 + u * 128 + q * 8 >= p.K) x[u] = make_uint4(0, 0, 0, 0);
+      if (k0 + u * NW * 32 + q * 8 >= p.K) x[u] = make_uint4(0, 0, 0, 0);
 #pragma unroll
       for (int t = 0; t < NT; ++t)
         acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v[u][t]), __builtin_bit_cast(bf16x8, x[u]), acc[t], 0, 0, 0);
@@ -141,11 +141,15 @@ __global__ __launch_bounds__(256) void route_mfma_kernel(RouteArgs p, const uint
 #pragma unroll
   for (int t = 0; t < NT; ++t) *reinterpret_cast<f32x4*>(&z_s[wave][r16][t * 16 + q * 4]) = acc[t];
   __syncthreads();
-  for (int x = tid; x < 16 * NT * 16; x += 256) {
+  for (int x = tid; x < 16 * NT * 16; x += NW * 64) {
     const int t = x / (NT * 16), e = x % (NT * 16);
-    z_s[0][t][e] = (z_s[0][t][e] + z_s[1][t][e]) + (z_s[2][t][e] + z_s[3][t][e]);
+    float v = z_s[0][t][e];
+#pragma unroll
+    for (int i = 1; i < NW; ++i) v += z_s[i][t][e];
+    z_s[0][t][e] = v;
   }
   __syncthreads();
+  if (tid >= 256) return;
   const int64_t m = m0 + (tid >> 4);
   constexpr int NE = NT < 4 ? 4 : NT;
   choose<NE>(z_s[0][tid >> 4], p.Ex, p.top, tid & 15, [&](int j, int e, float z) {
@@ -170,11 +174,17 @@ __global__ __launch_bounds__(SORT_WAVES * 64) void moe_sort_kernel(const int* id
   __syncthreads();
   const int per = ((A + SORT_WAVES - 1) / SORT_WAVES + 63) / 64 * 64, i0 = wave * per, i1 = i0 + per < A ? i0 + per : A;
   int own = 0;
-#pragma unroll 4
-  for (int i = i0 + lane; i < i1; i += 64) {
-    const int id = ids[i];
-    own += id == e;
-    atomicAdd(&count_s[id], 1);
+  constexpr int U = 8;  // reads together
+  for (int ib = i0; ib < i1; ib += 64 * U) {
+    int id[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) id[u] = ids[ib + u * 64 + lane < i1 ? ib + u * 64 + lane : i0];
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+      if (ib + u * 64 + lane < i1) {
+        own += id[u] == e;
+        atomicAdd(&count_s[id[u]], 1);
+      }
   }
 #pragma unroll
   for (int o = 32; o; o >>= 1) own += __shfl_xor(own, o, 64);
@@ -192,16 +202,22 @@ __global__ __launch_bounds__(SORT_WAVES * 64) void moe_sort_kernel(const int* id
   const int cnt = count_s[e];
   int at = off;
   for (int w = 0; w < wave; ++w) at += own_s[w];
-  for (int ib = i0; ib < i1; ib += 64) {
-    const int i = ib + lane;
-    const bool mine = i < i1 && ids[i] == e;
-    const uint64_t b = __builtin_amdgcn_ballot_w64(mine);
-    if (mine) {
-      const int s = at + __popcll(b & ((1ull << lane) - 1));
-      rows[s] = i;
-      slots[i] = s;
+  for (int ib = i0; ib < i1; ib += 64 * U) {
+    int id[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) id[u] = ids[ib + u * 64 + lane < i1 ? ib + u * 64 + lane : i0];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int i = ib + u * 64 + lane;
+      const bool mine = i < i1 && id[u] == e;
+      const uint64_t b = __builtin_amdgcn_ballot_w64(mine);
+      if (mine) {
+        const int s = at + __popcll(b & ((1ull << lane) - 1));
+        rows[s] = i;
+        slots[i] = s;
+      }
+      at += __popcll(b);
     }
-    at += __popcll(b);
   }
   if (e == 0 && tid == 0) tiles[0] = make_int4(total, 0, 0, 0);
   for (int t = tid; t * TM < cnt && 1 + t0 + t < n_tiles; t += SORT_WAVES * 64)
@@ -528,10 +544,11 @@ extern "C" int aqs_moe_route(const void* h, int64_t ldh, int dtype, const void* 
   if (dtype == AQ_BF16 && K % 8 == 0 && ldh % 8 == 0 && !bad_ptr16(h) && !bad_ptr16(w) && Ex <= 224) {
     const unsigned grid = (unsigned)((M + 15) / 16);
     const uint16_t *hp = (const uint16_t*)h, *wp = (const uint16_t*)w;
-    if (Ex <= 32) route_mfma_kernel<2, 8><<<grid, 256, 0, st>>>(p, hp, wp);
-    else if (Ex <= 64) route_mfma_kernel<4, 6><<<grid, 256, 0, st>>>(p, hp, wp);
-    else if (Ex <= 128) route_mfma_kernel<8, 3><<<grid, 256, 0, st>>>(p, hp, wp);
-    else route_mfma_kernel<14, 2><<<grid, 256, 0, st>>>(p, hp, wp);
+    if (Ex <= 32) route_mfma_kernel<2, 8, 8><<<grid, 512, 0, st>>>(p, hp, wp);
+    else if (Ex <= 64) route_mfma_kernel<4, 8, 8><<<grid, 512, 0, st>>>(p, hp, wp);
+    else if (Ex <= 96) route_mfma_kernel<6, 5, 8><<<grid, 512, 0, st>>>(p, hp, wp);
+    else if (Ex <= 128) route_mfma_kernel<8, 6, 4><<<grid, 256, 0, st>>>(p, hp, wp);
+    else route_mfma_kernel<14, 3, 4><<<grid, 256, 0, st>>>(p, hp, wp);
     return launched();
   }
   SQ_DISPATCH(dtype, (route_any_kernel<T><<<dim3((unsigned)((M + 3) / 4)), 256, 0, st>>>(p, (const T*)h, (const T*)w)));

@@ -314,7 +314,7 @@ typedef float f32x16 __attribute__((ext_vector_type(16)));
 constexpr int WQ = 128, WK = 64;
 
 template <int DP, int EP>
-__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DP + EP <= 256 ? 2 : 1))) void attn_window_kernel(
+__global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu(DP + EP <= 320 ? 2 : 1))) void attn_window_kernel(
     AttnDims a, AttnKV<uint16_t> kv, AttnOut oo, float scale_log2e, const uint16_t* q, uint16_t* out, int B) {
   constexpr int KP = DP + 8, VP = WK + 4, DS = DP / 16, DT = EP / 32, KC = DP / 32, VC = EP / 32;
   extern __shared__ __align__(16) uint16_t lds[];

@@ -645,7 +645,8 @@ extern "C" int aqs_latent_decode(const void* proj, int64_t ld, int64_t o_kv, int
   };
   using std::integral_constant;
   int rc = AQ_OK;
-  if (dtype == AQ_BF16 && R <= 512 && rot <= 128) {
+  // a few heads in all are faster with a workgroup each (8.6 against 12.5 us for 16 heads over 1024 positions, one sequence)
+  if (dtype == AQ_BF16 && R <= 512 && rot <= 128 && B * H > 16) {
     if (R <= 64) rc = cores(integral_constant<int, 64>{}, integral_constant<int, 6>{});
     else if (R <= 128) rc = cores(integral_constant<int, 128>{}, integral_constant<int, 8>{});
     else if (R <= 256) rc = cores(integral_constant<int, 256>{}, integral_constant<int, 12>{});

@@ -105,8 +105,9 @@ __global__ __launch_bounds__(256) void route_any_kernel(RouteArgs p, const T* h,
   });
 }
 
-// bf16 on the matrix cores: 16 tokens per workgroup, every wavefront all experts over its share of the contraction (steps
-// of 32 in turn).  NT: tiles of 16 experts; KU: steps whose operands are requested together; NW: wavefronts.
+// bf16 on the matrix cores: 16 tokens per workgroup, every wavefront all experts over its share of the contraction.  NT:
+// tiles of 16 experts; KU: products whose operands are requested together (in pairs that read whole cache lines
+// of a row); NW: wavefronts.
 template <int NT, int KU, int NW>
 __global__ __launch_bounds__(NW * 64) void route_mfma_kernel(RouteArgs p, const uint16_t* h, const uint16_t* w) {
   constexpr int ZP = NT * 16 + 4;
@@ -120,18 +121,20 @@ __global__ __launch_bounds__(NW * 64) void route_mfma_kernel(RouteArgs p, const 
   f32x4 acc[NT];
 #pragma unroll
   for (int t = 0; t < NT; ++t) acc[t] = f32x4{0, 0, 0, 0};
-  for (int k0 = wave * 32; k0 < p.K; k0 += NW * 32 * KU) {
+  static_assert(KU % 2 == 0, "whole cache lines");
+  for (int k0 = wave * 64; k0 < p.K; k0 += NW * 32 * KU) {
     uint4 x[KU], v[KU][NT];
 #pragma unroll
     for (int u = 0; u < KU; ++u) {
-      const int k = k0 + u * NW * 32 + q * 8, kc = k < p.K ? k : 0;
+      const int k = k0 + u / 2 * NW * 64 + (q * 2 + u % 2) * 8, kc = k < p.K ? k : 0;
       x[u] = *reinterpret_cast<const uint4*>(hr + kc);
 #pragma unroll
       for (int t = 0; t < NT; ++t) v[u][t] = *reinterpret_cast<const uint4*>(wr[t] + kc);
     }
+    __builtin_amdgcn_sched_barrier(0);  // all of them are requested before the first is waited for
 #pragma unroll
     for (int u = 0; u < KU; ++u) {
-      if (k0 + u * NW * 32 + q * 8 >= p.K) x[u] = make_uint4(0, 0, 0, 0);
+      if (k0 + u / 2 * NW * 64 + (q * 2 + u % 2) * 8 >= p.K) x[u] = make_uint4(0, 0, 0, 0);
 #pragma unroll
       for (int t = 0; t < NT; ++t)
         acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, v[u][t]), __builtin_bit_cast(bf16x8, x[u]), acc[t], 0, 0, 0);
@@ -546,9 +549,9 @@ extern "C" int aqs_moe_route(const void* h, int64_t ldh, int dtype, const void* 
     const uint16_t *hp = (const uint16_t*)h, *wp = (const uint16_t*)w;
     if (Ex <= 32) route_mfma_kernel<2, 8, 8><<<grid, 512, 0, st>>>(p, hp, wp);
     else if (Ex <= 64) route_mfma_kernel<4, 8, 8><<<grid, 512, 0, st>>>(p, hp, wp);
-    else if (Ex <= 96) route_mfma_kernel<6, 5, 8><<<grid, 512, 0, st>>>(p, hp, wp);
+    else if (Ex <= 96) route_mfma_kernel<6, 4, 8><<<grid, 512, 0, st>>>(p, hp, wp);
     else if (Ex <= 128) route_mfma_kernel<8, 6, 4><<<grid, 256, 0, st>>>(p, hp, wp);
-    else route_mfma_kernel<14, 3, 4><<<grid, 256, 0, st>>>(p, hp, wp);
+    else route_mfma_kernel<14, 2, 4><<<grid, 256, 0, st>>>(p, hp, wp);
     return launched();
   }
   SQ_DISPATCH(dtype, (route_any_kernel<T><<<dim3((unsigned)((M + 3) / 4)), 256, 0, st>>>(p, (const T*)h, (const T*)w)));

@@ -258,18 +258,24 @@ __global__ __launch_bounds__(256) void latent_absorb_kernel(LatentArgs a, const 
 
 // One head per workgroup, any type: 16 lanes share a key, PC pieces of 4 elements each, and keep what they read of it for
 // the value sum.  part [B, H, NS, R + 4]: numerators, maximum, denominator of a slice of `span` positions.
+// four elements, kept as they are until they are used
 template <typename T>
-__device__ __forceinline__ void load4(const T* p, float (&o)[4]);
+struct Raw4;
 template <>
-__device__ __forceinline__ void load4<float>(const float* p, float (&o)[4]) {
-  load_vec<4>(p, o);
-}
+struct Raw4<float> {
+  float4 v;
+  __device__ __forceinline__ void load(const float* p) { v = *reinterpret_cast<const float4*>(p); }
+  __device__ __forceinline__ void get(float* o) const { o[0] = v.x, o[1] = v.y, o[2] = v.z, o[3] = v.w; }
+};
 template <>
-__device__ __forceinline__ void load4<bf16>(const bf16* p, float (&o)[4]) {
-  const uint2 v = *reinterpret_cast<const uint2*>(p);
-  o[0] = __uint_as_float(v.x << 16), o[1] = __uint_as_float(v.x & 0xffff0000u);
-  o[2] = __uint_as_float(v.y << 16), o[3] = __uint_as_float(v.y & 0xffff0000u);
-}
+struct Raw4<bf16> {
+  uint2 v;
+  __device__ __forceinline__ void load(const bf16* p) { v = *reinterpret_cast<const uint2*>(p); }
+  __device__ __forceinline__ void get(float* o) const {
+    o[0] = __uint_as_float(v.x << 16), o[1] = __uint_as_float(v.x & 0xffff0000u);
+    o[2] = __uint_as_float(v.y << 16), o[3] = __uint_as_float(v.y & 0xffff0000u);
+  }
+};
 
 template <typename T, int PC>
 __global__ __launch_bounds__(256) void latent_decode_any_kernel(LatentArgs a, float scale_log2e, const T* qa, const T* kc, float* part,
@@ -287,36 +293,51 @@ __global__ __launch_bounds__(256) void latent_decode_any_kernel(LatentArgs a, fl
 #pragma unroll
   for (int c = 0; c < PC; ++c) {
     const int d = (c * 16 + ch) * 4;
-    load4<T>(qr + (d < DK ? d : 0), q[c]);
+    Raw4<T> x;
+    x.load(qr + (d < DK ? d : 0));
+    x.get(q[c]);
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       q[c][e] = d < DK ? q[c][e] * scale_log2e : 0.0f;
       acc[c][e] = 0.0f;
     }
   }
-  for (int tb = t0; tb < t1; tb += 16) {
-    const int t = tb + grp;
-    const int64_t pr = t < t1 ? page_row(a, b, t) : -1;
-    const T* kr = kc + (pr >= 0 ? pr : 0) * DK;
-    float k[PC][4], s = 0.0f;
+  // AH keys of this group of lanes are requested together
+  constexpr int AH = (sizeof(T) == 2 ? 4 : 2) / (PC > 9 ? 2 : 1);
+  for (int tb = t0; tb < t1; tb += 16 * AH) {
+    Raw4<T> kr[AH][PC];
+    bool on[AH];
 #pragma unroll
-    for (int c = 0; c < PC; ++c) {
-      const int d = (c * 16 + ch) * 4;
-      load4<T>(kr + (d < DK ? d : 0), k[c]);
+    for (int x = 0; x < AH; ++x) {
+      const int t = tb + x * 16 + grp;
+      const int64_t pr = t < t1 ? page_row(a, b, t) : -1;
+      on[x] = pr >= 0 && t >= lo;
+      const T* src = kc + (pr >= 0 ? pr : 0) * DK;
+#pragma unroll
+      for (int c = 0; c < PC; ++c) {
+        const int d = (c * 16 + ch) * 4;
+        kr[x][c].load(src + (d < DK ? d : 0));
+      }
     }
+    __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
-    for (int c = 0; c < PC; ++c)
+    for (int x = 0; x < AH; ++x) {
+      float k[PC][4], s = 0.0f;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) s = fmaf(k[c][e], q[c][e], s);
-    s = row16_sum(s);
-    const bool on = pr >= 0 && t >= lo;
-    const float mn = on ? fmaxf(m, s) : m, al = __builtin_amdgcn_exp2f(m - mn), w = on ? __builtin_amdgcn_exp2f(s - mn) : 0.0f;
-    m = mn;
-    l = l * al + w;
+      for (int c = 0; c < PC; ++c) {
+        kr[x][c].get(k[c]);
 #pragma unroll
-    for (int c = 0; c < PC; ++c)
+        for (int e = 0; e < 4; ++e) s = fmaf(k[c][e], q[c][e], s);
+      }
+      s = row16_sum(s);
+      const float mn = on[x] ? fmaxf(m, s) : m, al = __builtin_amdgcn_exp2f(m - mn), w = on[x] ? __builtin_amdgcn_exp2f(s - mn) : 0.0f;
+      m = mn;
+      l = l * al + w;
 #pragma unroll
-      for (int e = 0; e < 4; ++e) acc[c][e] = fmaf(w, on ? k[c][e] : 0.0f, acc[c][e] * al);
+      for (int c = 0; c < PC; ++c)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[c][e] = fmaf(w, on[x] ? k[c][e] : 0.0f, acc[c][e] * al);
+    }
   }
   if (ch == 0) m_s[grp] = m, l_s[grp] = l;
 #pragma unroll
@@ -472,6 +493,14 @@ __global__ __launch_bounds__(256) void latent_out_kernel(LatentArgs a, int E, co
   int n = (pos - lo / 64 * 64) / span + 1;
   n = n < NS ? n : NS;
   const float* src = part + ((int64_t)b * a.H + h) * NS * (R + 4);
+  // the first slices' numerators are requested before their weights are known
+  constexpr int PRE = 16;
+  float pre[2][PRE];
+#pragma unroll
+  for (int c = 0; c < 2; ++c)
+#pragma unroll
+    for (int i = 0; i < PRE; ++i) pre[c][i] = src[(int64_t)(i < n ? i : 0) * (R + 4) + (c * 256 + tid < R ? c * 256 + tid : 0)];
+  __builtin_amdgcn_sched_barrier(0);
   if (wave == 0) {
     const float* ml = src + (int64_t)(lane < n ? lane : 0) * (R + 4) + R;
     const float m = lane < n ? ml[0] : MASKED, l = ml[1], mx = wave_max(m);
@@ -479,9 +508,18 @@ __global__ __launch_bounds__(256) void latent_out_kernel(LatentArgs a, int E, co
     w_s[lane] = e / den;
   }
   __syncthreads();
-  for (int d = tid; d < R; d += 256) {
+#pragma unroll
+  for (int c = 0; c < 2; ++c) {
+    const int d = c * 256 + tid;
     float v = 0.0f;
-#pragma unroll 8
+#pragma unroll
+    for (int i = 0; i < PRE; ++i) v = fmaf(pre[c][i], w_s[i], v);  // weight zero past the last slice
+    if (d >= R) break;
+    for (int i = PRE; i < n; ++i) v = fmaf(src[(int64_t)i * (R + 4) + d], w_s[i], v);
+    o_s[d] = v;
+  }
+  for (int d = 512 + tid; d < R; d += 256) {
+    float v = 0.0f;
     for (int i = 0; i < n; ++i) v = fmaf(src[(int64_t)i * (R + 4) + d], w_s[i], v);
     o_s[d] = v;
   }

@@ -516,10 +516,38 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const float* z, const T* 
     rows(sw, Fs);
     dot_rows<T, R>(wr, sact + (int64_t)m * Fs, Fs, lane, acc);
   }
-  choose_any(z + (int64_t)m * Ex, Ex, top, lane & 15, [&](int j, int e, float) {
-    rows(w + (int64_t)__builtin_amdgcn_readfirstlane(e) * N * F, F);
-    dot_rows<T, R>(wr, act + ((int64_t)m * top + j) * F, F, lane, acc);
-  });
+  int mine = 0;  // lane j: expert j
+  choose_any(z + (int64_t)m * Ex, Ex, top, lane & 15, [&](int j, int e, float) { mine = lane == j ? e : mine; });
+  // the experts' rows as one sequence of pieces of 512, four pieces together
+  constexpr int U = 4;
+  const int steps = (F + 511) / 512, total = top * steps;
+  int j = 0, st = 0;
+  for (int s0 = 0; s0 < total; s0 += U) {
+    Raw8<T> wv[R][U], xv[U];
+    bool on[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int f = st * 512 + lane * 8, fc = f < F ? f : 0;
+      on[u] = f < F && s0 + u < total;
+      xv[u].load(act + ((int64_t)m * top + j) * F + fc);
+      rows(w + (int64_t)__builtin_amdgcn_readlane(mine, j) * N * F, F);
+#pragma unroll
+      for (int i = 0; i < R; ++i) wv[i][u].load(wr[i] + fc);
+      if (++st == steps) st = 0, j = j + 1 < top ? j + 1 : j;
+    }
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      float f[8], g[8];
+      xv[u].get(f);
+#pragma unroll
+      for (int i = 0; i < R; ++i) {
+        wv[i][u].get(g);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) acc[i] = fmaf(g[e], on[u] ? f[e] : 0.0f, acc[i]);
+      }
+    }
+  }
 #pragma unroll
   for (int i = 0; i < R; ++i) {
     const float s = wave_sum(acc[i]);
@@ -613,7 +641,7 @@ extern "C" int aqs_moe_product(int glu, const void* x, int64_t ldx, int dtype, c
 // whether the two launches below serve these sizes
 extern "C" int aqs_moe_step_ok(int64_t M, int64_t N, int64_t F, int64_t Fs, int64_t Ex, int64_t top) {
   return M > 0 && M <= 8 && N > 0 && N % 8 == 0 && F > 0 && F % 8 == 0 && Fs >= 0 && Fs % 8 == 0 && Ex > 0 && Ex <= MAX_EXPERTS && top > 0 &&
-         top <= Ex;
+         top <= Ex && top <= 64;
 }
 
 // h [M, K], z [M, Ex] logits, w [Ex, 2 F, K] -> act [M * top, F]
